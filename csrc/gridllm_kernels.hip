@@ -21,63 +21,7 @@
 //
 // Build: hipcc --offload-arch=gfx950 -O3 -shared -fPIC
 
-#include <hip/hip_runtime.h>
-#include <math.h>
-#include <float.h>
-
-typedef unsigned short bf16_t;
-typedef unsigned int u32;
-
-#define WAVE 64
-#define DEV_INLINE __device__ __forceinline__
-
-DEV_INLINE float bf2f(bf16_t v) {
-    u32 u = ((u32)v) << 16;
-    return __uint_as_float(u);
-}
-
-DEV_INLINE bf16_t f2bf(float f) {
-    u32 u = __float_as_uint(f);
-    // round-to-nearest-even; NaN-safe (quiet the NaN)
-    if ((u & 0x7fffffffu) > 0x7f800000u) return (bf16_t)0x7fc0;
-    u32 r = (u + 0x7fffu + ((u >> 16) & 1u)) >> 16;
-    return (bf16_t)r;
-}
-
-// unpack 8 bf16 from a uint4 into f32[8]
-DEV_INLINE void unpack8(const uint4 v, float* f) {
-    const u32 w[4] = {v.x, v.y, v.z, v.w};
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        f[2 * i]     = __uint_as_float((w[i] & 0xffffu) << 16);
-        f[2 * i + 1] = __uint_as_float(w[i] & 0xffff0000u);
-    }
-}
-
-// pack f32[8] -> uint4 of 8 bf16
-DEV_INLINE uint4 pack8(const float* f) {
-    uint4 v;
-    u32* w = (u32*)&v;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        u32 lo = (u32)f2bf(f[2 * i]);
-        u32 hi = (u32)f2bf(f[2 * i + 1]);
-        w[i] = lo | (hi << 16);
-    }
-    return v;
-}
-
-DEV_INLINE float wave_reduce_sum(float x) {
-#pragma unroll
-    for (int off = 32; off > 0; off >>= 1) x += __shfl_xor(x, off, WAVE);
-    return x;
-}
-
-DEV_INLINE float wave_reduce_max(float x) {
-#pragma unroll
-    for (int off = 32; off > 0; off >>= 1) x = fmaxf(x, __shfl_xor(x, off, WAVE));
-    return x;
-}
+#include "gridllm_attention.h"
 
 // ===========================================================================
 // RMSNorm (optionally fused residual add):
@@ -183,13 +127,13 @@ k_rope(bf16_t* __restrict__ q, bf16_t* __restrict__ k,
 }
 
 // ===========================================================================
-// SwiGLU: out[n, F] = silu(gateup[n, 0:F]) * gateup[n, F:2F]   (bf16)
+// Gated linear unit: out[n, F] = act(gateup[n, 0:F], gateup[n, F:2F])  (bf16)
 // Fused epilogue for the gate/up projection (one GEMM outputs [n, 2F]).
 // ===========================================================================
 
 __global__ void __launch_bounds__(256)
 k_swiglu(bf16_t* __restrict__ out, const bf16_t* __restrict__ gateup,
-         long n, int F) {
+         long n, int F, const GluParams glu) {
     const int fc = F >> 3;                    // uint4 chunks per half-row
     const long total = n * fc;
     for (long idx = blockIdx.x * 256L + threadIdx.x; idx < total;
@@ -203,9 +147,7 @@ k_swiglu(bf16_t* __restrict__ out, const bf16_t* __restrict__ gateup,
         unpack8(uv, u);
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
-            float x = g[i];
-            float sig = 1.f / (1.f + __expf(-x));
-            g[i] = x * sig * u[i];
+            g[i] = glu_act(g[i], u[i], glu);
         }
         ((uint4*)(out + r * (long)F))[c] = pack8(g);
     }
@@ -285,362 +227,6 @@ k_kv_append(bf16_t* __restrict__ kc, bf16_t* __restrict__ vc,
 }
 
 // ===========================================================================
-// GQA decode attention (flash-decode style).
-//   q:   [B, Hq, D] bf16 (one new token per sequence)
-//   kc/vc: [B, Hk, Smax, D] bf16
-//   seqlen: [B] int32 (number of valid keys, including the current token)
-//   out: [B, Hq, D] bf16
-//   ws (nsplit>1): f32 [B, Hk, G, nsplit, D+2]  (unnormalized acc, m, l)
-//
-// Block = 256 thr = 4 waves, one block per (b, hk, split). Each wave owns
-// key-blocks of 64 (one key per lane), keeps per-(g) online-softmax state,
-// then the 4 waves combine in LDS. G = Hq/Hk (q-heads per kv-head) so each
-// K/V row is read once and reused for all G query heads.
-// Constraints: D in {64, 128}; G <= 8; D % 8 == 0.
-// ===========================================================================
-
-#define MAXG 8
-
-template <int D, int G>
-__global__ void __launch_bounds__(256, 3)
-k_attn_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
-              const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc,
-              const int* __restrict__ seqlen, const int* __restrict__ slot_map,
-              float* __restrict__ ws,
-              int B, int Hk, int Smax, int nsplit, float scale) {
-    const int split = blockIdx.x % nsplit;
-    const int hk = (blockIdx.x / nsplit) % Hk;
-    const int b = blockIdx.x / (nsplit * Hk);
-    const int bc = slot_map ? slot_map[b] : b;   // cache slot for this row
-    const int lane = threadIdx.x & 63;
-    const int wid = threadIdx.x >> 6;
-
-    __shared__ float q_lds[G * D];
-    __shared__ float red[4][G * (D > 64 ? D : 64)];
-    __shared__ float wml[4][G][2];            // per-wave m, l
-
-    const int seq = seqlen[b];
-    // split range, 64-aligned chunks
-    const int chunks = (seq + 63) >> 6;
-    const int per = (chunks + nsplit - 1) / nsplit;
-    const int c0 = split * per;
-    const int c1 = min(chunks, c0 + per);
-    const int s0 = c0 << 6;
-    const int s1 = min(seq, c1 << 6);
-
-    // stage q (scaled) into LDS as f32
-    const int Hq = Hk * G;
-    for (int i = threadIdx.x; i < G * D; i += 256) {
-        int g = i / D, d = i % D;
-        // log2-domain softmax: fold log2(e) into the q prescale so every
-        // exp becomes a native v_exp_f32 exp2 (identical values:
-        // exp2((x-m)*log2e) == exp(x-m))
-        q_lds[i] = bf2f(q[((long)b * Hq + hk * (long)G + g) * D + d])
-                   * (scale * 1.4426950408889634f);
-    }
-    __syncthreads();
-
-    // per-wave online softmax state.
-    // P.V layout: the wave reads RPI = 64/(D/8) V-rows per b128-load
-    // iteration — lane covers row-group rg = lane/DV and d = (lane%DV)*8
-    // + 0..7 — so a 64-key block takes 64/RPI wide-load iterations instead
-    // of 64 row-at-a-time u32 iterations (which measured as a serial
-    // L2-latency chain, 3.2 TB/s). Each lane holds PARTIAL sums over its
-    // row group; one shfl_xor ladder at the end totals them.
-    float m[G], l[G];
-    constexpr int DV = D / 8;          // lanes per V row
-    constexpr int RPI = 64 / DV;       // V rows per iteration
-    float facc[G][8];
-#pragma unroll
-    for (int g = 0; g < G; ++g) {
-        m[g] = -INFINITY;
-        l[g] = 0.f;
-#pragma unroll
-        for (int i = 0; i < 8; ++i) facc[g][i] = 0.f;
-    }
-    const int rg = lane / DV;
-    const int d8 = (lane % DV) * 8;
-
-    const bf16_t* kbase = kc + ((long)bc * Hk + hk) * Smax * D;
-    const bf16_t* vbase = vc + ((long)bc * Hk + hk) * Smax * D;
-
-    for (int kb = s0 + wid * 64; kb < s1; kb += 256) {
-        const int j = kb + lane;
-        const bool valid = j < s1;
-        float s[G];
-#pragma unroll
-        for (int g = 0; g < G; ++g) s[g] = 0.f;
-        if (valid) {
-            const bf16_t* krow = kbase + (long)j * D;
-#pragma unroll
-            for (int dd = 0; dd < D; dd += 8) {
-                uint4 kv = *(const uint4*)(krow + dd);
-                float kf[8];
-                unpack8(kv, kf);
-#pragma unroll
-                for (int g = 0; g < G; ++g) {
-                    float a = 0.f;
-#pragma unroll
-                    for (int i = 0; i < 8; ++i) a += kf[i] * q_lds[g * D + dd + i];
-                    s[g] += a;
-                }
-            }
-        }
-        // online softmax update per g; store p into LDS (reuse red[] rows)
-#pragma unroll
-        for (int g = 0; g < G; ++g) {
-            float sv = valid ? s[g] : -INFINITY;
-            float bmax = wave_reduce_max(sv);
-            float mn = fmaxf(m[g], bmax);
-            // guard: all-invalid block -> bmax=-inf, mn may stay -inf
-            float alpha = (m[g] == -INFINITY) ? 0.f : exp2f(m[g] - mn);
-            float p = (sv == -INFINITY) ? 0.f : exp2f(sv - mn);
-            l[g] = l[g] * alpha + wave_reduce_sum(p);
-            if (mn != m[g]) {          // defer-rescale: skip when max held
-#pragma unroll
-                for (int i = 0; i < 8; ++i) facc[g][i] *= alpha;
-            }
-            m[g] = mn;
-            red[wid][g * 64 + lane] = p;      // per-wave scratch: p for 64 keys
-        }
-        // wave-local LDS visibility (no cross-wave traffic here)
-        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-        // accumulate P·V: RPI rows per iteration, one b128 load per lane
-        const int jmax = min(64, s1 - kb);
-        for (int jb = 0; jb < jmax; jb += RPI) {
-            const int j2 = jb + rg;
-            const uint4 vv = *(const uint4*)(
-                vbase + (long)(kb + min(j2, jmax - 1)) * D + d8);
-            float vf[8];
-            unpack8(vv, vf);
-#pragma unroll
-            for (int g = 0; g < G; ++g) {
-                const float p = (j2 < jmax) ? red[wid][g * 64 + j2] : 0.f;
-#pragma unroll
-                for (int i = 0; i < 8; ++i)
-                    facc[g][i] = fmaf(p, vf[i], facc[g][i]);
-            }
-        }
-    }
-
-    // total each lane's row-group partials: after the ladder every lane
-    // holds the full sum for its d = d8 + 0..7 slice
-#pragma unroll
-    for (int g = 0; g < G; ++g)
-#pragma unroll
-        for (int i = 0; i < 8; ++i)
-#pragma unroll
-            for (int off = 32; off >= DV; off >>= 1)
-                facc[g][i] += __shfl_xor(facc[g][i], off, WAVE);
-
-    // cross-wave combine in LDS
-#pragma unroll
-    for (int g = 0; g < G; ++g) {
-        wml[wid][g][0] = m[g];
-        wml[wid][g][1] = l[g];
-    }
-    __syncthreads();
-#pragma unroll
-    for (int g = 0; g < G; ++g) {
-        float M = fmaxf(fmaxf(wml[0][g][0], wml[1][g][0]),
-                        fmaxf(wml[2][g][0], wml[3][g][0]));
-        float f = (m[g] == -INFINITY) ? 0.f : exp2f(m[g] - M);
-        if (lane < DV)
-#pragma unroll
-            for (int i = 0; i < 8; ++i)
-                red[wid][g * D + d8 + i] = facc[g][i] * f;
-        if (lane == g % 64) wml[wid][g][1] = l[g] * f;  // scaled l (one lane writes)
-    }
-    __syncthreads();
-
-    // final reduction over 4 waves + output
-    for (int i = threadIdx.x; i < G * D; i += 256) {
-        const int g = i / D, d = i % D;
-        float a = red[0][g * D + d] + red[1][g * D + d] +
-                  red[2][g * D + d] + red[3][g * D + d];
-        float L = wml[0][g][1] + wml[1][g][1] + wml[2][g][1] + wml[3][g][1];
-        if (nsplit == 1) {
-            out[((long)b * Hq + hk * (long)G + g) * D + d] =
-                f2bf(L > 0.f ? a / L : 0.f);
-        } else {
-            float M = fmaxf(fmaxf(wml[0][g][0], wml[1][g][0]),
-                            fmaxf(wml[2][g][0], wml[3][g][0]));
-            float* wsp = ws + ((((long)b * Hk + hk) * G + g) * nsplit + split) * (D + 2);
-            wsp[d] = a;
-            if (d == 0) {
-                wsp[D] = M;
-                wsp[D + 1] = L;
-            }
-        }
-    }
-}
-
-// ===========================================================================
-// GQA decode attention, ONE WAVE per (b, hk[, split]) — the large-batch
-// variant. At serving batches B*Hk >= ~2048 the chip holds every block
-// resident (16 waves/CU), so per-wave independence beats the 4-wave
-// cooperative block: no q-staging barrier, no cross-wave LDS combine, no
-// idle waves when seq/64 < 4. Same math as k_attn_decode; V phase reads
-// RPI rows per b128 iteration with an end shfl ladder.
-// ===========================================================================
-
-template <int D, int G>
-__global__ void __launch_bounds__(64, 3)
-k_attn_decode1(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
-               const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc,
-               const int* __restrict__ seqlen,
-               const int* __restrict__ slot_map,
-               float* __restrict__ ws,
-               int B, int Hk, int Smax, int nsplit, float scale) {
-    const int split = blockIdx.x % nsplit;
-    const int hk = (blockIdx.x / nsplit) % Hk;
-    const int b = blockIdx.x / (nsplit * Hk);
-    const int bc = slot_map ? slot_map[b] : b;
-    const int lane = threadIdx.x;
-
-    __shared__ float q_lds[G * D];
-    __shared__ float p_lds[G * 64];
-
-    const int seq = seqlen[b];
-    const int chunks = (seq + 63) >> 6;
-    const int per = (chunks + nsplit - 1) / nsplit;
-    const int s0 = (split * per) << 6;
-    const int s1 = min(seq, (split * per + per) << 6);
-
-    const int Hq = Hk * G;
-    for (int i = lane; i < G * D; i += 64)
-        q_lds[i] = bf2f(q[((long)b * Hq + hk * (long)G + i / D) * D
-                          + i % D]) * (scale * 1.4426950408889634f);
-    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-
-    float m[G], l[G];
-    constexpr int DV = D / 8;
-    constexpr int RPI = 64 / DV;
-    float facc[G][8];
-#pragma unroll
-    for (int g = 0; g < G; ++g) {
-        m[g] = -INFINITY;
-        l[g] = 0.f;
-#pragma unroll
-        for (int i = 0; i < 8; ++i) facc[g][i] = 0.f;
-    }
-    const int rg = lane / DV;
-    const int d8 = (lane % DV) * 8;
-
-    const bf16_t* kbase = kc + ((long)bc * Hk + hk) * (long)Smax * D;
-    const bf16_t* vbase = vc + ((long)bc * Hk + hk) * (long)Smax * D;
-
-    for (int kb = s0; kb < s1; kb += 64) {
-        const int j = kb + lane;
-        const bool valid = j < s1;
-        float s[G];
-#pragma unroll
-        for (int g = 0; g < G; ++g) s[g] = 0.f;
-        if (valid) {
-            const bf16_t* krow = kbase + (long)j * D;
-#pragma unroll
-            for (int dd = 0; dd < D; dd += 8) {
-                uint4 kv = *(const uint4*)(krow + dd);
-                float kf[8];
-                unpack8(kv, kf);
-#pragma unroll
-                for (int g = 0; g < G; ++g) {
-                    float a = 0.f;
-#pragma unroll
-                    for (int i = 0; i < 8; ++i)
-                        a += kf[i] * q_lds[g * D + dd + i];
-                    s[g] += a;
-                }
-            }
-        }
-#pragma unroll
-        for (int g = 0; g < G; ++g) {
-            float sv = valid ? s[g] : -INFINITY;
-            float bmax = wave_reduce_max(sv);
-            float mn = fmaxf(m[g], bmax);
-            float alpha = (m[g] == -INFINITY) ? 0.f : exp2f(m[g] - mn);
-            float p = (sv == -INFINITY) ? 0.f : exp2f(sv - mn);
-            l[g] = l[g] * alpha + wave_reduce_sum(p);
-            if (mn != m[g]) {          // defer-rescale: skip when max held
-#pragma unroll
-                for (int i = 0; i < 8; ++i) facc[g][i] *= alpha;
-            }
-            m[g] = mn;
-            p_lds[g * 64 + lane] = p;
-        }
-        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-        // P.V: RPI rows per b128 iteration; p read from same-wave LDS
-        // (an LDS hop, not shfl: it bounds how far the scheduler can
-        // interleave the K and V phases — shfl spilled 1.5 KB here)
-        const int jmax = min(64, s1 - kb);
-        for (int jb = 0; jb < jmax; jb += RPI) {
-            const int j2 = jb + rg;
-            const uint4 vv = *(const uint4*)(
-                vbase + (long)(kb + min(j2, jmax - 1)) * D + d8);
-            float vf[8];
-            unpack8(vv, vf);
-#pragma unroll
-            for (int g = 0; g < G; ++g) {
-                const float p = (j2 < jmax) ? p_lds[g * 64 + j2] : 0.f;
-#pragma unroll
-                for (int i = 0; i < 8; ++i)
-                    facc[g][i] = fmaf(p, vf[i], facc[g][i]);
-            }
-        }
-    }
-
-#pragma unroll
-    for (int g = 0; g < G; ++g)
-#pragma unroll
-        for (int i = 0; i < 8; ++i)
-#pragma unroll
-            for (int off = 32; off >= DV; off >>= 1)
-                facc[g][i] += __shfl_xor(facc[g][i], off, WAVE);
-
-    if (lane < DV) {
-#pragma unroll
-        for (int g = 0; g < G; ++g) {
-            if (nsplit == 1) {
-                const float L = l[g];
-#pragma unroll
-                for (int i = 0; i < 8; ++i)
-                    out[((long)b * Hq + hk * (long)G + g) * D + d8 + i] =
-                        f2bf(L > 0.f ? facc[g][i] / L : 0.f);
-            } else {
-                float* wsp = ws + ((((long)b * Hk + hk) * G + g) * nsplit
-                                   + split) * (D + 2);
-#pragma unroll
-                for (int i = 0; i < 8; ++i) wsp[d8 + i] = facc[g][i];
-                if (lane == 0) {
-                    wsp[D] = m[g];
-                    wsp[D + 1] = l[g];
-                }
-            }
-        }
-    }
-}
-
-// Combine split-S partials: grid = B*Hq blocks, D threads.
-__global__ void
-k_attn_combine(bf16_t* __restrict__ out, const float* __restrict__ ws,
-               int Hq, int D, int nsplit) {
-    const long bh = blockIdx.x;               // b*Hq + hq  == (b*Hk + hk)*G + g
-    const int d = threadIdx.x;
-    const float* base = ws + bh * (long)nsplit * (D + 2);
-    float M = -INFINITY;
-    for (int s = 0; s < nsplit; ++s) M = fmaxf(M, base[s * (D + 2) + D]);
-    float num = 0.f, den = 0.f;
-    for (int s = 0; s < nsplit; ++s) {
-        const float* p = base + s * (long)(D + 2);
-        float ms = p[D];
-        float f = (ms == -INFINITY) ? 0.f : exp2f(ms - M);
-        num += f * p[d];
-        den += f * p[D + 1];
-    }
-    out[bh * D + d] = f2bf(den > 0.f ? num / den : 0.f);
-}
-
-// ===========================================================================
 // Skinny-M weight-streaming GEMM:  out[M,N] = x[M,K] @ W[N,K]^T   (bf16 I/O)
 //
 // The decode-path projection GEMMs (M = batch <= 256, W = torch linear
@@ -660,9 +246,6 @@ k_attn_combine(bf16_t* __restrict__ out, const float* __restrict__ ws,
 // partials in ws, combined by k_gemm_combine.
 // Constraints: N % 64 == 0, K % 32 == 0, M <= 16*MT.
 // ===========================================================================
-
-typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
-typedef __attribute__((ext_vector_type(4))) float f32x4;
 
 template <int MT>
 __global__ void __launch_bounds__(256, 2)
@@ -784,11 +367,7 @@ k_gemm_skinny(bf16_t* __restrict__ out, float* __restrict__ ws,
 // Constraints: N % 128 == 0 (64 at MT=4), K % 64 == 0, kslice % 64 == 0.
 // ===========================================================================
 
-DEV_INLINE float silu_mul(float g, float u) {
-    return g * (1.f / (1.f + __expf(-g))) * u;
-}
-
-// EPI: 0 = plain store; 1 = fused SwiGLU epilogue — W rows are interleaved
+// EPI: 0 = plain store; 1 = fused gated-linear-unit epilogue — W rows are interleaved
 // in 128-row groups [64 gate | 64 up] so each BN=128 block holds matching
 // gate/up column pairs and writes out[M, N/2] = silu(g)*u directly (the
 // separate k_swiglu pass and its gateup HBM round trip disappear).
@@ -796,7 +375,8 @@ template <int MT, int BN, int NB, int EPI = 0, int WAVES = 8, int BK = 64>
 __global__ void __launch_bounds__(WAVES * 64)
 k_gemm_proj(bf16_t* __restrict__ out, float* __restrict__ ws,
             const bf16_t* __restrict__ x, const bf16_t* __restrict__ w,
-            int M, int N, int K, int splitk, int kslice) {
+            int M, int N, int K, int splitk, int kslice,
+            const GluParams glu) {
     constexpr int R = WAVES * 16 * MT;  // x rows staged (>= M)
     constexpr int XI = R * BK / (512 * WAVES);   // x glds per wave per tile
     constexpr int WI = BN * BK / (512 * WAVES);  // w glds per wave per tile
@@ -927,8 +507,8 @@ k_gemm_proj(bf16_t* __restrict__ out, float* __restrict__ ws,
                     const int m = m0 + (wid * MT + t) * 16 + orow0 + r;
                     if (m < M)
                         out[(long)m * (N >> 1) + (n0 >> 1) + c * 16 + fr] =
-                            f2bf(silu_mul(acc[t][c][r],
-                                          acc[t][c + BN / 32][r]));
+                            f2bf(glu_act(acc[t][c][r],
+                                         acc[t][c + BN / 32][r], glu));
                 }
         return;
     }
@@ -954,18 +534,19 @@ k_gemm_proj(bf16_t* __restrict__ out, float* __restrict__ ws,
 template <int MT, int BN, int NB, int EPI = 0, int WAVES = 8, int BK = 64>
 static void launch_gemm_proj(hipStream_t st, bf16_t* out, float* ws,
                              const bf16_t* x, const bf16_t* w, int M, int N,
-                             int K, int splitk, int kslice, int mtiles = 1) {
+                             int K, int splitk, int kslice, int mtiles = 1,
+                             const GluParams glu = {1.f, INFINITY, 0.f}) {
     dim3 grid((unsigned)((N / BN) * splitk), (unsigned)mtiles),
         blk(WAVES * 64);
     k_gemm_proj<MT, BN, NB, EPI, WAVES, BK><<<grid, blk, 0, st>>>(
-        out, ws, x, w, M, N, K, splitk, kslice);
+        out, ws, x, w, M, N, K, splitk, kslice, glu);
 }
 
 // Combine split-K slabs of an INTERLEAVED gate/up projection with the
 // SwiGLU epilogue applied during the combine: out[M, N/2] bf16.
 __global__ void __launch_bounds__(256)
 k_gemm_combine_swiglu(bf16_t* __restrict__ out, const float* __restrict__ ws,
-                      int M, int N, int splitk) {
+                      int M, int N, int splitk, const GluParams glu) {
     const int no = N >> 1;
     const long mn = (long)M * N;
     const long total = (long)M * (no >> 1);       // u32 (2-col) units
@@ -980,8 +561,8 @@ k_gemm_combine_swiglu(bf16_t* __restrict__ out, const float* __restrict__ ws,
             const float* p = ws + (long)k * mn + gidx;
             g0 += p[0]; g1 += p[1]; u0 += p[64]; u1 += p[65];
         }
-        u32 lo = (u32)f2bf(silu_mul(g0, u0)) |
-                 ((u32)f2bf(silu_mul(g1, u1)) << 16);
+        u32 lo = (u32)f2bf(glu_act(g0, u0, glu)) |
+                 ((u32)f2bf(glu_act(g1, u1, glu)) << 16);
         *(u32*)(out + m * (long)no + j) = lo;
     }
 }
@@ -991,7 +572,7 @@ k_gemm_combine_swiglu(bf16_t* __restrict__ out, const float* __restrict__ ws,
 // weights: out[n, F] from gu[n, 2F].
 __global__ void __launch_bounds__(256)
 k_swiglu_il(bf16_t* __restrict__ out, const bf16_t* __restrict__ gu,
-            long n, int F) {
+            long n, int F, const GluParams glu) {
     const int fc = F >> 3;                        // 8-col units per out row
     const long total = n * fc;
     for (long idx = blockIdx.x * 256L + threadIdx.x; idx < total;
@@ -1006,7 +587,7 @@ k_swiglu_il(bf16_t* __restrict__ out, const bf16_t* __restrict__ gu,
         unpack8(gv, g);
         unpack8(uv, u);
 #pragma unroll
-        for (int i = 0; i < 8; ++i) g[i] = silu_mul(g[i], u[i]);
+        for (int i = 0; i < 8; ++i) g[i] = glu_act(g[i], u[i], glu);
         ((uint4*)(out + r * (long)F))[j >> 3] = pack8(g);
     }
 }
@@ -1028,187 +609,6 @@ k_gemm_combine(bf16_t* __restrict__ out, const float* __restrict__ ws,
     }
 }
 
-// ===========================================================================
-// GQA prefill attention — flash-style on MFMA (bf16), reads K/V straight
-// from the slot cache (no permuted host-side views).
-//   q:   [T, Hq, D] bf16 (roped)
-//   kc/vc: [slots, Hk, Smax, D] bf16
-//   out: [T, Hq, D] bf16
-// Workgroup = 4 waves; wave w owns 32 q-rows (q0 + w*32) of ONE q-head;
-// K/V walked in 32-row tiles with online softmax (guide App. B prefill).
-//
-// Layout trick (guide §5.5 "swapped QK^T"): S^T = mfma(A=K, B=Q) puts a
-// whole q-row's scores in ONE lane (C col = lane&31 = q), so the softmax
-// row-reduce is 15 in-register fmax + one shfl_xor(32) — no LDS. P is then
-// routed to the PV MFMA's B-operand layout through a per-wave LDS scratch
-// (paired b32 writes -> b128 fragment reads, same-wave lgkmcnt wait only),
-// and O^T = mfma(A=V^T, B=P) accumulates with V staged TRANSPOSED in LDS
-// (transpose once per tile, cooperative; A-fragments then read b128-clean).
-// mfma_f32_32x32x16_bf16 maps (guide §3):
-//   A[i][k]: lane l holds i = l&31, k = (l>>5)*8 + 0..7
-//   B[k][j]: lane l holds j = l&31, same k chunk
-//   C/D[i][j]: col j = l&31, row i = (reg&3) + 8*(reg>>2) + 4*(l>>5)
-// Constraints: D in {64, 128}; Hq % Hk == 0.
-// ===========================================================================
-
-typedef __attribute__((ext_vector_type(16))) float f32x16;
-
-// Shared body: one 128-q-row tile of one q-head for one sequence.
-// q0 = first q row of this tile; vt/plds = caller's LDS buffers.
-template <int D>
-__device__ __forceinline__ void
-attn_prefill_tile(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
-                  const bf16_t* __restrict__ kc,
-                  const bf16_t* __restrict__ vc,
-                  int T, int Hq, int G, int Hk, int Smax, int slot,
-                  int s_total, int causal_off, float scale, int q0,
-                  bf16_t* vt, bf16_t* plds_all) {
-    constexpr int NS = D / 16;     // 16-wide d slices (QK^T fragments)
-    constexpr int NT = D / 32;     // 32-wide d tiles (output / V^T)
-    constexpr int VST = 40;        // padded k-stride of V^T tile (16B-mult)
-
-    const int lane = threadIdx.x & 63;
-    const int wid = threadIdx.x >> 6;
-    const int hi = lane >> 5;
-    const int ln = lane & 31;
-    const int hq = blockIdx.y;
-    const int hk = hq / G;
-    const int qw = q0 + wid * 32;
-
-    const bf16_t* kbase = kc + ((long)slot * Hk + hk) * (long)Smax * D;
-    const bf16_t* vbase = vc + ((long)slot * Hk + hk) * (long)Smax * D;
-
-    // Q fragments: lane holds Q[qw+ln][s*16 + hi*8 + 0..7] (B operand)
-    bf16x8 qf[NS];
-    {
-        const bf16_t* qrow =
-            q + ((long)min(qw + ln, T - 1) * Hq + hq) * D + hi * 8;
-#pragma unroll
-        for (int s = 0; s < NS; ++s) qf[s] = *(const bf16x8*)(qrow + s * 16);
-    }
-
-    const int q_abs = causal_off + qw + ln;   // this lane's absolute q pos
-    float m = -INFINITY, l = 0.f;
-    f32x16 acc[NT];
-#pragma unroll
-    for (int t = 0; t < NT; ++t)
-#pragma unroll
-        for (int r = 0; r < 16; ++r) acc[t][r] = 0.f;
-
-    // causal upper bound for the workgroup's LAST q-row
-    const int kmax = min(s_total, causal_off + q0 + 128);
-
-    for (int k0 = 0; k0 < kmax; k0 += 32) {
-        // ---- stage V^T tile (cooperative transpose) --------------------
-        __syncthreads();               // previous tile's vt readers done
-        {
-            constexpr int CPR = D / 8;            // b128 chunks per V row
-            for (int c = threadIdx.x; c < 32 * CPR; c += 256) {
-                const int kr = c / CPR;
-                const int d8 = (c % CPR) * 8;
-                uint4 v = *(const uint4*)(
-                    vbase + (long)min(k0 + kr, s_total - 1) * D + d8);
-                const bf16_t* pv = (const bf16_t*)&v;
-#pragma unroll
-                for (int j = 0; j < 8; ++j) vt[(d8 + j) * VST + kr] = pv[j];
-            }
-        }
-        __syncthreads();
-
-        // ---- S^T = K·Q^T (K fragments straight from HBM/L2) ------------
-        f32x16 s_acc;
-#pragma unroll
-        for (int r = 0; r < 16; ++r) s_acc[r] = 0.f;
-        {
-            const bf16_t* krow =
-                kbase + (long)min(k0 + ln, s_total - 1) * D + hi * 8;
-#pragma unroll
-            for (int s = 0; s < NS; ++s) {
-                const bf16x8 kf = *(const bf16x8*)(krow + s * 16);
-                s_acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(
-                    kf, qf[s], s_acc, 0, 0, 0);
-            }
-        }
-
-        // ---- mask + online softmax (lane owns one q-row) ---------------
-        float sv[16], tmax = -INFINITY;
-        const float scl2 = scale * 1.4426950408889634f;   // log2 domain
-#pragma unroll
-        for (int r = 0; r < 16; ++r) {
-            const int kg = k0 + (r & 3) + 8 * (r >> 2) + 4 * hi;
-            const bool ok = (kg < s_total) && (kg <= q_abs);
-            sv[r] = ok ? s_acc[r] * scl2 : -INFINITY;
-            tmax = fmaxf(tmax, sv[r]);
-        }
-        tmax = fmaxf(tmax, __shfl_xor(tmax, 32, WAVE));
-        const float mn = fmaxf(m, tmax);
-        const float alpha = (m == -INFINITY) ? 0.f : exp2f(m - mn);
-        float p[16], psum = 0.f;
-#pragma unroll
-        for (int r = 0; r < 16; ++r) {
-            p[r] = (sv[r] == -INFINITY) ? 0.f : exp2f(sv[r] - mn);
-            psum += p[r];
-        }
-        psum += __shfl_xor(psum, 32, WAVE);
-        l = l * alpha + psum;
-        m = mn;
-
-        // ---- P -> PV B-fragment layout via per-wave LDS scratch --------
-        // (kpos, q=ln) lands where slice sidx = kpos>>4, lane
-        // lr = ln + 32*((kpos>>3)&1), word i = kpos&7 will read it; regs
-        // pair (r, r+1) = (kpos, kpos+1) -> one packed b32 write.
-        bf16_t* ps = plds_all + wid * (2 * 64 * 8);
-#pragma unroll
-        for (int r = 0; r < 16; r += 2) {
-            const int kpos = (r & 3) + 8 * (r >> 2) + 4 * hi;
-            const int sidx = kpos >> 4;
-            const int lr = ln + 32 * ((kpos >> 3) & 1);
-            u32 w = (u32)f2bf(p[r]) | ((u32)f2bf(p[r + 1]) << 16);
-            *(u32*)(ps + (sidx * 64 + lr) * 8 + (kpos & 7)) = w;
-        }
-        // rescale output accumulators while the P writes land
-#pragma unroll
-        for (int t = 0; t < NT; ++t)
-#pragma unroll
-            for (int r = 0; r < 16; ++r) acc[t][r] *= alpha;
-        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-
-        // ---- O^T += V^T · P --------------------------------------------
-        bf16x8 pf[2];
-#pragma unroll
-        for (int s = 0; s < 2; ++s)
-            pf[s] = *(const bf16x8*)(ps + (s * 64 + lane) * 8);
-#pragma unroll
-        for (int t = 0; t < NT; ++t) {
-            const bf16_t* vrow = vt + (t * 32 + ln) * VST + hi * 8;
-#pragma unroll
-            for (int s = 0; s < 2; ++s) {
-                const bf16x8 vf = *(const bf16x8*)(vrow + s * 16);
-                acc[t] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(
-                    vf, pf[s], acc[t], 0, 0, 0);
-            }
-        }
-    }
-
-    // ---- normalize + store: lane holds O^T[*][q=ln] — one q-row --------
-    if (qw + ln < T) {
-        const float inv = (l > 0.f) ? 1.f / l : 0.f;
-        bf16_t* orow = out + ((long)(qw + ln) * Hq + hq) * D;
-#pragma unroll
-        for (int t = 0; t < NT; ++t) {
-#pragma unroll
-            for (int g = 0; g < 4; ++g) {
-                const int d = t * 32 + 8 * g + 4 * hi;
-                u32 lo = (u32)f2bf(acc[t][4 * g] * inv) |
-                         ((u32)f2bf(acc[t][4 * g + 1] * inv) << 16);
-                u32 h2 = (u32)f2bf(acc[t][4 * g + 2] * inv) |
-                         ((u32)f2bf(acc[t][4 * g + 3] * inv) << 16);
-                *(uint2*)(orow + d) = make_uint2(lo, h2);
-            }
-        }
-    }
-}
-
 template <int D>
 __global__ void __launch_bounds__(256, 2)
 k_attn_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
@@ -1218,9 +618,10 @@ k_attn_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
     constexpr int VST = 40;
     __shared__ __attribute__((aligned(16))) bf16_t vt[D * VST];
     __shared__ __attribute__((aligned(16))) bf16_t plds[4][2 * 64 * 8];
-    attn_prefill_tile<D>(out, q, kc, vc, T, Hq, G, Hk, Smax, slot, s_total,
-                         causal_off, scale, blockIdx.x * 128, vt,
-                         &plds[0][0]);
+    const SlotKV<D> kv{kc, vc, Hk, Smax};
+    const HeadEpilogue epi{nullptr, nullptr, 0};
+    attn_prefill_tile<D>(out, q, kv, T, Hq, G, slot, s_total, causal_off,
+                         scale, blockIdx.x * 128, vt, &plds[0][0], epi, 0);
 }
 
 // ===========================================================================
@@ -1244,9 +645,11 @@ k_attn_prefill_batch(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
     __shared__ __attribute__((aligned(16))) bf16_t vt[D * VST];
     __shared__ __attribute__((aligned(16))) bf16_t plds[4][2 * 64 * 8];
     const int4 m = meta[blockIdx.x];
+    const SlotKV<D> kv{kc, vc, Hk, Smax};
+    const HeadEpilogue epi{nullptr, nullptr, 0};
     attn_prefill_tile<D>(out + (long)m.x * Hq * D, q + (long)m.x * Hq * D,
-                         kc, vc, m.y, Hq, G, Hk, Smax, m.z, m.y,
-                         /*causal_off=*/0, scale, m.w, vt, &plds[0][0]);
+                         kv, m.y, Hq, G, m.z, m.y, /*causal_off=*/0, scale,
+                         m.w, vt, &plds[0][0], epi, 0);
 }
 
 template <int MT>
@@ -1329,9 +732,6 @@ __global__ __launch_bounds__(256, 4) void k_sample_gumbel(
 // All return hipError_t as int (0 == success); callers must check.
 // ===========================================================================
 
-#define LAUNCH_CHECK() do { hipError_t e = hipGetLastError(); \
-    if (e != hipSuccess) return (int)e; } while (0)
-
 template <int D>
 static int launch_attn_decode(hipStream_t st, bf16_t* out, const bf16_t* q,
                               const bf16_t* kc, const bf16_t* vc,
@@ -1343,14 +743,15 @@ static int launch_attn_decode(hipStream_t st, bf16_t* out, const bf16_t* q,
     // yields nsplit==1 whenever B*Hk >= 512, so this is the common case;
     // explicit nsplit>1 calls keep the 4-wave cooperative kernel)
     const bool onewave = nsplit == 1 && (B * Hk) >= 2048;
+    const SlotKV<D> kv{kc, vc, Hk, Smax};
+    const HeadEpilogue epi{nullptr, nullptr, 0};
     switch (G) {   // compile-time G keeps softmax state in registers
 #define CASE_G(GG) \
         case GG: if (onewave) k_attn_decode1<D, GG><<<grid, dim3(64), 0, st>>>( \
-                out, q, kc, vc, seqlen, slot_map, ws, B, Hk, Smax, nsplit, \
-                scale); \
+                out, q, kv, seqlen, 0, slot_map, ws, 1, nsplit, scale, epi); \
             else k_attn_decode<D, GG><<<grid, dim3(256), 0, st>>>( \
-                out, q, kc, vc, seqlen, slot_map, ws, B, Hk, Smax, nsplit, \
-                scale); break;
+                out, q, kv, seqlen, 0, slot_map, ws, 1, nsplit, scale, epi); \
+            break;
         CASE_G(1) CASE_G(2) CASE_G(3) CASE_G(4)
         CASE_G(5) CASE_G(6) CASE_G(7) CASE_G(8)
 #undef CASE_G
@@ -1384,13 +785,15 @@ int gl_rope(void* stream, void* q, void* k, const void* cost, const void* sint,
     return 0;
 }
 
-int gl_swiglu(void* stream, void* out, const void* gateup, long n, int f) {
+int gl_swiglu(void* stream, void* out, const void* gateup, long n, int f,
+              float alpha, float limit, float shift) {
     if (f % 8 != 0) return -100;
     long total = n * (f / 8);
     int grid = (int)min((total + 255) / 256, (long)2048);
     if (grid == 0) return 0;
     k_swiglu<<<dim3(grid), dim3(256), 0, (hipStream_t)stream>>>(
-        (bf16_t*)out, (const bf16_t*)gateup, n, f);
+        (bf16_t*)out, (const bf16_t*)gateup, n, f,
+        GluParams{alpha, limit, shift});
     LAUNCH_CHECK();
     return 0;
 }
@@ -1444,7 +847,8 @@ int gl_attn_decode(void* stream, void* out, const void* q, const void* kc,
     LAUNCH_CHECK();
     if (nsplit > 1) {
         k_attn_combine<<<dim3((unsigned)(B * Hq)), dim3(D), 0, st>>>(
-            (bf16_t*)out, (const float*)ws, Hq, D, nsplit);
+            (bf16_t*)out, (const float*)ws, Hq, D, nsplit,
+            HeadEpilogue{nullptr, nullptr, 0});
         LAUNCH_CHECK();
     }
     return 0;
@@ -1478,7 +882,9 @@ int gl_gemm_skinny(void* stream, void* out, void* ws, const void* x,
 
 int gl_gemm_proj(void* stream, void* out, void* ws, const void* x,
                  const void* w, int M, int N, int K, int splitk,
-                 int kslice, int fuse_swiglu, int variant, int mtiles) {
+                 int kslice, int fuse_swiglu, int variant, int mtiles,
+                 float alpha, float limit, float shift) {
+    const GluParams glu{alpha, limit, shift};
     if (K % 64 != 0 || kslice % 64 != 0) return -100;
     // m-tiled variant bounds ROWS PER TILE, not M: serving buckets 768/
     // 1024 hit hipBLASLt fallbacks measured at 0.7-1.6 TB/s (r02j b768
@@ -1497,21 +903,21 @@ int gl_gemm_proj(void* stream, void* out, void* ws, const void* x,
             if (rpt <= 64)
                 launch_gemm_proj<1, 128, 3, 1, 4>(st, (bf16_t*)out,
                     (float*)ws, (const bf16_t*)x, (const bf16_t*)w,
-                    M, N, K, splitk, kslice, mtiles);
+                    M, N, K, splitk, kslice, mtiles, glu);
             else if (rpt <= 128)
                 launch_gemm_proj<1, 128, 3, 1>(st, (bf16_t*)out, (float*)ws,
                     (const bf16_t*)x, (const bf16_t*)w, M, N, K, splitk,
-                    kslice, mtiles);
+                    kslice, mtiles, glu);
             else
                 launch_gemm_proj<2, 128, 3, 1>(st, (bf16_t*)out, (float*)ws,
                     (const bf16_t*)x, (const bf16_t*)w, M, N, K, splitk,
-                    kslice, mtiles);
+                    kslice, mtiles, glu);
             LAUNCH_CHECK();
             if (splitk > 1) {
                 long chunks = ((long)M * (N >> 2) + 255) / 256;
                 int grid = (int)min(chunks, (long)2048);
                 k_gemm_combine_swiglu<<<dim3(grid), dim3(256), 0, st>>>(
-                    (bf16_t*)out, (const float*)ws, M, N, splitk);
+                    (bf16_t*)out, (const float*)ws, M, N, splitk, glu);
                 LAUNCH_CHECK();
             }
             return 0;
@@ -1616,16 +1022,18 @@ int gl_gemm_proj(void* stream, void* out, void* ws, const void* x,
     if (fuse_swiglu) {
         if (mt <= 1)
             launch_gemm_proj<1, 128, 3, 1>(st, (bf16_t*)out, (float*)ws,
-                (const bf16_t*)x, (const bf16_t*)w, M, N, K, splitk, kslice);
+                (const bf16_t*)x, (const bf16_t*)w, M, N, K, splitk, kslice,
+                1, glu);
         else
             launch_gemm_proj<2, 128, 3, 1>(st, (bf16_t*)out, (float*)ws,
-                (const bf16_t*)x, (const bf16_t*)w, M, N, K, splitk, kslice);
+                (const bf16_t*)x, (const bf16_t*)w, M, N, K, splitk, kslice,
+                1, glu);
         LAUNCH_CHECK();
         if (splitk > 1) {
             long chunks = ((long)M * (N >> 2) + 255) / 256;
             int grid = (int)min(chunks, (long)2048);
             k_gemm_combine_swiglu<<<dim3(grid), dim3(256), 0, st>>>(
-                (bf16_t*)out, (const float*)ws, M, N, splitk);
+                (bf16_t*)out, (const float*)ws, M, N, splitk, glu);
             LAUNCH_CHECK();
         }
         return 0;
@@ -1661,13 +1069,15 @@ int gl_sample_gumbel(void* stream, void* out, const void* logits,
     return 0;
 }
 
-int gl_swiglu_il(void* stream, void* out, const void* gu, long n, int f) {
+int gl_swiglu_il(void* stream, void* out, const void* gu, long n, int f,
+                 float alpha, float limit, float shift) {
     if (f % 64 != 0) return -100;
     hipStream_t st = (hipStream_t)stream;
     long total = n * (f >> 3);
     int grid = (int)min((total + 255) / 256, (long)4096);
     k_swiglu_il<<<dim3(grid), dim3(256), 0, st>>>(
-        (bf16_t*)out, (const bf16_t*)gu, n, f);
+        (bf16_t*)out, (const bf16_t*)gu, n, f,
+        GluParams{alpha, limit, shift});
     LAUNCH_CHECK();
     return 0;
 }

@@ -182,6 +182,15 @@ class LlamaModel:
                 attn_norm=torch.ones(s.hidden, dtype=self.dtype, device=self.device),
                 mlp_norm=torch.ones(s.hidden, dtype=self.dtype, device=self.device)))
 
+    def gemm_shapes(self) -> tuple[list, list]:
+        """(n, k) of the decode projections, and of the gate/up ones."""
+        s, d = self.spec, self.spec.head_dim
+        return ([((self.hq_l + 2 * self.hkv_l) * d, s.hidden),   # qkv
+                 (s.hidden, self.hq_l * d),                      # o
+                 (s.hidden, self.f_l),                           # down
+                 (s.vocab, s.hidden)],                           # lm_head
+                [(2 * self.f_l, s.hidden)])
+
     def interleave_gateup(self) -> None:
         """Reorder each wgateup's rows into 128-row groups [64 gate |
         64 up] so the fused-SwiGLU projection kernel (ops.gemm_proj with

@@ -12,6 +12,7 @@ from typing import Optional, Tuple
 import torch
 
 from gridllm_amd.ops import reference
+from gridllm_amd.ops.reference import SWIGLU, Glu
 from gridllm_amd.ops.hip_ops import HipExtensionMissing, available as hip_available
 
 __all__ = [
@@ -58,11 +59,11 @@ def rope_kv(qkv: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
                              hq, hk, d)
 
 
-def swiglu(gateup: torch.Tensor) -> torch.Tensor:
+def swiglu(gateup: torch.Tensor, glu: Glu = SWIGLU) -> torch.Tensor:
     if _on_gpu(gateup):
         from gridllm_amd.ops import hip_ops
-        return hip_ops.swiglu(gateup)
-    return reference.swiglu(gateup)
+        return hip_ops.swiglu(gateup, glu=glu)
+    return reference.swiglu(gateup, glu)
 
 
 def kv_append(kcache: torch.Tensor, vcache: torch.Tensor, k_new: torch.Tensor,

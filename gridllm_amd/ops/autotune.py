@@ -17,6 +17,7 @@ import torch
 import torch.nn.functional as F
 
 from gridllm_amd.ops import hip_ops
+from gridllm_amd.ops.reference import SWIGLU, Glu
 from gridllm_amd.utils.logging import get_logger
 
 log = get_logger("autotune")
@@ -164,16 +165,18 @@ def tune_gateup(m: int, n: int, k: int, device) -> tuple[str, int]:
     return best
 
 
-def linear_gateup(x: torch.Tensor, w_il: torch.Tensor) -> torch.Tensor:
-    """Fused gate/up projection + SwiGLU on an INTERLEAVED weight:
+def linear_gateup(x: torch.Tensor, w_il: torch.Tensor,
+                  glu: Glu = SWIGLU) -> torch.Tensor:
+    """Fused gate/up projection + gated linear unit on an INTERLEAVED weight:
     returns [M, F] activated. Dispatches through the tuned table."""
     c = _CHOICE_GU.get((x.shape[0], w_il.shape[0], w_il.shape[1]))
     if c is not None and c[0] == "proj":
-        return hip_ops.gemm_proj(x, w_il, splitk=c[1], fuse_swiglu=True)
+        return hip_ops.gemm_proj(x, w_il, splitk=c[1], fuse_swiglu=True,
+                                 glu=glu)
     if c is not None and c[0] == "projm":
         return hip_ops.gemm_proj(x, w_il, splitk=c[1], fuse_swiglu=True,
-                                 mtiles=c[2])
-    return hip_ops.swiglu_il(F.linear(x, w_il))
+                                 mtiles=c[2], glu=glu)
+    return hip_ops.swiglu_il(F.linear(x, w_il), glu=glu)
 
 
 def choice(m: int, n: int, k: int) -> Optional[tuple[str, int]]:
@@ -197,25 +200,18 @@ def linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
 
 
 def tune_model_shapes(model, buckets) -> None:
-    """Pre-tune every decode GEMM shape for the given batch buckets."""
-    s = model.spec
-    d = s.head_dim
-    shapes = [
-        ((s.heads // model.tp.size + 2 * (s.kv_heads // model.tp.size)) * d,
-         s.hidden),                               # qkv
-        (s.hidden, (s.heads // model.tp.size) * d),   # o
-        (s.hidden, s.intermediate // model.tp.size),      # down
-        (s.vocab, s.hidden),                      # lm_head
-    ]
-    gu_shape = (2 * s.intermediate // model.tp.size, s.hidden)
+    """Pre-tune every decode GEMM shape for the given batch buckets. The
+    model lists its plain projections and its gate/up projections as (n, k)."""
+    shapes, gu_shapes = model.gemm_shapes()
     t0 = time.monotonic()
     for m in buckets:
         for n, k in shapes:
             tune_shape(m, n, k, model.device)
-        if getattr(model, "gateup_il", False):
-            tune_gateup(m, gu_shape[0], gu_shape[1], model.device)
-        else:
-            tune_shape(m, gu_shape[0], gu_shape[1], model.device)
+        for n, k in gu_shapes:
+            if getattr(model, "gateup_il", False):
+                tune_gateup(m, n, k, model.device)
+            else:
+                tune_shape(m, n, k, model.device)
     picked = sum(1 for v in _CHOICE.values() if v[0] == "ours")
     log.performance("gemm autotune done", shapes=len(_CHOICE),
                     ours=picked, ms=int((time.monotonic() - t0) * 1000))

@@ -1,55 +1,80 @@
-"""In-tree build of the HIP kernel library for gfx950.
+"""In-tree build of the HIP kernel libraries for gfx950.
 
-Builds csrc/gridllm_kernels.hip -> gridllm_amd/ops/libgridllm_hip.so with a
-direct hipcc invocation (no hipify, no CUDA-compat layer). The .so is
-git-ignored but ships with the repo snapshot to GPU boxes.
+Each entry of LIBS is one source under csrc/ and the shared library it
+becomes next to this file, by a direct hipcc invocation (no hipify, no
+CUDA-compat layer). The libraries are git-ignored. Libraries are compiled in
+parallel; a file lock keeps two processes from building the same one.
 """
 
 from __future__ import annotations
 
+import fcntl
+import glob
 import os
 import subprocess
 import sys
+from concurrent.futures import ThreadPoolExecutor
+from typing import Iterable, Optional
 
 PKG_DIR = os.path.dirname(os.path.abspath(__file__))
 REPO_ROOT = os.path.dirname(os.path.dirname(PKG_DIR))
-SRC = os.path.join(REPO_ROOT, "csrc", "gridllm_kernels.hip")
-OUT = os.path.join(PKG_DIR, "libgridllm_hip.so")
+CSRC = os.path.join(REPO_ROOT, "csrc")
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950")
 
+# library name -> source. "hip": what every model shares and the Llama
+# family's attention; "hybrid": layer-list models (paged attention, mLSTM,
+# routed experts)
+LIBS = {"hip": "gridllm_kernels.hip"}
 
-def needs_build() -> bool:
-    if not os.path.exists(OUT):
+# hipcc otherwise forms packed-FP32 instructions from plain float code; some
+# of their forms give wrong results on this hardware, so all HIP code is
+# compiled without the feature (the host pass warns that it does not know it)
+FLAGS = [f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-shared", "-fPIC",
+         "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+
+
+def lib_path(name: str) -> str:
+    return os.path.join(PKG_DIR, f"libgridllm_{name}.so")
+
+
+def needs_build(name: str) -> bool:
+    out = lib_path(name)
+    if not os.path.exists(out):
         return True
-    return os.path.getmtime(SRC) > os.path.getmtime(OUT)
+    srcs = [os.path.join(CSRC, LIBS[name])] + glob.glob(
+        os.path.join(CSRC, "*.h"))
+    return max(map(os.path.getmtime, srcs)) > os.path.getmtime(out)
 
 
-def build(force: bool = False, asan: bool = False) -> str:
-    """asan=True (or GRIDLLM_ASAN=1): AddressSanitizer on the HOST side
-    of the library (launch wrappers, workspace sizing, pointer math) —
-    the sanitizer pass the round-1 verdict asked for (weak 7). Run the
-    process with the ASan runtime preloaded: scripts/asan_check.sh."""
-    asan = asan or os.environ.get("GRIDLLM_ASAN") == "1"
-    out = OUT if not asan else OUT.replace(".so", ".asan.so")
-    if not force and not asan and not needs_build():
+def _build_one(name: str, force: bool) -> str:
+    out = lib_path(name)
+    if not force and not needs_build(name):
         return out
-    cmd = [
-        HIPCC, f"--offload-arch={ARCH}", "-O3", "-std=c++17",
-        "-shared", "-fPIC", SRC, "-o", out,
-    ]
-    if asan:
-        # host-code ASan only: device code is exercised by the
-        # GRIDLLM_VALIDATE pre-launch range checks + numerics tests
-        cmd.insert(4, "-fsanitize=address")
-        cmd.insert(5, "-shared-libsan")
-    proc = subprocess.run(cmd, capture_output=True, text=True)
-    if proc.returncode != 0:
-        raise RuntimeError(
-            f"hipcc build failed (rc={proc.returncode}):\n{proc.stderr[-4000:]}")
+    with open(out + ".lock", "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        if not force and not needs_build(name):
+            return out                  # another process has just built it
+        tmp = f"{out}.{os.getpid()}"
+        proc = subprocess.run(
+            [HIPCC, *FLAGS, os.path.join(CSRC, LIBS[name]), "-o", tmp],
+            capture_output=True, text=True)
+        if proc.returncode != 0:
+            raise RuntimeError(f"hipcc build of {LIBS[name]} failed "
+                               f"(rc={proc.returncode}):\n"
+                               f"{proc.stderr[-4000:]}")
+        os.replace(tmp, out)
     return out
 
 
+def build(force: bool = False,
+          names: Optional[Iterable[str]] = None) -> list[str]:
+    """Build the named libraries (all by default); returns their paths."""
+    names = list(LIBS if names is None else names)
+    with ThreadPoolExecutor(max_workers=len(names)) as ex:
+        return list(ex.map(lambda n: _build_one(n, force), names))
+
+
 if __name__ == "__main__":
-    path = build(force="--force" in sys.argv)
-    print(f"built {path}")
+    for path in build(force="--force" in sys.argv):
+        print(f"built {path}")

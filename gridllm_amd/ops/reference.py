@@ -6,9 +6,21 @@ oracle the HIP kernels are tested against (tests/test_ops_gpu.py).
 
 from __future__ import annotations
 
-from typing import Optional, Tuple
+from typing import NamedTuple, Optional, Tuple
 
 import torch
+
+
+class Glu(NamedTuple):
+    """A gated linear unit by its constants: the gate is capped at `limit`,
+    the linear part clamped to +-limit and moved by `shift`;
+    y = g * sigmoid(alpha * g) * (u + shift)."""
+    alpha: float = 1.0
+    limit: float = float("inf")
+    shift: float = 0.0
+
+
+SWIGLU = Glu()
 
 
 def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float,
@@ -50,11 +62,12 @@ def rope(q: torch.Tensor, k: torch.Tensor, cos: torch.Tensor,
     return rot(q), rot(k)
 
 
-def swiglu(gateup: torch.Tensor) -> torch.Tensor:
+def swiglu(gateup: torch.Tensor, glu: Glu = SWIGLU) -> torch.Tensor:
     f = gateup.shape[-1] // 2
-    g = gateup[..., :f].float()
-    u = gateup[..., f:].float()
-    return (g * torch.sigmoid(g) * u).to(gateup.dtype)
+    g = gateup[..., :f].float().clamp(max=glu.limit)
+    u = gateup[..., f:].float().clamp(-glu.limit, glu.limit)
+    return (g * torch.sigmoid(glu.alpha * g) * (u + glu.shift)
+            ).to(gateup.dtype)
 
 
 def rope_kv(qkv: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor,
