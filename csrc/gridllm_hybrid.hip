@@ -1,0 +1,1446 @@
+// gfx950 kernels of the layer-list models: a decoder whose layers each name a
+// mixer (grouped softmax attention over a paged cache, or mLSTM with a matrix
+// memory per sequence) and a feed-forward (dense gated, or routed experts).
+//
+// Conventions
+//  * T is the element type of activations, weights and the KV cache: bf16, or
+//    f32 for the exact mode. The residual stream, norms, scores, gates, router
+//    logits and recurrent state are f32 in both.
+//  * Widths and head sizes are padded by the host to multiples of 64 with zero
+//    weights, so rows are 16-byte aligned and padding stays zero; the true
+//    sizes enter only where a mean is taken.
+//  * The tokens of a step are ordered decode rows first (one token of a
+//    sequence each), then the prompt portions, each a contiguous segment.
+//
+// Exported extern "C" with an explicit stream; nothing here allocates.
+
+#include "gridllm_attention.h"
+
+DEV_INLINE float ld(const bf16_t* p) { return bf2f(*p); }
+DEV_INLINE float ld(const float* p) { return *p; }
+DEV_INLINE void st(bf16_t* p, float v) { *p = f2bf(v); }
+DEV_INLINE void st(float* p, float v) { *p = v; }
+DEV_INLINE void ld8(const bf16_t* p, float* f) { unpack8(*(const uint4*)p, f); }
+DEV_INLINE void ld8(const float* p, float* f) {
+    *(float4*)f = ((const float4*)p)[0];
+    *(float4*)(f + 4) = ((const float4*)p)[1];
+}
+DEV_INLINE void st8(bf16_t* p, const float* f) { *(uint4*)p = pack8(f); }
+DEV_INLINE void st8(float* p, const float* f) {
+    ((float4*)p)[0] = *(const float4*)f;
+    ((float4*)p)[1] = *(const float4*)(f + 4);
+}
+DEV_INLINE float sigmoidf_(float z) { return 1.f / (1.f + expf(-z)); }
+
+// sum over a block of 256 threads; every thread gets it
+DEV_INLINE float block_sum(float v, float* red) {
+    v = wave_reduce_sum(v);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    return red[0] + red[1] + red[2] + red[3];
+}
+
+// ===========================================================================
+// x = embed[token] + pos_table[position], f32; xb = the same in T
+// ===========================================================================
+template <class T>
+__global__ void __launch_bounds__(256)
+k_embed_pos(float* __restrict__ x, T* __restrict__ xb,
+            const T* __restrict__ emb, const T* __restrict__ ptab,
+            const long long* __restrict__ tok, const int* __restrict__ pos,
+            int W, int vocab, int max_pos) {
+    const long n = blockIdx.x;
+    const long t = min(max(tok[n], 0ll), (long long)vocab - 1);
+    const long p = min(max(pos[n], 0), max_pos - 1);
+    for (int c = threadIdx.x * 8; c < W; c += 2048) {
+        float a[8], b[8];
+        ld8(emb + t * W + c, a);
+        ld8(ptab + p * W + c, b);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) a[i] += b[i];
+        st8(x + n * W + c, a);
+        if (xb) st8(xb + n * W + c, a);
+    }
+}
+
+// ===========================================================================
+// Norm of a sublayer's output, added to the residual:
+//   x += y * (1 / sqrt(mean(y^2) + eps)) * (w_off + w);  xb = T(x)
+// TOP > 0 (routed experts): y is sum_k wt[n, k] * ye[n * top + k].
+// W <= 8192 (a row is kept in registers); the mean is over Wtrue elements.
+// ===========================================================================
+template <class T, bool MOE>
+__global__ void __launch_bounds__(256)
+k_post_norm(float* __restrict__ x, T* __restrict__ xb,
+            const T* __restrict__ y, const float* __restrict__ wt, int top,
+            const float* __restrict__ w, float w_off, int W, int Wtrue,
+            float eps) {
+    __shared__ float red[4];
+    const long n = blockIdx.x;
+    float v[4][8];
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int c = (j * 256 + threadIdx.x) * 8;
+        if (c < W) {
+            if (MOE) {
+#pragma unroll
+                for (int i = 0; i < 8; ++i) v[j][i] = 0.f;
+                for (int k = 0; k < top; ++k) {
+                    float f[8];
+                    const float g = wt[n * top + k];
+                    ld8(y + (n * top + k) * (long)W + c, f);
+#pragma unroll
+                    for (int i = 0; i < 8; ++i) v[j][i] += g * f[i];
+                }
+            } else {
+                ld8(y + n * W + c, v[j]);
+            }
+#pragma unroll
+            for (int i = 0; i < 8; ++i) ss += v[j][i] * v[j][i];
+        }
+    }
+    const float rs = 1.f / sqrtf(block_sum(ss, red) / (float)Wtrue + eps);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int c = (j * 256 + threadIdx.x) * 8;
+        if (c < W) {
+            float a[8], g[8];
+            ld8(x + n * W + c, a);
+            ld8(w + c, g);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) a[i] += v[j][i] * rs * (w_off + g[i]);
+            st8(x + n * W + c, a);
+            if (xb) st8(xb + n * W + c, a);
+        }
+    }
+}
+
+// out[r] = norm(x[rows[r]]) in T; rows null = identity
+template <class T>
+__global__ void __launch_bounds__(256)
+k_norm_rows(T* __restrict__ out, const float* __restrict__ x,
+            const int* __restrict__ rows, const float* __restrict__ w,
+            float w_off, int W, int Wtrue, float eps) {
+    __shared__ float red[4];
+    const long n = rows ? rows[blockIdx.x] : blockIdx.x;
+    float ss = 0.f;
+    for (int c = threadIdx.x * 8; c < W; c += 2048) {
+        float a[8];
+        ld8(x + n * W + c, a);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) ss += a[i] * a[i];
+    }
+    const float rs = 1.f / sqrtf(block_sum(ss, red) / (float)Wtrue + eps);
+    for (int c = threadIdx.x * 8; c < W; c += 2048) {
+        float a[8], g[8];
+        ld8(x + n * W + c, a);
+        ld8(w + c, g);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) a[i] *= rs * (w_off + g[i]);
+        st8(out + (long)blockIdx.x * W + c, a);
+    }
+}
+
+// out = glu(gu[:, :F], gu[:, F:]), f32
+__global__ void __launch_bounds__(256)
+k_glu_f32(float* __restrict__ out, const float* __restrict__ gu, long n,
+          int F, const GluParams p) {
+    for (long i = blockIdx.x * 256L + threadIdx.x; i < n * F;
+         i += gridDim.x * 256L) {
+        const long r = i / F, c = i % F;
+        float g = fminf(gu[r * 2 * F + c], p.limit);
+        float u = fminf(fmaxf(gu[r * 2 * F + F + c], -p.limit), p.limit);
+        out[i] = g / (1.f + expf(-p.alpha * g)) * (u + p.shift);
+    }
+}
+
+// ===========================================================================
+// Projection to a few f32 outputs (router logits, recurrence gates):
+//   out[n, j] = sum_k x[n, k] w[j, k] + bias[j], bf16 inputs, f32 result.
+// One block per 16 rows x 16 outputs; its 4 waves split K and add up in LDS.
+// K % 32 == 0. Fragments load straight from memory (both k-contiguous).
+// ===========================================================================
+__global__ void __launch_bounds__(256)
+k_proj_f32(float* __restrict__ out, const bf16_t* __restrict__ x,
+           const bf16_t* __restrict__ w, const float* __restrict__ bias,
+           int M, int N, int K) {
+    __shared__ float red[4][16][17];
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    const int fr = lane & 15, kg = (lane >> 4) * 8;
+    const int m0 = blockIdx.x * 16, n0 = blockIdx.y * 16;
+    const bf16_t* xr = x + (long)min(m0 + fr, M - 1) * K + kg;
+    const bf16_t* wr = w + (long)min(n0 + fr, N - 1) * K + kg;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    const int steps = K >> 5;
+#pragma unroll 4
+    for (int s = wid; s < steps; s += 4)
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+            *(const bf16x8*)(xr + s * 32), *(const bf16x8*)(wr + s * 32),
+            acc, 0, 0, 0);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) red[wid][(lane >> 4) * 4 + r][fr] = acc[r];
+    __syncthreads();
+    const int i = threadIdx.x >> 4, j = threadIdx.x & 15;
+    if (m0 + i < M && n0 + j < N)
+        out[(long)(m0 + i) * N + n0 + j] =
+            red[0][i][j] + red[1][i][j] + red[2][i][j] + red[3][i][j] +
+            (bias ? bias[n0 + j] : 0.f);
+}
+
+// ===========================================================================
+// Attention prologue: unit-RMS q and k (no weight), query temperature, and
+// the write of k and v into the paged cache, from one projection row
+//   [H*P q | G*P k | G*P v | ...], row stride ld.
+// temperature(p) = 1 + coef * ln(floor((p + 1) / every) + 1).
+// One wave per (token, head).
+// ===========================================================================
+template <class T, int P>
+__global__ void __launch_bounds__(256)
+k_qknorm_kv(const T* __restrict__ qkv, T* __restrict__ q_out,
+            T* __restrict__ kc, T* __restrict__ vc,
+            const int* __restrict__ table, int per_slot,
+            const int* __restrict__ pos, const int* __restrict__ slot,
+            int N, int H, int G, int ld_, int dim, float eps, float coef,
+            int every) {
+    constexpr int V = P / 64;
+    const int nh = H + 2 * G;
+    const long item = blockIdx.x * 4L + (threadIdx.x >> 6);
+    if (item >= (long)N * nh) return;
+    const int n = (int)(item / nh), h = (int)(item % nh);
+    const int lane = threadIdx.x & 63;
+    const T* src = qkv + (long)n * ld_ + (long)h * P + lane * V;
+    const int p = pos[n];
+    float f[V];
+#pragma unroll
+    for (int i = 0; i < V; ++i) f[i] = ld(src + i);
+    T* dst;
+    if (h < H) {
+        dst = q_out + ((long)n * H + h) * P;
+    } else {
+        const int blk = p / KV_PAGE;
+        if (blk >= per_slot) return;
+        const int hk = (h - H) % G;
+        const long page = table[(long)slot[n] * per_slot + blk];
+        dst = (h < H + G ? kc : vc) +
+              ((page * G + hk) * KV_PAGE + p % KV_PAGE) * P;
+    }
+    if (h < H + G) {
+        float ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < V; ++i) ss += f[i] * f[i];
+        float s = 1.f / sqrtf(wave_reduce_sum(ss) / (float)dim + eps);
+        if (h < H) s *= 1.f + coef * logf((float)((p + 1) / every) + 1.f);
+#pragma unroll
+        for (int i = 0; i < V; ++i) f[i] *= s;
+    }
+#pragma unroll
+    for (int i = 0; i < V; ++i) st(dst + lane * V + i, f[i]);
+}
+
+// Varlen prefill over the paged cache. meta row (8 ints): {q_off, len, slot,
+// q0, start}: rows [q0, q0 + 128) of the portion packed at q_off, whose first
+// token stands at position `start`.
+template <int D>
+__global__ void __launch_bounds__(256, D > 128 ? 1 : 2)
+k_paged_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
+                const PagedKV<D> kv, const int* __restrict__ meta, int Hq,
+                int G, float scale, const HeadEpilogue epi) {
+    __shared__ __attribute__((aligned(16))) bf16_t vt[D * 40];
+    __shared__ __attribute__((aligned(16))) bf16_t plds[4][2 * 64 * 8];
+    const int* m = meta + blockIdx.x * 8;
+    const int q_off = m[0], len = m[1], start = m[4];
+    attn_prefill_tile<D>(out + (long)q_off * Hq * D,
+                         q + (long)q_off * Hq * D, kv, len, Hq, G, m[2],
+                         start + len, start, scale, m[3], vt, &plds[0][0],
+                         epi, q_off);
+}
+
+// Exact mode: one block per (row, query head), f32 cache, any position.
+template <int P>
+__global__ void __launch_bounds__(256)
+k_attn_rows_f32(float* __restrict__ out, const float* __restrict__ q,
+                const float* __restrict__ kc, const float* __restrict__ vc,
+                const int* __restrict__ table, int per_slot,
+                const int* __restrict__ pos, const int* __restrict__ slot,
+                int H, int G, float scale, const float* __restrict__ sink,
+                const float* __restrict__ gate, int gate_ld) {
+    const int n = blockIdx.x / H, h = blockIdx.x % H;
+    const int hk = h / (H / G);
+    const int* tab = table + (long)slot[n] * per_slot;
+    const int seq = min(pos[n] + 1, per_slot * KV_PAGE);
+    __shared__ float qs[P], sc[256], red[4], acc_s[256];
+    for (int i = threadIdx.x; i < P; i += 256)
+        qs[i] = q[((long)n * H + h) * P + i];
+    __syncthreads();
+    constexpr int NG = 256 / P;
+    const int c = threadIdx.x % P, grp = threadIdx.x / P;
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    float m = sink ? sink[h] : -INFINITY, l = sink ? 1.f : 0.f, acc = 0.f;
+    for (int k0 = 0; k0 < seq; k0 += 256) {
+        const int j = k0 + threadIdx.x;
+        float s = -INFINITY;
+        if (j < seq) {
+            const float* kr = kc + (((long)tab[j / KV_PAGE] * G + hk) * KV_PAGE
+                                    + j % KV_PAGE) * P;
+            s = 0.f;
+            for (int i = 0; i < P; i += 4) {
+                const float4 kv = *(const float4*)(kr + i);
+                s += kv.x * qs[i] + kv.y * qs[i + 1] + kv.z * qs[i + 2] +
+                     kv.w * qs[i + 3];
+            }
+            s *= scale;
+        }
+        float mx = wave_reduce_max(s);
+        if (lane == 0) red[wid] = mx;
+        __syncthreads();
+        mx = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
+        const float mn = fmaxf(m, mx);
+        const float alpha = (m == -INFINITY) ? 0.f : expf(m - mn);
+        const float p = (j < seq) ? expf(s - mn) : 0.f;
+        sc[threadIdx.x] = p;
+        m = mn;
+        __syncthreads();                       // red read, sc written
+        const float ps = wave_reduce_sum(p);
+        if (lane == 0) red[wid] = ps;
+        acc *= alpha;
+        const int jn = min(256, seq - k0);
+        for (int t = grp; t < jn; t += NG) {
+            const int jj = k0 + t;
+            acc += sc[t] * vc[(((long)tab[jj / KV_PAGE] * G + hk) * KV_PAGE +
+                               jj % KV_PAGE) * P + c];
+        }
+        __syncthreads();
+        l = l * alpha + red[0] + red[1] + red[2] + red[3];
+        __syncthreads();
+    }
+    acc_s[threadIdx.x] = acc;
+    __syncthreads();
+    if (threadIdx.x < P) {
+        float a = 0.f;
+        for (int g = 0; g < NG; ++g) a += acc_s[g * P + threadIdx.x];
+        float f = l > 0.f ? 1.f / l : 0.f;
+        if (gate) f *= sigmoidf_(gate[(long)n * gate_ld + h]);
+        out[((long)n * H + h) * P + threadIdx.x] = a * f;
+    }
+}
+
+// ===========================================================================
+// mLSTM: matrix memory with exponential gates, per head
+//   i = cap tanh(zi / cap);  f = logsigmoid(cap tanh(zf / cap))
+//   m' = max(f + m, i);  keep = exp(f + m - m');  put = exp(i - m')
+//   S = keep S + put v k^T;  n = keep n + put k
+//   o = S q / (max(|n . q|, exp(-m')) + 1e-6),  q scaled by dim^-1/2
+// The state of a slot is f32 [H][DV + 1][DK]: row r < DV is S[:, r] over the
+// key dimension, and row DV is n, which is the memory of the constant value
+// 1, so one update serves both. m is f32 [H]. A segment that starts at
+// position 0 takes the state as zero whatever the slot holds.
+// Projection row: [H*DK q | H*DK k | H*DV v | H*DV out gate | ...], stride ld;
+// gate row: [H zi | H zf], f32, biases included.
+// ===========================================================================
+DEV_INLINE void mlstm_gates(const float* gr, int h, int H, float cap,
+                            float& i, float& f) {
+    i = cap * tanhf(gr[h] / cap);
+    const float z = cap * tanhf(gr[H + h] / cap);
+    f = fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
+}
+
+// seg (int4): {first token, length, slot, start position}; null: row r is a
+// segment of one token at pos[r] of slot[r].
+DEV_INLINE int4 segment(const int4* seg, const int* pos, const int* slot,
+                        int r) {
+    if (seg) return seg[r];
+    return make_int4(r, 1, slot[r], pos[r]);
+}
+
+// Token by token. Block = (segment, head, `rpb` state rows); LPR lanes hold
+// one row of DK as NJ float4 each, and a wave works on 64 / LPR rows at once,
+// U of them in flight.
+template <class T, int LPR, int NJ>
+__global__ void __launch_bounds__(256)
+k_mlstm_step(float* __restrict__ o, float* __restrict__ S,
+             const float* __restrict__ mst, const T* __restrict__ qkv,
+             const float* __restrict__ gr, const int4* __restrict__ segs,
+             const int* __restrict__ pos, const int* __restrict__ slot,
+             int H, int DK, int DV, int ld_, float qscale, float cap,
+             int rpb) {
+    constexpr int RW = 64 / LPR;
+    constexpr int U = NJ == 1 ? 4 : 2;
+    const int4 sg = segment(segs, pos, slot, blockIdx.x);
+    const int h = blockIdx.y;
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    const int c0 = (lane % LPR) * 4, rl = lane / LPR;
+    const int rbeg = blockIdx.z * rpb, rend = min(DV + 1, rbeg + rpb);
+    float* Sb = S + ((long)sg.z * H + h) * (DV + 1) * DK;
+    float m = sg.w == 0 ? 0.f : mst[(long)sg.z * H + h];
+    for (int t = 0; t < sg.y; ++t) {
+        const long n = sg.x + t;
+        const bool fresh = sg.w + t == 0;
+        float gi, gf;
+        mlstm_gates(gr + n * 2 * H, h, H, cap, gi, gf);
+        const float mn = fmaxf(gf + m, gi);
+        const float keep = expf(gf + m - mn), put = expf(gi - mn);
+        m = mn;
+        const T* row = qkv + n * ld_;
+        float qv[NJ][4], kv[NJ][4];
+#pragma unroll
+        for (int j = 0; j < NJ; ++j) {
+            const int c = c0 + j * LPR * 4;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const bool in = c < DK;
+                qv[j][i] = in ? ld(row + h * DK + c + i) * qscale : 0.f;
+                kv[j][i] = in ? ld(row + (H + h) * DK + c + i) * put : 0.f;
+            }
+        }
+        const T* vrow = row + 2 * H * DK + h * DV;
+        for (int r0 = rbeg + wid * RW * U; r0 < rend; r0 += 4 * RW * U) {
+            float4 s[U][NJ];
+            float v[U];
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const int r = r0 + u * RW + rl;
+                v[u] = r < DV ? ld(vrow + r) : 1.f;
+                if (r >= rend) v[u] = 0.f;
+#pragma unroll
+                for (int j = 0; j < NJ; ++j) {
+                    const int c = c0 + j * LPR * 4;
+                    s[u][j] = make_float4(0.f, 0.f, 0.f, 0.f);
+                    if (!fresh && r < rend && c < DK)
+                        s[u][j] = *(const float4*)(Sb + (long)r * DK + c);
+                }
+            }
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const int r = r0 + u * RW + rl;
+                float a = 0.f;
+#pragma unroll
+                for (int j = 0; j < NJ; ++j) {
+                    const int c = c0 + j * LPR * 4;
+                    float4 z = s[u][j];
+                    z.x = keep * z.x + kv[j][0] * v[u];
+                    z.y = keep * z.y + kv[j][1] * v[u];
+                    z.z = keep * z.z + kv[j][2] * v[u];
+                    z.w = keep * z.w + kv[j][3] * v[u];
+                    a += z.x * qv[j][0] + z.y * qv[j][1] + z.z * qv[j][2] +
+                         z.w * qv[j][3];
+                    if (r < rend && c < DK)
+                        *(float4*)(Sb + (long)r * DK + c) = z;
+                }
+#pragma unroll
+                for (int off = LPR / 2; off > 0; off >>= 1)
+                    a += __shfl_xor(a, off, WAVE);
+                if (lane % LPR == 0 && r < rend)
+                    o[(n * H + h) * (DV + 1) + r] = a;
+            }
+        }
+    }
+}
+
+// o -> T out[n, H*DV]: unit RMS per head, times norm, times sigmoid of the
+// output gate. Items [0, nseg) are segments of the token-by-token kernel, whose
+// o still lacks its denominator and whose m is advanced here; the nplain
+// tokens from plain0 on are finished sums. One wave per (item, head).
+template <class T>
+__global__ void __launch_bounds__(256)
+k_mlstm_out(T* __restrict__ out, const float* __restrict__ o,
+            float* __restrict__ mst, const T* __restrict__ qkv,
+            const float* __restrict__ gr, const int4* __restrict__ segs,
+            const int* __restrict__ pos, const int* __restrict__ slot,
+            const float* __restrict__ norm, int nseg, int plain0, int nplain,
+            int H, int DK, int DV, int ld_, int dvtrue, float cap,
+            float eps) {
+    const long item = blockIdx.x * 4L + (threadIdx.x >> 6);
+    if (item >= (long)(nseg + nplain) * H) return;
+    const int it = (int)(item / H), h = (int)(item % H);
+    const int lane = threadIdx.x & 63;
+    int4 sg;
+    float m = 0.f;
+    const bool is_seg = it < nseg;
+    if (is_seg) {
+        sg = segment(segs, pos, slot, it);
+        if (sg.w != 0) m = mst[(long)sg.z * H + h];
+    } else {
+        sg = make_int4(plain0 + it - nseg, 1, 0, 0);
+    }
+    for (int t = 0; t < sg.y; ++t) {
+        const long n = sg.x + t;
+        const float* ob = o + (n * H + h) * (DV + 1);
+        float inv = 1.f;
+        if (is_seg) {
+            float gi, gf;
+            mlstm_gates(gr + n * 2 * H, h, H, cap, gi, gf);
+            m = fmaxf(gf + m, gi);
+            inv = 1.f / (fmaxf(fabsf(ob[DV]), expf(-m)) + 1e-6f);
+        }
+        float ss = 0.f;
+        for (int c = lane; c < DV; c += 64) {
+            const float v = ob[c] * inv;
+            ss += v * v;
+        }
+        const float rs =
+            inv / sqrtf(wave_reduce_sum(ss) / (float)dvtrue + eps);
+        const T* g = qkv + n * ld_ + (long)H * (2 * DK + DV) + (long)h * DV;
+        for (int c = lane; c < DV; c += 64)
+            st(out + (n * H + h) * DV + c,
+               ob[c] * rs * norm[h * DV + c] * sigmoidf_(ld(g + c)));
+    }
+    if (is_seg && lane == 0) mst[(long)sg.z * H + h] = m;
+}
+
+// ---------------------------------------------------------------------------
+// Prompt portions in chunks of 64 tokens. With F_t the running sum of f
+// inside a chunk, a_s = i_s - F_s and M_t = max(m_in, max_{s<=t} a_s):
+//   m_t = F_t + M_t
+//   S_t = exp(m_in - M_t) S_in + sum_{s<=t} exp(a_s - M_t) v_s k_s^T
+// so a chunk's own contribution (state kernel), the state that enters each
+// chunk (scan kernel), and the outputs (out kernel) separate; the first and
+// the last run over all chunks at once on the matrix cores. Where a product
+// takes f32 factors (state, weighted keys) they are split into two bf16 parts.
+//
+// chunk (int4): {first token, length, segment, -}
+// seg   (int4): {slot, start position, first chunk, chunks}
+// dS: f32 [chunks][H][DV + 1][DK]; the scan leaves the entering state there as
+// (hi | lo << 16) bf16 pairs. scal: f32 [chunks][H][4] = {max a, F total,
+// m of the slot before the step, m_in}.
+// ---------------------------------------------------------------------------
+#define MCH 64
+#define MLD 72      // padded row of 64 tokens in LDS
+
+// running sum of f, a, running max of a; lane = token, wave-wide
+DEV_INLINE void chunk_scan(const float* gr, int tok0, int clen, int h, int H,
+                           float cap, float& F, float& a, float& amax) {
+    const int t = threadIdx.x & 63;
+    float gi = -INFINITY, gf = 0.f;
+    if (t < clen) mlstm_gates(gr + (long)(tok0 + t) * 2 * H, h, H, cap, gi, gf);
+    F = gf;
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) {
+        const float u = __shfl_up(F, off, WAVE);
+        if (t >= off) F += u;
+    }
+    a = gi - F;
+    amax = a;
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) {
+        const float u = __shfl_up(amax, off, WAVE);
+        if (t >= off) amax = fmaxf(amax, u);
+    }
+}
+
+__global__ void __launch_bounds__(256)
+k_mlstm_chunk_state(float* __restrict__ dS, float* __restrict__ scal,
+                    const float* __restrict__ mst,
+                    const bf16_t* __restrict__ qkv,
+                    const float* __restrict__ gr,
+                    const int4* __restrict__ chunks,
+                    const int4* __restrict__ segs, int H, int DK, int DV,
+                    int ld_, float cap) {
+    __shared__ __attribute__((aligned(16))) bf16_t vt[64 * MLD];
+    __shared__ __attribute__((aligned(16))) bf16_t kh[64 * MLD];
+    __shared__ __attribute__((aligned(16))) bf16_t kl[64 * MLD];
+    __shared__ float wgt[MCH];
+    const int4 ch = chunks[blockIdx.x];
+    const int h = blockIdx.y;
+    const int nd = DK / 64;
+    const int d0 = (blockIdx.z % nd) * 64, v0 = (blockIdx.z / nd) * 64;
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    if (wid == 0) {
+        float F, a, amax;
+        chunk_scan(gr, ch.x, ch.y, h, H, cap, F, a, amax);
+        const float A = __shfl(amax, 63, WAVE);
+        wgt[lane] = lane < ch.y ? expf(a - A) : 0.f;
+        if (blockIdx.z == 0 && lane == 63) {
+            const int4 sg = segs[ch.z];
+            float* sp = scal + ((long)blockIdx.x * H + h) * 4;
+            sp[0] = A;
+            sp[1] = F;
+            sp[2] = sg.y == 0 ? 0.f : mst[(long)sg.x * H + h];
+        }
+    }
+    __syncthreads();
+    for (int i = threadIdx.x; i < 512; i += 256) {
+        const int t = i & 63, c8 = (i >> 6) * 8;   // a wave spans 64 tokens
+        const bf16_t* row = qkv + (long)(ch.x + min(t, ch.y - 1)) * ld_;
+        float f[8];
+        ld8(row + (H + h) * DK + d0 + c8, f);
+        const uint4 vv = *(const uint4*)(row + 2 * H * DK + h * DV + v0 + c8);
+        const bf16_t* pv = (const bf16_t*)&vv;
+        const float w = wgt[t];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+            const float x = f[j] * w;
+            const bf16_t hi = f2bf(x);
+            kh[(c8 + j) * MLD + t] = hi;
+            kl[(c8 + j) * MLD + t] = f2bf(x - bf2f(hi));
+            vt[(c8 + j) * MLD + t] = pv[j];
+        }
+    }
+    __syncthreads();
+    float* Db = dS + ((long)blockIdx.x * H + h) * (DV + 1) * DK;
+    const int fr = lane & 15, kg = (lane >> 4) * 8;
+    f32x4 acc[4];
+#pragma unroll
+    for (int c = 0; c < 4; ++c) acc[c] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ks = 0; ks < 2; ++ks) {
+        const bf16x8 a =
+            *(const bf16x8*)(vt + (wid * 16 + fr) * MLD + ks * 32 + kg);
+#pragma unroll
+        for (int c = 0; c < 4; ++c) {
+            const int at = (c * 16 + fr) * MLD + ks * 32 + kg;
+            acc[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                a, *(const bf16x8*)(kh + at), acc[c], 0, 0, 0);
+            acc[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                a, *(const bf16x8*)(kl + at), acc[c], 0, 0, 0);
+        }
+    }
+#pragma unroll
+    for (int c = 0; c < 4; ++c)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+            Db[(long)(v0 + wid * 16 + (lane >> 4) * 4 + r) * DK + d0 + c * 16 +
+               fr] = acc[c][r];
+    if (v0 == 0 && threadIdx.x < 64) {
+        float s = 0.f;
+        for (int t = 0; t < MCH; ++t)
+            s += bf2f(kh[lane * MLD + t]) + bf2f(kl[lane * MLD + t]);
+        Db[(long)DV * DK + d0 + lane] = s;
+    }
+}
+
+__global__ void __launch_bounds__(256)
+k_mlstm_chunk_scan(float* __restrict__ dS, float* __restrict__ scal,
+                   float* __restrict__ S, float* __restrict__ mst,
+                   const int4* __restrict__ segs, int H, int DK, int DV) {
+    const int4 sg = segs[blockIdx.x];
+    const int h = blockIdx.y;
+    const long size = (long)(DV + 1) * DK;
+    const long e = (blockIdx.z * 256L + threadIdx.x) * 4;
+    if (e >= size) return;
+    float* Sb = S + ((long)sg.x * H + h) * size + e;
+    float4 s = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (sg.y != 0) s = *(const float4*)Sb;
+    float m = scal[((long)sg.z * H + h) * 4 + 2];
+    const long cs = (long)H * size;
+    float* Db = dS + ((long)sg.z * H + h) * size + e;
+    constexpr int U = 4;
+    for (int c = 0; c < sg.w; c += U) {
+        float4 d[U];
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+            if (c + u < sg.w) d[u] = *(const float4*)(Db + (c + u) * cs);
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            if (c + u >= sg.w) break;
+            float* sp = scal + ((long)(sg.z + c + u) * H + h) * 4;
+            const float A = sp[0], Ft = sp[1];
+            if (e == 0) sp[3] = m;
+            uint4 pk;
+            const float sv[4] = {s.x, s.y, s.z, s.w};
+            u32* pp = (u32*)&pk;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const bf16_t hi = f2bf(sv[i]);
+                pp[i] = (u32)hi | ((u32)f2bf(sv[i] - bf2f(hi)) << 16);
+            }
+            *(uint4*)(Db + (c + u) * cs) = pk;
+            const float M = fmaxf(m, A);
+            const float keep = expf(m - M), put = expf(A - M);
+            s.x = keep * s.x + put * d[u].x;
+            s.y = keep * s.y + put * d[u].y;
+            s.z = keep * s.z + put * d[u].z;
+            s.w = keep * s.w + put * d[u].w;
+            m = Ft + M;
+        }
+    }
+    *(float4*)Sb = s;
+    if (e == 0) mst[(long)sg.x * H + h] = m;
+}
+
+// 8 (hi | lo << 16) pairs -> the two bf16 fragments
+DEV_INLINE void split8(const u32* p, bf16x8& hi, bf16x8& lo) {
+    const uint4 x = ((const uint4*)p)[0], y = ((const uint4*)p)[1];
+    uint4 a, b;
+    a.x = (x.x & 0xffffu) | (x.y << 16);  b.x = (x.x >> 16) | (x.y & 0xffff0000u);
+    a.y = (x.z & 0xffffu) | (x.w << 16);  b.y = (x.z >> 16) | (x.w & 0xffff0000u);
+    a.z = (y.x & 0xffffu) | (y.y << 16);  b.z = (y.x >> 16) | (y.y & 0xffff0000u);
+    a.w = (y.z & 0xffffu) | (y.w << 16);  b.w = (y.z >> 16) | (y.w & 0xffff0000u);
+    hi = *(bf16x8*)&a;
+    lo = *(bf16x8*)&b;
+}
+
+// Block = (chunk, head, 128 value columns); a wave owns 16 tokens.
+__global__ void __launch_bounds__(256, 2)
+k_mlstm_chunk_out(float* __restrict__ o, const float* __restrict__ dS,
+                  const float* __restrict__ scal,
+                  const bf16_t* __restrict__ qkv,
+                  const float* __restrict__ gr,
+                  const int4* __restrict__ chunks, int H, int DK, int DV,
+                  int ld_, float qscale, float cap) {
+    __shared__ __attribute__((aligned(16))) bf16_t vt[128 * MLD];
+    __shared__ __attribute__((aligned(16))) bf16_t ps[64 * MLD];
+    __shared__ float sa[MCH], sM[MCH], sm[MCH], sin_[MCH], snq[MCH];
+    const int4 ch = chunks[blockIdx.x];
+    const int h = blockIdx.y, v0 = blockIdx.z * 128;
+    const int nv = min(128, DV - v0);
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    if (wid == 0) {
+        float F, a, amax;
+        chunk_scan(gr, ch.x, ch.y, h, H, cap, F, a, amax);
+        const float m_in = scal[((long)blockIdx.x * H + h) * 4 + 3];
+        const float M = fmaxf(m_in, amax);
+        sa[lane] = a;
+        sM[lane] = M;
+        sm[lane] = F + M;
+        sin_[lane] = expf(m_in - M);
+    }
+    for (int i = threadIdx.x; i < 64 * (nv / 8); i += 256) {
+        const int t = i & 63, c8 = (i >> 6) * 8;
+        const uint4 vv = *(const uint4*)(
+            qkv + (long)(ch.x + min(t, ch.y - 1)) * ld_ + 2 * H * DK + h * DV +
+            v0 + c8);
+        const bf16_t* pv = (const bf16_t*)&vv;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) vt[(c8 + j) * MLD + t] = pv[j];
+    }
+    __syncthreads();
+    const int fr = lane & 15, kg = (lane >> 4) * 8, r0 = wid * 16;
+    const u32* Sb = (const u32*)dS + ((long)blockIdx.x * H + h) * (DV + 1) * DK;
+    const bf16_t* qr = qkv + (long)(ch.x + min(r0 + fr, ch.y - 1)) * ld_ +
+                       h * DK + kg;
+
+    // ---- scores of this wave's tokens against the chunk's keys, and n . q
+    f32x4 sc[4];
+    const bf16_t* kr[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        sc[j] = (f32x4){0.f, 0.f, 0.f, 0.f};
+        kr[j] = qkv + (long)(ch.x + min(j * 16 + fr, ch.y - 1)) * ld_ +
+                (H + h) * DK + kg;
+    }
+    float nq = 0.f;
+    for (int k0 = 0; k0 < DK; k0 += 32) {
+        const bf16x8 a = *(const bf16x8*)(qr + k0);
+        float qf[8];
+        unpack8(*(const uint4*)&a, qf);
+        const u32* np = Sb + (long)DV * DK + k0 + kg;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            const u32 w = np[i];
+            nq += qf[i] * (__uint_as_float(w << 16) +
+                           __uint_as_float(w & 0xffff0000u));
+        }
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+            if (j <= wid)
+                sc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                    a, *(const bf16x8*)(kr[j] + k0), sc[j], 0, 0, 0);
+    }
+    nq += __shfl_xor(nq, 16, WAVE);
+    nq += __shfl_xor(nq, 32, WAVE);
+    if (lane < 16) snq[r0 + lane] = nq;
+    float den[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        if (j > (wid | 1)) continue;
+        const int key = j * 16 + fr;
+        const float ak = sa[key];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int row = r0 + (lane >> 4) * 4 + r;
+            const float p = (key <= row && key < ch.y)
+                ? sc[j][r] * qscale * expf(ak - sM[row]) : 0.f;
+            den[r] += p;
+            ps[row * MLD + key] = f2bf(p);
+        }
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+#pragma unroll
+        for (int off = 8; off > 0; off >>= 1)
+            den[r] += __shfl_xor(den[r], off, WAVE);
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");   // own rows only
+
+    // ---- what the entering state gives, then the chunk's own values
+    f32x4 acc[8];
+#pragma unroll
+    for (int c = 0; c < 8; ++c) acc[c] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int k0 = 0; k0 < DK; k0 += 32) {
+        const bf16x8 a = *(const bf16x8*)(qr + k0);
+#pragma unroll
+        for (int c = 0; c < 8; ++c) {
+            if (c * 16 >= nv) continue;
+            bf16x8 hi, lo;
+            split8(Sb + (long)(v0 + c * 16 + fr) * DK + k0 + kg, hi, lo);
+            acc[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, hi, acc[c],
+                                                             0, 0, 0);
+            acc[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, lo, acc[c],
+                                                             0, 0, 0);
+        }
+    }
+    float inv[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+        const int row = r0 + (lane >> 4) * 4 + r;
+        const float in = sin_[row] * qscale;
+        const float d = den[r] + in * snq[row];
+        inv[r] = 1.f / (fmaxf(fabsf(d), expf(-sm[row])) + 1e-6f);
+#pragma unroll
+        for (int c = 0; c < 8; ++c) acc[c][r] *= in;
+    }
+    for (int ks = 0; ks <= (wid >> 1); ++ks) {
+        const bf16x8 a = *(const bf16x8*)(ps + (r0 + fr) * MLD + ks * 32 + kg);
+#pragma unroll
+        for (int c = 0; c < 8; ++c) {
+            if (c * 16 >= nv) continue;
+            acc[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                a, *(const bf16x8*)(vt + (c * 16 + fr) * MLD + ks * 32 + kg),
+                acc[c], 0, 0, 0);
+        }
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+        const int row = r0 + (lane >> 4) * 4 + r;
+        if (row >= ch.y) continue;
+        float* ob = o + ((long)(ch.x + row) * H + h) * (DV + 1) + v0 + fr;
+#pragma unroll
+        for (int c = 0; c < 8; ++c)
+            if (c * 16 < nv) ob[c * 16] = acc[c][r] * inv[r];
+    }
+}
+
+// ===========================================================================
+// Routed experts.
+//   route:   top experts of every token by f32 logits (ties: lower index),
+//            softmax over the chosen; counts per expert and each pair's rank
+//   scatter: pairs (token * top + k) sorted by expert, and the tile list
+//            {expert, first sorted row, rows, -}; unused tiles have expert -1
+//   gemm:    rows of one expert against its weights, once for the up
+//            projection (gathers token rows, squared ReLU) and once for the
+//            down projection (writes each pair's row back in pair order)
+// The weighted sum over a token's pairs is taken in k_post_norm.
+// ===========================================================================
+template <int VPL>
+__global__ void __launch_bounds__(256)
+k_moe_route(int* __restrict__ idx, float* __restrict__ wt,
+            int* __restrict__ rank, int* __restrict__ counts,
+            const float* __restrict__ z, int N, int E, int top) {
+    const int n = blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (n >= N) return;
+    const int lane = threadIdx.x & 63;
+    float v[VPL];
+#pragma unroll
+    for (int i = 0; i < VPL; ++i) {
+        const int e = i * 64 + lane;
+        v[i] = e < E ? z[(long)n * E + e] : -INFINITY;
+    }
+    float first = 0.f, sum = 0.f, mine = 0.f;
+    for (int k = 0; k < top; ++k) {
+        float best = -INFINITY;
+        int bi = 0x7fffffff;
+#pragma unroll
+        for (int i = 0; i < VPL; ++i)
+            if (v[i] > best) { best = v[i]; bi = i * 64 + lane; }
+#pragma unroll
+        for (int off = 32; off > 0; off >>= 1) {
+            const float ob = __shfl_xor(best, off, WAVE);
+            const int oi = __shfl_xor(bi, off, WAVE);
+            if (ob > best || (ob == best && oi < bi)) { best = ob; bi = oi; }
+        }
+        if (bi >= E) bi = k;           // only if logits are not numbers
+        if (k == 0) first = best;
+        const float p = expf(best - first);
+        sum += p;
+        if (lane == k) mine = p;       // top <= 64
+#pragma unroll
+        for (int i = 0; i < VPL; ++i)
+            if (i * 64 + lane == bi) v[i] = -INFINITY;
+        if (lane == 0) {
+            idx[(long)n * top + k] = bi;
+            rank[(long)n * top + k] = atomicAdd(counts + bi, 1);
+        }
+    }
+    if (lane < top) wt[(long)n * top + lane] = mine / sum;
+}
+
+__global__ void __launch_bounds__(256)
+k_moe_scatter(int* __restrict__ sorted, int4* __restrict__ tiles,
+              const int* __restrict__ idx, const int* __restrict__ rank,
+              const int* __restrict__ counts, int pairs, int E, int bm,
+              int max_tiles) {
+    __shared__ int off[1025], toff[1025];
+    for (int e = threadIdx.x; e < E; e += 256) off[e + 1] = counts[e];
+    if (threadIdx.x == 0) off[0] = toff[0] = 0;
+    __syncthreads();
+    if (threadIdx.x < 64) {            // one wave scans, 64 experts a turn
+        int base = 0, tbase = 0;
+        for (int e0 = 0; e0 < E; e0 += 64) {
+            const int e = e0 + threadIdx.x;
+            int c = e < E ? off[e + 1] : 0;
+            int t = (c + bm - 1) / bm;
+#pragma unroll
+            for (int s = 1; s < 64; s <<= 1) {
+                const int a = __shfl_up(c, s, WAVE);
+                const int b = __shfl_up(t, s, WAVE);
+                if ((int)threadIdx.x >= s) { c += a; t += b; }
+            }
+            if (e < E) { off[e + 1] = base + c; toff[e + 1] = tbase + t; }
+            base += __shfl(c, 63, WAVE);
+            tbase += __shfl(t, 63, WAVE);
+        }
+    }
+    __syncthreads();
+    const int i = blockIdx.x * 256 + threadIdx.x;
+    if (i < pairs) sorted[off[idx[i]] + rank[i]] = i;
+    if (blockIdx.x == 0) {
+        for (int e = threadIdx.x; e < E; e += 256) {
+            const int n = off[e + 1] - off[e];
+            for (int t = 0; t * bm < n; ++t)
+                if (toff[e] + t < max_tiles)
+                    tiles[toff[e] + t] = make_int4(e, off[e] + t * bm,
+                                                   min(bm, n - t * bm), 0);
+        }
+        for (int t = toff[E] + threadIdx.x; t < max_tiles; t += 256)
+            tiles[t] = make_int4(-1, 0, 0, 0);
+    }
+}
+
+DEV_INLINE float sq_relu(float v) {
+    v = fmaxf(v, 0.f);
+    return v * v;
+}
+
+// Large batches: 128 rows x 128 columns per block, 4 waves of 64 x 64, both
+// operands through LDS by global_load_lds (source addresses pre-swizzled so
+// that the lane-linear image reads back without bank conflicts), NB buffers.
+// UP: row r of the tile is token sorted[row0 + r] / top, squared ReLU, output
+// in sorted order. Otherwise row r is sorted row row0 + r and its output goes
+// to pair order. K % 64 == 0, N % 64 == 0.
+template <bool UP, int NB>
+__global__ void __launch_bounds__(256, 2)
+k_moe_gemm(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
+           const bf16_t* __restrict__ w, const int4* __restrict__ tiles,
+           const int* __restrict__ sorted, int top, int N, int K,
+           int ntn) {
+    constexpr int BK = 64, TB = 256 * BK, GL = 8;
+    __shared__ __attribute__((aligned(16))) bf16_t lds[NB * TB];
+    const int4 tl = tiles[blockIdx.x / ntn];
+    if (tl.x < 0) return;
+    const int n0 = (blockIdx.x % ntn) * 128;
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    const int fr = lane & 15, kg = (lane >> 4) * 8;
+    const int lrow = lane >> 3, lkb = (lane & 7) * 16;
+    const char* src[GL];
+#pragma unroll
+    for (int i = 0; i < GL; ++i) {     // pieces of 8 rows: 16 of x, 16 of w
+        const int piece = (i < 4 ? wid * 4 + i : 16 + wid * 4 + i - 4);
+        const int row = (piece & 15) * 8 + lrow;
+        const bf16_t* p;
+        if (piece < 16) {
+            const int r = tl.y + min(row, tl.z - 1);
+            p = x + (long)(UP ? sorted[r] / top : r) * K;
+        } else {
+            p = w + ((long)tl.x * N + min(n0 + row, N - 1)) * K;
+        }
+        src[i] = (const char*)p + (lkb ^ ((row & 7) << 4));
+    }
+    auto issue = [&](int buf, int kt) {
+#pragma unroll
+        for (int i = 0; i < GL; ++i) {
+            const int piece = (i < 4 ? wid * 4 + i : 16 + wid * 4 + i - 4);
+            __builtin_amdgcn_global_load_lds(
+                (const __attribute__((address_space(1))) unsigned int*)
+                    (src[i] + (long)kt * BK * 2),
+                (__attribute__((address_space(3))) unsigned int*)
+                    (lds + buf * TB + piece * 512), 16, 0, 0);
+        }
+    };
+    f32x4 acc[4][4];
+#pragma unroll
+    for (int a = 0; a < 4; ++a)
+#pragma unroll
+        for (int b = 0; b < 4; ++b) acc[a][b] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    const int nt = K / BK;
+    const int wr = (wid >> 1) * 64, wc = (wid & 1) * 64;
+#pragma unroll
+    for (int u = 0; u < NB - 1; ++u)
+        if (u < nt) issue(u, u);
+    for (int kt = 0; kt < nt; ++kt) {
+        if (kt + NB - 1 < nt)
+            asm volatile("s_waitcnt vmcnt(%0)" :: "i"(GL * (NB - 2)) : "memory");
+        else
+            asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __builtin_amdgcn_s_barrier();
+        if (kt + NB - 1 < nt) issue((kt + NB - 1) % NB, kt + NB - 1);
+        const char* xb = (const char*)(lds + (kt % NB) * TB);
+        const char* wb = xb + 128 * BK * 2;
+#pragma unroll
+        for (int kc = 0; kc < 2; ++kc) {
+            bf16x8 b[4];
+#pragma unroll
+            for (int c = 0; c < 4; ++c) {
+                const int row = wc + c * 16 + fr;
+                b[c] = *(const bf16x8*)(wb + row * 128 +
+                    (((kc * 32 + kg) * 2) ^ ((row & 7) << 4)));
+            }
+#pragma unroll
+            for (int a = 0; a < 4; ++a) {
+                const int row = wr + a * 16 + fr;
+                const bf16x8 av = *(const bf16x8*)(xb + row * 128 +
+                    (((kc * 32 + kg) * 2) ^ ((row & 7) << 4)));
+#pragma unroll
+                for (int c = 0; c < 4; ++c)
+                    acc[a][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                        av, b[c], acc[a][c], 0, 0, 0);
+            }
+        }
+    }
+#pragma unroll
+    for (int a = 0; a < 4; ++a)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int m = wr + a * 16 + (lane >> 4) * 4 + r;
+            if (m >= tl.z) continue;
+            const long dst = UP ? tl.y + m : sorted[tl.y + m];
+#pragma unroll
+            for (int c = 0; c < 4; ++c) {
+                const int n = n0 + wc + c * 16 + fr;
+                if (n < N)
+                    out[dst * N + n] =
+                        f2bf(UP ? sq_relu(acc[a][c][r]) : acc[a][c][r]);
+            }
+        }
+}
+
+// Small batches (weight streaming): up to 16 * MT rows of an expert against 64
+// columns; a wave owns 16 columns and streams its weights once, straight into
+// MFMA fragments, while the rows pass through LDS in panels of KS.
+template <bool UP, int MT>
+__global__ void __launch_bounds__(256)
+k_moe_gemm_skinny(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
+                  const bf16_t* __restrict__ w,
+                  const int4* __restrict__ tiles,
+                  const int* __restrict__ sorted, int top, int N, int K,
+                  int ntn) {
+    constexpr int KS = 256, ROWS = MT * 16;
+    __shared__ __attribute__((aligned(16))) bf16_t xs[ROWS * KS];
+    const int4 tl = tiles[blockIdx.x / ntn];
+    if (tl.x < 0) return;
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    const int fr = lane & 15, kg = (lane >> 4) * 8;
+    const int n0 = (blockIdx.x % ntn) * 64 + wid * 16;
+    const bf16_t* wrow = w + ((long)tl.x * N + n0 + fr) * K + kg;
+    f32x4 acc[MT];
+#pragma unroll
+    for (int t = 0; t < MT; ++t) acc[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    const bf16_t* xrow[MT * 2];
+#pragma unroll
+    for (int i = 0; i < MT * 2; ++i) {
+        const int r = tl.y + min((int)((threadIdx.x >> 5) + i * 8), tl.z - 1);
+        xrow[i] = x + (long)(UP ? sorted[r] / top : r) * K;
+    }
+    const int kc = (threadIdx.x & 31) * 8;
+    for (int kp = 0; kp < K; kp += KS) {
+        bf16x8 b[8];
+#pragma unroll
+        for (int u = 0; u < 8; ++u)
+            b[u] = __builtin_nontemporal_load(
+                (const bf16x8*)(wrow + min(kp + u * 32, K - 32)));
+        if (kp > 0) __syncthreads();
+#pragma unroll
+        for (int i = 0; i < MT * 2; ++i) {
+            const int row = (threadIdx.x >> 5) + i * 8;
+            const uint4 v = *(const uint4*)(xrow[i] + min(kp + kc, K - 8));
+            *(uint4*)((char*)xs + (((row * KS + kc) * 2) ^ ((row & 15) << 4))) = v;
+        }
+        __syncthreads();
+        const int nch = min(KS, K - kp) >> 5;
+#pragma unroll
+        for (int u = 0; u < 8; ++u) {
+            if (u >= nch) break;
+#pragma unroll
+            for (int t = 0; t < MT; ++t) {
+                const int row = t * 16 + fr;
+                acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                    *(const bf16x8*)((const char*)xs +
+                        (((row * KS + u * 32 + kg) * 2) ^ ((row & 15) << 4))),
+                    b[u], acc[t], 0, 0, 0);
+            }
+        }
+    }
+#pragma unroll
+    for (int t = 0; t < MT; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int m = t * 16 + (lane >> 4) * 4 + r;
+            if (m >= tl.z) continue;
+            const long dst = UP ? tl.y + m : sorted[tl.y + m];
+            out[dst * N + n0 + fr] = f2bf(UP ? sq_relu(acc[t][r]) : acc[t][r]);
+        }
+}
+
+// Exact mode: 16 rows x 64 columns per block, f32 products.
+template <bool UP>
+__global__ void __launch_bounds__(256)
+k_moe_gemm_f32(float* __restrict__ out, const float* __restrict__ x,
+               const float* __restrict__ w, const int4* __restrict__ tiles,
+               const int* __restrict__ sorted, int top, int N, int K,
+               int ntn) {
+    __shared__ float xs[16][33], ws[64][33];
+    const int4 tl = tiles[blockIdx.x / ntn];
+    if (tl.x < 0) return;
+    const int n0 = (blockIdx.x % ntn) * 64;
+    const int col = threadIdx.x & 63, r4 = (threadIdx.x >> 6) * 4;
+    float acc[4] = {0.f, 0.f, 0.f, 0.f};
+    for (int k0 = 0; k0 < K; k0 += 32) {
+        for (int i = threadIdx.x; i < 16 * 32; i += 256) {
+            const int r = tl.y + min(i >> 5, tl.z - 1);
+            xs[i >> 5][i & 31] =
+                x[(long)(UP ? sorted[r] / top : r) * K + k0 + (i & 31)];
+        }
+        for (int i = threadIdx.x; i < 64 * 32; i += 256)
+            ws[i >> 5][i & 31] =
+                w[((long)tl.x * N + n0 + (i >> 5)) * K + k0 + (i & 31)];
+        __syncthreads();
+#pragma unroll
+        for (int k = 0; k < 32; ++k) {
+            const float wv = ws[col][k];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) acc[r] += xs[r4 + r][k] * wv;
+        }
+        __syncthreads();
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+        if (r4 + r >= tl.z) continue;
+        const long dst = UP ? tl.y + r4 + r : sorted[tl.y + r4 + r];
+        out[dst * N + n0 + col] = UP ? sq_relu(acc[r]) : acc[r];
+    }
+}
+
+// ===========================================================================
+// Entry points. f32 != 0 selects the exact mode. 0 = success.
+// ===========================================================================
+template <int D, int G>
+static void launch_paged_decode(hipStream_t st, void* out, const void* q,
+                                const PagedKV<D>& kv, const int* pos,
+                                const int* slot, float* ws, int B, int ngrp,
+                                int nsplit, float scale,
+                                const HeadEpilogue& epi) {
+    const dim3 grid((unsigned)(B * kv.Hk * ngrp * nsplit));
+    if (nsplit == 1 && B * kv.Hk * ngrp >= 2048)
+        k_attn_decode1<D, G><<<grid, dim3(64), 0, st>>>(
+            (bf16_t*)out, (const bf16_t*)q, kv, pos, 1, slot, ws, ngrp,
+            nsplit, scale, epi);
+    else
+        k_attn_decode<D, G><<<grid, dim3(256), 0, st>>>(
+            (bf16_t*)out, (const bf16_t*)q, kv, pos, 1, slot, ws, ngrp,
+            nsplit, scale, epi);
+}
+
+template <int D>
+static int paged_decode(hipStream_t st, void* out, const void* q,
+                        const void* kc, const void* vc, const int* table,
+                        int per_slot, const int* pos, const int* slot,
+                        float* ws, int B, int Hq, int Hk, int nsplit,
+                        float scale, const HeadEpilogue& epi) {
+    const PagedKV<D> kv{(const bf16_t*)kc, (const bf16_t*)vc, table, Hk,
+                        per_slot};
+    const int per = Hq / Hk;
+    int g = per;
+    if (g > MAXG) for (g = MAXG; per % g; --g) {}
+    switch (g) {
+#define CASE_G(GG) case GG: launch_paged_decode<D, GG>(st, out, q, kv, pos, \
+        slot, ws, B, per / GG, nsplit, scale, epi); break;
+        CASE_G(1) CASE_G(2) CASE_G(3) CASE_G(4)
+        CASE_G(5) CASE_G(6) CASE_G(7) CASE_G(8)
+#undef CASE_G
+        default: return -102;
+    }
+    LAUNCH_CHECK();
+    if (nsplit > 1) {
+        k_attn_combine<<<dim3((unsigned)(B * Hq)), dim3(D), 0, st>>>(
+            (bf16_t*)out, ws, Hq, D, nsplit, epi);
+        LAUNCH_CHECK();
+    }
+    return 0;
+}
+
+extern "C" {
+
+int gh_embed_pos(void* stream, int f32, void* x, void* xb, const void* emb,
+                 const void* ptab, const void* tok, const void* pos, int N,
+                 int W, int vocab, int max_pos) {
+    if (W % 64 || N < 1) return -100;
+    hipStream_t st_ = (hipStream_t)stream;
+    if (f32)
+        k_embed_pos<float><<<N, 256, 0, st_>>>((float*)x, (float*)xb,
+            (const float*)emb, (const float*)ptab, (const long long*)tok,
+            (const int*)pos, W, vocab, max_pos);
+    else
+        k_embed_pos<bf16_t><<<N, 256, 0, st_>>>((float*)x, (bf16_t*)xb,
+            (const bf16_t*)emb, (const bf16_t*)ptab, (const long long*)tok,
+            (const int*)pos, W, vocab, max_pos);
+    LAUNCH_CHECK();
+    return 0;
+}
+
+int gh_post_norm(void* stream, int f32, void* x, void* xb, const void* y,
+                 const void* wt, int top, const void* w, float w_off, int N,
+                 int W, int Wtrue, float eps) {
+    if (W % 64 || W > 8192 || N < 1) return -100;
+    hipStream_t st_ = (hipStream_t)stream;
+#define GO(T, M) k_post_norm<T, M><<<N, 256, 0, st_>>>((float*)x, (T*)xb, \
+        (const T*)y, (const float*)wt, top, (const float*)w, w_off, W, Wtrue, \
+        eps)
+    if (f32) { if (wt) GO(float, true); else GO(float, false); }
+    else { if (wt) GO(bf16_t, true); else GO(bf16_t, false); }
+#undef GO
+    LAUNCH_CHECK();
+    return 0;
+}
+
+int gh_norm_rows(void* stream, int f32, void* out, const void* x,
+                 const void* rows, const void* w, float w_off, int M, int W,
+                 int Wtrue, float eps) {
+    if (W % 64 || M < 1) return -100;
+    hipStream_t st_ = (hipStream_t)stream;
+    if (f32)
+        k_norm_rows<float><<<M, 256, 0, st_>>>((float*)out, (const float*)x,
+            (const int*)rows, (const float*)w, w_off, W, Wtrue, eps);
+    else
+        k_norm_rows<bf16_t><<<M, 256, 0, st_>>>((bf16_t*)out, (const float*)x,
+            (const int*)rows, (const float*)w, w_off, W, Wtrue, eps);
+    LAUNCH_CHECK();
+    return 0;
+}
+
+int gh_glu_f32(void* stream, void* out, const void* gu, long n, int F,
+               float alpha, float limit, float shift) {
+    if (n < 1) return -100;
+    const int grid = (int)min((n * F + 255) / 256, (long)4096);
+    k_glu_f32<<<grid, 256, 0, (hipStream_t)stream>>>(
+        (float*)out, (const float*)gu, n, F, GluParams{alpha, limit, shift});
+    LAUNCH_CHECK();
+    return 0;
+}
+
+int gh_proj_f32(void* stream, void* out, const void* x, const void* w,
+                const void* bias, int M, int N, int K) {
+    if (K % 32 || M < 1 || N < 1) return -100;
+    k_proj_f32<<<dim3((M + 15) / 16, (N + 15) / 16), 256, 0,
+                 (hipStream_t)stream>>>((float*)out, (const bf16_t*)x,
+        (const bf16_t*)w, (const float*)bias, M, N, K);
+    LAUNCH_CHECK();
+    return 0;
+}
+
+int gh_qknorm_kv(void* stream, int f32, const void* qkv, void* q_out,
+                 void* kc, void* vc, const void* table, int per_slot,
+                 const void* pos, const void* slot, int N, int H, int G,
+                 int P, int ld_, int dim, float eps, float coef, int every) {
+    if (N < 1 || H % G || every < 1) return -100;
+    hipStream_t st_ = (hipStream_t)stream;
+    const unsigned grid = (unsigned)(((long)N * (H + 2 * G) + 3) / 4);
+#define GO(T, PP) k_qknorm_kv<T, PP><<<grid, 256, 0, st_>>>((const T*)qkv, \
+        (T*)q_out, (T*)kc, (T*)vc, (const int*)table, per_slot, \
+        (const int*)pos, (const int*)slot, N, H, G, ld_, dim, eps, coef, every)
+    if (P == 64) { if (f32) GO(float, 64); else GO(bf16_t, 64); }
+    else if (P == 128) { if (f32) GO(float, 128); else GO(bf16_t, 128); }
+    else if (P == 256) { if (f32) GO(float, 256); else GO(bf16_t, 256); }
+    else return -101;
+#undef GO
+    LAUNCH_CHECK();
+    return 0;
+}
+
+int gh_paged_decode(void* stream, void* out, const void* q, const void* kc,
+                    const void* vc, const void* table, int per_slot,
+                    const void* pos, const void* slot, void* ws, int B,
+                    int Hq, int Hk, int D, int nsplit, float scale,
+                    const void* sink, const void* gate, int gate_ld) {
+    if (B < 1 || Hq % Hk || nsplit < 1) return -100;
+    const HeadEpilogue epi{(const float*)sink, (const bf16_t*)gate, gate_ld};
+    hipStream_t st_ = (hipStream_t)stream;
+#define GO(DD) return paged_decode<DD>(st_, out, q, kc, vc, \
+        (const int*)table, per_slot, (const int*)pos, (const int*)slot, \
+        (float*)ws, B, Hq, Hk, nsplit, scale, epi)
+    if (D == 64) GO(64);
+    if (D == 128) GO(128);
+    if (D == 256) GO(256);
+#undef GO
+    return -101;
+}
+
+int gh_paged_prefill(void* stream, void* out, const void* q, const void* kc,
+                     const void* vc, const void* table, int per_slot,
+                     const void* meta, int ntiles, int Hq, int Hk, int D,
+                     float scale, const void* sink, const void* gate,
+                     int gate_ld) {
+    if (ntiles < 1 || Hq % Hk) return -100;
+    const HeadEpilogue epi{(const float*)sink, (const bf16_t*)gate, gate_ld};
+    hipStream_t st_ = (hipStream_t)stream;
+#define GO(DD) k_paged_prefill<DD><<<dim3(ntiles, Hq), 256, 0, st_>>>( \
+        (bf16_t*)out, (const bf16_t*)q, \
+        PagedKV<DD>{(const bf16_t*)kc, (const bf16_t*)vc, (const int*)table, \
+                    Hk, per_slot}, (const int*)meta, Hq, Hq / Hk, scale, epi)
+    if (D == 64) GO(64);
+    else if (D == 128) GO(128);
+    else if (D == 256) GO(256);
+    else return -101;
+#undef GO
+    LAUNCH_CHECK();
+    return 0;
+}
+
+int gh_attn_rows_f32(void* stream, void* out, const void* q, const void* kc,
+                     const void* vc, const void* table, int per_slot,
+                     const void* pos, const void* slot, int N, int H, int G,
+                     int P, float scale, const void* sink, const void* gate,
+                     int gate_ld) {
+    if (N < 1 || H % G) return -100;
+    hipStream_t st_ = (hipStream_t)stream;
+#define GO(PP) k_attn_rows_f32<PP><<<(unsigned)((long)N * H), 256, 0, st_>>>( \
+        (float*)out, (const float*)q, (const float*)kc, (const float*)vc, \
+        (const int*)table, per_slot, (const int*)pos, (const int*)slot, H, G, \
+        scale, (const float*)sink, (const float*)gate, gate_ld)
+    if (P == 64) GO(64);
+    else if (P == 128) GO(128);
+    else if (P == 256) GO(256);
+    else return -101;
+#undef GO
+    LAUNCH_CHECK();
+    return 0;
+}
+
+int gh_mlstm_step(void* stream, int f32, void* o, void* S, const void* mst,
+                  const void* qkv, const void* gr, const void* segs,
+                  const void* pos, const void* slot, int nseg, int H, int DK,
+                  int DV, int ld_, float qscale, float cap, int rpb) {
+    if (nseg < 1 || DK % 64 || DV % 64 || DK > 1024 || rpb < 1) return -100;
+    hipStream_t st_ = (hipStream_t)stream;
+    const dim3 grid((unsigned)nseg, (unsigned)H,
+                    (unsigned)((DV + 1 + rpb - 1) / rpb));
+#define GO(T, L, J) k_mlstm_step<T, L, J><<<grid, 256, 0, st_>>>((float*)o, \
+        (float*)S, (const float*)mst, (const T*)qkv, (const float*)gr, \
+        (const int4*)segs, (const int*)pos, (const int*)slot, H, DK, DV, ld_, \
+        qscale, cap, rpb)
+#define PICK(T) do { if (DK <= 64) GO(T, 16, 1); \
+        else if (DK <= 128) GO(T, 32, 1); else if (DK <= 256) GO(T, 64, 1); \
+        else if (DK <= 512) GO(T, 64, 2); else GO(T, 64, 4); } while (0)
+    if (f32) PICK(float); else PICK(bf16_t);
+#undef PICK
+#undef GO
+    LAUNCH_CHECK();
+    return 0;
+}
+
+int gh_mlstm_out(void* stream, int f32, void* out, const void* o, void* mst,
+                 const void* qkv, const void* gr, const void* segs,
+                 const void* pos, const void* slot, const void* norm,
+                 int nseg, int plain0, int nplain, int H, int DK, int DV,
+                 int ld_, int dvtrue, float cap, float eps) {
+    if (nseg + nplain < 1) return -100;
+    hipStream_t st_ = (hipStream_t)stream;
+    const unsigned grid = (unsigned)(((long)(nseg + nplain) * H + 3) / 4);
+#define GO(T) k_mlstm_out<T><<<grid, 256, 0, st_>>>((T*)out, \
+        (const float*)o, (float*)mst, (const T*)qkv, (const float*)gr, \
+        (const int4*)segs, (const int*)pos, (const int*)slot, \
+        (const float*)norm, nseg, plain0, nplain, H, DK, DV, ld_, dvtrue, \
+        cap, eps)
+    if (f32) GO(float); else GO(bf16_t);
+#undef GO
+    LAUNCH_CHECK();
+    return 0;
+}
+
+int gh_mlstm_chunks(void* stream, void* o, void* S, void* mst, void* dS,
+                    void* scal, const void* qkv, const void* gr,
+                    const void* chunks, const void* segs, int nchunks,
+                    int nseg, int H, int DK, int DV, int ld_, float qscale,
+                    float cap) {
+    if (nchunks < 1 || nseg < 1 || DK % 64 || DV % 64) return -100;
+    hipStream_t st_ = (hipStream_t)stream;
+    k_mlstm_chunk_state<<<dim3(nchunks, H, (DK / 64) * (DV / 64)), 256, 0,
+                          st_>>>((float*)dS, (float*)scal, (const float*)mst,
+        (const bf16_t*)qkv, (const float*)gr, (const int4*)chunks,
+        (const int4*)segs, H, DK, DV, ld_, cap);
+    LAUNCH_CHECK();
+    const long quads = (long)(DV + 1) * DK / 4;
+    k_mlstm_chunk_scan<<<dim3(nseg, H, (unsigned)((quads + 255) / 256)), 256,
+                         0, st_>>>((float*)dS, (float*)scal, (float*)S,
+        (float*)mst, (const int4*)segs, H, DK, DV);
+    LAUNCH_CHECK();
+    k_mlstm_chunk_out<<<dim3(nchunks, H, (DV + 127) / 128), 256, 0, st_>>>(
+        (float*)o, (const float*)dS, (const float*)scal, (const bf16_t*)qkv,
+        (const float*)gr, (const int4*)chunks, H, DK, DV, ld_, qscale, cap);
+    LAUNCH_CHECK();
+    return 0;
+}
+
+int gh_moe_route(void* stream, void* idx, void* wt, void* rank, void* counts,
+                 void* sorted, void* tiles, const void* z, int N, int E,
+                 int top, int bm, int max_tiles) {
+    if (N < 1 || E < 1 || E > 1024 || top < 1 || top > 64 || top > E)
+        return -100;
+    hipStream_t st_ = (hipStream_t)stream;
+#define GO(V) k_moe_route<V><<<(N + 3) / 4, 256, 0, st_>>>((int*)idx, \
+        (float*)wt, (int*)rank, (int*)counts, (const float*)z, N, E, top)
+    if (E <= 64) GO(1);
+    else if (E <= 256) GO(4);
+    else GO(16);
+#undef GO
+    LAUNCH_CHECK();
+    const long pairs = (long)N * top;
+    k_moe_scatter<<<(unsigned)((pairs + 255) / 256), 256, 0, st_>>>(
+        (int*)sorted, (int4*)tiles, (const int*)idx, (const int*)rank,
+        (const int*)counts, (int)pairs, E, bm, max_tiles);
+    LAUNCH_CHECK();
+    return 0;
+}
+
+// bm: rows per tile of the list: 16, 32 or 64 (weight streaming) or 128
+int gh_moe_gemm(void* stream, int f32, int up, void* out, const void* x,
+                const void* w, const void* tiles, const void* sorted,
+                int top, int N, int K, int bm, int max_tiles) {
+    if (N % 64 || K % 64 || max_tiles < 1) return -100;
+    hipStream_t st_ = (hipStream_t)stream;
+    if (f32) {
+        if (bm != 16) return -103;
+        const int ntn = N / 64;
+        const unsigned grid = (unsigned)(max_tiles * ntn);
+#define GO(U) k_moe_gemm_f32<U><<<grid, 256, 0, st_>>>((float*)out, \
+        (const float*)x, (const float*)w, (const int4*)tiles, \
+        (const int*)sorted, top, N, K, ntn)
+        if (up) GO(true); else GO(false);
+#undef GO
+        LAUNCH_CHECK();
+        return 0;
+    }
+#define ARGS (bf16_t*)out, (const bf16_t*)x, (const bf16_t*)w, \
+        (const int4*)tiles, (const int*)sorted, top, N, K, ntn
+    if (bm == 128) {
+        const int ntn = (N + 127) / 128;
+        const unsigned grid = (unsigned)(max_tiles * ntn);
+        if (up) k_moe_gemm<true, 2><<<grid, 256, 0, st_>>>(ARGS);
+        else k_moe_gemm<false, 2><<<grid, 256, 0, st_>>>(ARGS);
+    } else {
+        const int ntn = N / 64;
+        const unsigned grid = (unsigned)(max_tiles * ntn);
+#define GO(M) do { \
+        if (up) k_moe_gemm_skinny<true, M><<<grid, 256, 0, st_>>>(ARGS); \
+        else k_moe_gemm_skinny<false, M><<<grid, 256, 0, st_>>>(ARGS); \
+        } while (0)
+        if (bm == 16) GO(1);
+        else if (bm == 32) GO(2);
+        else if (bm == 64) GO(4);
+        else return -103;
+#undef GO
+    }
+#undef ARGS
+    LAUNCH_CHECK();
+    return 0;
+}
+
+}  // extern "C"

@@ -8,7 +8,10 @@ llama3:70b).
 
 from __future__ import annotations
 
+import json
+import os
 from dataclasses import dataclass, replace
+from typing import Callable, Optional, Union
 
 
 @dataclass(frozen=True)
@@ -40,10 +43,223 @@ class ModelSpec:
         return self.layers * per_layer + emb + h
 
 
-_SPECS: dict[str, ModelSpec] = {}
+# ------------------------------------------------------ layer-list designs
+# A model whose layers each name a mixer and a feed-forward; a layer may use
+# the weights of another one (with a cache or state of its own).
 
 
-def _reg(spec: ModelSpec, *aliases: str) -> None:
+@dataclass(frozen=True)
+class AttentionMixer:
+    """Grouped softmax attention: unit-RMS q and k, a query temperature
+    1 + q_coef ln(floor((p + 1) / q_every) + 1), a sink term and an output
+    gate per head; no rotation."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    q_coef: float = 0.0
+    q_every: int = 1
+
+    def params(self, width: int) -> int:
+        h, g = self.heads, self.kv_heads
+        return width * (h * self.dim + g * (self.dim + self.vdim) + h
+                        + h * self.vdim) + h
+
+
+@dataclass(frozen=True)
+class MlstmMixer:
+    """mLSTM: a matrix memory per head, exponential input gate, log-sigmoid
+    forget gate, both soft-capped at gate_cap."""
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float
+
+    def params(self, width: int) -> int:
+        h = self.heads
+        return width * h * (2 * self.dim + 3 * self.vdim + 2) \
+            + 2 * h + h * self.vdim
+
+
+@dataclass(frozen=True)
+class DenseFF:
+    """Gated feed-forward, act(g, u) = g sigmoid(alpha g) (u + shift) with g
+    capped at limit and u clamped to +-limit."""
+    ff: int
+    limit: float
+    alpha: float = 1.702
+    shift: float = 1.0
+
+    def params(self, width: int) -> int:
+        return 3 * width * self.ff
+
+
+@dataclass(frozen=True)
+class RoutedFF:
+    """Routed experts with squared ReLU; weights are the softmax over the
+    chosen logits."""
+    experts: int
+    top: int
+    ff: int
+
+    def params(self, width: int) -> int:
+        return self.experts * width * (2 * self.ff + 1)
+
+
+@dataclass(frozen=True)
+class LayerSpec:
+    mixer: Union[AttentionMixer, MlstmMixer]
+    ff: Union[DenseFF, RoutedFF, None] = None
+    weights_of: Optional[int] = None
+
+
+@dataclass(frozen=True)
+class HybridSpec:
+    name: str
+    vocab: int
+    hidden: int
+    layers: tuple[LayerSpec, ...]
+    norm_eps: float
+    positions: int                 # rows of the learned position table
+    max_seq_len: int = 0           # 0 -> positions
+
+    def __post_init__(self) -> None:
+        if not 0 < self.max_seq_len <= self.positions:
+            object.__setattr__(self, "max_seq_len", self.positions)
+        if not self.layers:
+            raise ValueError(f"{self.name}: no layers")
+        for i, ly in enumerate(self.layers):
+            j = self.owner(i)
+            own = self.layers[j]
+            if (ly.mixer, ly.ff) != (own.mixer, own.ff):
+                raise ValueError(f"layer {i} uses layer {j}'s weights but "
+                                 "differs from it")
+            mx, ff = ly.mixer, ly.ff
+            if isinstance(mx, AttentionMixer) and mx.heads % mx.kv_heads:
+                raise ValueError(f"layer {i}: {mx.heads} heads over "
+                                 f"{mx.kv_heads} key/value heads")
+            if isinstance(ff, RoutedFF) and not 0 < ff.top <= ff.experts:
+                raise ValueError(f"layer {i}: top {ff.top} of {ff.experts}")
+
+    def owner(self, i: int) -> int:
+        """The layer whose tensors layer i uses (itself, usually)."""
+        seen = {i}
+        while (j := self.layers[i].weights_of) is not None:
+            if not 0 <= j < len(self.layers) or j in seen:
+                raise ValueError(f"layer {i}: weights_of {j}")
+            seen.add(j)
+            i = j
+        return i
+
+    @property
+    def params(self) -> int:
+        w = self.hidden
+        total = (self.vocab + self.positions + 1) * w
+        for ly in self.layers:
+            if ly.weights_of is None:
+                total += ly.mixer.params(w) + w
+                if ly.ff is not None:
+                    total += ly.ff.params(w) + w
+        return total
+
+
+Spec = Union[ModelSpec, HybridSpec]
+
+
+def _take(d: dict, what: str, keys: tuple, optional: tuple = ()) -> dict:
+    """d, if it has all of keys and nothing beyond keys and optional."""
+    missing = [k for k in keys if k not in d]
+    extra = [k for k in d if k not in keys and k not in optional]
+    if missing or extra:
+        raise ValueError(f"config: {what} lacks {missing}, has unknown "
+                         f"{extra}")
+    return d
+
+
+def _read_mixer(kind: str, d: dict):
+    if kind == "attention":
+        _take(d, "attention mixer",
+              ("heads", "kv_heads", "dim", "vdim", "scale"), ("q_temp",))
+        t = d.get("q_temp")
+        extra = {}
+        if t is not None:
+            _take(t, "q_temp", ("coef", "every"))
+            extra = {"q_coef": float(t["coef"]), "q_every": int(t["every"])}
+        return AttentionMixer(heads=d["heads"], kv_heads=d["kv_heads"],
+                              dim=d["dim"], vdim=d["vdim"],
+                              scale=float(d["scale"]), **extra)
+    if kind == "mlstm":
+        _take(d, "mlstm mixer", ("heads", "dim", "vdim", "gate_cap"))
+        return MlstmMixer(heads=d["heads"], dim=d["dim"], vdim=d["vdim"],
+                          gate_cap=float(d["gate_cap"]))
+    raise ValueError(f"config: unknown mixer {kind!r}")
+
+
+def _read_ff(d: Optional[dict]):
+    if d is None:
+        return None
+    if d.get("kind") == "dense":
+        _take(d, "dense mlp", ("kind", "ff", "limit"))
+        return DenseFF(ff=d["ff"], limit=float(d["limit"]))
+    if d.get("kind") == "moe":
+        _take(d, "moe mlp", ("kind", "expert", "router"))
+        _take(d["expert"], "expert", ("ff",))
+        r = _take(d["router"], "router", ("experts", "top"))
+        return RoutedFF(experts=r["experts"], top=r["top"],
+                        ff=d["expert"]["ff"])
+    raise ValueError(f"config: unknown mlp kind {d.get('kind')!r}")
+
+
+def read_birepel(cfg: dict, name: str = "birepel") -> HybridSpec:
+    """Birepel's config.json -> spec."""
+    layers = tuple(
+        LayerSpec(mixer=_read_mixer(ly["type"], ly["mixer"]),
+                  ff=_read_ff(ly.get("mlp")), weights_of=ly.get("weights_of"))
+        for ly in cfg["layers"])
+    return HybridSpec(name=name, vocab=cfg["vocab"], hidden=cfg["width"],
+                      layers=layers, norm_eps=float(cfg["norm"]["eps"]),
+                      positions=cfg["max_positions"])
+
+
+# "architecture" in config.json -> reader. Checkpoints without that key (HF
+# layout) are loaded into the architecture that the model name gives.
+_READERS: dict[str, Callable[[dict, str], Spec]] = {"Birepel": read_birepel}
+
+
+def spec_from_dir(path: str) -> Optional[Spec]:
+    """Spec that a checkpoint folder's own config.json gives, or None if it
+    leaves the architecture to the model name."""
+    f = os.path.join(path, "config.json")
+    if not path or not os.path.isfile(f):
+        return None
+    with open(f) as fh:
+        cfg = json.load(fh)
+    arch = cfg.get("architecture")
+    if arch is None:
+        return None
+    if arch not in _READERS:
+        raise ValueError(f"{f}: unknown architecture {arch!r}; known: "
+                         f"{sorted(_READERS)}")
+    return _READERS[arch](cfg, f"{arch.lower()}:custom")
+
+
+def resolve_spec(model: str, weights_path: str = "",
+                 max_seq_len: int = 0) -> Spec:
+    """Spec of what an engine is to serve: a checkpoint folder that describes
+    itself wins over the name."""
+    spec = spec_from_dir(weights_path)
+    if spec is None:
+        return get_spec(model, max_seq_len)
+    if spec.name not in _SPECS or _SPECS[spec.name] != spec:
+        register_spec(spec)
+    return replace(spec, max_seq_len=max_seq_len) if max_seq_len else spec
+
+
+_SPECS: dict[str, Spec] = {}
+
+
+def _reg(spec: Spec, *aliases: str) -> None:
     _SPECS[spec.name] = spec
     for a in aliases:
         _SPECS[a] = spec
@@ -95,7 +311,40 @@ _reg(ModelSpec("tiny-qwen", hidden=128, layers=2, heads=4, kv_heads=2,
      "tiny-qwen:latest")
 
 
-def get_spec(name: str, max_seq_len: int = 0) -> ModelSpec:
+# Birepel: xLSTM-style mLSTM layers with a few softmax-attention layers between
+# them, routed experts, the last attention layer sharing an earlier one's
+# weights. "tiny-birepel" for CPU tests and CI; the other has layers of a real
+# model's size
+def birepel_stack(name: str, *, vocab: int, hidden: int, attn: AttentionMixer,
+                  rec: MlstmMixer, dense: DenseFF, routed: RoutedFF,
+                  blocks: int, positions: int) -> HybridSpec:
+    """A dense-fed mLSTM layer, then `blocks` times (attention, 2 x mLSTM) fed
+    by experts, then the first attention layer once more."""
+    layers = [LayerSpec(rec, dense)]
+    for _ in range(blocks):
+        layers += [LayerSpec(attn, routed)] + [LayerSpec(rec, routed)] * 2
+    layers.append(LayerSpec(attn, routed, weights_of=1))
+    return HybridSpec(name, vocab=vocab, hidden=hidden, layers=tuple(layers),
+                      norm_eps=1e-5, positions=positions)
+
+
+_reg(birepel_stack("tiny-birepel", vocab=512, hidden=128, blocks=1,
+                   positions=256,
+                   attn=AttentionMixer(4, 2, 32, 32, 32 ** -0.5, 0.1, 64),
+                   rec=MlstmMixer(2, 32, 48, 15.0), dense=DenseFF(256, 7.0),
+                   routed=RoutedFF(8, 2, 64)),
+     "tiny-birepel:latest")
+_reg(birepel_stack("birepel:3b", vocab=128256, hidden=3072, blocks=2,
+                   positions=16384,
+                   attn=AttentionMixer(24, 8, 128, 128, 128 ** -0.5, 0.1,
+                                       8192),
+                   rec=MlstmMixer(12, 128, 256, 15.0),
+                   dense=DenseFF(8192, 7.0),
+                   routed=RoutedFF(64, 8, 1024)),
+     "birepel-3b")
+
+
+def get_spec(name: str, max_seq_len: int = 0) -> Spec:
     key = name.strip()
     if key not in _SPECS:
         raise KeyError(f"unknown model {name!r}; known: {sorted(set(_SPECS))}")
@@ -109,7 +358,7 @@ def list_specs() -> list[str]:
     return sorted({s.name for s in _SPECS.values()})
 
 
-def register_spec(spec: ModelSpec, *aliases: str) -> None:
+def register_spec(spec: Spec, *aliases: str) -> None:
     """Register a custom architecture at runtime (tests, custom configs)."""
     _reg(spec, *aliases)
 

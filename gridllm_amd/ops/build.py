@@ -25,7 +25,7 @@ ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950")
 # library name -> source. "hip": what every model shares and the Llama
 # family's attention; "hybrid": layer-list models (paged attention, mLSTM,
 # routed experts)
-LIBS = {"hip": "gridllm_kernels.hip"}
+LIBS = {"hip": "gridllm_kernels.hip", "hybrid": "gridllm_hybrid.hip"}
 
 # hipcc otherwise forms packed-FP32 instructions from plain float code; some
 # of their forms give wrong results on this hardware, so all HIP code is

@@ -1,0 +1,38 @@
+"""Ops of the layer-list models: HIP kernels for tensors on the GPU, the
+PyTorch reference for tensors on the CPU (see hip_hybrid for what each does)."""
+
+from __future__ import annotations
+
+import torch
+
+from gridllm_amd.ops import hip_hybrid, reference_hybrid
+from gridllm_amd.ops import reference
+from gridllm_amd.ops.reference_hybrid import StepMeta  # noqa: F401
+
+
+def _dispatch(name: str):
+    hip, ref = getattr(hip_hybrid, name), getattr(reference_hybrid, name)
+
+    def op(t: torch.Tensor, *args, **kw):
+        return (hip if t.is_cuda else ref)(t, *args, **kw)
+
+    op.__name__, op.__doc__ = name, hip.__doc__
+    return op
+
+
+embed_pos = _dispatch("embed_pos")
+post_norm = _dispatch("post_norm")
+norm_rows = _dispatch("norm_rows")
+proj_f32 = _dispatch("proj_f32")
+qknorm_kv = _dispatch("qknorm_kv")
+paged_attn = _dispatch("paged_attn")
+mlstm = _dispatch("mlstm")
+moe = _dispatch("moe")
+
+
+def glu(gateup: torch.Tensor, p: reference.Glu) -> torch.Tensor:
+    """act(gateup[:, :F], gateup[:, F:]) in the input's type."""
+    if gateup.is_cuda and gateup.dtype == torch.float32:
+        return hip_hybrid.glu_f32(gateup, p)
+    from gridllm_amd import ops
+    return ops.swiglu(gateup, p)
