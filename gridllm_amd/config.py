@@ -138,6 +138,9 @@ class EngineConfig:
     use_hipgraph: bool = True                  # capture decode step in a hipGraph
     autotune: bool = True                      # per-shape GEMM dispatch tuning
     context_shift: bool = True                 # slide the KV window past max_seq
+    kv_tokens: int = 0         # paged models: KV pool in tokens; 0 -> max_batch
+                               # sequences of full length
+    prefill_chunk: int = 8192  # mixed-step models: prompt tokens per step
     weights_path: str = ""                     # safetensors dir; empty -> random init
     seed: int = 0
 
@@ -153,6 +156,8 @@ class EngineConfig:
             use_hipgraph=_env_int("ENGINE_HIPGRAPH", 1, 0, 1) == 1,
             autotune=_env_int("ENGINE_AUTOTUNE", 1, 0, 1) == 1,
             context_shift=_env_int("ENGINE_CONTEXT_SHIFT", 1, 0, 1) == 1,
+            kv_tokens=_env_int("ENGINE_KV_TOKENS", 0),
+            prefill_chunk=_env_int("ENGINE_PREFILL_CHUNK", 8192, 1),
             weights_path=_env_str("ENGINE_WEIGHTS", ""),
             seed=_env_int("ENGINE_SEED", 0),
         )

@@ -247,6 +247,7 @@ class Batcher:
                                 or op.get("frequency_penalty"))
                 use_async = (inflight is not None
                              and not eng.tp.enabled
+                             and not eng.mixed
                              and all(_async_ok(op) for _, op, *_ in items))
                 try:
                     if use_async:

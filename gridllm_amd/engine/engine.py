@@ -24,8 +24,8 @@ from gridllm_amd.config import EngineConfig
 from gridllm_amd.engine import chat as chat_mod
 from gridllm_amd.engine.sampler import SamplerState, sample
 from gridllm_amd.engine.tokenizer import load_tokenizer
-from gridllm_amd.models.llama import LlamaModel
-from gridllm_amd.models.registry import get_spec
+from gridllm_amd.models import model_class
+from gridllm_amd.models.registry import resolve_spec
 from gridllm_amd.parallel.tp import TPContext
 from gridllm_amd.types import SamplingOptions
 from gridllm_amd.utils.logging import get_logger
@@ -71,6 +71,8 @@ class _Row:
     t_decode_ns: int = 0           # wall clock when prefill+first token done
     cur_len: int = 0               # storage length in the KV slot
     constraint: object = None      # grammar automaton (format="json")
+    todo: list[int] = field(default_factory=list)   # prompt tokens not run yet
+                                   # (models with mixed steps)
 
 
 class InferenceEngine:
@@ -88,18 +90,30 @@ class InferenceEngine:
         dtype = self.cfg.dtype
         if not self.is_gpu and dtype != "fp32":
             dtype = "fp32"          # CPU reference path runs fp32
-        spec = get_spec(self.cfg.model, self.cfg.max_seq_len)
+        if self.cfg.max_batch_size < 1:
+            raise ValueError("max_batch_size must be at least 1")
+        spec = resolve_spec(self.cfg.model, self.cfg.weights_path,
+                            self.cfg.max_seq_len)
         t0 = time.monotonic_ns()
+        import glob as _glob
+        import os as _os
+        have_weights = bool(self.cfg.weights_path) and bool(_glob.glob(
+            _os.path.join(self.cfg.weights_path, "*.safetensors")))
+        cls = model_class(spec)
+        # a model with mixed steps runs portions of prompts beside decoded
+        # tokens; its KV memory is a pool of tokens, not of full-length slots
+        self.mixed = getattr(cls, "supports_mixed", False)
+        self.shift_ok = (self.cfg.context_shift
+                         and getattr(cls, "supports_shift", True))
+        extra = {"kv_tokens": self.cfg.kv_tokens,
+                 "random_init": not have_weights} if self.mixed else {}
         # +1 scratch slot for hipGraph warmup/padding rows
-        self.model = LlamaModel(spec, device=str(self.device), dtype=dtype,
-                                tp=self.tp, seed=self.cfg.seed,
-                                kv_slots=self.cfg.max_batch_size + 1,
-                                max_seq=self.cfg.max_seq_len)
+        self.model = cls(spec, device=str(self.device), dtype=dtype,
+                         tp=self.tp, seed=self.cfg.seed,
+                         kv_slots=self.cfg.max_batch_size + 1,
+                         max_seq=self.cfg.max_seq_len, **extra)
         if self.cfg.weights_path:
-            import glob as _glob
-            import os as _os
-            if _glob.glob(_os.path.join(self.cfg.weights_path,
-                                        "*.safetensors")):
+            if have_weights:
                 n = self.model.load_safetensors(self.cfg.weights_path)
                 log.performance("weights loaded", tensors=n,
                                 path=self.cfg.weights_path)
@@ -238,6 +252,7 @@ class InferenceEngine:
         slots_t: optional prebuilt device int32 slot tensor (callers that
         also sample by slot share ONE upload per step)."""
         b = len(token_ids)
+        self.model.cache.prepare_decode(slot_ids)
         if self._graph_ok():
             bucket = self._bucket(b)
             try:
@@ -270,6 +285,88 @@ class InferenceEngine:
         slots = slots_t if slots_t is not None else torch.as_tensor(
             slot_ids, dtype=torch.int32, device=self.device)
         return self.model.forward_decode(tokens, slots)
+
+    # -------------------------------------------------------- mixed steps
+    # (models with supports_mixed: the step that generation runs on, and the
+    #  way to feed given tokens, e.g. to replay a trace)
+
+    def open_sequence(self, tokens: int = 0) -> int:
+        """A fresh sequence; `tokens` > 0 sets memory aside for that many,
+        otherwise it grows while there is some. Returns its slot."""
+        with self._lock:
+            return self.model.cache.alloc(tokens)
+
+    def close_sequence(self, slot: int) -> None:
+        with self._lock:
+            self.model.cache.free(slot)
+
+    def run_step(self, entries: Sequence[tuple]) -> torch.Tensor:
+        """Run one batch of (slot, token ids, wanted places) and return the
+        logits f32 [wanted, vocab] in that order."""
+        with self._lock:
+            return self._run_step(entries)
+
+    def _run_step(self, entries: Sequence[tuple]) -> torch.Tensor:
+        if not self.mixed:
+            raise NotImplementedError(
+                f"{self.spec.name} has no mixed steps")
+        lens = self.model.cache.lens
+        if all(len(ids) == 1 and lens[sl] > 0 for sl, ids, _ in entries):
+            # nothing but decoding: the captured step
+            for _, ids, _ in entries:
+                if not 0 <= ids[0] < self.spec.vocab:
+                    raise ValueError("token id outside of the vocabulary")
+            logits = self._decode_step([ids[0] for _, ids, _ in entries],
+                                       [sl for sl, _, _ in entries])
+            if all(list(w) == [0] for _, _, w in entries):
+                return logits
+            return logits[[i for i, e in enumerate(entries) for _ in e[2]]]
+        return self.model.forward_step(entries)
+
+    def _mixed_step(self, active: list["_Row"]) -> list["_Row"]:
+        """One step in which some rows still have prompt tokens to run: the
+        others decode their next token beside as many prompt tokens, in order
+        of admission, as the step's budget takes. Returns the rows still
+        running."""
+        for r in active:
+            if r.todo and self._cancelled(r):
+                r.result.done_reason = "cancelled"
+                r.result.cancelled = True
+                self._retire(r)
+        active = [r for r in active if not r.done]
+        left = self.cfg.prefill_chunk
+        entries, emitting = [], []
+        for r in active:
+            if not r.todo:
+                entries.append((r.slot, [r.last_token], [0]))
+                emitting.append(r)
+                r.cur_len += 1
+                continue
+            part = r.todo[:left]
+            if not part:
+                continue
+            left -= len(part)
+            r.todo = r.todo[len(part):]
+            entries.append((r.slot, part, [] if r.todo else [len(part) - 1]))
+            if not r.todo:
+                emitting.append(r)
+        if not entries:
+            return active
+        logits = self._run_step(entries)
+        if not emitting:
+            return active
+        slots = self.model.up.upload(
+            np.asarray([r.slot for r in emitting], dtype=np.int64))
+        toks = self._sample_batch(logits, emitting, slots)
+        t1 = time.monotonic_ns()
+        for r, tok in zip(emitting, toks):
+            first = r.t_decode_ns == 0
+            if first:
+                r.result.prompt_eval_duration = t1 - r.t_start_ns
+                r.t_decode_ns = t1
+            if not (self._emit(r, tok) and (r.max_new > 1 or not first)):
+                self._retire(r)
+        return [r for r in active if not r.done]
 
     # ------------------------------------------------------------- sampling
 
@@ -349,7 +446,7 @@ class InferenceEngine:
                 hiddens = []
                 for j0 in range(0, len(chunk), nslots):
                     part = token_lists[j0:j0 + nslots]
-                    slots = [self.model.cache.alloc() for _ in part]
+                    slots = [self.model.cache.alloc(len(t)) for t in part]
                     try:
                         _, h = self.model.forward_prefill_batch(
                             part, slots, return_hidden=True)
@@ -464,6 +561,13 @@ class InferenceEngine:
             return rows
 
     def _start_rows(self, items: list[tuple]) -> list["_Row"]:
+        if self.mixed:
+            # nothing runs yet: the prompts go through the next steps
+            rows, id_lists = self._make_rows(items)
+            for row, ids in zip(rows, id_lists):
+                row.todo = list(ids)
+            self.sampler.admit(rows, self.spec.vocab)
+            return rows
         rows, logits, slots_t = self._prefill_rows(items)
         try:
             toks = self._sample_batch(logits, rows, slots_t)  # syncs
@@ -479,7 +583,8 @@ class InferenceEngine:
                 self._retire(row)
         return rows
 
-    def _prefill_rows(self, items: list[tuple]):
+    def _make_rows(self, items: list[tuple]):
+        """Rows with a cache slot each, and their prompts' token ids."""
         t0 = time.monotonic_ns()
         rows: list[_Row] = []
         id_lists: list[list[int]] = []
@@ -491,8 +596,6 @@ class InferenceEngine:
                 if opts.num_ctx:
                     ids = ids[-max(16, min(opts.num_ctx,
                                            self.model.max_seq - 8)):]
-                slot = self.model.cache.alloc()
-                slots.append(slot)
                 id_lists.append(ids)
                 stops = list(opts.stop or [])
                 if extra_stops:
@@ -504,7 +607,7 @@ class InferenceEngine:
                 max_new = opts.num_predict \
                     if opts.num_predict and opts.num_predict > 0 \
                     else (1 << 30)
-                if self.cfg.context_shift:
+                if self.shift_ok:
                     # the KV window slides, so generation is bounded by the
                     # rope table (original absolute positions), not max_seq
                     max_new = min(max_new,
@@ -528,6 +631,11 @@ class InferenceEngine:
                         from gridllm_amd.engine.schema_constraints import \
                             JsonSchemaByteConstraint
                         constraint = JsonSchemaByteConstraint(opts.format)
+                # tokens the slot may come to hold (a pipelined retire runs
+                # one decode step too many)
+                slot = self.model.cache.alloc(
+                    min(self.model.max_seq, len(ids) + max_new + 1))
+                slots.append(slot)
                 row = _Row(slot=slot,
                            state=SamplerState.create(opts, self.device),
                            decoder=self.tokenizer.decode_stream(),
@@ -544,6 +652,11 @@ class InferenceEngine:
             for sl in slots:          # release what this batch allocated
                 self.model.cache.free(sl)
             raise
+        return rows, id_lists
+
+    def _prefill_rows(self, items: list[tuple]):
+        rows, id_lists = self._make_rows(items)
+        slots = [r.slot for r in rows]
         try:
             # ONE pinned upload for every prompt's ids (one blocking H2D
             # per prompt measured ~1.5 ms each against a busy stream)
@@ -581,7 +694,9 @@ class InferenceEngine:
 
     def _step_rows(self, active: list["_Row"]) -> list["_Row"]:
         """One batched decode step; returns the rows still running."""
-        if self.cfg.context_shift:
+        if any(r.todo for r in active):
+            return self._mixed_step(active)
+        if self.shift_ok:
             for r in active:
                 if r.cur_len >= self.model.max_seq:
                     r.cur_len = self.model.shift_slot(r.slot)
@@ -619,7 +734,7 @@ class InferenceEngine:
         if self.tp.enabled:
             return False
         for r in rows:
-            if r.constraint is not None or r.state.has_penalty:
+            if r.todo or r.constraint is not None or r.state.has_penalty:
                 return False
             if r.cur_len + 2 > self.model.max_seq:
                 return False
@@ -673,7 +788,7 @@ class InferenceEngine:
         with self._lock:
             import numpy as np
             b = len(rows)
-            if self.cfg.context_shift:
+            if self.shift_ok:
                 for r in rows:
                     if r.cur_len >= self.model.max_seq:
                         r.cur_len = self.model.shift_slot(r.slot)
@@ -735,6 +850,8 @@ class InferenceEngine:
                         ap["ids_dev"][up[3].clamp(min=0)], tokens_dev)
                 slots64 = up[2]
                 slots32 = slots64.to(torch.int32)
+            if self.mixed:
+                self.model.cache.prepare_decode([r.slot for r in rows])
             if self._graph_ok():
                 bucket = self._bucket(b)
                 try:

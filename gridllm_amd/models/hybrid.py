@@ -92,6 +92,8 @@ class HybridModel:
         self.device = torch.device(device)
         self.dtype = _DTYPES[dtype]
         self.max_seq = min(max_seq or spec.max_seq_len, spec.positions)
+        if kv_tokens:                      # one sequence has to fit the pool
+            self.max_seq = min(self.max_seq, pad64(kv_tokens))
         self.rope_len = self.max_seq       # bound of positions
         self.width = pad64(spec.hidden)
         if self.width > 8192:

@@ -73,7 +73,10 @@ class KVCache:
         if slot in self._free:
             self._free.remove(slot)
 
-    def alloc(self) -> int:
+    def prepare_decode(self, slots) -> None:
+        """Slots are contiguous: nothing to assign ahead of a step."""
+
+    def alloc(self, tokens: int = 0) -> int:
         """HOST-ONLY bookkeeping: seq_lens/rope_off for the slot are
         (re)initialized by the next prefill's batched scatter — a per-slot
         scalar device write here measured ~0.5 ms of stream-sync stall per
@@ -94,6 +97,9 @@ class KVCache:
 
 
 class LlamaModel:
+    supports_mixed = False
+    supports_shift = True
+
     def __init__(self, spec: ModelSpec, device: str = "cpu",
                  dtype: str = "bf16", tp: Optional[TPContext] = None,
                  seed: int = 0, kv_slots: int = 64, max_seq: int = 0):

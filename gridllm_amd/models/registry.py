@@ -30,6 +30,23 @@ class ModelSpec:
     tie_embeddings: bool = True
     qkv_bias: bool = False         # Qwen2-family: bias on q/k/v projections
 
+    family = "llama"
+
+    def model_info(self) -> dict:
+        """Ollama-style model_info of /api/show."""
+        return {
+            "general.architecture": "llama",
+            "general.parameter_count": self.params,
+            "llama.block_count": self.layers,
+            "llama.embedding_length": self.hidden,
+            "llama.attention.head_count": self.heads,
+            "llama.attention.head_count_kv": self.kv_heads,
+            "llama.feed_forward_length": self.intermediate,
+            "llama.context_length": self.max_seq_len,
+            "llama.vocab_size": self.vocab,
+            "llama.rope.freq_base": self.rope_theta,
+        }
+
     @property
     def params(self) -> int:
         h, f, v = self.hidden, self.intermediate, self.vocab
@@ -152,6 +169,31 @@ class HybridSpec:
             i = j
         return i
 
+    family = "birepel"
+
+    def model_info(self) -> dict:
+        """Ollama-style model_info of /api/show."""
+        attn = [ly.mixer for ly in self.layers
+                if isinstance(ly.mixer, AttentionMixer)]
+        routed = [ly.ff for ly in self.layers if isinstance(ly.ff, RoutedFF)]
+        f = self.family
+        info = {
+            "general.architecture": f,
+            "general.parameter_count": self.params,
+            f"{f}.block_count": len(self.layers),
+            f"{f}.embedding_length": self.hidden,
+            f"{f}.context_length": self.max_seq_len,
+            f"{f}.vocab_size": self.vocab,
+        }
+        if attn:
+            info |= {f"{f}.attention.block_count": len(attn),
+                     f"{f}.attention.head_count": attn[0].heads,
+                     f"{f}.attention.head_count_kv": attn[0].kv_heads}
+        if routed:
+            info |= {f"{f}.expert_count": routed[0].experts,
+                     f"{f}.expert_used_count": routed[0].top}
+        return info
+
     @property
     def params(self) -> int:
         w = self.hidden
@@ -227,9 +269,9 @@ def read_birepel(cfg: dict, name: str = "birepel") -> HybridSpec:
 _READERS: dict[str, Callable[[dict, str], Spec]] = {"Birepel": read_birepel}
 
 
-def spec_from_dir(path: str) -> Optional[Spec]:
-    """Spec that a checkpoint folder's own config.json gives, or None if it
-    leaves the architecture to the model name."""
+def spec_from_dir(path: str, name: str = "") -> Optional[Spec]:
+    """Spec that a checkpoint folder's own config.json gives, under `name`, or
+    None if it leaves the architecture to the model name."""
     f = os.path.join(path, "config.json")
     if not path or not os.path.isfile(f):
         return None
@@ -241,14 +283,14 @@ def spec_from_dir(path: str) -> Optional[Spec]:
     if arch not in _READERS:
         raise ValueError(f"{f}: unknown architecture {arch!r}; known: "
                          f"{sorted(_READERS)}")
-    return _READERS[arch](cfg, f"{arch.lower()}:custom")
+    return _READERS[arch](cfg, name or f"{arch.lower()}:custom")
 
 
 def resolve_spec(model: str, weights_path: str = "",
                  max_seq_len: int = 0) -> Spec:
     """Spec of what an engine is to serve: a checkpoint folder that describes
     itself wins over the name."""
-    spec = spec_from_dir(weights_path)
+    spec = spec_from_dir(weights_path, model if model not in _SPECS else "")
     if spec is None:
         return get_spec(model, max_seq_len)
     if spec.name not in _SPECS or _SPECS[spec.name] != spec:

@@ -331,24 +331,13 @@ def build_router(scheduler: JobScheduler, registry: WorkerRegistry) -> APIRouter
         try:
             from gridllm_amd.models.registry import get_spec
             spec = get_spec(model)
-            info = {
-                "general.architecture": "llama",
-                "general.parameter_count": spec.params,
-                "llama.block_count": spec.layers,
-                "llama.embedding_length": spec.hidden,
-                "llama.attention.head_count": spec.heads,
-                "llama.attention.head_count_kv": spec.kv_heads,
-                "llama.feed_forward_length": spec.intermediate,
-                "llama.context_length": spec.max_seq_len,
-                "llama.vocab_size": spec.vocab,
-                "llama.rope.freq_base": spec.rope_theta,
-            }
+            info, family = spec.model_info(), spec.family
         except KeyError:
-            info = {}
+            info, family = {}, "llama"
         return JSONResponse({
             "modelfile": "", "parameters": "", "template": "",
             "details": {"parent_model": "", "format": "safetensors",
-                        "family": "llama", "families": ["llama"],
+                        "family": family, "families": [family],
                         "parameter_size": "", "quantization_level": "BF16"},
             "model_info": info,
             "capabilities": ["completion", "chat", "embedding"],
