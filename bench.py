@@ -500,14 +500,123 @@ def engine_mode(args, rank, world, local_rank, dist, device, on_gpu):
         print(json.dumps(out))
 
 
+def layers_mode(args, rank, world, local_rank, dist, device, on_gpu):
+    """Prefill and decode throughput of a layer-list model beside a Llama of
+    the same widths, heads and active feed-forward size (random weights, no
+    serving glue): one step function call per timed iteration, decode through
+    the captured graphs."""
+    from dataclasses import replace
+
+    from gridllm_amd.config import EngineConfig
+    from gridllm_amd.engine import InferenceEngine
+    from gridllm_amd.models.registry import (AttentionMixer, ModelSpec,
+                                             get_spec, register_spec)
+
+    if args.layers_model:
+        name = args.layers_model
+    else:
+        name = "birepel:3b" if on_gpu else "tiny-birepel"
+    spec = get_spec(name)
+    mx = next(ly.mixer for ly in spec.layers
+              if isinstance(ly.mixer, AttentionMixer))
+    ff = next((f.top * f.ff for f in (ly.ff for ly in spec.layers)
+               if hasattr(f, "top")), spec.layers[0].ff.ff)
+    twin = ModelSpec(f"{name}-llama-twin", hidden=spec.hidden,
+                     layers=len(spec.layers), heads=mx.heads,
+                     kv_heads=mx.kv_heads, head_dim=mx.dim, intermediate=ff,
+                     vocab=spec.vocab, max_seq_len=spec.max_seq_len)
+    register_spec(twin)
+    # (sequences, tokens each) and (rows, context)
+    prefills = [(1, 8192), (8, 1024), (1, 512)] if on_gpu else [(2, 32)]
+    decodes = [(1, 1024), (16, 1024), (64, 1024), (256, 1024)] \
+        if on_gpu else [(2, 32)]
+    top_b = max(b for b, _ in decodes + prefills)
+    results = {}
+    for which, sp in (("model", spec), ("llama_twin", twin)):
+        register_spec(replace(sp, max_seq_len=8192 if on_gpu else 128))
+        eng = InferenceEngine(EngineConfig(
+            model=sp.name, device=device, dtype="bf16" if on_gpu else "fp32",
+            max_seq_len=8192 if on_gpu else 128, max_batch_size=top_b,
+            use_hipgraph=on_gpu))
+        m, cache, out = eng.model, eng.model.cache, {}
+
+        def timed(fn, reset=lambda: None):
+            for _ in range(args.warmup):
+                fn()
+                reset()
+            total = 0.0
+            for _ in range(args.steps):
+                eng._sync()
+                t0 = time.monotonic()
+                fn()
+                eng._sync()
+                total += time.monotonic() - t0
+                reset()
+            return total / args.steps
+
+        for b, t in prefills:
+            toks = [torch.randint(0, sp.vocab, (t,), device=eng.device)
+                    for _ in range(b)]
+            slots = []
+
+            def run():
+                slots[:] = [cache.alloc(t) for _ in toks]
+                if b == 1:
+                    m.forward_prefill(toks[0], slots[0])
+                else:
+                    m.forward_prefill_batch(toks, slots)
+
+            def give_back():
+                for sl in slots:
+                    cache.free(sl)
+
+            dt = timed(run, give_back)
+            out[f"prefill_{b}x{t}_tok_s"] = round(b * t / dt, 1)
+        for b, ctx in decodes:
+            slots = [cache.alloc(2 * ctx) for _ in range(b)]
+            for i in range(0, b, 8):
+                part = slots[i:i + 8]
+                toks = [torch.randint(0, sp.vocab, (ctx,), device=eng.device)
+                        for _ in part]
+                if len(part) == 1:
+                    m.forward_prefill(toks[0], part[0])
+                else:
+                    m.forward_prefill_batch(toks, part)
+            ids = [1 + i % 100 for i in range(b)]
+            dt = timed(lambda: eng._decode_step(ids, slots))
+            out[f"decode_b{b}_tok_s"] = round(b / dt, 1)
+            for sl in slots:
+                cache.free(sl)
+        results[which] = out
+        results[which + "_params"] = sp.params
+        del eng, m, cache
+        if on_gpu:
+            torch.cuda.empty_cache()
+    if rank == 0:
+        key = f"decode_b{decodes[-1][0]}_tok_s"
+        print(json.dumps({
+            "metric": f"decode tokens/sec, {name} layers, batch "
+                      f"{decodes[-1][0]} (raw engine step)",
+            "value": results["model"][key], "unit": "tokens/s",
+            "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+            "ms_per_step": round(1000.0 * decodes[-1][0]
+                                 / results["model"][key], 3),
+            "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+            "dtype": "bf16" if on_gpu else "fp32", "data": "synthetic",
+            "config": {"model": name, "mode": "layers", **results}}))
+
+
 def main() -> None:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=8)
     ap.add_argument("--warmup", type=int, default=2)
-    ap.add_argument("--mode", choices=["serving", "engine"],
+    ap.add_argument("--mode", choices=["serving", "engine", "layers"],
                     default="serving")
     ap.add_argument("--model", default="llama3.2:3b")
+    ap.add_argument("--layers-model", default="",
+                    help="layers: layer-list model to time beside its "
+                         "Llama twin (default birepel:3b)")
     ap.add_argument("--concurrency", type=int, default=1024,
                     help="serving: concurrent streams per GPU")
     ap.add_argument("--num-predict", type=int, default=128,
@@ -551,6 +660,8 @@ def main() -> None:
 
     if args.mode == "serving":
         serving_mode(args, rank, world, local_rank, dist, device, on_gpu)
+    elif args.mode == "layers":
+        layers_mode(args, rank, world, local_rank, dist, device, on_gpu)
     else:
         engine_mode(args, rank, world, local_rank, dist, device, on_gpu)
 

@@ -158,7 +158,8 @@ class PagedCache:
             return
         ch = np.asarray(self._changes, dtype=np.int64).T
         self._changes = []
-        dev = self._upload(ch) if self._upload else torch.from_numpy(ch.copy())
+        dev = self._upload(ch) if self._upload else \
+            torch.from_numpy(np.ascontiguousarray(ch)).to(self.device)
         self.table.view(-1).index_copy_(0, dev[0], dev[1].to(torch.int32))
 
     @property

@@ -25,6 +25,28 @@ def query_temperature(pos, coef, every):
     return 1 + coef * torch.log(steps.to(torch.float64) + 1)
 
 
+def attend(q, k, v, scale, sink=None):
+    """Causal softmax attention of one sequence, a sink in the denominator.
+    q [t, H, d], k [t, G, d], v [t, G, dv] -> [t, H, dv]."""
+    t, H, _ = q.shape
+    G, dv = k.shape[1], v.shape[2]
+    pos = torch.arange(t)
+    out = torch.zeros(t, H, dv, dtype=q.dtype)
+    for hd in range(H):
+        kv = hd // (H // G)
+        s = q[:, hd] @ k[:, kv].T * scale
+        s = s.masked_fill(pos[None, :] > pos[:, None], float("-inf"))
+        top = s.max(-1).values
+        if sink is not None:
+            top = torch.maximum(top, sink[hd])
+        e = torch.exp(s - top[:, None])
+        den = e.sum(-1)
+        if sink is not None:
+            den = den + torch.exp(sink[hd] - top)
+        out[:, hd] = (e @ v[:, kv]) / den[:, None]
+    return out
+
+
 def attention(h, w, c, eps):
     """Grouped causal attention: unit-RMS q and k, a query temperature, one
     extra sink term per head in the denominator, one output gate per head."""
@@ -33,22 +55,10 @@ def attention(h, w, c, eps):
     q = rms((h @ w["q"].T).view(t, H, d), eps)
     k = rms((h @ w["k"].T).view(t, G, d), eps)
     v = (h @ w["v"].T).view(t, G, dv)
-    pos = torch.arange(t)
-    temp = query_temperature(pos, c["q_temp"]["coef"],
+    temp = query_temperature(torch.arange(t), c["q_temp"]["coef"],
                              c["q_temp"]["every"]).to(h.dtype)
-    q = q * temp.view(t, 1, 1)
-    gate = torch.sigmoid(h @ w["g"].T)
-    out = torch.zeros(t, H, dv, dtype=h.dtype)
-    for hd in range(H):
-        kv = hd // (H // G)
-        s = q[:, hd] @ k[:, kv].T * c["scale"]
-        s = s.masked_fill(pos[None, :] > pos[:, None], float("-inf"))
-        e = torch.exp(s - torch.maximum(s.max(-1, keepdim=True).values,
-                                        w["sink"][hd]))
-        top = torch.maximum(s.max(-1).values, w["sink"][hd])
-        den = e.sum(-1) + torch.exp(w["sink"][hd] - top)
-        out[:, hd] = (e @ v[:, kv]) / den[:, None]
-    out = out * gate[:, :, None]
+    out = attend(q * temp.view(t, 1, 1), k, v, c["scale"], w["sink"])
+    out = out * torch.sigmoid(h @ w["g"].T)[:, :, None]
     return out.reshape(t, H * dv) @ w["o"].T
 
 
@@ -57,36 +67,44 @@ def soft_cap(x, cap):
 
 
 def mlstm_step(S, n, m, q, k, v, i, f):
-    """One token of one head. S [dim, vdim], n [dim], m scalar; q already
+    """One token of every head. S [H, dim, vdim], n [H, dim], m [H]; q already
     scaled; i and f are the logarithms of the gates. Returns o and the state."""
     m_new = torch.maximum(f + m, i)
     keep, put = torch.exp(f + m - m_new), torch.exp(i - m_new)
-    S = keep * S + put * torch.outer(k, v)
-    n = keep * n + put * k
-    den = torch.maximum((n @ q).abs(), torch.exp(-m_new)) + 1e-6
-    return (q @ S) / den, S, n, m_new
+    S = keep[:, None, None] * S + put[:, None, None] * k[:, :, None] * v[:, None]
+    n = keep[:, None] * n + put[:, None] * k
+    den = torch.maximum((n * q).sum(-1).abs(), torch.exp(-m_new)) + 1e-6
+    return (S * q[:, :, None]).sum(1) / den[:, None], S, n, m_new
+
+
+def mlstm_run(q, k, v, i, f):
+    """One sequence from a zero state. q, k [t, H, d], v [t, H, dv],
+    log gates [t, H] -> o [t, H, dv]."""
+    t, H, d = q.shape
+    S = torch.zeros(H, d, v.shape[2], dtype=q.dtype)
+    n = torch.zeros(H, d, dtype=q.dtype)
+    m = torch.zeros(H, dtype=q.dtype)
+    o = []
+    for p in range(t):
+        out, S, n, m = mlstm_step(S, n, m, q[p], k[p], v[p], i[p], f[p])
+        o.append(out)
+    return torch.stack(o)
+
+
+def mlstm_log_gates(zi, zf, cap):
+    return soft_cap(zi, cap), torch.nn.functional.logsigmoid(soft_cap(zf, cap))
 
 
 def mlstm(h, w, c, eps):
     t = h.shape[0]
     H, d, dv = c["heads"], c["dim"], c["vdim"]
-    q = (h @ w["q"].T).view(t, H, d) * d ** -0.5
-    k = (h @ w["k"].T).view(t, H, d)
-    v = (h @ w["v"].T).view(t, H, dv)
-    i = soft_cap(h @ w["i"].T + w["i.b"], c["gate_cap"])
-    f = torch.nn.functional.logsigmoid(
-        soft_cap(h @ w["f"].T + w["f.b"], c["gate_cap"]))
-    o = torch.zeros(t, H, dv, dtype=h.dtype)
-    for hd in range(H):
-        S = torch.zeros(d, dv, dtype=h.dtype)
-        n = torch.zeros(d, dtype=h.dtype)
-        m = torch.zeros((), dtype=h.dtype)
-        for p in range(t):
-            o[p, hd], S, n, m = mlstm_step(S, n, m, q[p, hd], k[p, hd],
-                                           v[p, hd], i[p, hd], f[p, hd])
+    i, f = mlstm_log_gates(h @ w["i"].T + w["i.b"], h @ w["f"].T + w["f.b"],
+                           c["gate_cap"])
+    o = mlstm_run((h @ w["q"].T).view(t, H, d) * d ** -0.5,
+                  (h @ w["k"].T).view(t, H, d), (h @ w["v"].T).view(t, H, dv),
+                  i, f)
     o = rms(o, eps).reshape(t, H * dv) * w["norm"]
-    o = o * torch.sigmoid(h @ w["g"].T)
-    return o @ w["o"].T
+    return (o * torch.sigmoid(h @ w["g"].T)) @ w["o"].T
 
 
 def clamped_glu(g, u, limit):

@@ -1,0 +1,769 @@
+"""Layer-list models (Birepel) against the plain implementation in
+hybrid_oracle: on the CPU in f32, on the GPU in f32 and bf16."""
+
+import io
+import json
+import os
+import subprocess
+import sys
+import time
+
+import numpy as np
+import pytest
+import torch
+
+sys.path.insert(0, os.path.dirname(os.path.abspath(__file__)))
+import hybrid_oracle as oracle  # noqa: E402
+
+from gridllm_amd.config import EngineConfig  # noqa: E402
+from gridllm_amd.engine import InferenceEngine  # noqa: E402
+from gridllm_amd.models.hybrid import HybridModel  # noqa: E402
+from gridllm_amd.models.paged import PagedCache  # noqa: E402
+from gridllm_amd.models.registry import (get_spec, read_birepel,  # noqa: E402
+                                         resolve_spec)
+from gridllm_amd.ops import hybrid as hops  # noqa: E402
+from gridllm_amd.ops.hybrid import StepMeta  # noqa: E402
+
+REPO = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+RUNS = [pytest.param(("cpu", "fp32"), id="cpu"),
+        pytest.param(("cuda:0", "fp32"), id="gpu-f32", marks=pytest.mark.gpu),
+        pytest.param(("cuda:0", "bf16"), id="gpu-bf16", marks=pytest.mark.gpu)]
+EXACT = RUNS[:2]
+
+
+@pytest.fixture(autouse=True)
+def one_thread():
+    """Thousands of tiny CPU products: threads only get in their way."""
+    n = torch.get_num_threads()
+    torch.set_num_threads(1)
+    yield
+    torch.set_num_threads(n)
+
+
+def attn(heads=4, kv_heads=2, dim=32, vdim=32, scale=0.2, coef=0.25, every=16):
+    return {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim,
+            "scale": scale, "q_temp": {"coef": coef, "every": every}}
+
+
+def rec(heads=2, dim=32, vdim=32, gate_cap=6.0):
+    return {"heads": heads, "dim": dim, "vdim": vdim, "gate_cap": gate_cap}
+
+
+def dense(ff=96, limit=0.8):
+    return {"kind": "dense", "ff": ff, "limit": limit}
+
+
+def routed(experts=5, top=2, ff=40):
+    return {"kind": "moe", "expert": {"ff": ff},
+            "router": {"experts": experts, "top": top}}
+
+
+def config(*layers, vocab=130, width=96, positions=512, eps=1e-5):
+    """layers: (mixer, mlp) or (mixer, mlp, weights_of)."""
+    out = []
+    for ly in layers:
+        d = {"type": "attention" if "kv_heads" in ly[0] else "mlstm",
+             "mixer": ly[0], "mlp": ly[1]}
+        if len(ly) > 2:
+            d["weights_of"] = ly[2]
+        out.append(d)
+    return {"architecture": "Birepel", "layers": out, "vocab": vocab,
+            "width": width, "max_positions": positions, "norm": {"eps": eps}}
+
+
+# every branch at once, sizes that need padding, a shared layer ahead of and
+# behind its owner
+FULL = config((attn(6, 3, 40, 24), None),
+              (rec(3, 40, 72), dense()),
+              (attn(4, 1, 72, 80, every=5), routed()),
+              (rec(1, 24, 16, gate_cap=2.5), routed(4, 4, 24)),
+              (rec(3, 40, 72), dense(), 1),
+              (attn(4, 1, 72, 80, every=5), routed(), 2))
+
+
+def weights_of(cfg, seed=0):
+    return oracle.random_weights(cfg, seed)
+
+
+def build(cfg, run, seed=0, slots=5, pool=0, W=None):
+    dev, dtype = run
+    m = HybridModel(read_birepel(cfg), device=dev, dtype=dtype,
+                    kv_slots=slots, kv_tokens=pool, random_init=False)
+    W = W or weights_of(cfg, seed)
+    m._assemble(lambda name: W[name].to(dev))
+    if dev != "cpu" and dtype == "bf16":
+        m.interleave_gateup()
+    return m
+
+
+def tokens(n, cfg=FULL, seed=0):
+    return np.random.default_rng(seed).integers(0, cfg["vocab"], n).tolist()
+
+
+def feed(m, slot, ids, sizes):
+    """Run ids in portions of `sizes` (the last one repeats); all logits."""
+    out, at, k = [], 0, 0
+    while at < len(ids):
+        n = sizes[min(k, len(sizes) - 1)]
+        part = ids[at:at + n]
+        out.append(m.forward_step([(slot, part, list(range(len(part))))]))
+        at, k = at + len(part), k + 1
+    return torch.cat(out).cpu()
+
+
+def whole(m, ids):
+    slot = m.cache.alloc(0)
+    out = feed(m, slot, ids, [len(ids)])
+    m.cache.free(slot)
+    return out
+
+
+def errors(got, want):
+    """Per row: rms difference over the row's own rms."""
+    want = want.to(torch.float64)
+    d = got.cpu().to(torch.float64) - want
+    return (d.pow(2).mean(-1) / want.pow(2).mean(-1)).sqrt()
+
+
+def close(got, want, run, exact=2e-4, coarse=0.04, odd=0.04):
+    """f32: every row. bf16: all but a few rows in which a close call of the
+    router went the other way."""
+    e = errors(got, want)
+    if run[1] == "fp32":
+        assert float(e.max()) < exact, float(e.max())
+    else:
+        bad = int((e > coarse).sum())
+        assert bad <= odd * len(e), (bad, len(e), float(e.max()))
+
+
+# ------------------------------------------------------------ each mechanism
+
+ALONE = {
+    "attention": config((attn(), None)),
+    "attention-one-kv-head": config((attn(12, 1, 64, 64), None)),
+    "attention-own-kv-heads": config((attn(3, 3, 96, 128), None)),
+    "attention-wide-heads": config((attn(2, 1, 160, 136, scale=0.1), None)),
+    "attention-no-temperature": config((attn(coef=0.0, every=1), None)),
+    "mlstm": config((rec(), None)),
+    "mlstm-narrow-keys": config((rec(2, 48, 200), None)),
+    "mlstm-wide-keys": config((rec(1, 130, 40), None)),
+    "mlstm-widest-keys": config((rec(1, 300, 64), None)),
+    "mlstm-one-head": config((rec(1, 64, 64, gate_cap=1.0), None)),
+    "dense": config((rec(1, 16, 16), dense(200, 0.5))),
+    "dense-wide-limit": config((rec(1, 16, 16), dense(64, 100.0))),
+    "routed": config((rec(1, 16, 16), routed(7, 3, 64))),
+    "routed-one": config((rec(1, 16, 16), routed(9, 1, 24))),
+    "routed-all": config((rec(1, 16, 16), routed(3, 3, 72))),
+    "routed-many": config((rec(1, 16, 16), routed(80, 6, 16))),
+    "wide-residual": config((rec(), dense()), width=200),
+    "coarse-eps": config((attn(), dense()), eps=0.05),
+}
+
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("name", sorted(ALONE))
+def test_mechanism_alone(name, run):
+    cfg = ALONE[name]
+    m = build(cfg, run)
+    ids = tokens(150, cfg)
+    trail = []
+    slot = m.cache.alloc(0)
+    got = m.forward_step([(slot, ids, list(range(len(ids))))], trail=trail)
+    want, layers = oracle.forward(cfg, weights_of(cfg), ids)
+    close(got, want, run)
+    close(trail[-1], layers[-1], run)
+
+
+@pytest.mark.parametrize("run", RUNS)
+def test_all_layers(run):
+    m = build(FULL, run)
+    ids = tokens(200)
+    trail = []
+    slot = m.cache.alloc(0)
+    got = m.forward_step([(slot, ids, list(range(200)))], trail=trail)
+    want, layers = oracle.forward(FULL, weights_of(FULL), ids)
+    for a, b in zip(trail, layers):
+        close(a, b, run, coarse=0.1, odd=0.1)
+    close(got, want, run, coarse=0.1, odd=0.1)
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("batch", [3, 40, 130, 600])
+def test_experts_at_every_tile_size(batch):
+    """The mean number of rows per expert picks the GEMM; all of them agree."""
+    e, w, f, top = 6, 128, 192, 2
+    g = torch.Generator().manual_seed(3)
+    x = torch.randn(batch, w, generator=g).bfloat16()
+    z = torch.randn(batch, e, generator=g)
+    up = (torch.randn(e, f, w, generator=g) * w ** -0.5).bfloat16()
+    dn = (torch.randn(e, w, f, generator=g) * f ** -0.5).bfloat16()
+    # one expert far more popular than the others
+    z[:, 2] += 2.0
+    ye, wt = hops.moe(x.cuda(), z.cuda(), up.cuda(), dn.cuda(), top)
+    idx = torch.topk(z, top).indices
+    sm = torch.softmax(torch.topk(z, top).values, -1)
+    assert torch.allclose(wt.cpu(), sm, atol=1e-6)
+    a = torch.relu(torch.einsum("nw,nkfw->nkf", x.float(), up[idx].float()))
+    want = torch.einsum("nkf,nkwf->nkw", (a ** 2).bfloat16().float(),
+                        dn[idx].float())
+    assert float(errors(ye.view(batch, top, w), want).max()) < 0.02
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("m", [1, 64, 100, 300])
+def test_fused_gate_projection_takes_the_constants(m):
+    """Every gated-unit path with a limit that cuts: the plain op, the
+    interleaved one, and the projection with the fused epilogue."""
+    from gridllm_amd.ops import hip_ops
+    from gridllm_amd.ops.reference import Glu
+    glu = Glu(1.702, 0.6, 1.0)
+    f, k = 256, 192
+    g = torch.Generator().manual_seed(m)
+    x = torch.randn(m, k, generator=g).bfloat16().cuda()
+    w = (torch.randn(2 * f, k, generator=g) * k ** -0.5).bfloat16().cuda()
+    il = w.view(2, f // 64, 64, k).transpose(0, 1).reshape(2 * f, k).contiguous()
+    gu = (x.float() @ w.float().T).cpu().double()
+    want = oracle.clamped_glu(gu[:, :f], gu[:, f:], 0.6)
+    rows = torch.nn.functional.linear(x, w)
+    outs = [hip_ops.swiglu(rows, glu=glu),
+            hip_ops.swiglu_il(torch.nn.functional.linear(x, il), glu=glu)]
+    if m <= 256:
+        outs += [hip_ops.gemm_proj(x, il, splitk=s, fuse_swiglu=True, glu=glu)
+                 for s in (1, 3)]
+    for got in outs:
+        assert float(errors(got, want).max()) < 0.02
+    exact = hops.glu((x.float() @ w.float().T), glu)
+    assert float(errors(exact, want).max()) < 1e-4
+
+
+# ------------------------------------------- keys and tokens that stand out
+
+def meta_for(cache, slot, start, ln, dev):
+    """Step of one entry, as forward_step lays it out."""
+    def t(a, w):
+        return torch.tensor(a, dtype=torch.int32, device=dev).view(-1, w)
+    st = StepMeta(nd=1 if ln == 1 else 0,
+                  pos=torch.arange(start, start + ln, dtype=torch.int32,
+                                   device=dev),
+                  slot=torch.full((ln,), slot, dtype=torch.int32, device=dev),
+                  table=cache.table, max_len=cache.max_seq)
+    if ln > 1:
+        st.segs = t([[0, ln, slot, start]], 4)
+        st.tiles = t([[0, ln, slot, q, start, 0, 0, 0]
+                      for q in range(0, ln, 128)], 8)
+        st.chunks = t([[c, min(64, ln - c), 0, 0]
+                       for c in range(0, ln, 64)], 4)
+        st.chunk_segs = t([[slot, start, 0, -(-ln // 64)]], 4)
+    return st
+
+
+def portions(n, how):
+    cuts, at = [], 0
+    while at < n:
+        ln = min(how[min(len(cuts), len(how) - 1)], n - at)
+        cuts.append((at, ln))
+        at += ln
+    return cuts
+
+
+CUTS = {"whole": [300], "decode-tail": [190, 1], "pairs": [250, 2],
+        "odd": [63, 2, 1, 64, 65]}
+
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("how", sorted(CUTS))
+def test_one_key_stands_out(how, run):
+    """Every query looks for one key: the first, the neighbours of page
+    borders, itself, the previous one; for some it is the next one, which it
+    must not see. Sinks from negligible to dominating."""
+    dev, dtype = run
+    H, G, d, n = 4, 2, 64, 300
+    cfg = config((attn(H, G, d, d), None), positions=320)
+    cache = PagedCache(read_birepel(cfg), 3, 320, torch.device(dev),
+                       torch.float32 if dtype == "fp32" else torch.bfloat16)
+    cache.alloc(70)                       # page 1 and 2 belong to another
+    slot = cache.alloc(0)
+    g = torch.Generator().manual_seed(5)
+    k = torch.randn(n, G, d, generator=g)
+    v = torch.randn(n, G, d, generator=g)
+    gate = torch.randn(n, H, generator=g)
+    near = [0, 1, 62, 63, 64, 65, 127, 128, 191, 192, 255, 256]
+    q = torch.zeros(n, H, d)
+    for p in range(n):
+        for h in range(H):
+            targets = [t for t in near if t <= p] + [p, max(p - 1, 0),
+                                                     min(p + 1, n - 1)]
+            q[p, h] = k[targets[(p * 7 + h * 5) % len(targets)], h // (H // G)]
+    sink = torch.tensor([-30.0, 0.0, 6.0, 14.0])
+    row = torch.cat([q.view(n, -1), k.view(n, -1), v.view(n, -1), gate], 1)
+    row = torch.nn.functional.pad(row, (0, 60)).to(cache.k[0].dtype)
+    coef, every, scale = 0.3, 32, 0.125
+    rr = row.double()
+    qd, kd, vd, gd, _ = rr.split([H * d, G * d, G * d, H, 60], dim=1)
+    temp = oracle.query_temperature(torch.arange(n), coef, every)
+    want = oracle.attend(
+        oracle.rms(qd.view(n, H, d), 1e-5) * temp.view(n, 1, 1),
+        oracle.rms(kd.view(n, G, d), 1e-5), vd.view(n, G, d), scale,
+        sink.double()) * torch.sigmoid(gd)[:, :, None]
+    got = []
+    for at, ln in portions(n, CUTS[how]):
+        cache.extend([slot], [ln])
+        st = meta_for(cache, slot, at, ln, dev)
+        part = row[at:at + ln].to(dev).contiguous()
+        qn = hops.qknorm_kv(part, cache.k[0], cache.v[0], st, H, G, d, 1e-5,
+                            coef, every)
+        got.append(hops.paged_attn(
+            qn, cache.k[0], cache.v[0], st, scale, sink.to(dev),
+            part[:, (H + 2 * G) * d:(H + 2 * G) * d + H]))
+    got = torch.cat(got).cpu().double()
+    assert float((got - want).abs().max()) < (1e-4 if dtype == "fp32"
+                                              else 0.06)
+
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("how", sorted(CUTS))
+@pytest.mark.parametrize("dk,dv", [(64, 64), (128, 192)])
+def test_one_token_is_remembered(how, run, dk, dv):
+    """A token with a wide open input gate, at the first place and around
+    chunk borders, is what later queries recall; one head forgets at once, one
+    keeps everything, one sees a deep forget in the middle."""
+    dev, dtype = run
+    H, n, cap = 3, 300, 15.0
+    cfg = config((rec(H, dk, dv, cap), None), positions=320)
+    cache = PagedCache(read_birepel(cfg), 3, 320, torch.device(dev),
+                       torch.float32)
+    slot = cache.alloc(0)
+    S, mst = cache.S[0], cache.m[0]
+    S[slot], mst[slot] = 7.0, 3.0         # a predecessor's state
+    g = torch.Generator().manual_seed(7)
+    el = torch.float32 if dtype == "fp32" else torch.bfloat16
+    q, k = torch.randn(2, n, H, dk, generator=g)
+    v, gate = torch.randn(2, n, H, dv, generator=g)
+    zi = torch.full((n, H), -9.0)
+    zf = torch.full((n, H), 30.0)
+    loud = [0, 63, 64, 65, 128, 191, 192, 250]
+    for t in loud:
+        zi[t] = 9.0
+    for p in range(n):
+        q[p] = k[max([t for t in loud if t <= p])] * 2
+    zf[:, 1] = 4.0
+    zf[:, 2] = torch.where(torch.arange(n) == 100, -40.0, 6.0)
+    row = torch.cat([q.reshape(n, -1), k.reshape(n, -1), v.reshape(n, -1),
+                     gate.reshape(n, -1)], 1).to(el)
+    gates = torch.cat([zi, zf], 1)
+    rr = row.double()
+    qd, kd, vd, gd = rr.split([H * dk, H * dk, H * dv, H * dv], dim=1)
+    li, lf = oracle.mlstm_log_gates(zi.double(), zf.double(), cap)
+    o = oracle.mlstm_run(qd.view(n, H, dk) * dk ** -0.5, kd.view(n, H, dk),
+                         vd.view(n, H, dv), li, lf)
+    norm = torch.randn(H * dv, generator=g)
+    want = oracle.rms(o, 1e-5).reshape(n, -1) * norm.double() * \
+        torch.sigmoid(gd)
+    got = []
+    for at, ln in portions(n, CUTS[how]):
+        cache.extend([slot], [ln])
+        got.append(hops.mlstm(row[at:at + ln].to(dev).contiguous(),
+                              gates[at:at + ln].to(dev).contiguous(), S, mst,
+                              norm.to(dev), meta_for(cache, slot, at, ln, dev),
+                              dk, dv, cap, 1e-5))
+    got = torch.cat(got).cpu().double()
+    e = errors(got.view(n, H, dv).transpose(1, 2).reshape(n, -1),
+               want.view(n, H, dv).transpose(1, 2).reshape(n, -1))
+    assert float(e.max()) < (3e-4 if dtype == "fp32" else 0.02)
+
+
+# ----------------------------------------------- cuts, batches, pages, slots
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("sizes", [[1], [2], [3], [63, 2], [64], [100, 1],
+                                   [130, 1, 7]], ids=str)
+def test_cuts_do_not_matter(sizes, run):
+    m = build(FULL, run)
+    ids = tokens(140, seed=1)
+    want, _ = oracle.forward(FULL, weights_of(FULL), ids)
+    slot = m.cache.alloc(0)
+    close(feed(m, slot, ids, sizes), want, run, coarse=0.1, odd=0.1)
+
+
+@pytest.mark.parametrize("run", RUNS)
+def test_unequal_batch_against_each_alone(run):
+    m = build(FULL, run)
+    seqs = {s: tokens(n, seed=s) for s, n in ((1, 150), (2, 3), (3, 70),
+                                              (4, 97))}
+    want = {s: oracle.forward(FULL, weights_of(FULL), ids)[0]
+            for s, ids in seqs.items()}
+    # portions of some beside single tokens of others; one pauses
+    steps = [{1: 64, 2: 1, 3: 2}, {1: 5, 3: 63, 4: 30}, {1: 1, 3: 1, 4: 2},
+             {1: 60, 2: 1, 4: 64}, {1: 1, 2: 1, 3: 1, 4: 1}, {3: 2}, {1: 18},
+             {1: 1, 3: 1}]
+    slots = {s: m.cache.alloc(0) for s in seqs}
+    at = {s: 0 for s in seqs}
+    got = {s: [] for s in seqs}
+    for st in steps:
+        out = m.forward_step([(slots[s], seqs[s][at[s]:at[s] + n],
+                               list(range(n))) for s, n in st.items()]).cpu()
+        for (s, n), part in zip(st.items(), out.split(list(st.values()))):
+            got[s].append(part)
+            at[s] += n
+    assert at == {s: len(v) for s, v in seqs.items()}
+    for s in seqs:
+        close(torch.cat(got[s]), want[s], run, coarse=0.1, odd=0.2)
+
+
+@pytest.mark.parametrize("run", RUNS)
+def test_wanted_places_come_in_order(run):
+    m = build(FULL, run)
+    a, b = tokens(20, seed=1), tokens(30, seed=2)
+    wa, wb = whole(m, a), whole(m, b)
+    s1, s2, s3 = (m.cache.alloc(0) for _ in range(3))
+    out = m.forward_step([(s1, a, [19, 3]), (s3, [5], []),
+                          (s2, b, [7, 7, 0])]).cpu()
+    close(out, torch.cat([wa[[19, 3]], wb[[7, 7, 0]]]), run, exact=1e-4,
+          coarse=0.1, odd=0.4)
+    assert m.forward_step([(s1, [1, 2], [])]).shape == (0, FULL["vocab"])
+
+
+@pytest.mark.parametrize("run", RUNS)
+def test_pages_and_slots_are_used_again(run):
+    """A pool that only fits if everything is given back, in an order that
+    scatters the pages of later sequences."""
+    m = build(FULL, run, slots=3, pool=64 * 7)
+    first = {}
+    for rnd in range(3):
+        s1, s2 = m.cache.alloc(0), m.cache.alloc(0)
+        a, b = tokens(150, seed=10), tokens(140, seed=11)
+        ga, gb = [], []
+        for i in range(0, 150, 30):           # interleave the page demand
+            ga.append(m.forward_step([(s1, a[i:i + 30], [0, 29])]))
+            if i < 140:
+                part = b[i:i + 30]
+                gb.append(m.forward_step([(s2, part, [len(part) - 1])]))
+        first.setdefault("a", torch.cat(ga).cpu())
+        first.setdefault("b", torch.cat(gb).cpu())
+        close(torch.cat(ga).cpu(), first["a"], run, exact=1e-4,
+              coarse=0.1, odd=0.1)
+        close(torch.cat(gb).cpu(), first["b"], run, exact=1e-4,
+              coarse=0.1, odd=0.1)
+        m.cache.free(s2 if rnd else s1)
+        s3 = m.cache.alloc(0)
+        c = tokens(130, seed=12)
+        close(feed(m, s3, c, [100, 1])[[0, 129]],
+              oracle.forward(FULL, weights_of(FULL), c)[0][[0, 129]], run,
+              coarse=0.1, odd=0.5)
+        m.cache.free(s3)
+        m.cache.free(s1 if rnd else s2)
+    assert len(m.cache._free_pages) == 7 and m.cache.n_free == 1
+
+
+def test_pool_promises():
+    spec = read_birepel(config((attn(), None), positions=256))
+    c = PagedCache(spec, 4, 256, torch.device("cpu"), torch.float32,
+                   pool_tokens=64 * 8)
+    assert c.n_free == 2                       # two of full length
+    a = c.alloc(130)                           # three pages set aside
+    assert c.n_free == 1
+    b = c.alloc(0)
+    c.extend([b], [256])
+    with pytest.raises(RuntimeError, match="pages"):
+        c.alloc(128)                           # only one is not spoken for
+    c.extend([a], [130])
+    with pytest.raises(RuntimeError, match="cache for"):
+        c.extend([b], [1])                     # longer than the cache's bound
+    d = c.alloc(0)
+    c.extend([d], [64])
+    with pytest.raises(RuntimeError, match="out of pages"):
+        c.extend([d], [1])
+    held = [set(c._held[s]) for s in (a, b, d)]
+    assert sum(map(len, held)) == len(set().union(*held)) == 8
+    assert 0 not in set().union(*held)
+    for s in (a, b, d):
+        c.free(s)
+    assert c.n_free == 2 and c._owed == 0 and len(c._free_pages) == 8
+    for _ in range(4):
+        c.alloc(0)
+    with pytest.raises(RuntimeError, match="slots"):
+        c.alloc(0)
+
+
+def test_bad_steps_are_refused():
+    m = build(FULL, ("cpu", "fp32"))
+    s = m.cache.alloc(0)
+    for entries in ([(s, [], [])], [(s, [1], [1])], [(s, [1], []), (s, [2], [])],
+                    [(s, [FULL["vocab"]], [])], [(s, [-1], [])]):
+        with pytest.raises(ValueError):
+            m.forward_step(entries)
+
+
+# ------------------------------------------------- configuration and weights
+
+def test_config_reader():
+    spec = read_birepel(FULL)
+    assert [spec.owner(i) for i in range(6)] == [0, 1, 2, 3, 1, 2]
+    assert spec.params == sum(v.numel() for v in weights_of(FULL).values())
+    assert spec.max_seq_len == FULL["max_positions"]
+
+    def broken(change):
+        c = json.loads(json.dumps(FULL))
+        change(c)
+        with pytest.raises((ValueError, KeyError)):
+            read_birepel(c)
+
+    broken(lambda c: c["layers"][0]["mixer"].pop("scale"))
+    broken(lambda c: c["layers"][0]["mixer"].update(window=64))
+    broken(lambda c: c["layers"][0].update(type="conv"))
+    broken(lambda c: c["layers"][1]["mlp"].update(kind="other"))
+    broken(lambda c: c["layers"][4]["mixer"].update(heads=2))
+    broken(lambda c: c["layers"][4].update(weights_of=4))
+    broken(lambda c: c["layers"][2]["mlp"]["router"].update(top=6))
+    broken(lambda c: c["layers"][0]["mixer"].update(kv_heads=4))
+
+
+@pytest.fixture
+def checkpoint(tmp_path):
+    from safetensors.torch import save_file
+    save_file(weights_of(FULL, 3), str(tmp_path / "model.safetensors"))
+    (tmp_path / "config.json").write_text(json.dumps(FULL))
+    return tmp_path
+
+
+def test_checkpoint_describes_itself(checkpoint):
+    spec = resolve_spec("llama3.2:1b", str(checkpoint))
+    assert (spec.family, spec.name) == ("birepel", "birepel:custom")
+    assert resolve_spec("mine", str(checkpoint), 100).max_seq_len == 100
+    assert get_spec("mine").hidden == FULL["width"]
+    (checkpoint / "config.json").write_text('{"architecture": "Else"}')
+    with pytest.raises(ValueError, match="unknown architecture"):
+        resolve_spec("mine", str(checkpoint))
+
+
+def test_checkpoint_errors(checkpoint):
+    from safetensors.torch import save_file
+    m = HybridModel(read_birepel(FULL), dtype="fp32", random_init=False)
+    assert m.load_safetensors(str(checkpoint)) == len(weights_of(FULL))
+    W = weights_of(FULL, 3)
+    W["l0.norm1"] = W["l0.norm1"][:-1].clone()
+    save_file(W, str(checkpoint / "model.safetensors"))
+    with pytest.raises(ValueError, match="l0.norm1"):
+        m.load_safetensors(str(checkpoint))
+    del W["l0.norm1"]
+    save_file(W, str(checkpoint / "model.safetensors"))
+    with pytest.raises(KeyError, match="l0.norm1"):
+        m.load_safetensors(str(checkpoint))
+
+
+# --------------------------------------------------- engine and its schedule
+
+def engine_for(checkpoint, run, **kw):
+    kw = {"max_seq_len": 256, "max_batch_size": 4, "autotune": False} | kw
+    return InferenceEngine(EngineConfig(
+        weights_path=str(checkpoint), device=run[0], dtype=run[1], **kw))
+
+
+def greedy(ids, steps, seed=3):
+    """Greedy continuation by the plain implementation, and how far the
+    winner stood above the second at each step."""
+    W, ids, gaps = weights_of(FULL, seed), list(ids), []
+    for _ in range(steps):
+        z = oracle.forward(FULL, W, ids)[0][-1]
+        top = torch.topk(z, 2)
+        gaps.append(float(top.values[0] - top.values[1]))
+        ids.append(int(top.indices[0]))
+    return ids[-steps:], gaps
+
+
+GREEDY = {"temperature": 0.0, "num_predict": 8}
+# bytes below the vocabulary's size
+PROMPTS = ["3 + 4 = ", "x", "A much longer prompt, so that it takes more than "
+           "one page and a few portions to run it all ...... ", "!"]
+
+
+class _Bytes:
+    """Prompts as bytes; every id decodes to something, none ends a text."""
+    eos_id = -1
+
+    def encode(self, text):
+        return [b % FULL["vocab"] for b in text.encode()]
+
+    def decode(self, ids):
+        return "".join(chr(33 + i % 90) for i in ids)
+
+    def decode_stream(self):
+        tok = self
+
+        class D:
+            def push(self, i):
+                return tok.decode([i])
+        return D()
+
+
+@pytest.mark.parametrize("run", EXACT)
+@pytest.mark.parametrize("chunk", [8192, 5])
+def test_greedy_generation(checkpoint, run, chunk):
+    """Through generate, generate_batch and the continuous batcher, with whole
+    prompts and with portions of five tokens beside decoding rows."""
+    from gridllm_amd.engine.batcher import Batcher
+    eng = engine_for(checkpoint, run, prefill_chunk=chunk)
+    eng.tokenizer = _Bytes()
+    want, gaps = zip(*(greedy(eng.tokenizer.encode(p), 8) for p in PROMPTS))
+    assert min(min(g) for g in gaps) > 1e-3        # no close call in the test
+    free = eng.model.cache.n_free
+    assert [eng.generate(p, GREEDY).token_ids for p in PROMPTS] == list(want)
+    out = eng.generate_batch([(p, GREEDY) for p in PROMPTS])
+    assert [r.token_ids for r in out] == list(want)
+    assert all(r.prompt_eval_duration > 0 and r.done_reason == "length"
+               for r in out)
+    b = Batcher(eng)
+    try:
+        futs = [b.submit_generate(p, GREEDY) for p in PROMPTS * 3]
+        assert [f.result(60).token_ids for f in futs] == list(want) * 3
+        deadline = time.time() + 10
+        while eng.model.cache.n_free != free and time.time() < deadline:
+            time.sleep(0.02)
+    finally:
+        b.shutdown()
+    assert eng.model.cache.n_free == free
+    assert len(eng.embed(["abc", "defg"])[1]) == FULL["width"]
+
+
+def test_small_pool_serves_more_than_it_holds(checkpoint):
+    """A pool for two full sequences, a dozen requests in flight."""
+    from gridllm_amd.engine.batcher import Batcher
+    eng = engine_for(checkpoint, ("cpu", "fp32"), kv_tokens=512)
+    eng.tokenizer = _Bytes()
+    want = [eng.generate(p, GREEDY).token_ids for p in PROMPTS]
+    b = Batcher(eng)
+    try:
+        futs = [b.submit_generate(p, GREEDY) for p in PROMPTS * 3]
+        assert [f.result(60).token_ids for f in futs] == want * 3
+    finally:
+        b.shutdown()
+
+
+def test_cancel_while_the_prompt_runs(checkpoint):
+    import threading
+    eng = engine_for(checkpoint, ("cpu", "fp32"), prefill_chunk=4)
+    eng.tokenizer = _Bytes()
+    ev = threading.Event()
+    free = eng.model.cache.n_free
+    rows = eng.start_rows([(PROMPTS[2], GREEDY, None, ev, None),
+                           (PROMPTS[1], GREEDY, None, None, None)])
+    rows = eng.step_rows(rows)
+    ev.set()
+    done = []
+    while rows:
+        left = eng.step_rows(rows)
+        done += [r for r in rows if r.done]
+        rows = left
+    assert sorted(r.result.done_reason for r in done) == ["cancelled",
+                                                          "length"]
+    assert eng.model.cache.n_free == free
+
+
+def test_context_ends_without_a_shift(checkpoint):
+    eng = engine_for(checkpoint, ("cpu", "fp32"), max_seq_len=40)
+    eng.tokenizer = _Bytes()
+    r = eng.generate("0123456789", {"temperature": 0.0})
+    assert r.done_reason == "length" and 10 + r.eval_count <= 40
+
+
+def test_registered_model_serves():
+    eng = InferenceEngine(EngineConfig(model="tiny-birepel", device="cpu",
+                                       max_batch_size=2, max_seq_len=128))
+    r = eng.generate("hello", {"temperature": 0.7, "seed": 5,
+                               "num_predict": 6})
+    assert r.eval_count == 6
+    assert "tiny-birepel" in eng.model_names()
+    assert eng.spec.model_info()["general.architecture"] == "birepel"
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", ["fp32", "bf16"])
+def test_long_decode_by_captured_graphs(checkpoint, dtype):
+    """Decode-only steps replay captured graphs, between eager mixed steps and
+    synchronizations; every step against the eager model, 150 tokens long and
+    over page borders."""
+    eng = engine_for(checkpoint, ("cuda:0", dtype))
+    assert eng._graph_ok() and eng._graphs
+    W = weights_of(FULL, 3)
+    ref = build(FULL, ("cuda:0", dtype), W=W)
+    ids = {i: tokens(190, seed=20 + i) for i in range(3)}
+    a = {i: eng.open_sequence() for i in ids}
+    b = {i: ref.cache.alloc(0) for i in ids}
+    start = {0: 40, 1: 2, 2: 33}
+    at = dict(start)
+    eng.run_step([(a[i], ids[i][:n], []) for i, n in start.items()])
+    ref.forward_step([(b[i], ids[i][:n], []) for i, n in start.items()])
+    for step in range(150):
+        live = [i for i in ids if not (i == 1 and step % 3 == 0)]
+        n = {i: 2 if step % 31 == 30 and i == 2 else 1 for i in live}
+        ent = [(i, ids[i][at[i]:at[i] + n[i]], [0]) for i in live
+               if at[i] + n[i] <= 190]
+        got = eng.run_step([(a[i], t, w) for i, t, w in ent])
+        want = ref.forward_step([(b[i], t, w) for i, t, w in ent])
+        close(got, want.cpu(), ("cuda:0", dtype), exact=1e-4, coarse=0.1, odd=0.4)
+        for i, t, _ in ent:
+            at[i] += len(t)
+        if step % 10 == 0:
+            torch.cuda.synchronize()
+    close(eng.run_step([(a[0], [7], [0])]),
+          oracle.forward(FULL, W, ids[0][:at[0]] + [7])[0][-1:],
+          ("cuda:0", dtype), odd=1.0)
+
+
+# ------------------------------------------------------------------- traces
+
+def trace_lines():
+    a, b = tokens(80, seed=1), tokens(3, seed=2)
+    steps = [{"step": 0, "entries": [
+                 {"id": "a", "tokens": a[:70], "want": [0, 69]},
+                 {"id": "b", "tokens": b[:1], "want": [0]}], "end": []},
+             {"step": 1, "entries": [
+                 {"id": "b", "tokens": b[1:], "want": []}], "end": ["b"]},
+             {"step": 2, "entries": [
+                 {"id": "a", "tokens": a[70:71], "want": [0]}], "end": []},
+             {"step": 3, "entries": [
+                 {"id": "c", "tokens": b, "want": [2]},
+                 {"id": "a", "tokens": a[71:], "want": [8]}],
+              "end": ["a", "c"]}]
+    W = weights_of(FULL, 3)
+    la, lb = (oracle.forward(FULL, W, t)[0] for t in (a, b))
+    want = {0: torch.stack([la[0], la[69], lb[0]]), 2: la[70:71],
+            3: torch.stack([lb[2], la[79]])}
+    return "".join(json.dumps(s) + "\n" for s in steps), want
+
+
+def check_trace(out, want, run):
+    assert sorted(os.listdir(out)) == [f"{k}.f32" for k in sorted(want)]
+    for k, w in want.items():
+        got = np.fromfile(os.path.join(out, f"{k}.f32"), dtype="<f4")
+        close(torch.from_numpy(got).view(w.shape), w, run, coarse=0.1, odd=0.5)
+
+
+@pytest.mark.parametrize("run", RUNS)
+def test_trace_replay(checkpoint, tmp_path, run):
+    from gridllm_amd import trace
+    lines, want = trace_lines()
+    out = tmp_path / "out"
+    out.mkdir()
+    eng = trace.make_engine(str(checkpoint),
+                            {"fp32": "float32", "bf16": "bfloat16"}[run[1]],
+                            256, run[0])
+    acks = io.StringIO()
+    trace.replay(eng, io.StringIO(lines), str(out), acks)
+    assert acks.getvalue() == "".join(f"done {i}\n" for i in range(4))
+    assert eng.model.cache.pages == 4 and len(eng.model.cache._free_pages) == 4
+    check_trace(out, want, run)
+
+
+def test_trace_program(checkpoint, tmp_path):
+    lines, want = trace_lines()
+    out = tmp_path / "out"
+    out.mkdir()
+    r = subprocess.run([os.path.join(REPO, "bin", "trace_run"), "--model",
+                        str(checkpoint), "--dtype", "float32", "--out",
+                        str(out), "--max-tokens", "256", "--device", "cpu"],
+                       input=lines, capture_output=True, text=True, timeout=120)
+    assert r.returncode == 0, r.stderr[-2000:]
+    assert [x for x in r.stdout.splitlines() if x.startswith("done")] == [
+        f"done {i}" for i in range(4)]
+    check_trace(out, want, ("cpu", "fp32"))
