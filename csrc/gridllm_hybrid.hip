@@ -30,6 +30,19 @@ DEV_INLINE void st8(float* p, const float* f) {
     ((float4*)p)[0] = *(const float4*)f;
     ((float4*)p)[1] = *(const float4*)(f + 4);
 }
+DEV_INLINE void ld4(const bf16_t* p, float* f) {
+    const uint2 v = *(const uint2*)p;
+    f[0] = __uint_as_float(v.x << 16);
+    f[1] = __uint_as_float(v.x & 0xffff0000u);
+    f[2] = __uint_as_float(v.y << 16);
+    f[3] = __uint_as_float(v.y & 0xffff0000u);
+}
+DEV_INLINE void ld4(const float* p, float* f) { *(float4*)f = *(const float4*)p; }
+DEV_INLINE void st4(bf16_t* p, const float* f) {
+    *(uint2*)p = make_uint2((u32)f2bf(f[0]) | ((u32)f2bf(f[1]) << 16),
+                            (u32)f2bf(f[2]) | ((u32)f2bf(f[3]) << 16));
+}
+DEV_INLINE void st4(float* p, const float* f) { *(float4*)p = *(const float4*)f; }
 DEV_INLINE float sigmoidf_(float z) { return 1.f / (1.f + expf(-z)); }
 
 // sum over a block of 256 threads; every thread gets it
@@ -86,12 +99,18 @@ k_post_norm(float* __restrict__ x, T* __restrict__ xb,
             if (MOE) {
 #pragma unroll
                 for (int i = 0; i < 8; ++i) v[j][i] = 0.f;
-                for (int k = 0; k < top; ++k) {
-                    float f[8];
-                    const float g = wt[n * top + k];
-                    ld8(y + (n * top + k) * (long)W + c, f);
+                for (int k0 = 0; k0 < top; k0 += 4) {   // 4 rows in flight
+                    float f[4][8], g[4];
 #pragma unroll
-                    for (int i = 0; i < 8; ++i) v[j][i] += g * f[i];
+                    for (int k = 0; k < 4; ++k) {
+                        const long r = n * top + min(k0 + k, top - 1);
+                        g[k] = k0 + k < top ? wt[r] : 0.f;
+                        ld8(y + r * W + c, f[k]);
+                    }
+#pragma unroll
+                    for (int k = 0; k < 4; ++k)
+#pragma unroll
+                        for (int i = 0; i < 8; ++i) v[j][i] += g[k] * f[k][i];
                 }
             } else {
                 ld8(y + n * W + c, v[j]);
@@ -158,34 +177,61 @@ k_glu_f32(float* __restrict__ out, const float* __restrict__ gu, long n,
 // ===========================================================================
 // Projection to a few f32 outputs (router logits, recurrence gates):
 //   out[n, j] = sum_k x[n, k] w[j, k] + bias[j], bf16 inputs, f32 result.
-// One block per 16 rows x 16 outputs; its 4 waves split K and add up in LDS.
-// K % 32 == 0. Fragments load straight from memory (both k-contiguous).
+// One block per 16 rows x 16 NT outputs; its 8 waves split K and add up in
+// LDS, each with U steps of loads in flight. Fragments load straight from
+// memory (both operands are k-contiguous). K % 32 == 0.
 // ===========================================================================
-__global__ void __launch_bounds__(256)
+template <int NT>
+__global__ void __launch_bounds__(512)
 k_proj_f32(float* __restrict__ out, const bf16_t* __restrict__ x,
            const bf16_t* __restrict__ w, const float* __restrict__ bias,
            int M, int N, int K) {
-    __shared__ float red[4][16][17];
+    constexpr int U = NT == 1 ? 6 : 4;
+    __shared__ float red[8][16][16 * NT + 1];
     const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
     const int fr = lane & 15, kg = (lane >> 4) * 8;
-    const int m0 = blockIdx.x * 16, n0 = blockIdx.y * 16;
+    const int m0 = blockIdx.x * 16, n0 = blockIdx.y * 16 * NT;
     const bf16_t* xr = x + (long)min(m0 + fr, M - 1) * K + kg;
-    const bf16_t* wr = w + (long)min(n0 + fr, N - 1) * K + kg;
-    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-    const int steps = K >> 5;
-#pragma unroll 4
-    for (int s = wid; s < steps; s += 4)
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-            *(const bf16x8*)(xr + s * 32), *(const bf16x8*)(wr + s * 32),
-            acc, 0, 0, 0);
+    const bf16_t* wr[NT];
+    f32x4 acc[NT];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) red[wid][(lane >> 4) * 4 + r][fr] = acc[r];
+    for (int t = 0; t < NT; ++t) {
+        wr[t] = w + (long)min(n0 + t * 16 + fr, N - 1) * K + kg;
+        acc[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    }
+    const int steps = K >> 5;
+    for (int s0 = wid; s0 < steps; s0 += 8 * U) {
+        bf16x8 a[U], b[U][NT];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const int s = min(s0 + u * 8, steps - 1);
+            a[u] = *(const bf16x8*)(xr + s * 32);
+#pragma unroll
+            for (int t = 0; t < NT; ++t)
+                b[u][t] = *(const bf16x8*)(wr[t] + s * 32);
+        }
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+            if (s0 + u * 8 < steps)
+#pragma unroll
+                for (int t = 0; t < NT; ++t)
+                    acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                        a[u], b[u][t], acc[t], 0, 0, 0);
+    }
+#pragma unroll
+    for (int t = 0; t < NT; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+            red[wid][(lane >> 4) * 4 + r][t * 16 + fr] = acc[t][r];
     __syncthreads();
-    const int i = threadIdx.x >> 4, j = threadIdx.x & 15;
-    if (m0 + i < M && n0 + j < N)
-        out[(long)(m0 + i) * N + n0 + j] =
-            red[0][i][j] + red[1][i][j] + red[2][i][j] + red[3][i][j] +
-            (bias ? bias[n0 + j] : 0.f);
+    for (int e = threadIdx.x; e < 256 * NT; e += 512) {
+        const int i = e / (16 * NT), j = e % (16 * NT);
+        if (m0 + i >= M || n0 + j >= N) continue;
+        float v = bias ? bias[n0 + j] : 0.f;
+#pragma unroll
+        for (int k = 0; k < 8; ++k) v += red[k][i][j];
+        out[(long)(m0 + i) * N + n0 + j] = v;
+    }
 }
 
 // ===========================================================================
@@ -431,13 +477,14 @@ k_mlstm_step(float* __restrict__ o, float* __restrict__ S,
                 for (int off = LPR / 2; off > 0; off >>= 1)
                     a += __shfl_xor(a, off, WAVE);
                 if (lane % LPR == 0 && r < rend)
-                    o[(n * H + h) * (DV + 1) + r] = a;
+                    o[(n * H + h) * (DV + 4) + r] = a;
             }
         }
     }
 }
 
-// o -> T out[n, H*DV]: unit RMS per head, times norm, times sigmoid of the
+// o (f32 rows of DV + 4 per token and head: DV sums, n . q, padding)
+// -> T out[n, H*DV]: unit RMS per head, times norm, times sigmoid of the
 // output gate. Items [0, nseg) are segments of the token-by-token kernel, whose
 // o still lacks its denominator and whose m is advanced here; the nplain
 // tokens from plain0 on are finished sums. One wave per (item, head).
@@ -465,7 +512,7 @@ k_mlstm_out(T* __restrict__ out, const float* __restrict__ o,
     }
     for (int t = 0; t < sg.y; ++t) {
         const long n = sg.x + t;
-        const float* ob = o + (n * H + h) * (DV + 1);
+        const float* ob = o + (n * H + h) * (DV + 4);
         float inv = 1.f;
         if (is_seg) {
             float gi, gf;
@@ -474,16 +521,25 @@ k_mlstm_out(T* __restrict__ out, const float* __restrict__ o,
             inv = 1.f / (fmaxf(fabsf(ob[DV]), expf(-m)) + 1e-6f);
         }
         float ss = 0.f;
-        for (int c = lane; c < DV; c += 64) {
-            const float v = ob[c] * inv;
-            ss += v * v;
+        for (int c = lane * 4; c < DV; c += 256) {
+            const float4 v = *(const float4*)(ob + c);
+            ss += (v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w) * inv * inv;
         }
         const float rs =
             inv / sqrtf(wave_reduce_sum(ss) / (float)dvtrue + eps);
         const T* g = qkv + n * ld_ + (long)H * (2 * DK + DV) + (long)h * DV;
-        for (int c = lane; c < DV; c += 64)
-            st(out + (n * H + h) * DV + c,
-               ob[c] * rs * norm[h * DV + c] * sigmoidf_(ld(g + c)));
+        T* dst = out + (n * H + h) * DV;
+        for (int c = lane * 4; c < DV; c += 256) {
+            const float4 v = *(const float4*)(ob + c);
+            const float4 w = *(const float4*)(norm + h * DV + c);
+            float z[4];
+            ld4(g + c, z);
+            const float r[4] = {v.x * rs * w.x * sigmoidf_(z[0]),
+                                v.y * rs * w.y * sigmoidf_(z[1]),
+                                v.z * rs * w.z * sigmoidf_(z[2]),
+                                v.w * rs * w.w * sigmoidf_(z[3])};
+            st4(dst + c, r);
+        }
     }
     if (is_seg && lane == 0) mst[(long)sg.z * H + h] = m;
 }
@@ -624,7 +680,7 @@ k_mlstm_chunk_scan(float* __restrict__ dS, float* __restrict__ scal,
     float m = scal[((long)sg.z * H + h) * 4 + 2];
     const long cs = (long)H * size;
     float* Db = dS + ((long)sg.z * H + h) * size + e;
-    constexpr int U = 4;
+    constexpr int U = 8;
     for (int c = 0; c < sg.w; c += U) {
         float4 d[U];
 #pragma unroll
@@ -803,7 +859,7 @@ k_mlstm_chunk_out(float* __restrict__ o, const float* __restrict__ dS,
     for (int r = 0; r < 4; ++r) {
         const int row = r0 + (lane >> 4) * 4 + r;
         if (row >= ch.y) continue;
-        float* ob = o + ((long)(ch.x + row) * H + h) * (DV + 1) + v0 + fr;
+        float* ob = o + ((long)(ch.x + row) * H + h) * (DV + 4) + v0 + fr;
 #pragma unroll
         for (int c = 0; c < 8; ++c)
             if (c * 16 < nv) ob[c * 16] = acc[c][r] * inv[r];
@@ -815,53 +871,80 @@ k_mlstm_chunk_out(float* __restrict__ o, const float* __restrict__ dS,
 //   route:   top experts of every token by f32 logits (ties: lower index),
 //            softmax over the chosen; counts per expert and each pair's rank
 //   scatter: pairs (token * top + k) sorted by expert, and the tile list
-//            {expert, first sorted row, rows, -}; unused tiles have expert -1
+//            {expert, first sorted row, rows, -}; entry max_tiles holds the
+//            number of tiles
 //   gemm:    rows of one expert against its weights, once for the up
 //            projection (gathers token rows, squared ReLU) and once for the
 //            down projection (writes each pair's row back in pair order)
 // The weighted sum over a token's pairs is taken in k_post_norm.
 // ===========================================================================
+//
+// A wave routes `tpw` tokens, one expert per lane and VPL experts deep. The
+// place of an expert among a token's logits is the number of larger ones, so
+// the chosen fall out of one pass over the lanes. Counts are gathered per
+// block in LDS and added up once per block and expert.
 template <int VPL>
 __global__ void __launch_bounds__(256)
 k_moe_route(int* __restrict__ idx, float* __restrict__ wt,
             int* __restrict__ rank, int* __restrict__ counts,
-            const float* __restrict__ z, int N, int E, int top) {
-    const int n = blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (n >= N) return;
-    const int lane = threadIdx.x & 63;
-    float v[VPL];
+            const float* __restrict__ z, int N, int E, int top, int tpw) {
+    __shared__ int cnt[VPL * 64], base[VPL * 64];
+    for (int e = threadIdx.x; e < VPL * 64; e += 256) cnt[e] = 0;
+    __syncthreads();
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    const int n0 = (blockIdx.x * 4 + wid) * tpw;
+    for (int n = n0; n < min(N, n0 + tpw); ++n) {
+        float v[VPL];
+        int place[VPL];
 #pragma unroll
-    for (int i = 0; i < VPL; ++i) {
-        const int e = i * 64 + lane;
-        v[i] = e < E ? z[(long)n * E + e] : -INFINITY;
-    }
-    float first = 0.f, sum = 0.f, mine = 0.f;
-    for (int k = 0; k < top; ++k) {
-        float best = -INFINITY;
-        int bi = 0x7fffffff;
-#pragma unroll
-        for (int i = 0; i < VPL; ++i)
-            if (v[i] > best) { best = v[i]; bi = i * 64 + lane; }
-#pragma unroll
-        for (int off = 32; off > 0; off >>= 1) {
-            const float ob = __shfl_xor(best, off, WAVE);
-            const int oi = __shfl_xor(bi, off, WAVE);
-            if (ob > best || (ob == best && oi < bi)) { best = ob; bi = oi; }
+        for (int i = 0; i < VPL; ++i) {
+            const int e = i * 64 + lane;
+            v[i] = e < E ? z[(long)n * E + e] : -INFINITY;
+            if (v[i] != v[i]) v[i] = -INFINITY;   // keeps the choice in range
+            place[i] = 0;
         }
-        if (bi >= E) bi = k;           // only if logits are not numbers
-        if (k == 0) first = best;
-        const float p = expf(best - first);
-        sum += p;
-        if (lane == k) mine = p;       // top <= 64
 #pragma unroll
-        for (int i = 0; i < VPL; ++i)
-            if (i * 64 + lane == bi) v[i] = -INFINITY;
-        if (lane == 0) {
-            idx[(long)n * top + k] = bi;
-            rank[(long)n * top + k] = atomicAdd(counts + bi, 1);
+        for (int j = 0; j < VPL; ++j) {
+            const int last = min(64, E - j * 64);
+            for (int l = 0; l < last; ++l) {
+                const float o = __uint_as_float(
+                    __builtin_amdgcn_readlane(__float_as_uint(v[j]), l));
+                const int e = j * 64 + l;
+#pragma unroll
+                for (int i = 0; i < VPL; ++i)
+                    place[i] += o > v[i] || (o == v[i] && e < i * 64 + lane);
+            }
+        }
+        float mx = v[0];
+#pragma unroll
+        for (int i = 1; i < VPL; ++i) mx = fmaxf(mx, v[i]);
+        mx = wave_reduce_max(mx);
+        float p[VPL], sum = 0.f;
+#pragma unroll
+        for (int i = 0; i < VPL; ++i) {
+            const bool in = place[i] < top && i * 64 + lane < E;
+            p[i] = in ? expf(v[i] - mx) : 0.f;
+            sum += p[i];
+        }
+        sum = wave_reduce_sum(sum);
+#pragma unroll
+        for (int i = 0; i < VPL; ++i) {
+            const int e = i * 64 + lane;
+            if (place[i] >= top || e >= E) continue;
+            const long at = (long)n * top + place[i];
+            idx[at] = e;
+            wt[at] = p[i] / sum;
+            rank[at] = atomicAdd(cnt + e, 1);       // within the block
         }
     }
-    if (lane < top) wt[(long)n * top + lane] = mine / sum;
+    __syncthreads();
+    for (int e = threadIdx.x; e < E; e += 256)
+        base[e] = cnt[e] ? atomicAdd(counts + e, cnt[e]) : 0;
+    __syncthreads();
+    const long p0 = (long)blockIdx.x * 4 * tpw * top;
+    const long p1 = min((long)N * top, p0 + 4L * tpw * top);
+    for (long at = p0 + threadIdx.x; at < p1; at += 256)
+        rank[at] += base[idx[at]];
 }
 
 __global__ void __launch_bounds__(256)
@@ -892,7 +975,10 @@ k_moe_scatter(int* __restrict__ sorted, int4* __restrict__ tiles,
     }
     __syncthreads();
     const int i = blockIdx.x * 256 + threadIdx.x;
-    if (i < pairs) sorted[off[idx[i]] + rank[i]] = i;
+    if (i < pairs) {
+        const int at = off[idx[i]] + rank[i];
+        if (at >= 0 && at < pairs) sorted[at] = i;
+    }
     if (blockIdx.x == 0) {
         for (int e = threadIdx.x; e < E; e += 256) {
             const int n = off[e + 1] - off[e];
@@ -901,8 +987,8 @@ k_moe_scatter(int* __restrict__ sorted, int4* __restrict__ tiles,
                     tiles[toff[e] + t] = make_int4(e, off[e] + t * bm,
                                                    min(bm, n - t * bm), 0);
         }
-        for (int t = toff[E] + threadIdx.x; t < max_tiles; t += 256)
-            tiles[t] = make_int4(-1, 0, 0, 0);
+        if (threadIdx.x == 0)
+            tiles[max_tiles] = make_int4(min(toff[E], max_tiles), 0, 0, 0);
     }
 }
 
@@ -911,23 +997,41 @@ DEV_INLINE float sq_relu(float v) {
     return v * v;
 }
 
+// Work item of this block: tiles of neighbouring numbers (the columns of one
+// row tile, then the next row tile of the expert) go to the same XCD, whose L2
+// then holds the rows and weights they share. Blocks are dealt to the 8 XCDs
+// in turn, and only the tiles in use are counted. Returns false if none is
+// left for the block.
+DEV_INLINE bool moe_work(const int4* tiles, int max_tiles, int ntn, int4& tl,
+                         int& nt) {
+    const int total = tiles[max_tiles].x * ntn;
+    const int per = (total + 7) >> 3;
+    const int i = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
+    if ((int)(blockIdx.x >> 3) >= per || i >= total) return false;
+    tl = tiles[i / ntn];
+    nt = i % ntn;
+    return true;
+}
+
 // Large batches: 128 rows x 128 columns per block, 4 waves of 64 x 64, both
 // operands through LDS by global_load_lds (source addresses pre-swizzled so
 // that the lane-linear image reads back without bank conflicts), NB buffers.
 // UP: row r of the tile is token sorted[row0 + r] / top, squared ReLU, output
 // in sorted order. Otherwise row r is sorted row row0 + r and its output goes
-// to pair order. K % 64 == 0, N % 64 == 0.
+// to pair order. The MFMA computes W x^T, so a lane ends up with 4 neighbouring
+// columns of one row. K % 64 == 0, N % 64 == 0.
 template <bool UP, int NB>
 __global__ void __launch_bounds__(256, 2)
 k_moe_gemm(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
            const bf16_t* __restrict__ w, const int4* __restrict__ tiles,
-           const int* __restrict__ sorted, int top, int N, int K,
-           int ntn) {
+           const int* __restrict__ sorted, int top, int N, int K, int ntn,
+           int max_tiles) {
     constexpr int BK = 64, TB = 256 * BK, GL = 8;
     __shared__ __attribute__((aligned(16))) bf16_t lds[NB * TB];
-    const int4 tl = tiles[blockIdx.x / ntn];
-    if (tl.x < 0) return;
-    const int n0 = (blockIdx.x % ntn) * 128;
+    int4 tl;
+    int nti;
+    if (!moe_work(tiles, max_tiles, ntn, tl, nti)) return;
+    const int n0 = nti * 128;
     const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
     const int fr = lane & 15, kg = (lane >> 4) * 8;
     const int lrow = lane >> 3, lkb = (lane & 7) * 16;
@@ -992,52 +1096,55 @@ k_moe_gemm(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
 #pragma unroll
                 for (int c = 0; c < 4; ++c)
                     acc[a][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                        av, b[c], acc[a][c], 0, 0, 0);
+                        b[c], av, acc[a][c], 0, 0, 0);
             }
         }
     }
 #pragma unroll
-    for (int a = 0; a < 4; ++a)
+    for (int a = 0; a < 4; ++a) {
+        const int m = wr + a * 16 + fr;
+        if (m >= tl.z) continue;
+        bf16_t* orow = out + (UP ? (long)tl.y + m : sorted[tl.y + m]) * (long)N;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const int m = wr + a * 16 + (lane >> 4) * 4 + r;
-            if (m >= tl.z) continue;
-            const long dst = UP ? tl.y + m : sorted[tl.y + m];
+        for (int c = 0; c < 4; ++c) {
+            const int n = n0 + wc + c * 16 + (lane >> 4) * 4;
+            float f[4];
 #pragma unroll
-            for (int c = 0; c < 4; ++c) {
-                const int n = n0 + wc + c * 16 + fr;
-                if (n < N)
-                    out[dst * N + n] =
-                        f2bf(UP ? sq_relu(acc[a][c][r]) : acc[a][c][r]);
-            }
+            for (int r = 0; r < 4; ++r)
+                f[r] = UP ? sq_relu(acc[a][c][r]) : acc[a][c][r];
+            if (n < N) st4(orow + n, f);
         }
+    }
 }
 
-// Small batches (weight streaming): up to 16 * MT rows of an expert against 64
-// columns; a wave owns 16 columns and streams its weights once, straight into
-// MFMA fragments, while the rows pass through LDS in panels of KS.
+// Medium batches (weight streaming): up to 16 * MT rows of an expert against
+// 64 columns; a wave owns 16 columns and streams its weights once, straight
+// into MFMA fragments, while the rows pass through LDS in panels of KS. Rows
+// that the tile does not have are neither staged nor multiplied.
 template <bool UP, int MT>
 __global__ void __launch_bounds__(256)
 k_moe_gemm_skinny(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
                   const bf16_t* __restrict__ w,
                   const int4* __restrict__ tiles,
                   const int* __restrict__ sorted, int top, int N, int K,
-                  int ntn) {
+                  int ntn, int max_tiles) {
     constexpr int KS = 256, ROWS = MT * 16;
     __shared__ __attribute__((aligned(16))) bf16_t xs[ROWS * KS];
-    const int4 tl = tiles[blockIdx.x / ntn];
-    if (tl.x < 0) return;
+    int4 tl;
+    int nti;
+    if (!moe_work(tiles, max_tiles, ntn, tl, nti)) return;
     const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
     const int fr = lane & 15, kg = (lane >> 4) * 8;
-    const int n0 = (blockIdx.x % ntn) * 64 + wid * 16;
+    const int n0 = nti * 64 + wid * 16;
     const bf16_t* wrow = w + ((long)tl.x * N + n0 + fr) * K + kg;
     f32x4 acc[MT];
 #pragma unroll
     for (int t = 0; t < MT; ++t) acc[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
     const bf16_t* xrow[MT * 2];
+    const int r0 = threadIdx.x >> 5;
 #pragma unroll
     for (int i = 0; i < MT * 2; ++i) {
-        const int r = tl.y + min((int)((threadIdx.x >> 5) + i * 8), tl.z - 1);
+        const int r = tl.y + min(r0 + i * 8, tl.z - 1);
         xrow[i] = x + (long)(UP ? sorted[r] / top : r) * K;
     }
     const int kc = (threadIdx.x & 31) * 8;
@@ -1050,34 +1157,81 @@ k_moe_gemm_skinny(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
         if (kp > 0) __syncthreads();
 #pragma unroll
         for (int i = 0; i < MT * 2; ++i) {
-            const int row = (threadIdx.x >> 5) + i * 8;
+            const int row = r0 + i * 8;
+            if (row >= tl.z) continue;
             const uint4 v = *(const uint4*)(xrow[i] + min(kp + kc, K - 8));
             *(uint4*)((char*)xs + (((row * KS + kc) * 2) ^ ((row & 15) << 4))) = v;
         }
         __syncthreads();
         const int nch = min(KS, K - kp) >> 5;
 #pragma unroll
-        for (int u = 0; u < 8; ++u) {
-            if (u >= nch) break;
+        for (int t = 0; t < MT; ++t) {
+            if (t * 16 >= tl.z) break;
+            const int row = t * 16 + fr;
 #pragma unroll
-            for (int t = 0; t < MT; ++t) {
-                const int row = t * 16 + fr;
+            for (int u = 0; u < 8; ++u) {
+                if (u >= nch) break;
                 acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                    *(const bf16x8*)((const char*)xs +
+                    b[u], *(const bf16x8*)((const char*)xs +
                         (((row * KS + u * 32 + kg) * 2) ^ ((row & 15) << 4))),
-                    b[u], acc[t], 0, 0, 0);
+                    acc[t], 0, 0, 0);
             }
         }
     }
 #pragma unroll
-    for (int t = 0; t < MT; ++t)
+    for (int t = 0; t < MT; ++t) {
+        const int m = t * 16 + fr;
+        if (m >= tl.z) continue;
+        float f[4];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const int m = t * 16 + (lane >> 4) * 4 + r;
-            if (m >= tl.z) continue;
-            const long dst = UP ? tl.y + m : sorted[tl.y + m];
-            out[dst * N + n0 + fr] = f2bf(UP ? sq_relu(acc[t][r]) : acc[t][r]);
+        for (int r = 0; r < 4; ++r) f[r] = UP ? sq_relu(acc[t][r]) : acc[t][r];
+        st4(out + (UP ? (long)tl.y + m : sorted[tl.y + m]) * (long)N + n0 +
+            (lane >> 4) * 4, f);
+    }
+}
+
+// Smallest batches: up to 16 rows against 16 columns per block, K split over
+// the 4 waves, so that a handful of experts still fills the chip.
+template <bool UP>
+__global__ void __launch_bounds__(256)
+k_moe_gemm_few(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
+               const bf16_t* __restrict__ w, const int4* __restrict__ tiles,
+               const int* __restrict__ sorted, int top, int N, int K,
+               int ntn, int max_tiles) {
+    constexpr int U = 8;
+    __shared__ __attribute__((aligned(16))) float red[4][16][20];
+    int4 tl;
+    int nti;
+    if (!moe_work(tiles, max_tiles, ntn, tl, nti)) return;
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    const int fr = lane & 15, kg = (lane >> 4) * 8;
+    const int n0 = nti * 16;
+    const bf16_t* wr = w + ((long)tl.x * N + n0 + fr) * K + kg;
+    const int r = tl.y + min(fr, tl.z - 1);
+    const bf16_t* xr = x + (long)(UP ? sorted[r] / top : r) * K + kg;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    const int steps = K >> 5;
+    for (int s0 = wid; s0 < steps; s0 += 4 * U) {
+        bf16x8 a[U], b[U];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const int s = min(s0 + u * 4, steps - 1);
+            b[u] = __builtin_nontemporal_load((const bf16x8*)(wr + s * 32));
+            a[u] = *(const bf16x8*)(xr + s * 32);
         }
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+            if (s0 + u * 4 < steps)
+                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(b[u], a[u], acc,
+                                                              0, 0, 0);
+    }
+    *(f32x4*)&red[wid][fr][(lane >> 4) * 4] = acc;
+    __syncthreads();
+    const int m = threadIdx.x >> 4, c = threadIdx.x & 15;
+    if (m >= tl.z) return;
+    const float v = red[0][m][c] + red[1][m][c] + red[2][m][c] + red[3][m][c];
+    out[(UP ? (long)tl.y + m : sorted[tl.y + m]) * (long)N + n0 + c] =
+        f2bf(UP ? sq_relu(v) : v);
 }
 
 // Exact mode: 16 rows x 64 columns per block, f32 products.
@@ -1086,11 +1240,12 @@ __global__ void __launch_bounds__(256)
 k_moe_gemm_f32(float* __restrict__ out, const float* __restrict__ x,
                const float* __restrict__ w, const int4* __restrict__ tiles,
                const int* __restrict__ sorted, int top, int N, int K,
-               int ntn) {
+               int ntn, int max_tiles) {
     __shared__ float xs[16][33], ws[64][33];
-    const int4 tl = tiles[blockIdx.x / ntn];
-    if (tl.x < 0) return;
-    const int n0 = (blockIdx.x % ntn) * 64;
+    int4 tl;
+    int nti;
+    if (!moe_work(tiles, max_tiles, ntn, tl, nti)) return;
+    const int n0 = nti * 64;
     const int col = threadIdx.x & 63, r4 = (threadIdx.x >> 6) * 4;
     float acc[4] = {0.f, 0.f, 0.f, 0.f};
     for (int k0 = 0; k0 < K; k0 += 32) {
@@ -1229,9 +1384,15 @@ int gh_glu_f32(void* stream, void* out, const void* gu, long n, int F,
 int gh_proj_f32(void* stream, void* out, const void* x, const void* w,
                 const void* bias, int M, int N, int K) {
     if (K % 32 || M < 1 || N < 1) return -100;
-    k_proj_f32<<<dim3((M + 15) / 16, (N + 15) / 16), 256, 0,
-                 (hipStream_t)stream>>>((float*)out, (const bf16_t*)x,
-        (const bf16_t*)w, (const float*)bias, M, N, K);
+    hipStream_t st_ = (hipStream_t)stream;
+#define GO(NT) k_proj_f32<NT><<<dim3((M + 15) / 16, \
+        (N + 16 * NT - 1) / (16 * NT)), 512, 0, st_>>>((float*)out, \
+        (const bf16_t*)x, (const bf16_t*)w, (const float*)bias, M, N, K)
+    // few rows: narrow blocks, so that more of them stream the weights
+    if (M <= 512 || N <= 16) GO(1);
+    else if (N <= 32) GO(2);
+    else GO(4);
+#undef GO
     LAUNCH_CHECK();
     return 0;
 }
@@ -1382,11 +1543,12 @@ int gh_mlstm_chunks(void* stream, void* o, void* S, void* mst, void* dS,
 int gh_moe_route(void* stream, void* idx, void* wt, void* rank, void* counts,
                  void* sorted, void* tiles, const void* z, int N, int E,
                  int top, int bm, int max_tiles) {
-    if (N < 1 || E < 1 || E > 1024 || top < 1 || top > 64 || top > E)
+    if (N < 1 || E < 1 || E > 1024 || top < 1 || top > E)
         return -100;
     hipStream_t st_ = (hipStream_t)stream;
-#define GO(V) k_moe_route<V><<<(N + 3) / 4, 256, 0, st_>>>((int*)idx, \
-        (float*)wt, (int*)rank, (int*)counts, (const float*)z, N, E, top)
+#define GO(V) k_moe_route<V><<<(N + 4 * tpw - 1) / (4 * tpw), 256, 0, st_>>>((int*)idx, \
+        (float*)wt, (int*)rank, (int*)counts, (const float*)z, N, E, top, tpw)
+    const int tpw = min(max(N / 1024, 1), 16);
     if (E <= 64) GO(1);
     else if (E <= 256) GO(4);
     else GO(16);
@@ -1409,25 +1571,30 @@ int gh_moe_gemm(void* stream, int f32, int up, void* out, const void* x,
     if (f32) {
         if (bm != 16) return -103;
         const int ntn = N / 64;
-        const unsigned grid = (unsigned)(max_tiles * ntn);
+        const unsigned grid = (unsigned)((max_tiles * ntn + 7) / 8 * 8);
 #define GO(U) k_moe_gemm_f32<U><<<grid, 256, 0, st_>>>((float*)out, \
         (const float*)x, (const float*)w, (const int4*)tiles, \
-        (const int*)sorted, top, N, K, ntn)
+        (const int*)sorted, top, N, K, ntn, max_tiles)
         if (up) GO(true); else GO(false);
 #undef GO
         LAUNCH_CHECK();
         return 0;
     }
 #define ARGS (bf16_t*)out, (const bf16_t*)x, (const bf16_t*)w, \
-        (const int4*)tiles, (const int*)sorted, top, N, K, ntn
+        (const int4*)tiles, (const int*)sorted, top, N, K, ntn, max_tiles
     if (bm == 128) {
         const int ntn = (N + 127) / 128;
-        const unsigned grid = (unsigned)(max_tiles * ntn);
+        const unsigned grid = (unsigned)((max_tiles * ntn + 7) / 8 * 8);
         if (up) k_moe_gemm<true, 2><<<grid, 256, 0, st_>>>(ARGS);
         else k_moe_gemm<false, 2><<<grid, 256, 0, st_>>>(ARGS);
+    } else if (bm == 16 && max_tiles * (N / 64) < 1024) {
+        const int ntn = N / 16;
+        const unsigned grid = (unsigned)((max_tiles * ntn + 7) / 8 * 8);
+        if (up) k_moe_gemm_few<true><<<grid, 256, 0, st_>>>(ARGS);
+        else k_moe_gemm_few<false><<<grid, 256, 0, st_>>>(ARGS);
     } else {
         const int ntn = N / 64;
-        const unsigned grid = (unsigned)(max_tiles * ntn);
+        const unsigned grid = (unsigned)((max_tiles * ntn + 7) / 8 * 8);
 #define GO(M) do { \
         if (up) k_moe_gemm_skinny<true, M><<<grid, 256, 0, st_>>>(ARGS); \
         else k_moe_gemm_skinny<false, M><<<grid, 256, 0, st_>>>(ARGS); \

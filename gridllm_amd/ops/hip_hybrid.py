@@ -209,7 +209,7 @@ def mlstm(qkv: torch.Tensor, gates: torch.Tensor, S: torch.Tensor,
     assert ld >= h * (2 * dk + 2 * dv) and gates.shape == (n, 2 * h)
     f = _f32(qkv)
     qscale = dim ** -0.5
-    o = torch.empty(n, h, dv + 1, dtype=torch.float32, device=qkv.device)
+    o = torch.empty(n, h, dv + 4, dtype=torch.float32, device=qkv.device)
     segs, nseg = (st.segs, st.segs.shape[0]) if f and st.segs is not None \
         else (None, st.nd)
     if nseg:
@@ -256,7 +256,7 @@ def moe(x: torch.Tensor, logits: torch.Tensor, up: torch.Tensor,
     ints = torch.empty(3 * pairs, dtype=torch.int32, device=dev)
     idx, rank, order = ints[:pairs], ints[pairs:2 * pairs], ints[2 * pairs:]
     counts = torch.zeros(e, dtype=torch.int32, device=dev)
-    tiles = torch.empty(max_tiles, 4, dtype=torch.int32, device=dev)
+    tiles = torch.empty(max_tiles + 1, 4, dtype=torch.int32, device=dev)
     wt = torch.empty(n, top, dtype=torch.float32, device=dev)
     _call("gh_moe_route", idx, wt, rank, counts, order, tiles, logits, n, e,
           top, bm, max_tiles)
