@@ -1013,9 +1013,10 @@ DEV_INLINE bool moe_work(const int4* tiles, int max_tiles, int ntn, int4& tl,
     return true;
 }
 
-// Large batches: 128 rows x 128 columns per block, 4 waves of 64 x 64, both
+// 128 rows x 128 columns per block, 4 waves of 64 x 64, both
 // operands through LDS by global_load_lds (source addresses pre-swizzled so
 // that the lane-linear image reads back without bank conflicts), NB buffers.
+// With few rows per expert the same pipeline streams the weights.
 // UP: row r of the tile is token sorted[row0 + r] / top, squared ReLU, output
 // in sorted order. Otherwise row r is sorted row row0 + r and its output goes
 // to pair order. The MFMA computes W x^T, so a lane ends up with 4 neighbouring
@@ -1117,81 +1118,8 @@ k_moe_gemm(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
     }
 }
 
-// Medium batches (weight streaming): up to 16 * MT rows of an expert against
-// 64 columns; a wave owns 16 columns and streams its weights once, straight
-// into MFMA fragments, while the rows pass through LDS in panels of KS. Rows
-// that the tile does not have are neither staged nor multiplied.
-template <bool UP, int MT>
-__global__ void __launch_bounds__(256)
-k_moe_gemm_skinny(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
-                  const bf16_t* __restrict__ w,
-                  const int4* __restrict__ tiles,
-                  const int* __restrict__ sorted, int top, int N, int K,
-                  int ntn, int max_tiles) {
-    constexpr int KS = 256, ROWS = MT * 16;
-    __shared__ __attribute__((aligned(16))) bf16_t xs[ROWS * KS];
-    int4 tl;
-    int nti;
-    if (!moe_work(tiles, max_tiles, ntn, tl, nti)) return;
-    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
-    const int fr = lane & 15, kg = (lane >> 4) * 8;
-    const int n0 = nti * 64 + wid * 16;
-    const bf16_t* wrow = w + ((long)tl.x * N + n0 + fr) * K + kg;
-    f32x4 acc[MT];
-#pragma unroll
-    for (int t = 0; t < MT; ++t) acc[t] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    const bf16_t* xrow[MT * 2];
-    const int r0 = threadIdx.x >> 5;
-#pragma unroll
-    for (int i = 0; i < MT * 2; ++i) {
-        const int r = tl.y + min(r0 + i * 8, tl.z - 1);
-        xrow[i] = x + (long)(UP ? sorted[r] / top : r) * K;
-    }
-    const int kc = (threadIdx.x & 31) * 8;
-    for (int kp = 0; kp < K; kp += KS) {
-        bf16x8 b[8];
-#pragma unroll
-        for (int u = 0; u < 8; ++u)
-            b[u] = __builtin_nontemporal_load(
-                (const bf16x8*)(wrow + min(kp + u * 32, K - 32)));
-        if (kp > 0) __syncthreads();
-#pragma unroll
-        for (int i = 0; i < MT * 2; ++i) {
-            const int row = r0 + i * 8;
-            if (row >= tl.z) continue;
-            const uint4 v = *(const uint4*)(xrow[i] + min(kp + kc, K - 8));
-            *(uint4*)((char*)xs + (((row * KS + kc) * 2) ^ ((row & 15) << 4))) = v;
-        }
-        __syncthreads();
-        const int nch = min(KS, K - kp) >> 5;
-#pragma unroll
-        for (int t = 0; t < MT; ++t) {
-            if (t * 16 >= tl.z) break;
-            const int row = t * 16 + fr;
-#pragma unroll
-            for (int u = 0; u < 8; ++u) {
-                if (u >= nch) break;
-                acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                    b[u], *(const bf16x8*)((const char*)xs +
-                        (((row * KS + u * 32 + kg) * 2) ^ ((row & 15) << 4))),
-                    acc[t], 0, 0, 0);
-            }
-        }
-    }
-#pragma unroll
-    for (int t = 0; t < MT; ++t) {
-        const int m = t * 16 + fr;
-        if (m >= tl.z) continue;
-        float f[4];
-#pragma unroll
-        for (int r = 0; r < 4; ++r) f[r] = UP ? sq_relu(acc[t][r]) : acc[t][r];
-        st4(out + (UP ? (long)tl.y + m : sorted[tl.y + m]) * (long)N + n0 +
-            (lane >> 4) * 4, f);
-    }
-}
-
-// Smallest batches: up to 16 rows against 16 columns per block, K split over
-// the 4 waves, so that a handful of experts still fills the chip.
+// A few rows: up to 16 against 16 columns per block, K split over the 4 waves,
+// so that a handful of experts still fills the chip.
 template <bool UP>
 __global__ void __launch_bounds__(256)
 k_moe_gemm_few(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
@@ -1562,7 +1490,7 @@ int gh_moe_route(void* stream, void* idx, void* wt, void* rank, void* counts,
     return 0;
 }
 
-// bm: rows per tile of the list: 16, 32 or 64 (weight streaming) or 128
+// bm: rows per tile of the list: 16 (few pairs; the exact mode) or 128
 int gh_moe_gemm(void* stream, int f32, int up, void* out, const void* x,
                 const void* w, const void* tiles, const void* sorted,
                 int top, int N, int K, int bm, int max_tiles) {
@@ -1587,23 +1515,13 @@ int gh_moe_gemm(void* stream, int f32, int up, void* out, const void* x,
         const unsigned grid = (unsigned)((max_tiles * ntn + 7) / 8 * 8);
         if (up) k_moe_gemm<true, 2><<<grid, 256, 0, st_>>>(ARGS);
         else k_moe_gemm<false, 2><<<grid, 256, 0, st_>>>(ARGS);
-    } else if (bm == 16 && max_tiles * (N / 64) < 1024) {
+    } else if (bm == 16) {
         const int ntn = N / 16;
         const unsigned grid = (unsigned)((max_tiles * ntn + 7) / 8 * 8);
         if (up) k_moe_gemm_few<true><<<grid, 256, 0, st_>>>(ARGS);
         else k_moe_gemm_few<false><<<grid, 256, 0, st_>>>(ARGS);
     } else {
-        const int ntn = N / 64;
-        const unsigned grid = (unsigned)((max_tiles * ntn + 7) / 8 * 8);
-#define GO(M) do { \
-        if (up) k_moe_gemm_skinny<true, M><<<grid, 256, 0, st_>>>(ARGS); \
-        else k_moe_gemm_skinny<false, M><<<grid, 256, 0, st_>>>(ARGS); \
-        } while (0)
-        if (bm == 16) GO(1);
-        else if (bm == 32) GO(2);
-        else if (bm == 64) GO(4);
-        else return -103;
-#undef GO
+        return -103;
     }
 #undef ARGS
     LAUNCH_CHECK();

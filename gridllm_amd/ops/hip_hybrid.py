@@ -234,11 +234,9 @@ def mlstm(qkv: torch.Tensor, gates: torch.Tensor, S: torch.Tensor,
     return out
 
 
-def _tile_rows(pairs: int, experts: int) -> int:
-    """Rows per tile of the expert GEMMs, from the mean rows per expert."""
-    mean = pairs / experts
-    return 16 if mean <= 12 else 32 if mean <= 24 else \
-        64 if mean <= 48 else 128
+# up to this many (token, expert) pairs, mostly of different experts, the
+# 16-row kernel fills the chip better than 128 x 128 tiles do
+_FEW_PAIRS = 64
 
 
 def moe(x: torch.Tensor, logits: torch.Tensor, up: torch.Tensor,
@@ -251,7 +249,7 @@ def moe(x: torch.Tensor, logits: torch.Tensor, up: torch.Tensor,
     _dense(x, logits, up, down)
     dev, f = x.device, _f32(x)
     pairs = n * top
-    bm = 16 if f else _tile_rows(pairs, e)
+    bm = 16 if f or pairs <= _FEW_PAIRS else 128
     max_tiles = min(pairs, e + pairs // bm)
     ints = torch.empty(3 * pairs, dtype=torch.int32, device=dev)
     idx, rank, order = ints[:pairs], ints[pairs:2 * pairs], ints[2 * pairs:]
