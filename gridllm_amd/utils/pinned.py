@@ -4,8 +4,10 @@ A pageable `.to(device)` both enqueues BEHIND everything already on the
 stream and blocks the host until the copy lands — ~1.5 ms per call
 against a busy decode stream (round-2 serving profiles). Staging through
 a reusable pinned buffer with non_blocking=True enqueues without a host
-stall. Buffers are pooled per rounded capacity in a ring (depth 4) so a
-still-in-flight copy's staging is never rewritten by the next few calls.
+stall. Buffers are pooled per rounded capacity in a ring of 4, each with the
+event of its last copy: a buffer is rewritten only when that copy is done, so
+a host that runs many steps ahead of the stream waits here instead of changing
+data under a copy.
 """
 
 from __future__ import annotations
@@ -22,12 +24,16 @@ class PinnedUploader:
         self.is_gpu = self.device.type == "cuda"
         self._pool: dict = {}
 
-    def _stage(self, cap: int, dtype) -> torch.Tensor:
+    def _stage(self, cap: int, dtype):
+        """A free staging buffer and its event."""
         key = (cap, dtype)
         ring = self._pool.setdefault(key, [[None] * _RING, 0])
         i = ring[1] = (ring[1] + 1) % _RING
         if ring[0][i] is None:
-            ring[0][i] = torch.empty(cap, dtype=dtype, pin_memory=True)
+            ring[0][i] = (torch.empty(cap, dtype=dtype, pin_memory=True),
+                          torch.cuda.Event())
+        else:
+            ring[0][i][1].synchronize()
         return ring[0][i]
 
     def upload(self, arr: np.ndarray) -> torch.Tensor:
@@ -38,9 +44,10 @@ class PinnedUploader:
             return t
         n = t.numel()
         cap = max(16, 1 << (n - 1).bit_length()) if n else 16
-        stage = self._stage(cap, t.dtype)
+        stage, copied = self._stage(cap, t.dtype)
         flat = stage[:n]
         flat.copy_(t.view(-1))
         out = torch.empty(t.shape, dtype=t.dtype, device=self.device)
         out.view(-1).copy_(flat, non_blocking=True)
+        copied.record()
         return out

@@ -710,6 +710,21 @@ def test_long_decode_by_captured_graphs(checkpoint, dtype):
           ("cuda:0", dtype), odd=1.0)
 
 
+@pytest.mark.gpu
+def test_uploads_far_ahead_of_the_stream():
+    """Steps that nobody waits for queue up behind a busy stream; what they
+    uploaded must not change under them."""
+    from gridllm_amd.utils.pinned import PinnedUploader
+    up = PinnedUploader(torch.device("cuda:0"))
+    up.upload(np.zeros(100, dtype=np.int64))
+    a = torch.randn(4096, 4096, device="cuda:0")
+    torch.cuda.synchronize()
+    for _ in range(20):
+        a = a @ a * 1e-3
+    got = [up.upload(np.full(100, i, dtype=np.int64)) for i in range(12)]
+    assert [int(t.sum()) for t in got] == [100 * i for i in range(12)]
+
+
 # ------------------------------------------------------------------- traces
 
 def trace_lines():
