@@ -39,3 +39,12 @@ def test_bench_engine_mode_contract():
     assert REQUIRED <= set(res)
     assert res["value"] > 0
     assert res["config"]["mode"] == "engine"
+
+
+def test_bench_layers_mode_contract():
+    res = _run(["--mode", "layers", "--steps", "1", "--warmup", "1"])
+    assert REQUIRED <= set(res)
+    cfg = res["config"]
+    assert cfg["mode"] == "layers" and cfg["model"].keys() == \
+        cfg["llama_twin"].keys()
+    assert all(v > 0 for v in cfg["model"].values())

@@ -297,7 +297,7 @@ def test_one_key_stands_out(how, run):
     sink = torch.tensor([-30.0, 0.0, 6.0, 14.0])
     row = torch.cat([q.view(n, -1), k.view(n, -1), v.view(n, -1), gate], 1)
     row = torch.nn.functional.pad(row, (0, 60)).to(cache.k[0].dtype)
-    coef, every, scale = 0.3, 32, 0.125
+    coef, every, scale = 0.35, 32, 0.13
     rr = row.double()
     qd, kd, vd, gd, _ = rr.split([H * d, G * d, G * d, H, 60], dim=1)
     temp = oracle.query_temperature(torch.arange(n), coef, every)
