@@ -230,6 +230,177 @@ k_norm_rows(T* __restrict__ out, const float* __restrict__ x,
     }
 }
 
+// ===========================================================================
+// Norm in groups: a row's `groups` equal consecutive parts, each divided by
+// its own root mean square, times w (no offset).
+//   ADD:  x += norm(y) * wy;  out = norm(x) * w, if there is an out
+//   else: out[r] = norm(x[rows[r]]) * w
+// Columns from Wtrue on carry zeros. Squares are summed in pieces of GR columns
+// (the largest power of two up to 8 that divides a group), which meet in LDS:
+// group sums come out the same in every run. W <= 8192.
+// ===========================================================================
+struct Groups {
+    int count, size;
+};
+
+// v holds columns c .. c + 7 of j = 0 .. 3; factors 1 / rms by group into rs
+template <int GR>
+DEV_INLINE void group_factors(const float v[4][8], float* part, float* rs,
+                              int W, const Groups gp, float eps) {
+    __syncthreads();                       // part and rs are free
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int c = (j * 256 + threadIdx.x) * 8;
+        if (c < W)
+#pragma unroll
+            for (int i = 0; i < 8; i += GR) {
+                float s = 0.f;
+#pragma unroll
+                for (int k = 0; k < GR; ++k) s += v[j][i + k] * v[j][i + k];
+                part[(c + i) / GR] = s;
+            }
+    }
+    __syncthreads();
+    const int lane = threadIdx.x & 63, n = gp.size / GR;
+    for (int g = threadIdx.x >> 6; g < gp.count; g += 4) {
+        float s = 0.f;
+        for (int i = lane; i < n; i += 64) s += part[g * n + i];
+        s = wave_reduce_sum(s);
+        if (lane == 0) rs[g] = 1.f / sqrtf(s / (float)gp.size + eps);
+    }
+    __syncthreads();
+}
+
+// f *= rs of each column's group
+template <int GR>
+DEV_INLINE void scale_groups(float* f, const float* rs, int c,
+                             const Groups gp) {
+#pragma unroll
+    for (int i = 0; i < 8; i += GR) {
+        const float r = rs[min((c + i) / gp.size, gp.count - 1)];
+#pragma unroll
+        for (int k = 0; k < GR; ++k) f[i + k] *= r;
+    }
+}
+
+template <class T, bool ADD, int GR>
+__global__ void __launch_bounds__(256)
+k_group_norm(T* __restrict__ out, float* __restrict__ x,
+             const T* __restrict__ y, const int* __restrict__ rows,
+             const float* __restrict__ wy, const float* __restrict__ w, int W,
+             const Groups gp, float eps) {
+    extern __shared__ float part[];        // W / GR, then a factor per group
+    float* const rs = part + W / GR;
+    const long n = !ADD && rows ? rows[blockIdx.x] : blockIdx.x;
+    float v[4][8], a[4][8];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int c = (j * 256 + threadIdx.x) * 8;
+        if (c < W) {
+            ld8(x + n * W + c, a[j]);
+            if (ADD) ld8(y + n * W + c, v[j]);
+        }
+    }
+    if (ADD) {
+        group_factors<GR>(v, part, rs, W, gp, eps);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int c = (j * 256 + threadIdx.x) * 8;
+            if (c < W) {
+                float g[8];
+                ld8(wy + c, g);
+                scale_groups<GR>(v[j], rs, c, gp);
+#pragma unroll
+                for (int i = 0; i < 8; ++i) a[j][i] += v[j][i] * g[i];
+                st8(x + n * W + c, a[j]);
+            }
+        }
+        if (!out) return;
+    }
+    group_factors<GR>(a, part, rs, W, gp, eps);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int c = (j * 256 + threadIdx.x) * 8;
+        if (c < W) {
+            float g[8];
+            ld8(w + c, g);
+            scale_groups<GR>(a[j], rs, c, gp);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) a[j][i] *= g[i];
+            st8(out + (long)blockIdx.x * W + c, a[j]);
+        }
+    }
+}
+
+// ===========================================================================
+// PolyNorm: out = c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3, powers by element, N
+// dividing a row by its root mean square over Ftrue elements (columns behind
+// them are zero). NV > 0: a row of up to NV * 2048 columns stays in registers.
+// ===========================================================================
+template <class T, int NV>
+__global__ void __launch_bounds__(256)
+k_poly_norm(T* __restrict__ out, const T* __restrict__ z,
+            const float* __restrict__ coef, int F, int Ftrue, float eps) {
+    __shared__ float red[3][4];
+    constexpr int KEEP = NV ? NV : 1;
+    const long n = blockIdx.x;
+    float v[KEEP][8], ss[3] = {0.f, 0.f, 0.f};
+    auto add = [&](const float* f) {
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            const float q = f[i] * f[i];
+            ss[0] += q;
+            ss[1] += q * q;
+            ss[2] += q * q * q;
+        }
+    };
+    if (NV) {
+#pragma unroll
+        for (int j = 0; j < KEEP; ++j) {
+            const int c = (j * 256 + threadIdx.x) * 8;
+            if (c < F) {
+                ld8(z + n * F + c, v[j]);
+                add(v[j]);
+            }
+        }
+    } else {
+        for (int c = threadIdx.x * 8; c < F; c += 2048) {
+            ld8(z + n * F + c, v[0]);
+            add(v[0]);
+        }
+    }
+    float k[3];
+#pragma unroll
+    for (int i = 0; i < 3; ++i) {
+        const float s = wave_reduce_sum(ss[i]);
+        if ((threadIdx.x & 63) == 0) red[i][threadIdx.x >> 6] = s;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < 3; ++i)
+        k[i] = coef[i] / sqrtf((red[i][0] + red[i][1] + red[i][2] +
+                                red[i][3]) / (float)Ftrue + eps);
+    const float k3 = coef[3];
+    auto put = [&](float* f, int c) {
+#pragma unroll
+        for (int i = 0; i < 8; ++i)
+            f[i] = k3 + f[i] * (k[0] + f[i] * (k[1] + f[i] * k[2]));
+        st8(out + n * F + c, f);
+    };
+    if (NV) {
+#pragma unroll
+        for (int j = 0; j < KEEP; ++j) {
+            const int c = (j * 256 + threadIdx.x) * 8;
+            if (c < F) put(v[j], c);
+        }
+    } else {
+        for (int c = threadIdx.x * 8; c < F; c += 2048) {
+            ld8(z + n * F + c, v[0]);
+            put(v[0], c);
+        }
+    }
+}
+
 // out = glu(gu[:, :F], gu[:, F:]), f32
 __global__ void __launch_bounds__(256)
 k_glu_f32(float* __restrict__ out, const float* __restrict__ gu, long n,
@@ -1846,6 +2017,43 @@ int gh_norm_rows(void* stream, int f32, void* out, const void* x,
     else
         k_norm_rows<bf16_t><<<M, 256, 0, st_>>>((bf16_t*)out, (const float*)x,
             (const int*)rows, (const float*)w, w_off, W, Wtrue, eps);
+    LAUNCH_CHECK();
+    return 0;
+}
+
+int gh_group_norm(void* stream, int f32, void* out, void* x, const void* y,
+                  const void* rows, const void* wy, const void* w, int N,
+                  int W, int groups, int size, float eps) {
+    if (N < 1 || W % 8 || W > 8192 || groups < 1 || size < 1 ||
+        (long)groups * size > W || (!y && !out) || (y && rows)) return -100;
+    const int gr = size % 8 == 0 ? 8 : size % 4 == 0 ? 4 : size % 2 ? 1 : 2;
+    const int lds = (W / gr + groups) * 4;
+    if (lds > 64 * 1024) return -100;
+    const Groups gp{groups, size};
+#define GO(T, A, B) k_group_norm<T, A, B><<<N, 256, lds, \
+        (hipStream_t)stream>>>((T*)out, (float*)x, (const T*)y, \
+        (const int*)rows, (const float*)wy, (const float*)w, W, gp, eps)
+#define PICK(T, A) do { if (gr == 8) GO(T, A, 8); else if (gr == 4) \
+        GO(T, A, 4); else if (gr == 2) GO(T, A, 2); else GO(T, A, 1); \
+        } while (0)
+    if (f32) { if (y) PICK(float, true); else PICK(float, false); }
+    else { if (y) PICK(bf16_t, true); else PICK(bf16_t, false); }
+#undef PICK
+#undef GO
+    LAUNCH_CHECK();
+    return 0;
+}
+
+int gh_poly_norm(void* stream, int f32, void* out, const void* z,
+                 const void* coef, int N, int F, int Ftrue, float eps) {
+    if (N < 1 || F % 8 || Ftrue < 1 || Ftrue > F) return -100;
+#define GO(T, NV) k_poly_norm<T, NV><<<N, 256, 0, (hipStream_t)stream>>>( \
+        (T*)out, (const T*)z, (const float*)coef, F, Ftrue, eps)
+#define PICK(T) do { if (F <= 4096) GO(T, 2); else if (F <= 8192) GO(T, 4); \
+        else if (F <= 16384) GO(T, 8); else GO(T, 0); } while (0)
+    if (f32) PICK(float); else PICK(bf16_t);
+#undef PICK
+#undef GO
     LAUNCH_CHECK();
     return 0;
 }

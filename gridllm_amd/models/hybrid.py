@@ -1,6 +1,7 @@
-"""Layer-list models: a decoder in which every layer names its mixer (softmax
-or latent attention over a paged cache, mLSTM or gated linear attention with a
-state per sequence) and its feed-forward (dense gated, or routed experts).
+"""Layer-list models: a decoder in which every layer names its mixer (softmax,
+latent or talking-heads attention over a paged cache, mLSTM or gated linear
+attention with a state per sequence) and its feed-forward (dense gated, dense
+with PolyNorm, or routed experts).
 
 One step function serves prompts, portions of prompts and decoding, also mixed
 in one batch: `forward_step`. Its tokens are ordered decode rows first, so each
@@ -29,17 +30,20 @@ import torch
 from gridllm_amd.models.paged import (PAGE, PagedCache, head_pad, latent_pad,
                                       pad64)
 from gridllm_amd.models.registry import (AttentionMixer, DenseFF, GlaMixer,
-                                         HybridSpec, LatentMixer, RoutedFF)
+                                         HybridSpec, LatentMixer, PolyFF,
+                                         RoutedFF, TalkingMixer)
 from gridllm_amd.ops import hybrid as hops
 from gridllm_amd.ops.autotune import linear as _linear
 from gridllm_amd.ops.autotune import linear_gateup as _linear_gateup
-from gridllm_amd.ops.hybrid import Choice, DepthAverage, StepMeta
+from gridllm_amd.ops.hybrid import (ChunkPortions, Choice, DepthAverage,
+                                    StepMeta, Talk)
 from gridllm_amd.ops.reference import Glu
 from gridllm_amd.parallel.tp import TPContext
 
 _DTYPES = {"bf16": torch.bfloat16, "fp32": torch.float32}
-# portions of up to this many tokens run latent attention token by token
-# against the cached latents; for longer ones it pays to expand these
+# portions of up to this many tokens run latent and talking-heads attention
+# token by token against the cached rows; for longer ones it pays to lay out
+# keys and values
 _ABSORB = 16
 
 
@@ -65,6 +69,10 @@ class BlockWeights:
     wukv: Optional[torch.Tensor] = None       # [H, 2 P, KR]
     wa2: Optional[torch.Tensor] = None        # decays: [rank, H * DK]
     ba2: Optional[torch.Tensor] = None
+    talk: Optional[Talk] = None               # talking-heads attention
+    act: Optional[torch.Tensor] = None        # PolyNorm's numbers
+    pre1: Optional[torch.Tensor] = None       # norms ahead of the sublayers
+    pre2: Optional[torch.Tensor] = None
     corr: Optional[torch.Tensor] = None
     avg: Optional[torch.Tensor] = None        # depth average
     wgateup: Optional[torch.Tensor] = None
@@ -87,6 +95,14 @@ def _pad_heads(t: torch.Tensor, heads: int, to: int) -> torch.Tensor:
     d = t.shape[0] // heads
     t = t.view(heads, d, *t.shape[1:])
     return _pad(t, heads, to, *t.shape[2:]).reshape(heads * to, *t.shape[2:])
+
+
+def _pair_order(dim: int, rot_dims: int) -> torch.Tensor:
+    """Coordinates of a head such that the pairs (i, i + rot_dims / 2) become
+    neighbours, in front."""
+    i = torch.arange(rot_dims // 2)
+    pairs = torch.stack([i, i + rot_dims // 2], dim=1).flatten()
+    return torch.cat([pairs, torch.arange(rot_dims, dim)])
 
 
 class HybridModel:
@@ -113,7 +129,7 @@ class HybridModel:
             self.max_seq = pad64(kv_tokens)
         if kv_tokens:                      # one sequence has to fit the pool
             self.max_seq = min(self.max_seq, pad64(kv_tokens))
-        self.norm_off = 0.0 if spec.scalar_norms else 1.0
+        self.norm_off = 0.0 if spec.scalar_norms or spec.plain_norms else 1.0
         self.rope_len = self.max_seq       # bound of positions
         self.width = pad64(spec.hidden)
         if self.width > 8192:
@@ -125,17 +141,26 @@ class HybridModel:
                                 self.dtype, pool_tokens=kv_tokens,
                                 upload=self.up.upload)
         self.rot = self._rotations()
-        self.expands = dtype == "bf16" and any(self.rot)
+        mixers = [ly.mixer for ly in spec.layers]
+        # latents of prompt portions are expanded; keys within these chunk
+        # sizes laid out
+        self.expands = dtype == "bf16" and any(
+            isinstance(m, LatentMixer) for m in mixers)
+        self.chunks = sorted({m.chunk for m in mixers
+                              if isinstance(m, TalkingMixer)}) \
+            if dtype == "bf16" else []
         if random_init:
             self._init_weights(seed)
 
     def _rotations(self) -> list[Optional[tuple]]:
-        """Per latent-attention layer, cos and sin of position times frequency,
-        f32 [max_seq, R / 2]; 1 and 0 for pairs that are not rotated."""
+        """Per latent- or talking-heads-attention layer, cos and sin of position
+        times frequency, f32 [max_seq, R / 2]; 1 and 0 for pairs that are not
+        rotated."""
         made: dict[tuple, tuple] = {}
 
-        def table(mx: LatentMixer) -> tuple:
-            r = latent_pad(mx)[1]
+        def table(mx) -> tuple:
+            r = latent_pad(mx)[1] if isinstance(mx, LatentMixer) else \
+                -(-mx.rot_dims // 32) * 32
             key = (mx.rot_base, mx.rot_dims, r)
             if key not in made:
                 half = mx.rot_dims // 2
@@ -148,7 +173,8 @@ class HybridModel:
                                   for t in (a.cos(), a.sin()))
             return made[key]
 
-        return [table(ly.mixer) if isinstance(ly.mixer, LatentMixer) else None
+        return [table(ly.mixer)
+                if isinstance(ly.mixer, (LatentMixer, TalkingMixer)) else None
                 for ly in self.spec.layers]
 
     # -- weights -----------------------------------------------------------
@@ -171,10 +197,19 @@ class HybridModel:
             if ly.weights_of is not None:
                 continue
             p, mx, ff = f"l{i}.", ly.mixer, ly.ff
-            out |= {p + "norm1": norm} | self._mixer_shapes(p + "mix.", mx)
+            out |= self._mixer_shapes(p + "mix.", mx)
+            for k in (1, 2) if ff is not None else (1,):
+                out[f"{p}norm{k}"] = norm
+                if s.pre_norms:
+                    out[f"{p}norm{k}b"] = norm
+                if s.layer_scale:
+                    out[f"{p}ls{k}"] = (w,)
             if ff is None:
                 continue
-            out[p + "norm2"] = norm
+            if isinstance(ff, PolyFF):
+                out |= {p + "mlp.up": (ff.ff, w), p + "mlp.down": (w, ff.ff),
+                        p + "mlp.act": (4,)}
+                continue
             if isinstance(ff, DenseFF):
                 out |= {p + "mlp.gate": (ff.ff, w), p + "mlp.up": (ff.ff, w),
                         p + "mlp.down": (w, ff.ff)}
@@ -198,6 +233,12 @@ class HybridModel:
                     p + "dkv": (k + mx.rot_dim, w), p + "dkv.norm": (k,),
                     p + "uk": (h * mx.dim, k), p + "uv": (h * mx.vdim, k),
                     p + "g": (h, w), p + "o": (w, h * mx.vdim)}
+        if isinstance(mx, TalkingMixer):
+            q, k = h * mx.dim, mx.kv_heads * mx.dim
+            return {p + "q": (q, w), p + "q.b": (q,), p + "k": (k, w),
+                    p + "k.b": (k,), p + "q.norm": (mx.dim,),
+                    p + "k.norm": (mx.dim,), p + "talk": (h, h),
+                    p + "o": (w, q)}
         attn = isinstance(mx, AttentionMixer)
         kv = mx.kv_heads if attn else h
         out = {p + "q": (h * mx.dim, w), p + "k": (kv * mx.dim, w),
@@ -228,7 +269,14 @@ class HybridModel:
                 return t
             if last == "norm" and ".mix." in name:
                 return torch.ones(sh, device=self.device)
-            if last in ("norm", "norm1", "norm2"):
+            if last in ("ls1", "ls2"):
+                return torch.ones(sh, device=self.device)
+            if last == "act":              # odd powers, as an activation's
+                return torch.tensor([0.5, 0.0, 0.5, 0.0], device=self.device)
+            if last == "talk":             # mostly each head's own weights
+                return torch.eye(sh[0], device=self.device) + 0.02 * \
+                    torch.randn(sh, generator=gen, device=self.device)
+            if last in ("norm", "norm1", "norm2", "norm1b", "norm2b"):
                 return torch.full(sh, 1.0 - self.norm_off, device=self.device)
             if name.endswith("i.b") or last == "correction":
                 return torch.zeros(sh, device=self.device)
@@ -291,7 +339,7 @@ class HybridModel:
         built: dict[int, BlockWeights] = {}
         for i, ly in enumerate(s.layers):
             if ly.weights_of is None:
-                built[i] = self._assemble_layer(f"l{i}.", ly, get, mat, norm)
+                built[i] = self._assemble_layer(i, ly, get, mat, norm)
         self.layers = [built[s.owner(i)] for i in range(len(s.layers))]
         self.averages = [get(f"l{i}.dwa").float().contiguous()
                          for i in range(len(s.layers))] \
@@ -319,10 +367,46 @@ class HybridModel:
             qnorm=_pad(get(p + "dq.norm").float(), qr),
             kvnorm=_pad(get(p + "dkv.norm").float(), kr))
 
-    def _assemble_layer(self, p: str, ly, get, mat, norm) -> BlockWeights:
-        mx, ff, wp = ly.mixer, ly.ff, self.width
+    def _assemble_talk(self, i: int, mx: TalkingMixer, get, mat) -> dict:
+        p, h, g, d, pd = f"l{i}.mix.", mx.heads, mx.kv_heads, mx.dim, \
+            head_pad(mx)
+        order = _pair_order(d, mx.rot_dims).to(self.device)
+
+        def heads(t, n):            # rows [n * d, ...] reordered, padded
+            t = t.view(n, d, *t.shape[1:])[:, order]
+            return _pad_heads(t.reshape(n * d, *t.shape[2:]), n, pd)
+
+        talk = get(p + "talk").float().contiguous()
+        nh = -(-h // 8)             # heads of a wave in the tiled kernel
+        if nh <= 4:
+            lift = 0
+            if talk.abs().max() > 0:
+                lift = int(torch.log2(talk.abs().max()).ceil())
+            at = torch.tensor([k // nh * 4 + k % nh for k in range(h)],
+                              device=self.device)
+            talk16 = talk.new_zeros(32, 32)
+            talk16[at.unsqueeze(1), at] = talk * 2.0 ** -lift
+            talk16 = talk16.half()
+        return dict(
+            wmix=torch.cat([heads(mat(get(p + "q")), h),
+                            heads(mat(get(p + "k")), g)]),
+            # a head's columns in the order of its values
+            wo=_pad_heads(get(p + "o").to(self.dtype).T.reshape(h, d, -1)
+                          [:, order].reshape(h * d, -1), h, pd).T,
+            talk=Talk(h, d, mx.scale, mx.cap, mx.chunk, self.rot[i],
+                      torch.cat([heads(get(p + "q.b").float(), h),
+                                 heads(get(p + "k.b").float(), g)]),
+                      _pad(get(p + "q.norm").float()[order], pd),
+                      _pad(get(p + "k.norm").float()[order], pd), talk,
+                      *((talk16, 2.0 ** (lift - 14)) if nh <= 4 else ())))
+
+    def _assemble_layer(self, i: int, ly, get, mat, norm) -> BlockWeights:
+        s, mx, ff, wp, p = self.spec, ly.mixer, ly.ff, self.width, f"l{i}."
         h = mx.heads
-        if isinstance(mx, LatentMixer):
+        if isinstance(mx, TalkingMixer):
+            parts = self._assemble_talk(i, mx, get, mat)
+            dv = head_pad(mx)
+        elif isinstance(mx, LatentMixer):
             parts = self._assemble_latent(p + "mix.", mx, get, mat)
             dv = head_pad(mx)
         else:
@@ -330,14 +414,29 @@ class HybridModel:
         wmix = parts.pop("wmix")
         wmix = _pad(wmix, -(-wmix.shape[0] // 128) * 128, wp).contiguous()
         # columns of the output projection follow the padded heads
-        wo = _pad_heads(get(p + "mix.o").to(self.dtype).T, h, dv).T
+        wo = parts.pop("wo", None)
+        if wo is None:
+            wo = _pad_heads(get(p + "mix.o").to(self.dtype).T, h, dv).T
+
+        def norms(k):               # behind a sublayer (scaled), ahead of it
+            t = norm(get(f"{p}norm{k}b" if s.pre_norms else f"{p}norm{k}"))
+            if s.layer_scale:
+                t *= _pad(get(f"{p}ls{k}").float(), wp)
+            return t, norm(get(f"{p}norm{k}")) if s.pre_norms else None
+
+        norm1, pre1 = norms(1)
         w = BlockWeights(
             wmix=wmix, wo=_pad(wo, wp, h * dv).contiguous(),
-            norm1=norm(get(p + "norm1")), **parts)
+            norm1=norm1, pre1=pre1, **parts)
         if ff is None:
             return w
-        w.norm2 = norm(get(p + "norm2"))
+        w.norm2, w.pre2 = norms(2)
         fp = pad64(ff.ff)
+        if isinstance(ff, PolyFF):
+            w.up = mat(get(p + "mlp.up"), fp).contiguous()
+            w.down = mat(get(p + "mlp.down"), wp)
+            w.act = get(p + "mlp.act").float().contiguous()
+            return w
         if isinstance(ff, DenseFF):
             w.wgateup = torch.cat([mat(get(p + "mlp.gate"), fp),
                                    mat(get(p + "mlp.up"), fp)])
@@ -403,6 +502,8 @@ class HybridModel:
             if w.wgateup is not None:
                 gu.add(tuple(w.wgateup.shape))
                 plain.add(tuple(w.down.shape))
+            if w.act is not None:
+                plain |= {tuple(w.up.shape), tuple(w.down.shape)}
         return sorted(plain), sorted(gu)
 
     def interleave_gateup(self) -> None:
@@ -423,7 +524,10 @@ class HybridModel:
         if self.head is not self.embed:
             ts.append(self.head)
         for w in self.unique_layers():
-            ts += vars(w).values()
+            ts += [t for t in vars(w).values() if not isinstance(t, Talk)]
+            if w.talk is not None:
+                ts += [w.talk.bias, w.talk.qnorm, w.talk.knorm, w.talk.talk,
+                       w.talk.talk16]
         return sum(t.numel() * t.element_size() for t in ts if t is not None)
 
     # -- layers ------------------------------------------------------------
@@ -446,6 +550,10 @@ class HybridModel:
             o = hops.latent_attn(_linear(cq, w.wuq), c.lat[i], st, self.rot[i],
                                  w.wuk, w.wuv, w.wukv, mx.scale,
                                  rows[:, at:at + mx.heads])
+        elif isinstance(mx, TalkingMixer):
+            q = hops.talk_rows(rows, c.v[i], c.inv[i], st, w.talk, eps)
+            o = hops.talk_attn(q, c.v[i], c.inv[i], st,
+                               w.talk).view(xb.shape[0], -1)
         elif isinstance(mx, GlaMixer):
             u = hops.proj_f32(xb, w.wgates)
             o = hops.gla(rows, u, w.wa2, w.ba2, c.S[i], w.mnorm, st, mx.dim,
@@ -464,6 +572,10 @@ class HybridModel:
             act = _linear_gateup(xb, w.wgateup, glu) if self.gateup_il else \
                 hops.glu(_linear(xb, w.wgateup), glu)
             return _linear(act, w.down), None, None
+        if isinstance(ff, PolyFF):
+            z = hops.poly_norm(_linear(xb, w.up), w.act, ff.ff,
+                               self.spec.norm_eps)
+            return _linear(z, w.down), None, None
         assert isinstance(ff, RoutedFF)
         how = Choice(ff.top, w.corr, ff.groups, ff.keep,
                      1e-20 if ff.corrected else 0.0, ff.scale)
@@ -474,6 +586,8 @@ class HybridModel:
         """The residual stream behind the last layer, f32 [n, W]; trail
         collects it behind every layer."""
         s = self.spec
+        if s.pre_norms:
+            return self._run_between_norms(tokens, st, trail)
         n, size, norm = tokens.shape[0], (s.hidden, s.norm_eps), self.norm_off
         hist = None
         if s.depth_average:
@@ -509,11 +623,39 @@ class HybridModel:
                 trail.append(x[:, :s.hidden].clone())
         return x
 
+    def _run_between_norms(self, tokens: torch.Tensor, st: StepMeta,
+                           trail: Optional[list]) -> torch.Tensor:
+        """_run for sublayers between two norms: the norm behind one and the
+        norm ahead of the next are one kernel."""
+        s = self.spec
+        how = (s.norm_groups, s.hidden, s.norm_eps)
+        x, _ = hops.embed(tokens, st.pos, self.embed, self.pos_table)
+        h = hops.group_norm(x, None, self.layers[0].pre1, *how, self.dtype)
+        for i, (ly, w) in enumerate(zip(s.layers, self.layers)):
+            ahead = self.layers[i + 1].pre1 if i + 1 < len(s.layers) else None
+            y = self._mix(i, w, ly.mixer, h, st)
+            h = hops.join_norm(x, y, w.norm1, ahead if ly.ff is None
+                               else w.pre2, *how)
+            if ly.ff is not None:
+                y = self._feed(w, ly.ff, h)[0]
+                h = hops.join_norm(x, y, w.norm2, ahead, *how)
+            if trail is not None:
+                trail.append(x[:, :s.hidden].clone())
+        return x
+
+    def _normed(self, x: torch.Tensor, rows: Optional[torch.Tensor],
+                w: torch.Tensor) -> torch.Tensor:
+        s = self.spec
+        if s.norm_groups > 1:
+            return hops.group_norm(x, rows, w, s.norm_groups, s.hidden,
+                                   s.norm_eps, self.dtype)
+        return hops.norm_rows(x, rows, w, 0.0, s.hidden, s.norm_eps,
+                              self.dtype)
+
     def _head(self, x: torch.Tensor, rows: Optional[torch.Tensor]
               ) -> torch.Tensor:
-        h = hops.norm_rows(x, rows, self.head_norm, 0.0, self.spec.hidden,
-                           self.spec.norm_eps, self.dtype)
-        return _linear(h, self.head).float()
+        return _linear(self._normed(x, rows, self.head_norm),
+                       self.head).float()
 
     # -- steps -------------------------------------------------------------
 
@@ -569,6 +711,7 @@ class HybridModel:
                            for q0 in range(0, ln, 128)]
                 lrows += -(-total // 32) * 32
             off += ln
+        talks = [self._chunk_portions(segs, c) for c in self.chunks]
         ids_np = np.concatenate(toks)
         if ids_np.min() < 0 or ids_np.max() >= self.spec.vocab:
             raise ValueError("token id outside of the vocabulary")
@@ -577,6 +720,8 @@ class HybridModel:
         parts = [np.concatenate(pos), np.concatenate(slot), np.asarray(want),
                  np.asarray(segs), np.asarray(tiles), np.asarray(chunks),
                  np.asarray(csegs), np.asarray(litems), np.asarray(ltiles)]
+        for t in talks:
+            parts += t[1:]
         dev = self._upload_ints(parts)
         mixed = bool(tiles)
         st = StepMeta(nd=nd, pos=dev[0], slot=dev[1], table=self.cache.table,
@@ -588,6 +733,11 @@ class HybridModel:
                       absorbed=absorbed, lat_rows=lrows,
                       lat_items=dev[7].view(-1, 4) if litems else None,
                       lat_tiles=dev[8].view(-1, 8) if ltiles else None)
+        for k, (c, t) in enumerate(zip(self.chunks, talks)):
+            if t[0]:
+                items, t16, t128 = dev[9 + 3 * k:12 + 3 * k]
+                st.talk[c] = ChunkPortions(t[0], items.view(-1, 4),
+                                           t16.view(-1, 8), t128.view(-1, 8))
         x = self._run(tokens, st, trail)
         ends = np.asarray([[e[0] for e in entries],
                            [p + len(e[1]) for p, e in zip(starts, entries)]],
@@ -598,12 +748,39 @@ class HybridModel:
             torch.empty(0, self.spec.vocab, device=self.device)
         if not return_hidden:
             return logits
-        h = hops.norm_rows(x, None, self.final_norm, 0.0, self.spec.hidden,
-                           self.spec.norm_eps, self.dtype)
+        h = self._normed(x, None, self.final_norm)
         h = h[:, :self.spec.hidden].float()
         return logits, torch.stack(
             [h[first[i]:first[i] + len(e[1])].mean(0)
              for i, e in enumerate(entries)])
+
+    @staticmethod
+    def _chunk_portions(segs: list, chunk: int) -> tuple:
+        """Pages, items, 16-row and 128-row tiles of the longer portions (see
+        ChunkPortions)."""
+        pages, items, tiles = 0, [], {16: [], 128: []}
+        for off, ln, sl, p0 in segs:
+            if ln <= _ABSORB:
+                continue
+            page0 = p0 // chunk * chunk // PAGE
+            have = np.arange(page0, -(-(p0 + ln) // PAGE))
+            items.append(np.stack(
+                [have, np.full_like(have, sl), pages + have - page0,
+                 np.minimum(PAGE, p0 + ln - have * PAGE)], axis=1))
+            for rows, out in tiles.items():
+                q0 = np.arange(0, ln, rows)
+                t = np.zeros((len(q0), 8), dtype=np.int64)
+                t[:, :6] = (off, ln, pages, 0, p0, page0)
+                t[:, 3] = q0
+                out.append(t)
+            pages += len(have)
+        if not pages:
+            return 0, [], [], []
+        t16, t128 = (np.concatenate(t) for t in tiles.values())
+        # the kernel's blocks start in this order: long spans of keys first
+        span = (t16[:, 3] + t16[:, 4]) % chunk
+        t16 = t16[np.argsort(-span, kind="stable")]
+        return pages, np.concatenate(items), t16, t128
 
     def _upload_ints(self, parts: list) -> list[torch.Tensor]:
         """int32 arrays to the device in one copy; each starts at a multiple

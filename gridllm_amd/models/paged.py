@@ -2,7 +2,8 @@
 
 Two kinds of memory per sequence. Attention layers share one pool of pages of
 64 tokens (one page id holds a sequence's 64 tokens in every attention layer):
-keys and values, or one row of latent and rotated key part per token. Recurrent
+keys and values, one row of latent and rotated key part per token, or (where
+keys are made from the values) values and the inverse of their rms. Recurrent
 layers have a state of fixed size per slot. A sequence is a slot: a row of the
 page table plus its states.
 
@@ -25,7 +26,8 @@ import numpy as np
 import torch
 
 from gridllm_amd.models.registry import (AttentionMixer, GlaMixer,
-                                         HybridSpec, LatentMixer)
+                                         HybridSpec, LatentMixer,
+                                         TalkingMixer)
 
 PAGE = 64
 
@@ -41,10 +43,11 @@ def _next_of(sizes: tuple, n: int, what: str) -> int:
     raise ValueError(f"{what} of {n}: more than {sizes[-1]} is not supported")
 
 
-def head_pad(mixer: Union[AttentionMixer, LatentMixer]) -> int:
+def head_pad(mixer: Union[AttentionMixer, LatentMixer, TalkingMixer]) -> int:
     """Head size that the attention kernels run at: keys and values padded to
     the next of 64, 128, 256."""
-    return _next_of((64, 128, 256), max(mixer.dim, mixer.vdim),
+    return _next_of((64, 128, 256),
+                    max(mixer.dim, getattr(mixer, "vdim", 0)),
                     "attention heads")
 
 
@@ -72,11 +75,12 @@ class PagedCache:
         self.k: list[Optional[torch.Tensor]] = []
         self.v: list[Optional[torch.Tensor]] = []
         self.lat: list[Optional[torch.Tensor]] = []
+        self.inv: list[Optional[torch.Tensor]] = []
         self.S: list[Optional[torch.Tensor]] = []
         self.m: list[Optional[torch.Tensor]] = []
         for ly in spec.layers:
             mx = ly.mixer
-            k = v = lat = s = m = None
+            k = v = lat = inv = s = m = None
             if isinstance(mx, AttentionMixer):
                 shape = (pages + 1, mx.kv_heads, PAGE, head_pad(mx))
                 k = torch.zeros(shape, dtype=dtype, device=device)
@@ -84,6 +88,11 @@ class PagedCache:
             elif isinstance(mx, LatentMixer):
                 lat = torch.zeros(pages + 1, PAGE, sum(latent_pad(mx)),
                                   dtype=dtype, device=device)
+            elif isinstance(mx, TalkingMixer):
+                shape = (pages + 1, mx.kv_heads, PAGE)
+                v = torch.zeros(*shape, head_pad(mx), dtype=dtype,
+                                device=device)
+                inv = torch.zeros(shape, device=device)
             elif isinstance(mx, GlaMixer):
                 s = torch.zeros(slots, mx.heads, pad64(mx.vdim),
                                 pad64(mx.dim), device=device)
@@ -94,6 +103,7 @@ class PagedCache:
             self.k.append(k)
             self.v.append(v)
             self.lat.append(lat)
+            self.inv.append(inv)
             self.S.append(s)
             self.m.append(m)
         self.table = torch.zeros(slots, self.per_slot, dtype=torch.int32,
@@ -190,5 +200,6 @@ class PagedCache:
 
     def bytes(self) -> int:
         return sum(t.numel() * t.element_size()
-                   for ts in (self.k, self.v, self.lat, self.S, self.m)
+                   for ts in (self.k, self.v, self.lat, self.inv, self.S,
+                              self.m)
                    for t in ts if t is not None)

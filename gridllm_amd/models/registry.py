@@ -87,6 +87,29 @@ class AttentionMixer:
 
 
 @dataclass(frozen=True)
+class TalkingMixer:
+    """Grouped softmax attention whose values are the keys as projected (with a
+    bias, ahead of norm and rotation), so that values alone are cached. RMS norms
+    of q and k with a weight over the head; pairs (i, i + rot_dims / 2) of the
+    first rot_dims coordinates turn by p rot_base^(-2 i / rot_dims); scores are
+    soft-capped at `cap`; a query sees the keys of its own chunk of `chunk`
+    positions; 1 is added to the denominator; the heads' weights are mixed by a
+    matrix."""
+    heads: int
+    kv_heads: int
+    dim: int
+    scale: float
+    cap: float
+    chunk: int
+    rot_base: float
+    rot_dims: int
+
+    def params(self, width: int) -> int:
+        h, g, d = self.heads, self.kv_heads, self.dim
+        return (width + 1) * (h + g) * d + 2 * d + h * h + width * h * d
+
+
+@dataclass(frozen=True)
 class MlstmMixer:
     """mLSTM: a matrix memory per head, exponential input gate, log-sigmoid
     forget gate, both soft-capped at gate_cap."""
@@ -162,6 +185,16 @@ class DenseFF:
 
 
 @dataclass(frozen=True)
+class PolyFF:
+    """Ungated feed-forward with PolyNorm between its matrices: a N(z) + b N(z^2)
+    + c N(z^3) + e, N dividing by the root mean square."""
+    ff: int
+
+    def params(self, width: int) -> int:
+        return 2 * width * self.ff + 4
+
+
+@dataclass(frozen=True)
 class RoutedFF:
     """Routed experts: squared ReLU, or (gated) silu(gate) * up.
 
@@ -191,8 +224,9 @@ class RoutedFF:
 
 @dataclass(frozen=True)
 class LayerSpec:
-    mixer: Union[AttentionMixer, LatentMixer, MlstmMixer, GlaMixer]
-    ff: Union[DenseFF, RoutedFF, None] = None
+    mixer: Union[AttentionMixer, LatentMixer, TalkingMixer, MlstmMixer,
+                 GlaMixer]
+    ff: Union[DenseFF, PolyFF, RoutedFF, None] = None
     weights_of: Optional[int] = None
 
 
@@ -210,7 +244,11 @@ class HybridSpec:
     # x <- norm(post_alpha x + y)
     post_alpha: Optional[float] = None
     scalar_norms: bool = False     # one number per norm; else a vector, stored
-                                   # around zero
+    plain_norms: bool = False      # around zero, or as it is
+    # a norm ahead of every sublayer, too: x <- x + norm(y(norm(x)))
+    pre_norms: bool = False
+    norm_groups: int = 1           # equal parts of a row, each with its own rms
+    layer_scale: bool = False      # a vector on every sublayer's normed output
     embed_norm: bool = False
     # a layer passes on a weighted sum of its result, all earlier layers'
     # results and the embedding
@@ -224,6 +262,17 @@ class HybridSpec:
             object.__setattr__(self, "max_seq_len", bound)
         if not self.layers:
             raise ValueError(f"{self.name}: no layers")
+        if self.norm_groups < 1 or self.hidden % self.norm_groups:
+            raise ValueError(f"{self.name}: {self.norm_groups} norm groups of "
+                             f"a width of {self.hidden}")
+        if (self.norm_groups > 1 or self.layer_scale) and not self.pre_norms:
+            raise ValueError(f"{self.name}: grouped norms and layer scales go "
+                             "with norms on both sides")
+        if self.pre_norms and (self.post_alpha is not None or
+                               self.depth_average or self.embed_norm):
+            raise ValueError(f"{self.name}: norms on both sides exclude norms "
+                             "behind the sum, of the embedding, and depth "
+                             "averages")
         for i, ly in enumerate(self.layers):
             j = self.owner(i)
             own = self.layers[j]
@@ -231,13 +280,23 @@ class HybridSpec:
                 raise ValueError(f"layer {i} uses layer {j}'s weights but "
                                  "differs from it")
             mx, ff = ly.mixer, ly.ff
-            if isinstance(mx, AttentionMixer) and mx.heads % mx.kv_heads:
+            if isinstance(mx, (AttentionMixer, TalkingMixer)) and \
+                    mx.heads % mx.kv_heads:
                 raise ValueError(f"layer {i}: {mx.heads} heads over "
                                  f"{mx.kv_heads} key/value heads")
             if isinstance(mx, LatentMixer) and (
                     mx.rot_dims % 2 or not 0 <= mx.rot_dims <= mx.rot_dim):
                 raise ValueError(f"layer {i}: rotates {mx.rot_dims} of "
                                  f"{mx.rot_dim} dimensions")
+            if isinstance(mx, TalkingMixer):
+                if mx.rot_dims % 2 or not 0 <= mx.rot_dims <= mx.dim:
+                    raise ValueError(f"layer {i}: rotates {mx.rot_dims} of "
+                                     f"{mx.dim} dimensions")
+                if not (mx.cap > 0 and mx.chunk > 0):
+                    raise ValueError(f"layer {i}: cap {mx.cap}, chunks of "
+                                     f"{mx.chunk}")
+            if self.pre_norms and isinstance(ff, RoutedFF):
+                raise ValueError(f"layer {i}: routed experts between norms")
             if isinstance(ff, RoutedFF):
                 if ff.outputs % ff.groups or not 0 < ff.keep <= ff.groups:
                     raise ValueError(f"layer {i}: {ff.keep} of {ff.groups} "
@@ -259,7 +318,8 @@ class HybridSpec:
     def model_info(self) -> dict:
         """Ollama-style model_info of /api/show."""
         attn = [ly.mixer for ly in self.layers
-                if isinstance(ly.mixer, (AttentionMixer, LatentMixer))]
+                if isinstance(ly.mixer, (AttentionMixer, LatentMixer,
+                                         TalkingMixer))]
         routed = [ly.ff for ly in self.layers if isinstance(ly.ff, RoutedFF)]
         f = self.family
         info = {
@@ -280,6 +340,11 @@ class HybridSpec:
                          f"{f}.attention.q_lora_rank": attn[0].q_rank,
                          f"{f}.rope.dimension_count": attn[0].rot_dims,
                          f"{f}.rope.freq_base": attn[0].rot_base}
+            elif isinstance(attn[0], TalkingMixer):
+                info |= {f"{f}.attention.chunk_size": attn[0].chunk,
+                         f"{f}.attention.logit_softcapping": attn[0].cap,
+                         f"{f}.rope.dimension_count": attn[0].rot_dims,
+                         f"{f}.rope.freq_base": attn[0].rot_base}
         if routed:
             info |= {f"{f}.expert_count": routed[0].experts,
                      f"{f}.expert_used_count": routed[0].top}
@@ -289,15 +354,16 @@ class HybridSpec:
     def params(self) -> int:
         w = self.hidden
         norm = 1 if self.scalar_norms else w
+        sub = norm * (1 + self.pre_norms) + w * self.layer_scale
         total = (self.vocab * (1 if self.tied else 2) + self.positions) * w
         total += norm * (1 + self.embed_norm)
         for i, ly in enumerate(self.layers):
             if self.depth_average:
                 total += i + 2
             if ly.weights_of is None:
-                total += ly.mixer.params(w) + norm
+                total += ly.mixer.params(w) + sub
                 if ly.ff is not None:
-                    total += ly.ff.params(w) + norm
+                    total += ly.ff.params(w) + sub
         return total
 
 
@@ -415,10 +481,51 @@ def read_maferax(cfg: dict, name: str = "maferax", shape=None) -> HybridSpec:
 _MAFERAX = dict(family="maferax", scalar_norms=True, embed_norm=True,
                 depth_average=True, tied=False)
 
+def _read_vivepel_layer(i: int, ly: dict) -> LayerSpec:
+    _take(ly, f"layer {i}", ("type", "mixer"), ("mlp",))
+    kind, d, ff = ly["type"], ly["mixer"], ly.get("mlp")
+    if kind != "attention":
+        raise ValueError(f"config: unknown mixer {kind!r}")
+    _take(d, kind, ("heads", "kv_heads", "dim", "vdim", "scale", "softcap",
+                    "rot", "mask"))
+    rot = _take(d["rot"], "rot", ("base", "dims"))
+    mask = _take(d["mask"], "mask", ("size",))
+    if d["vdim"] != d["dim"]:
+        raise ValueError(f"config: values are keys, but of size {d['vdim']}, "
+                         f"not {d['dim']}")
+    mixer = TalkingMixer(
+        heads=d["heads"], kv_heads=d["kv_heads"], dim=d["dim"],
+        scale=float(d["scale"]), cap=float(d["softcap"]),
+        chunk=int(mask["size"]), rot_base=float(rot["base"]),
+        rot_dims=rot["dims"])
+    if ff is None:
+        return LayerSpec(mixer)
+    if ff.get("kind") != "dense":
+        raise ValueError(f"config: unknown mlp kind {ff.get('kind')!r}")
+    _take(ff, "dense mlp", ("kind", "ff"))
+    return LayerSpec(mixer, PolyFF(ff["ff"]))
+
+
+def read_vivepel(cfg: dict, name: str = "vivepel", shape=None) -> HybridSpec:
+    """Vivepel's config.json -> spec."""
+    _take(cfg, "model", ("layers", "vocab", "width", "norm"),
+          ("architecture",))
+    norm = _take(cfg["norm"], "norm", ("eps", "groups"))
+    return HybridSpec(
+        name=name, vocab=cfg["vocab"], hidden=cfg["width"],
+        layers=tuple(_read_vivepel_layer(i, ly)
+                     for i, ly in enumerate(cfg["layers"])),
+        norm_eps=float(norm["eps"]), norm_groups=norm["groups"], **_VIVEPEL)
+
+
+_VIVEPEL = dict(family="vivepel", plain_norms=True, pre_norms=True,
+                layer_scale=True, tied=False)
+
 # "architecture" in config.json -> reader. Checkpoints without that key (HF
 # layout) are loaded into the architecture that the model name gives.
 _READERS: dict[str, Callable[..., Spec]] = {"Birepel": read_birepel,
-                                            "Maferax": read_maferax}
+                                            "Maferax": read_maferax,
+                                            "Vivepel": read_vivepel}
 
 
 def _shape_reader(path: str) -> Callable[[str], Optional[tuple]]:
@@ -588,6 +695,28 @@ _reg(maferax_stack("maferax:5b", vocab=128256, hidden=3072, blocks=2,
                    routed=RoutedFF(64, 8, 1024, gated=True, corrected=True,
                                    groups=8, keep=4, identity=8, scale=2.0)),
      "maferax-5b")
+
+
+# Vivepel: talking-heads attention within chunks, PolyNorm feed-forwards, norms
+# in groups on both sides of every sublayer
+def vivepel_stack(name: str, *, vocab: int, hidden: int, attn: TalkingMixer,
+                  ff: int, layers: int, groups: int,
+                  max_seq_len: int) -> HybridSpec:
+    return HybridSpec(name, vocab=vocab, hidden=hidden,
+                      layers=(LayerSpec(attn, PolyFF(ff)),) * layers,
+                      norm_eps=1e-5, norm_groups=groups,
+                      max_seq_len=max_seq_len, **_VIVEPEL)
+
+
+_reg(vivepel_stack("tiny-vivepel", vocab=512, hidden=128, ff=256, layers=2,
+                   groups=4, max_seq_len=256,
+                   attn=TalkingMixer(4, 2, 32, 32 ** -0.5, 30.0, 48, 1e4, 16)),
+     "tiny-vivepel:latest")
+_reg(vivepel_stack("vivepel:2b", vocab=128256, hidden=3072, ff=12288,
+                   layers=8, groups=8, max_seq_len=16384,
+                   attn=TalkingMixer(24, 8, 128, 128 ** -0.5, 30.0, 4096, 5e5,
+                                     64)),
+     "vivepel-2b")
 
 
 def get_spec(name: str, max_seq_len: int = 0) -> Spec:

@@ -24,9 +24,10 @@ ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950")
 
 # library name -> source. "hip": what every model shares and the Llama
 # family's attention; "hybrid": layer-list models (paged attention, mLSTM,
-# gated linear attention, routed experts); "latent": their latent attention
+# gated linear attention, routed experts); "latent": their latent attention;
+# "talk": their talking-heads attention
 LIBS = {"hip": "gridllm_kernels.hip", "hybrid": "gridllm_hybrid.hip",
-        "latent": "gridllm_latent.hip"}
+        "latent": "gridllm_latent.hip", "talk": "gridllm_talk.hip"}
 
 # hipcc otherwise forms packed-FP32 instructions from plain float code; some
 # of their forms give wrong results on this hardware, so all HIP code is
@@ -37,6 +38,18 @@ FLAGS = [f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-shared", "-fPIC",
 
 def lib_path(name: str) -> str:
     return os.path.join(PKG_DIR, f"libgridllm_{name}.so")
+
+
+def libs_of(spec) -> list[str]:
+    """The libraries that a model of this spec calls."""
+    from gridllm_amd.models.registry import (HybridSpec, LatentMixer,
+                                             TalkingMixer)
+    if not isinstance(spec, HybridSpec):
+        return ["hip"]
+    mixers = [ly.mixer for ly in spec.layers]
+    return ["hip", "hybrid"] + [
+        lib for lib, kind in (("latent", LatentMixer), ("talk", TalkingMixer))
+        if any(isinstance(m, kind) for m in mixers)]
 
 
 def needs_build(name: str) -> bool:

@@ -1,6 +1,6 @@
-"""ctypes binding to libgridllm_hybrid.so and libgridllm_latent.so: the gfx950
-kernels of the layer-list models (csrc/gridllm_hybrid.hip and
-csrc/gridllm_latent.hip). Same contract as hip_ops: launches go onto torch's
+"""ctypes binding to libgridllm_hybrid.so, libgridllm_latent.so and
+libgridllm_talk.so: the gfx950 kernels of the layer-list models
+(csrc/gridllm_hybrid.hip, _latent.hip and _talk.hip). Same contract as hip_ops: launches go onto torch's
 current stream, a missing library raises, shapes are checked on the host before
 a launch.
 
@@ -21,10 +21,11 @@ from gridllm_amd.ops.build import lib_path
 from gridllm_amd.ops.hip_ops import (HipExtensionMissing, _check,
                                      _check_range)
 from gridllm_amd.ops.reference import Glu
-from gridllm_amd.ops.reference_hybrid import Choice, StepMeta
+from gridllm_amd.ops.reference_hybrid import Choice, StepMeta, Talk
 
 _libs: dict[str, ctypes.CDLL] = {}
 PAGE = 64
+LOG2E = 1.4426950408889634
 
 # argument kinds of each entry point after the stream: p pointer, i int,
 # l long, f float
@@ -33,6 +34,8 @@ _SIGS = {
     "gh_post_norm": "ippppipfiiif",
     "gh_sum_norm": "ipppppippffppiiiiif",
     "gh_norm_rows": "ippppfiiif",
+    "gh_group_norm": "ippppppiiiif",
+    "gh_poly_norm": "ipppiiif",
     "gh_glu_f32": "ppliffff",
     "gh_proj_f32": "ppppiii",
     "gh_qknorm_kv": "ipppppippiiiiiiffi",
@@ -52,8 +55,14 @@ _SIGS = {
     "gn_latent_attn_f32": "pppppippppiiiiiif",
     "gn_latent_gather": "pppipii",
     "gn_latent_prefill": "ppppipippiiiifpi",
+    "gt_talk_rows": "ipppppippppppiiiiiiiif",
+    "gt_talk_decode": "pppppippppppp" + "iiiiiiiifff",
+    "gt_talk_gather": "pppppipppipiiii",
+    "gt_talk_lse": "ppppiiiiifff",
+    "gt_talk_prefill": "pppppppiiiiiffff",
+    "gt_talk_plain": "ipppppipppppp" + "iiiiiiiff",
 }
-_LIB_OF = {"gh": "hybrid", "gn": "latent"}
+_LIB_OF = {"gh": "hybrid", "gn": "latent", "gt": "talk"}
 _KINDS = {"p": ctypes.c_void_p, "i": ctypes.c_int, "l": ctypes.c_long,
           "f": ctypes.c_float}
 
@@ -176,6 +185,48 @@ def norm_rows(x: torch.Tensor, rows: Optional[torch.Tensor], w: torch.Tensor,
     out = torch.empty(m, x.shape[1], dtype=dtype, device=x.device)
     _call("gh_norm_rows", _f32(out), out, x, rows, w, w_off, m, x.shape[1],
           width, eps)
+    return out
+
+
+def group_norm(x: torch.Tensor, rows: Optional[torch.Tensor], w: torch.Tensor,
+               groups: int, width: int, eps: float,
+               dtype: torch.dtype) -> torch.Tensor:
+    """norm(x[rows]) * w in dtype, each of `groups` equal parts of the first
+    `width` columns by its own mean; rows int32, None for all."""
+    m = x.shape[0] if rows is None else rows.shape[0]
+    _dense(x, rows, w)
+    assert w.shape == (x.shape[1],) and width % groups == 0
+    if rows is not None:
+        _check_range("group_norm.rows", rows, x.shape[0])
+    out = torch.empty(m, x.shape[1], dtype=dtype, device=x.device)
+    _call("gh_group_norm", _f32(out), out, x, None, rows, None, w, m,
+          x.shape[1], groups, width // groups, eps)
+    return out
+
+
+def join_norm(x: torch.Tensor, y: torch.Tensor, wy: torch.Tensor,
+              w: Optional[torch.Tensor], groups: int, width: int,
+              eps: float) -> Optional[torch.Tensor]:
+    """x += norm(y) * wy, in place; then norm(x) * w in y's type, if there is a
+    w. Norms as in group_norm."""
+    n, wp = x.shape
+    _dense(x, y, wy, w)
+    assert y.shape == x.shape and wy.shape == (wp,) and width % groups == 0
+    out = None if w is None else torch.empty_like(y)
+    _call("gh_group_norm", _f32(y), out, x, y, None, wy, w, n, wp, groups,
+          width // groups, eps)
+    return out
+
+
+def poly_norm(z: torch.Tensor, coef: torch.Tensor, ff: int,
+              eps: float) -> torch.Tensor:
+    """c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3, N dividing a row by its root mean
+    square over the first ff columns (the others are zero); coef f32 [4]."""
+    _dense(z, coef)
+    assert coef.shape == (4,) and 0 < ff <= z.shape[1]
+    out = torch.empty_like(z)
+    _call("gh_poly_norm", _f32(z), out, z, coef, z.shape[0], z.shape[1], ff,
+          eps)
     return out
 
 
@@ -437,4 +488,79 @@ def gla(rows: torch.Tensor, u: torch.Tensor, wa2: torch.Tensor,
     out = torch.empty(n, h * dv, dtype=rows.dtype, device=dev)
     _call("gh_rec_out", f, 1, out, o, None, rows, None, None, st.pos, st.slot,
           norm, 0, 0, n, h, dk, dv, ld, vdim, 0.0, eps)
+    return out
+
+
+def talk_rows(rows: torch.Tensor, vc: torch.Tensor, inv: torch.Tensor,
+              st: StepMeta, tk: Talk, eps: float) -> torch.Tensor:
+    """From projection rows [q H*P | k G*P | ...] without their bias: normed and
+    rotated queries [n, H, P]; k goes to the pages of vc [pages, G, 64, P], and
+    1 / rms(k) to inv f32 [pages, G, 64]."""
+    n, ld = rows.shape
+    h, (g, _, p) = tk.heads, vc.shape[1:]
+    _dense(rows, vc, inv, st.table, tk.bias, tk.qnorm, *tk.rot)
+    assert ld >= (h + g) * p and tk.bias.shape == ((h + g) * p,)
+    assert inv.shape == vc.shape[:3] and tk.qnorm.shape == (p,)
+    _check_range("talk_rows.slot", st.slot, st.table.shape[0])
+    q = torch.empty(n, h, p, dtype=rows.dtype, device=rows.device)
+    _call("gt_talk_rows", _f32(rows), rows, q, vc, inv, st.table,
+          st.table.shape[1], st.pos, st.slot, tk.bias, tk.qnorm, *tk.rot,
+          tk.rot[0].shape[0], n, h, g, p, 2 * tk.rot[0].shape[1], ld, tk.dim,
+          eps)
+    return q
+
+
+def _talk_sizes(tk: Talk, g: int, p: int) -> tuple[bool, bool]:
+    """Whether the one-pass and the tiled kernels take these sizes."""
+    h, nh = tk.heads, -(-tk.heads // 8)
+    one = h <= 64 and g * p <= 1024 and not (p == 256 and g > 2 and h > 32) \
+        and tk.cap <= 128
+    return one, one and nh <= 4 and nh * p <= 512
+
+
+def talk_tiled(tk: Talk, g: int, p: int) -> bool:
+    """Whether prompt portions of this mixer run the tiled kernels."""
+    return _talk_sizes(tk, g, p)[1]
+
+
+def talk_attn(q: torch.Tensor, vc: torch.Tensor, inv: torch.Tensor,
+              st: StepMeta, tk: Talk) -> torch.Tensor:
+    """Talking-heads attention of a step's tokens over their sequences' pages.
+    q/out [n, H, P]."""
+    n, h, p = q.shape
+    g, per, dev = vc.shape[1], st.table.shape[1], q.device
+    _dense(q, vc, inv, st.table, tk.knorm, tk.talk, tk.talk16, *tk.rot)
+    assert tk.talk.shape == (h, h) and tk.knorm.shape == (p,) and h % g == 0
+    out = torch.empty_like(q)
+    nrot, r = tk.rot[0].shape[0], 2 * tk.rot[0].shape[1]
+    one, tiled = _talk_sizes(tk, g, p)
+    cap = (2 * LOG2E * tk.scale / tk.cap, tk.cap * LOG2E,
+           max(0.0, tk.cap * LOG2E - 80.0))
+    if _f32(q) or not one:
+        _call("gt_talk_plain", _f32(q), out, q, vc, inv, st.table, per, st.pos,
+              st.slot, tk.knorm, tk.talk, *tk.rot, nrot, n, h, g, p, r,
+              tk.chunk, tk.scale, tk.cap)
+        return out
+    portions = st.talk.get(tk.chunk) if tiled else None
+    na = n if portions is None else st.absorbed
+    if na:
+        # a split's sums are as large as the values of 2 H keys
+        seen = min(st.max_len, tk.chunk)
+        nsplit = max(1, min(256 // na, -(-seen // max(128, 8 * h)), 32))
+        ws = torch.empty(na * nsplit * (g * h * p + h), dtype=torch.float32,
+                         device=dev) if nsplit > 1 else None
+        _call("gt_talk_decode", out, q, vc, inv, st.table, per, st.pos,
+              st.slot, ws, tk.knorm, tk.talk, *tk.rot, nrot, na, h, g, p, r,
+              tk.chunk, nsplit, *cap)
+    if portions is not None:
+        kx = torch.empty(2, portions.pages, g, PAGE * p, dtype=q.dtype,
+                         device=dev)
+        _call("gt_talk_gather", kx[0], kx[1], vc, inv, st.table, per, tk.knorm,
+              *tk.rot, nrot, portions.items, portions.items.shape[0], g, p, r)
+        lse = torch.empty(n, h, dtype=torch.float32, device=dev)
+        _call("gt_talk_lse", lse, q, kx[0], portions.tiles128,
+              portions.tiles128.shape[0], h, g, p, tk.chunk, *cap)
+        _call("gt_talk_prefill", out, q, kx[0], kx[1], lse, tk.talk16,
+              portions.tiles16, portions.tiles16.shape[0], h, g, p, tk.chunk,
+              *cap, tk.talk16_scale)
     return out

@@ -8,7 +8,7 @@ import torch
 from gridllm_amd.ops import hip_hybrid, reference_hybrid
 from gridllm_amd.ops import reference
 from gridllm_amd.ops.reference_hybrid import (  # noqa: F401
-    Choice, DepthAverage, StepMeta)
+    ChunkPortions, Choice, DepthAverage, StepMeta, Talk)
 
 
 def _dispatch(name: str):
@@ -25,11 +25,16 @@ embed = _dispatch("embed")
 post_norm = _dispatch("post_norm")
 sum_norm = _dispatch("sum_norm")
 norm_rows = _dispatch("norm_rows")
+group_norm = _dispatch("group_norm")
+join_norm = _dispatch("join_norm")
+poly_norm = _dispatch("poly_norm")
 proj_f32 = _dispatch("proj_f32")
 qknorm_kv = _dispatch("qknorm_kv")
 paged_attn = _dispatch("paged_attn")
 latent_rows = _dispatch("latent_rows")
 latent_attn = _dispatch("latent_attn")
+talk_rows = _dispatch("talk_rows")
+talk_attn = _dispatch("talk_attn")
 mlstm = _dispatch("mlstm")
 gla = _dispatch("gla")
 moe = _dispatch("moe")

@@ -4,13 +4,29 @@ step that both take."""
 
 from __future__ import annotations
 
-from dataclasses import dataclass
+from dataclasses import dataclass, field
 from typing import Optional
 
 import torch
 import torch.nn.functional as F
 
 PAGE = 64
+
+
+@dataclass
+class ChunkPortions:
+    """Prompt portions of a step as talking-heads attention takes them, for one
+    chunk size. The keys that they see are laid out in `pages` pages:
+    items    [*, 4] {page number, slot, page to write, rows} per page
+    tiles16  [*, 8] {first token, length, first page, first row, start, page
+             number of that page} per 16 rows of a portion, longest spans
+             first, and
+    tiles128 per 128 rows
+    """
+    pages: int
+    items: torch.Tensor
+    tiles16: torch.Tensor
+    tiles128: torch.Tensor
 
 
 @dataclass
@@ -48,6 +64,8 @@ class StepMeta:
     lat_rows: int = 0
     lat_items: Optional[torch.Tensor] = None
     lat_tiles: Optional[torch.Tensor] = None
+    # by chunk size: the portions behind the absorbed tokens
+    talk: dict[int, ChunkPortions] = field(default_factory=dict)
 
     def entries(self) -> list:
         """(first token, length, slot, start) of every entry, on the host."""
@@ -69,6 +87,27 @@ class Choice:
     keep: int = 1
     eps: float = 0.0
     scale: float = 1.0
+
+
+@dataclass
+class Talk:
+    """A talking-heads attention layer: its constants and weights. rot: cos and
+    sin tables [positions, R / 2] of neighbouring pairs; bias f32 [(H + G) * P]
+    of the projection; norms f32 [P]; talk f32 [H, H]."""
+    heads: int
+    dim: int
+    scale: float
+    cap: float
+    chunk: int
+    rot: tuple
+    bias: torch.Tensor
+    qnorm: torch.Tensor
+    knorm: torch.Tensor
+    talk: torch.Tensor
+    # talk in f16 in the tiled kernel's numbering of heads, and the factor that
+    # makes up for its scaling
+    talk16: Optional[torch.Tensor] = None
+    talk16_scale: float = 1.0
 
 
 @dataclass
@@ -129,6 +168,30 @@ def sum_norm(x, xo, xb, y, w, w_off, alpha, width, eps, pair_w=None,
 def norm_rows(x, rows, w, w_off, width, eps, dtype):
     z = x if rows is None else x[rows.long()]
     return _norm(z, w, w_off, width, eps).to(dtype)
+
+
+def group_norm(x, rows, w, groups, width, eps, dtype):
+    z = x if rows is None else x[rows.long()]
+    parts = z[:, :width].view(z.shape[0], groups, -1)
+    rs = torch.rsqrt(parts.pow(2).mean(-1, keepdim=True) + eps)
+    out = torch.zeros_like(z)
+    out[:, :width] = (parts * rs).flatten(1)
+    return (out * w).to(dtype)
+
+
+def join_norm(x, y, wy, w, groups, width, eps):
+    x += group_norm(y.float(), None, wy, groups, width, eps, torch.float32)
+    return None if w is None else group_norm(x, None, w, groups, width, eps,
+                                             y.dtype)
+
+
+def poly_norm(z, coef, ff, eps):
+    z, out = z.float(), coef[3]
+    for i in range(3):
+        q = z ** (i + 1)
+        out = out + coef[i] * q * torch.rsqrt(
+            q.pow(2).sum(-1, keepdim=True) / ff + eps)
+    return out
 
 
 def proj_f32(x, w, bias=None):
@@ -307,3 +370,46 @@ def moe(x, logits, up, down, how):
             a = torch.relu(a) ** 2
         ye[r] = (a @ down[e].float().T).to(x.dtype)
     return ye, wt, ident
+
+
+def talk_rows(rows, vc, inv, st, tk, eps):
+    n, h, (g, _, p) = rows.shape[0], tk.heads, vc.shape[1:]
+    cols = rows[:, :(h + g) * p].float() + tk.bias
+    q, v = cols.view(n, h + g, p).split([h, g], dim=1)
+    rs = torch.rsqrt(v.pow(2).sum(-1) / tk.dim + eps)
+    page = st.table[st.slot.long(), (st.pos // PAGE).long()].long()
+    off = (st.pos % PAGE).long()
+    vc[page, :, off] = v.to(vc.dtype)
+    inv[page, :, off] = rs
+    return _rotate_first(_norm(q, tk.qnorm, 0.0, tk.dim, eps), st.pos,
+                         tk.rot).to(rows.dtype)
+
+
+def _rotate_first(x, pos, rot):
+    """_rotate on the coordinates that the tables cover."""
+    r = 2 * rot[0].shape[1]
+    return torch.cat([_rotate(x[..., :r], pos, rot), x[..., r:]], dim=-1)
+
+
+def talk_attn(q, vc, inv, st, tk):
+    n, h, p = q.shape
+    g = vc.shape[1]
+    out = torch.empty_like(q)
+    for off, ln, slot, start in st.entries():
+        lo, total = start // tk.chunk * tk.chunk, start + ln
+        page, row = _rows_of(vc, st.table, slot, lo, total)
+        v = vc[page, :, row].float()
+        k = _rotate_first(v * inv[page, :, row].unsqueeze(-1) * tk.knorm,
+                          torch.arange(lo, total), tk.rot)
+        k, v = (t.repeat_interleave(h // g, dim=1) for t in (k, v))
+        s = torch.einsum("thd,shd->hts", q[off:off + ln].float(), k)
+        s = tk.cap * torch.tanh(s * tk.scale / tk.cap)
+        i = torch.arange(start, total).view(1, -1, 1)
+        j = torch.arange(lo, total).view(1, 1, -1)
+        s = s.masked_fill((j > i) | (j // tk.chunk != i // tk.chunk),
+                          float("-inf"))
+        s = torch.cat([s, torch.zeros(h, ln, 1)], dim=-1)
+        w = torch.softmax(s, dim=-1)[..., :-1]
+        w = torch.einsum("hg,gts->hts", tk.talk, w)
+        out[off:off + ln] = torch.einsum("hts,shd->thd", w, v).to(q.dtype)
+    return out

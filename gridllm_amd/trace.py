@@ -84,8 +84,11 @@ def main(argv: Optional[list[str]] = None) -> int:
     args = ap.parse_args(argv)
     os.environ.setdefault("LOG_LEVEL", "warn")
     if args.device != "cpu":
-        from gridllm_amd.ops.build import build
-        build()                            # compiles what is missing or stale
+        from gridllm_amd.models.registry import spec_from_dir
+        from gridllm_amd.ops.build import build, libs_of
+        spec = spec_from_dir(args.model)
+        # compiles what the model needs and is missing or stale
+        build(names=libs_of(spec) if spec else None)
     engine = make_engine(args.model, args.dtype, args.max_tokens, args.device)
     replay(engine, sys.stdin, args.out, sys.stdout)
     return 0
