@@ -502,12 +502,13 @@ def engine_mode(args, rank, world, local_rank, dist, device, on_gpu):
 
 def layers_twin(spec):
     """The closest model of another design at the size of a layer-list model,
-    and its key in the results: Birepel beside Maferax, layer by layer, and a
-    Llama of equal active feed-forward size beside Birepel."""
+    and its key in the results: Birepel beside Maferax, layer by layer, a Llama
+    of equal active feed-forward size beside Birepel, and of as many
+    feed-forward weights beside Vivepel."""
     from gridllm_amd.models.registry import (AttentionMixer, DenseFF,
                                              HybridSpec, LatentMixer,
                                              LayerSpec, MlstmMixer, ModelSpec,
-                                             RoutedFF)
+                                             PolyFF, RoutedFF, TalkingMixer)
     if spec.family == "maferax":
         layers = []
         for ly in spec.layers:
@@ -528,14 +529,16 @@ def layers_twin(spec):
             layers=tuple(layers), norm_eps=spec.norm_eps,
             positions=spec.max_seq_len)
     mx = next(ly.mixer for ly in spec.layers
-              if isinstance(ly.mixer, AttentionMixer))
+              if isinstance(ly.mixer, (AttentionMixer, TalkingMixer)))
     ff = next((f.top * f.ff for f in (ly.ff for ly in spec.layers)
                if hasattr(f, "top")), spec.layers[0].ff.ff)
+    if isinstance(spec.layers[0].ff, PolyFF):     # two matrices, not three
+        ff = max(64, ff * 2 // 3 // 64 * 64)
     return "llama_twin", ModelSpec(
         f"{spec.name}-llama-twin", hidden=spec.hidden,
         layers=len(spec.layers), heads=mx.heads, kv_heads=mx.kv_heads,
         head_dim=mx.dim, intermediate=ff, vocab=spec.vocab,
-        max_seq_len=spec.max_seq_len)
+        max_seq_len=spec.max_seq_len, tie_embeddings=spec.tied)
 
 
 def layers_mode(args, rank, world, local_rank, dist, device, on_gpu):
@@ -645,7 +648,7 @@ def main() -> None:
     ap.add_argument("--model", default="llama3.2:3b")
     ap.add_argument("--layers-model", default="",
                     help="layers: layer-list model to time beside its twin "
-                         "(default birepel:3b; maferax:5b is another)")
+                         "(default birepel:3b; others: maferax:5b, vivepel:2b)")
     ap.add_argument("--concurrency", type=int, default=1024,
                     help="serving: concurrent streams per GPU")
     ap.add_argument("--num-predict", type=int, default=128,

@@ -122,11 +122,12 @@ DEV_INLINE void split_tiles(int p, int chunk, int nsplit, int split, int* t0,
 // ===========================================================================
 template <int P, int GP, int HB>
 struct DecodeShape {
-    static constexpr int WAVES = GP * P / 16 < 8 ? GP * P / 16 : 8;
+    static constexpr int WAVES =
+        GP > 8 ? 16 : GP * P / 16 < 8 ? GP * P / 16 : 8;
     static constexpr int CW = GP * P / WAVES;     // columns of a wave
     static constexpr int QLD = P + 8, PLD = 40;
     static constexpr int TILE = GP * 32 * P;
-    static constexpr int IT = GP > 8 ? 4 : 2;     // score items of a wave
+    static_assert(P % CW == 0, "a wave has columns of one value head");
     // elements of LDS: two tiles, queries, weights; then f32 sums
     static constexpr int ELEMS = 2 * TILE + HB * 16 * (QLD + PLD);
     static constexpr int BYTES = ELEMS * 2 + HB * 16 * 2 * 4;
@@ -142,7 +143,7 @@ k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
               const float* __restrict__ talk, const Rotation rot, int N,
               int H, int G, int chunk, int nsplit, const Cap cap) {
     typedef DecodeShape<P, GP, HB> Sh;
-    constexpr int WAVES = Sh::WAVES, CW = Sh::CW, CH = P / 8, IT = Sh::IT;
+    constexpr int WAVES = Sh::WAVES, CW = Sh::CW, CH = P / 8, IT = 2;
     constexpr int NS = P / 32, NT = CW / 16, QLD = Sh::QLD, PLD = Sh::PLD;
     constexpr int LOADS = GP * 32 * CH / (WAVES * 64);
     extern __shared__ __attribute__((aligned(16))) bf16_t smem[];
@@ -153,7 +154,7 @@ k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
     const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
     const int fr = lane & 15, gq = lane >> 4;
     const int rep = H / G, rbn = (rep + 15) >> 4, items = 2 * G * rbn;
-    const int per = (items + WAVES - 1) / WAVES;    // up to IT
+    const int per = (items + WAVES - 1) / WAVES;    // 1 or 2, see IT
     const int p = min(pos[n], per_slot * PAGE - 1);
     const int lo = first_seen(p, chunk);
     int t0, t1;

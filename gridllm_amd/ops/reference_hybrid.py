@@ -388,6 +388,8 @@ def talk_rows(rows, vc, inv, st, tk, eps):
 def _rotate_first(x, pos, rot):
     """_rotate on the coordinates that the tables cover."""
     r = 2 * rot[0].shape[1]
+    if not r:
+        return x
     return torch.cat([_rotate(x[..., :r], pos, rot), x[..., r:]], dim=-1)
 
 

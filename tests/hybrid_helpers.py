@@ -6,7 +6,7 @@ import os
 import pytest
 import torch
 
-from gridllm_amd.ops.hybrid import StepMeta
+from gridllm_amd.ops.hybrid import ChunkPortions, StepMeta
 
 REPO = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 RUNS = [pytest.param(("cpu", "fp32"), id="cpu"),
@@ -60,9 +60,10 @@ def close(got, want, run, exact=2e-4, coarse=0.04, odd=0.04):
         assert bad <= odd * len(e), (bad, len(e), float(e.max()))
 
 
-def meta_for(cache, slot, start, ln, dev, absorb=16):
-    """Step of one entry, as forward_step lays it out. Latent attention takes
-    portions of up to `absorb` tokens one by one."""
+def meta_for(cache, slot, start, ln, dev, absorb=16, chunk=0):
+    """Step of one entry, as forward_step lays it out. Latent and talking-heads
+    attention take portions of up to `absorb` tokens one by one; `chunk` is the
+    latter's."""
     def t(a, w):
         return torch.tensor(a, dtype=torch.int32, device=dev).view(-1, w)
     st = StepMeta(nd=1 if ln == 1 else 0,
@@ -86,6 +87,14 @@ def meta_for(cache, slot, start, ln, dev, absorb=16):
             64, st.lat_rows - c)] for c in range(0, total, 64)], 4)
         st.lat_tiles = t([[0, ln, 0, q, start, 0, 0, 0]
                           for q in range(0, ln, 128)], 8)
+        if chunk:
+            p0 = start // chunk * chunk // 64          # first page seen
+            n = -(-total // 64) - p0
+            st.talk[chunk] = ChunkPortions(
+                n, t([[p0 + i, slot, i, min(64, total - 64 * (p0 + i))]
+                      for i in range(n)], 4),
+                *(t([[0, ln, 0, q, start, p0, 0, 0]
+                     for q in range(0, ln, k)], 8) for k in (16, 128)))
     return st
 
 
