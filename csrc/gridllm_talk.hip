@@ -34,9 +34,16 @@ struct Cap {
     float rate, top, rho;
 };
 
-DEV_INLINE float capped(float x, const Cap c) {
-    return c.top - 2.f * c.top * __builtin_amdgcn_rcpf(
+// `top` is c.top less what the exponent is taken relative to
+DEV_INLINE float capped(float x, const Cap c, float top) {
+    return top - 2.f * c.top * __builtin_amdgcn_rcpf(
         fast_exp2(x * c.rate) + 1.f);
+}
+
+// number of the wave in its block, in a scalar register: what depends on it
+// alone then needs no vector registers, and its branches no masks
+DEV_INLINE int wave_number() {
+    return __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
 }
 
 // 8 coordinates of a key, from coordinate c of its value on
@@ -115,8 +122,8 @@ DEV_INLINE void split_tiles(int p, int chunk, int nsplit, int split, int* t0,
 // Decode. Block: a row and a split of its keys; tiles of 32 keys of all G value
 // heads go through LDS (16-byte pieces XOR-swizzled by the row), the next one
 // in flight. Scores: up to 16 heads of one value head against 16 keys are one
-// item; the weights meet in LDS, and a wave then has
-// all heads' weights against CW columns of one value head.
+// item, and a wave has one or two of the same heads; the weights meet in LDS,
+// and a wave then has all heads' weights against CW columns of one value head.
 //   ws (nsplit > 1): sums [N][nsplit][G][H][P], and behind them the weights'
 //   sums [N][nsplit][H]
 // ===========================================================================
@@ -125,16 +132,20 @@ struct DecodeShape {
     static constexpr int WAVES =
         GP > 8 ? 16 : GP * P / 16 < 8 ? GP * P / 16 : 8;
     static constexpr int CW = GP * P / WAVES;     // columns of a wave
-    static constexpr int QLD = P + 8, PLD = 40;
+    static constexpr int PLD = 40;
     static constexpr int TILE = GP * 32 * P;
     static_assert(P % CW == 0, "a wave has columns of one value head");
-    // elements of LDS: two tiles, queries, weights; then f32 sums
-    static constexpr int ELEMS = 2 * TILE + HB * 16 * (QLD + PLD);
-    static constexpr int BYTES = ELEMS * 2 + HB * 16 * 2 * 4;
+    // LDS in bytes: two tiles and weights; then in f32 sums, 1 / rms of two
+    // tiles and, if it fits, the rotation of one
+    static constexpr int ELEMS = 2 * TILE + HB * 16 * PLD;
+    static constexpr int FIXED = ELEMS * 2 + (HB * 32 + GP * 64) * 4;
+    static constexpr int TABLE = 32 * P * 4;
+    static constexpr bool TAB = FIXED + TABLE <= 160 * 1024;
+    static constexpr int BYTES = FIXED + (TAB ? TABLE : 0);
 };
 
 template <int P, int GP, int HB>
-__global__ void __launch_bounds__((DecodeShape<P, GP, HB>::WAVES * 64), 2)
+__global__ void __launch_bounds__((DecodeShape<P, GP, HB>::WAVES * 64))
 k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
               const bf16_t* __restrict__ vc, const float* __restrict__ inv,
               const int* __restrict__ table, int per_slot,
@@ -144,14 +155,15 @@ k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
               int H, int G, int chunk, int nsplit, const Cap cap) {
     typedef DecodeShape<P, GP, HB> Sh;
     constexpr int WAVES = Sh::WAVES, CW = Sh::CW, CH = P / 8, IT = 2;
-    constexpr int NS = P / 32, NT = CW / 16, QLD = Sh::QLD, PLD = Sh::PLD;
+    constexpr int NS = P / 32, NT = CW / 16, PLD = Sh::PLD;
     constexpr int LOADS = GP * 32 * CH / (WAVES * 64);
     extern __shared__ __attribute__((aligned(16))) bf16_t smem[];
-    bf16_t* const qs = smem + 2 * Sh::TILE;
-    bf16_t* const pb = qs + HB * 16 * QLD;
+    bf16_t* const pb = smem + 2 * Sh::TILE;
     float* const ls = (float*)(smem + Sh::ELEMS);   // [2][HB * 16]
+    float* const ivs = ls + HB * 32;                // [2][GP][32]
+    float* const tabs = ivs + GP * 64;              // cos, sin [32][R / 2]
     const int n = blockIdx.x / nsplit, split = blockIdx.x % nsplit;
-    const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
+    const int lane = threadIdx.x & 63, wv = wave_number();
     const int fr = lane & 15, gq = lane >> 4;
     const int rep = H / G, rbn = (rep + 15) >> 4, items = 2 * G * rbn;
     const int per = (items + WAVES - 1) / WAVES;    // 1 or 2, see IT
@@ -163,8 +175,8 @@ k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
     const int rotated = 2 * rot.half;
 
     auto issue = [&](int t) {
-        const bf16_t* src = vc + (long)tab[t >> 1] * G * PAGE * P +
-                            (t & 1) * 32 * P;
+        const long page = tab[t >> 1];
+        const bf16_t* src = vc + page * G * PAGE * P + (t & 1) * 32 * P;
         bf16_t* dst = smem + (t & 1) * Sh::TILE;
 #pragma unroll
         for (int i = 0; i < LOADS; ++i) {
@@ -175,21 +187,46 @@ k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                                (c ^ (row & 7)) * 8,
                            dst + (i * WAVES + wv) * 512);
         }
+        const int kv = wv * 8 + (lane >> 3);       // 8 value heads a wave
+        if (wv * 8 < GP && kv < G)
+            load_lds16((const bf16_t*)(inv + (page * G + kv) * PAGE +
+                                       (t & 1) * 32 + (lane & 7) * 4),
+                       (bf16_t*)(ivs + (t & 1) * GP * 32 + wv * 256));
     };
-    if (t0 < t1) issue(t0);
-    // queries; where keys are not rotated, the keys' weights go into them
-    for (int i = threadIdx.x; i < HB * 16 * CH; i += WAVES * 64) {
-        const int h = i / CH, c = i % CH * 8;
-        float f[8] = {0, 0, 0, 0, 0, 0, 0, 0}, g[8];
-        if (h < H) {
-            ld8(q + ((long)n * H + h) * P + c, f);
-            if (c >= rotated) {
-                ld8(kw + c, g);
-#pragma unroll
-                for (int j = 0; j < 8; ++j) f[j] *= g[j];
-            }
+    // rotation of a tile's positions; 16-byte pieces swizzled by the row
+    const int pieces = rot.half / 4, twist = pieces % 8 ? 3 : 7;
+    auto issue_rotation = [&](int t) {
+        if (!Sh::TAB) return;
+        for (int i = wv * 64; i < 64 * pieces; i += WAVES * 64) {
+            const int pc = i + lane, row = pc / pieces, c = pc % pieces;
+            const float* src = row < 32 ? rot.cos_ : rot.sin_;
+            load_lds16((const bf16_t*)(
+                           src + (long)(t * 32 + (row & 31)) * rot.half +
+                           (c ^ (row & twist)) * 4),
+                       (bf16_t*)(tabs + i * 4));
         }
-        st8(qs + h * QLD + c, f);
+    };
+    if (t0 < t1) {
+        issue(t0);
+        issue_rotation(t0);
+    }
+    // this wave's scores: up to 16 heads of one value head, 16 or 32 keys.
+    // Where keys are not rotated, their weights go into the queries.
+    const int sg = min(wv * per >> 1, G * rbn - 1), kv = sg / rbn;
+    const int hr = sg % rbn * 16 + fr, h = kv * rep + min(hr, rep - 1);
+    const int mine = min(per, items - wv * per);
+    bf16x8 qf[NS];
+    float kwf[NS][8];
+#pragma unroll
+    for (int s = 0; s < NS; ++s) {
+        const int c = s * 32 + gq * 8;
+        float f[8];
+        ld8(q + ((long)n * H + h) * P + c, f);
+        ld8(kw + c, kwf[s]);
+        if (s * 32 >= rotated)
+#pragma unroll
+            for (int i = 0; i < 8; ++i) f[i] *= kwf[s][i];
+        qf[s] = to_bf16x8(f);
     }
     for (int i = threadIdx.x; i < HB * 16 * PLD / 2; i += WAVES * 64)
         ((u32*)pb)[i] = 0;
@@ -205,21 +242,13 @@ k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
 
     for (int t = t0; t < t1; ++t) {
         const bf16_t* tile = smem + (t & 1) * Sh::TILE;
-        const long page = tab[t >> 1];
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         lds_barrier();              // tile is there, the other one is free
         if (t + 1 < t1) issue(t + 1);
 #pragma unroll
         for (int it = 0; it < IT; ++it) {
-            const int item = wv * per + it;
-            if (it >= per || item >= items) continue;
-            const int sg = item >> 1, kb = item & 1;
-            const int kv = sg / rbn, hr = sg % rbn * 16 + fr;
-            const int h = kv * rep + min(hr, rep - 1);
-            const int row = kb * 16 + fr;
-            const float4 iv = *(const float4*)(
-                inv + (page * G + kv) * PAGE + (t & 1) * 32 + kb * 16 +
-                gq * 4);
+            if (it >= mine) continue;
+            const int kb = (wv * per + it) & 1, row = kb * 16 + fr;
             f32x4 sc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int s = 0; s < NS; ++s) {
@@ -229,18 +258,27 @@ k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                 bf16x8 kf = *(const bf16x8*)src;
                 if (s * 32 < rotated) {
                     float f[8];
-                    key8(f, src, 1.f, kw + c, c, t * 32 + row, rot);
+#pragma unroll
+                    for (int i = 0; i < 8; ++i)
+                        f[i] = (float)kf[i] * kwf[s][i];
+                    if (Sh::TAB) {
+                        const int at = (row * pieces + ((c >> 3) ^
+                                                        (row & twist))) * 4;
+                        rotate_by(f, tabs + at, tabs + 128 * pieces + at);
+                    } else {
+                        rotate8(f, c, t * 32 + row, rot);
+                    }
                     kf = to_bf16x8(f);
                 }
                 sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                    kf, *(const bf16x8*)(qs + h * QLD + c), sc, 0, 0, 0);
+                    kf, qf[s], sc, 0, 0, 0);
             }
-            const float ivr[4] = {iv.x, iv.y, iv.z, iv.w};
-            float e[4];
+            float e[4], iv[4];
+            ld4(ivs + (t & 1) * GP * 32 + kv * 32 + kb * 16 + gq * 4, iv);
             const int key = t * 32 + kb * 16 + gq * 4;
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-                e[r] = fast_exp2(capped(sc[r] * ivr[r], cap) - cap.rho);
+                e[r] = fast_exp2(capped(sc[r] * iv[r], cap, cap.top - cap.rho));
                 if (key + r < lo || key + r > p) e[r] = 0.f;
                 l[it] += e[r];
             }
@@ -249,6 +287,7 @@ k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                     make_uint2(pack2(e[0], e[1]), pack2(e[2], e[3]));
         }
         lds_barrier();              // weights are there
+        if (t + 1 < t1) issue_rotation(t + 1);
         if (vh >= G) continue;
         bf16x8 pf[HB];
 #pragma unroll
@@ -276,14 +315,11 @@ k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
     lds_barrier();                  // ls is cleared, also without a tile
 #pragma unroll
     for (int it = 0; it < IT; ++it) {
-        const int item = wv * per + it;
-        if (it >= per || item >= items) continue;
+        if (it >= mine) continue;
         float s = l[it];
         s += __shfl_xor(s, 16, WAVE);
         s += __shfl_xor(s, 32, WAVE);
-        const int sg = item >> 1, hr = sg % rbn * 16 + fr;
-        if (gq == 0 && hr < rep)
-            ls[(item & 1) * HB * 16 + sg / rbn * rep + hr] = s;
+        if (gq == 0 && hr < rep) ls[(((wv * per + it) & 1)) * HB * 16 + h] = s;
     }
     __syncthreads();
     if (nsplit > 1) {
@@ -339,66 +375,80 @@ k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
 }
 
 // Splits of a row added up, normalised and mixed. Block: a row, a value head,
-// 4 of its output heads. 256 threads: P / 4 columns by 1024 / P score heads.
-template <int P>
+// 32 columns; 256 threads are 32 score heads by 8 x 4 columns. H <= 64.
 __global__ void __launch_bounds__(256)
 k_talk_combine(bf16_t* __restrict__ out, const float* __restrict__ ws,
                const float* __restrict__ talk, const int* __restrict__ pos,
-               int per_slot, int N, int H, int G, int chunk, int nsplit,
-               float rho) {
-    constexpr int CQ = P / 4, GL = 256 / CQ;
-    __shared__ __attribute__((aligned(16))) float red[GL][4][P];
+               int per_slot, int N, int H, int G, int P, int chunk,
+               int nsplit, float rho) {
+    __shared__ __attribute__((aligned(16))) float red[4][4][32];
     __shared__ float nrm[64];
     const int n = blockIdx.x, kv = blockIdx.y, rep = H / G;
-    const int i0 = blockIdx.z * 4, c = (threadIdx.x % CQ) * 4;
-    const int gl = threadIdx.x / CQ;
+    const int c0 = blockIdx.z * 32, tid = threadIdx.x;
+    const int c = c0 + (tid & 7) * 4, g0 = tid >> 3;
     const int p = min(pos[n], per_slot * PAGE - 1);
     int t0, t1, live = 0;              // splits that have keys come first
     for (; live < nsplit; ++live) {
         split_tiles(p, chunk, nsplit, live, &t0, &t1);
         if (t0 >= t1) break;
     }
+    constexpr int U = 8;               // rows in flight
     const float* wl = ws + (long)N * nsplit * G * H * P + (long)n * nsplit * H;
-    if (threadIdx.x < H) {
+    if (tid < H) {
         float l = exp2f(-rho);
-        for (int s = 0; s < live; ++s) l += wl[s * H + threadIdx.x];
-        nrm[threadIdx.x] = 1.f / l;
-    }
-    __syncthreads();
-    float a[4][4] = {};
-    for (int g = gl; g < H; g += GL) {
-        float o[4] = {0.f, 0.f, 0.f, 0.f};
-        for (int s0 = 0; s0 < live; s0 += 4) {    // 4 rows in flight
-            float f[4][4];
+        for (int s0 = 0; s0 < live; s0 += U) {
+            float f[U];
 #pragma unroll
-            for (int s = 0; s < 4; ++s) {
-                const long at = (long)n * nsplit + min(s0 + s, live - 1);
-                ld4(ws + ((at * G + kv) * H + g) * P + c, f[s]);
-            }
+            for (int u = 0; u < U; ++u)
+                f[u] = wl[min(s0 + u, live - 1) * H + tid];
 #pragma unroll
-            for (int s = 0; s < 4; ++s)
-                if (s0 + s < live)
-#pragma unroll
-                    for (int j = 0; j < 4; ++j) o[j] += f[s][j];
+            for (int u = 0; u < U; ++u) l += s0 + u < live ? f[u] : 0.f;
         }
+        nrm[tid] = 1.f / l;
+    }
+    float o[2][4] = {};
 #pragma unroll
-        for (int i = 0; i < 4; ++i)
-            if (i0 + i < rep) {
+    for (int k = 0; k < 2; ++k) {
+        const int g = g0 + k * 32;
+        if (g >= H) break;
+        const float* src = ws + (((long)n * nsplit * G + kv) * H + g) * P + c;
+        for (int s0 = 0; s0 < live; s0 += U) {
+            float f[U][4];
+#pragma unroll
+            for (int u = 0; u < U; ++u)
+                ld4(src + (long)min(s0 + u, live - 1) * G * H * P, f[u]);
+#pragma unroll
+            for (int u = 0; u < U; ++u)
+                if (s0 + u < live)
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) o[k][j] += f[u][j];
+        }
+    }
+    for (int i0 = 0; i0 < rep; i0 += 4) {
+        __syncthreads();               // nrm is there, red is free
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            float a[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int k = 0; k < 2; ++k) {
+                const int g = g0 + k * 32;
+                if (g >= H || i0 + i >= rep) continue;
                 const float x = talk[(kv * rep + i0 + i) * H + g] * nrm[g];
 #pragma unroll
-                for (int j = 0; j < 4; ++j) a[i][j] += x * o[j];
+                for (int j = 0; j < 4; ++j) a[j] += x * o[k][j];
             }
-    }
 #pragma unroll
-    for (int i = 0; i < 4; ++i) st4(&red[gl][i][c], a[i]);
-    __syncthreads();
-    for (int e = threadIdx.x; e < 4 * P; e += 256) {
-        const int i = e / P, d = e % P;
-        if (i0 + i >= rep) continue;
-        float s = 0.f;
+            for (int j = 0; j < 4; ++j)
 #pragma unroll
-        for (int k = 0; k < GL; ++k) s += red[k][i][d];
-        out[((long)n * H + kv * rep + i0 + i) * P + d] = f2bf(s);
+                for (int off = 8; off < 64; off <<= 1)
+                    a[j] += __shfl_xor(a[j], off, WAVE);
+            if ((tid & 63) < 8) st4(&red[tid >> 6][i][(tid & 7) * 4], a);
+        }
+        __syncthreads();
+        const int i = tid >> 5, d = tid & 31;
+        if (i < 4 && i0 + i < rep)
+            out[((long)n * H + kv * rep + i0 + i) * P + c0 + d] =
+                f2bf(red[0][i][d] + red[1][i][d] + red[2][i][d] + red[3][i][d]);
     }
 }
 
@@ -465,58 +515,71 @@ __global__ void __launch_bounds__(256, 2)
 k_talk_lse(float* __restrict__ lse, const bf16_t* __restrict__ q,
            const bf16_t* __restrict__ kx, const int* __restrict__ meta,
            int ntiles, int H, int G, int chunk, const Cap cap) {
-    constexpr int NS = P / 16;
+    constexpr int NS = P / 16, CH = P / 8, LOADS = 32 * CH / 256;
+    __shared__ __attribute__((aligned(16))) bf16_t tile[2][32 * P];
     // neighbouring work (tiles of one head) on the same XCD, longest first
     const int total = ntiles * H, per = (total + 7) >> 3;
     const int i0 = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
     if ((int)(blockIdx.x >> 3) >= per || i0 >= total) return;
     const int h = i0 / ntiles, kv = h / (H / G);
-    const Tile tl(meta + (ntiles - 1 - i0 % ntiles) * 8);
-    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    const Tile tl(meta + (i0 % ntiles) * 8);
+    const int lane = threadIdx.x & 63, wid = wave_number();
     const int hi = lane >> 5, ln = lane & 31;
-    const int qw = tl.q0 + wid * 32;
-    if (qw >= tl.len) return;
-    const int qrow = min(qw + ln, tl.len - 1), qa = tl.start + qrow;
-    const int qlo = first_seen(qa, chunk);
+    const int qw = min(tl.q0 + wid * 32, tl.len - 1);   // (a wave without rows
+    const int qrow = min(qw + ln, tl.len - 1);          // repeats the last)
+    const int qa = tl.start + qrow, qlo = first_seen(qa, chunk);
     const int first = tl.start + qw, last = tl.start + min(qw + 31, tl.len - 1);
     const int all_lo = first_seen(last, chunk);     // seen by every row
-    bf16x8 qf[NS], kf[NS];
+    const int wave_lo = first_seen(first, chunk);
+    bf16x8 qf[NS];
     const bf16_t* qr = q + ((long)(tl.off + qrow) * H + h) * P + hi * 8;
 #pragma unroll
     for (int s = 0; s < NS; ++s) qf[s] = *(const bf16x8*)(qr + s * 16);
-    auto load = [&](int k0) {
-        const bf16_t* kr = kx + ((tl.at(k0) * G + kv) * PAGE + (k0 & 63) + ln)
-                                * P + hi * 8;
+    auto issue = [&](int k0) {
+        const bf16_t* src = kx + ((tl.at(k0) * G + kv) * PAGE + (k0 & 63)) * P;
 #pragma unroll
-        for (int s = 0; s < NS; ++s) kf[s] = *(const bf16x8*)(kr + s * 16);
+        for (int i = 0; i < LOADS; ++i) {
+            const int pc = i * 256 + threadIdx.x;
+            const int row = pc / CH, c = pc % CH;
+            load_lds16(src + row * P + (c ^ (row & 7)) * 8,
+                       tile[(k0 >> 5) & 1] + (i * 256 + wid * 64) * 8);
+        }
     };
-    const int begin = first_seen(first, chunk) & ~31;
+    const int begin = first_seen(tl.start + tl.q0, chunk) & ~31;
+    const int end = tl.start + min(tl.q0 + 127, tl.len - 1);
+    const float top = cap.top - cap.rho;
     float l = 0.f;
-    load(begin);
-    for (int k0 = begin; k0 <= last; k0 += 32) {
+    issue(begin);
+    for (int k0 = begin; k0 <= end; k0 += 32) {
+        const bf16_t* kt = tile[(k0 >> 5) & 1];
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        lds_barrier();              // tile is there, the other one is free
+        if (k0 + 32 <= end) issue(k0 + 32);
+        if (k0 > last || k0 + 31 < wave_lo) continue;
         f32x16 sv;
 #pragma unroll
         for (int r = 0; r < 16; ++r) sv[r] = 0.f;
 #pragma unroll
         for (int s = 0; s < NS; ++s)
-            sv = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf[s], qf[s], sv, 0,
-                                                         0, 0);
-        if (k0 + 32 <= last) load(k0 + 32);
+            sv = __builtin_amdgcn_mfma_f32_32x32x16_bf16(
+                *(const bf16x8*)(kt + ln * P +
+                                 ((s * 2 + hi) ^ (ln & 7)) * 8),
+                qf[s], sv, 0, 0, 0);
         if (k0 >= all_lo && k0 + 31 <= first) {
 #pragma unroll
             for (int r = 0; r < 16; ++r)
-                l += fast_exp2(capped(sv[r], cap) - cap.rho);
+                l += fast_exp2(capped(sv[r], cap, top));
         } else {
 #pragma unroll
             for (int r = 0; r < 16; ++r) {
                 const int key = k0 + (r & 3) + 8 * (r >> 2) + 4 * hi;
-                const float e = fast_exp2(capped(sv[r], cap) - cap.rho);
+                const float e = fast_exp2(capped(sv[r], cap, top));
                 l += key >= qlo && key <= qa ? e : 0.f;
             }
         }
     }
     l += __shfl_xor(l, 32, WAVE);
-    if (hi == 0 && qw + ln < tl.len)
+    if (hi == 0 && tl.q0 + wid * 32 + ln < tl.len)
         lse[(long)(tl.off + qrow) * H + h] =
             cap.rho + log2f(exp2f(-cap.rho) + l);
 }
@@ -525,13 +588,15 @@ k_talk_lse(float* __restrict__ lse, const bf16_t* __restrict__ q,
 // Mixed weights times values. Block: 16 rows of a portion, all heads; wave w
 // has heads w * NH .. + NH - 1, which are numbered w * 4 + 0 .. NH - 1 where
 // heads are a matrix dimension. Per 32 keys: a wave makes its heads' weights
-// (f16, times 2^14) and leaves them in LDS; one MFMA mixes 16 pairs of row and
-// key for 16 output heads; each wave applies its heads' mixed weights.
+// (f16, times 2^14) and leaves them in LDS; one MFMA mixes 16 keys of a row for
+// 16 output heads; each wave applies its heads' mixed weights. The three steps
+// work on three successive tiles between two barriers.
 //   talk: f16 [32][32] in that numbering; fin: factor of the result
+//   SAME: the heads of a wave share a value head
 // ===========================================================================
 #define LIFT 14.f
 
-template <int P, int NH>
+template <int P, int NH, bool SAME>
 __global__ void __launch_bounds__(512, 2)
 k_talk_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                const bf16_t* __restrict__ kx, const bf16_t* __restrict__ vx,
@@ -539,13 +604,14 @@ k_talk_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                const int* __restrict__ meta, int H, int G, int chunk,
                const Cap cap, float fin) {
     constexpr int NS = P / 32, NT = P / 16;
-    constexpr int LDR = 40;                   // a row of 32, padded
-    constexpr int QS = 32 * LDR + 8, HS = 16 * LDR + 8;
-    __shared__ __attribute__((aligned(16))) _Float16 pb[16 * QS];
-    __shared__ __attribute__((aligned(16))) bf16_t wb[32 * HS];
+    // a row of 32, and 32 or 16 such rows, padded against bank conflicts
+    constexpr int LDR = 36, QS = 32 * LDR + 4, HS = 16 * LDR + 4;
+    __shared__ __attribute__((aligned(16))) _Float16 pb[2][16 * QS];
+    __shared__ __attribute__((aligned(16))) bf16_t wb[2][32 * HS];
+    __shared__ __attribute__((aligned(16))) _Float16 tb[2 * 512];
     const Tile tl(meta + (long)blockIdx.x * 8);
     if (tl.len <= tl.q0) return;              // the same for the block
-    const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
+    const int lane = threadIdx.x & 63, wv = wave_number();
     const int fr = lane & 15, gq = lane >> 4, rep = H / G;
     const int nq = min(16, tl.len - tl.q0);
     const int row = tl.off + tl.q0 + min(fr, nq - 1);
@@ -553,7 +619,6 @@ k_talk_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
     const int qa = first + min(fr, nq - 1), qlo = first_seen(qa, chunk);
     const int all_lo = first_seen(last, chunk);
     const int h0 = wv * NH;
-    const int mine = max(0, min(NH, H - h0));
     const bool two = (H + NH - 1) / NH > 4;   // numbers above 16 occur
 
     bf16x8 qf[NH][NS], kf[2][NS], vf[NT];
@@ -562,26 +627,23 @@ k_talk_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
 #pragma unroll
     for (int i = 0; i < NH; ++i) {
         const int h = min(h0 + i, H - 1);
-        ls[i] = lse[(long)row * H + h] - LIFT;
+        ls[i] = cap.top - lse[(long)row * H + h] + LIFT;
         const bf16_t* qr = q + ((long)row * H + h) * P + gq * 8;
 #pragma unroll
         for (int s = 0; s < NS; ++s) qf[i][s] = *(const bf16x8*)(qr + s * 32);
 #pragma unroll
         for (int t = 0; t < NT; ++t) acc[i][t] = (f32x4){0.f, 0.f, 0.f, 0.f};
     }
-    f16x8 tf[2];
-#pragma unroll
-    for (int b = 0; b < 2; ++b)
-        tf[b] = *(const f16x8*)(talk + (b * 16 + fr) * 32 + gq * 8);
+    for (int i = threadIdx.x; i < 512; i += 512)   // in MFMA operand order
+        ((u32*)tb)[i] = ((const u32*)talk)[(i >> 8) * 256 + (i & 3) +
+                                           (i >> 2 & 15) * 16 +
+                                           (i >> 6 & 3) * 4];
 
-    auto load_k = [&](int kv, int k0) {
-        const bf16_t* kr = kx + ((tl.at(k0) * G + kv) * PAGE + (k0 & 63) + fr)
-                                * P + gq * 8;
+    auto load_k = [&](int kv, int k0, int b) {        // 16 keys
+        const bf16_t* kr = kx + ((tl.at(k0) * G + kv) * PAGE + (k0 & 63) +
+                                 b * 16 + fr) * P + gq * 8;
 #pragma unroll
-        for (int b = 0; b < 2; ++b)
-#pragma unroll
-            for (int s = 0; s < NS; ++s)
-                kf[b][s] = *(const bf16x8*)(kr + b * 16 * P + s * 32);
+        for (int s = 0; s < NS; ++s) kf[b][s] = *(const bf16x8*)(kr + s * 32);
     };
     auto load_v = [&](int kv, int k0) {
         const bf16_t* vr = vx + ((tl.at(k0) * G + kv) * P + fr) * PAGE +
@@ -591,99 +653,116 @@ k_talk_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
             vf[t] = *(const bf16x8*)(vr + t * 16 * PAGE);
     };
     const int begin = first_seen(first, chunk) & ~31;
-    const int kv0 = min(h0, H - 1) / rep;
-    int have = kv0;
-    if (mine) {
-        load_k(kv0, begin);
-    } else {                                  // numbers without a head
+    // value head of a wave's head (the last head stands in for missing ones:
+    // their column of talk is zero, and nobody stores their result)
+    auto value_head = [&](int i) { return min(h0 + i, H - 1) / rep; };
+    auto other = [&](int i) {                 // not the head's before
+        return !SAME && (i == 0 || value_head(i) != value_head(i - 1));
+    };
+    const int kv0 = value_head(0), now0 = (begin >> 5) & 1;
+    for (int i = threadIdx.x; i < 8 * QS; i += 512) ((u32*)pb[now0 ^ 1])[i] = 0;
+    for (int i = threadIdx.x; i < 16 * HS; i += 512) ((u32*)wb[now0])[i] = 0;
+    if (SAME) load_v(kv0, begin);
+    lds_barrier();
+    // Tile k0: weights; tile k0 - 32: mixing; tile k0 - 64: values. Where there
+    // is no such tile the weights are zero. Keys take over the registers of
+    // the values.
+    const int tail = last & ~31;
+    for (int k0 = begin; k0 <= tail + 64; k0 += 32) {
+        const int now = (k0 >> 5) & 1, kt = min(k0, tail);
+        bf16x8 w[NH];
 #pragma unroll
-        for (int j = 0; j < 8; ++j)
-            *(uint2*)(pb + fr * QS +
-                      ((j >> 2) * 16 + gq * 4 + (j & 3)) * LDR + wv * 4) =
-                make_uint2(0, 0);
-    }
-    for (int k0 = begin; k0 <= last; k0 += 32) {
-        const bool whole = k0 >= all_lo && k0 + 31 <= first;
-        if (mine) {
-            _Float16 ph[8][4];
+        for (int i = 0; i < NH; ++i) {
+            const bf16_t* wr =
+                wb[now] + (wv * 4 + i) * HS + fr * LDR + gq * 8;
+            w[i] = __builtin_shufflevector(
+                *(const bf16x4*)wr, *(const bf16x4*)(wr + 4), 0, 1, 2, 3, 4, 5,
+                6, 7);
+        }
+        if (SAME) {
 #pragma unroll
-            for (int j = 0; j < 8; ++j)
+            for (int b = 0; b < 2; ++b) {
 #pragma unroll
-                for (int i = NH; i < 4; ++i) ph[j][i] = (_Float16)0.f;
+                for (int t = b * NT / 2; t < (b + 1) * NT / 2; ++t)
+#pragma unroll
+                    for (int i = 0; i < NH; ++i)
+                        acc[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                            vf[t], w[i], acc[i][t], 0, 0, 0);
+                load_k(kv0, kt, b);
+            }
+        } else {
 #pragma unroll
             for (int i = 0; i < NH; ++i) {
-                if (i < mine) {
-                    const int kv = (h0 + i) / rep;
-                    if (kv != have) load_k(have = kv, k0);
-                    f32x4 sc[2];
+                if (other(i)) load_v(value_head(i), max(k0 - 64, begin));
 #pragma unroll
-                    for (int b = 0; b < 2; ++b) {
-                        sc[b] = (f32x4){0.f, 0.f, 0.f, 0.f};
+                for (int t = 0; t < NT; ++t)
+                    acc[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                        vf[t], w[i], acc[i][t], 0, 0, 0);
+            }
+        }
+        const bool whole = k0 >= all_lo && k0 + 31 <= first;
+        u32 pw[8][2];                         // heads 0 | 1 and 2 | 3
 #pragma unroll
-                        for (int s = 0; s < NS; ++s)
-                            sc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                                kf[b][s], qf[i][s], sc[b], 0, 0, 0);
-                    }
+        for (int j = 0; j < 8; ++j) pw[j][0] = pw[j][1] = 0;
 #pragma unroll
-                    for (int j = 0; j < 8; ++j) {
-                        float e = fast_exp2(capped(sc[j >> 2][j & 3], cap) -
-                                            ls[i]);
-                        if (!whole) {
-                            const int key = k0 + (j >> 2) * 16 + gq * 4 +
-                                            (j & 3);
-                            if (key < qlo || key > qa) e = 0.f;
-                        }
-                        ph[j][i] = (_Float16)e;
-                    }
-                } else {
+        for (int i = 0; i < NH; ++i) {
+            if (other(i)) {
+                load_k(value_head(i), kt, 0);
+                load_k(value_head(i), kt, 1);
+            }
+            f32x4 sc[2];
 #pragma unroll
-                    for (int j = 0; j < 8; ++j) ph[j][i] = (_Float16)0.f;
-                }
+            for (int b = 0; b < 2; ++b) {
+                sc[b] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int s = 0; s < NS; ++s)
+                    sc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                        kf[b][s], qf[i][s], sc[b], 0, 0, 0);
             }
 #pragma unroll
-            for (int j = 0; j < 8; ++j)
-                *(f16x4*)(pb + fr * QS +
-                          ((j >> 2) * 16 + gq * 4 + (j & 3)) * LDR + wv * 4) =
-                    (f16x4){ph[j][0], ph[j][1], ph[j][2], ph[j][3]};
-            // for the second half of this tile, and for the next tile
-            load_v(kv0, k0);
-            if (k0 + 32 <= last) load_k(have = kv0, k0 + 32);
+            for (int j = 0; j < 8; ++j) {
+                float e =
+                    fast_exp2(capped(sc[j >> 2][j & 3], cap, ls[i]));
+                if (!whole) {
+                    const int key = k0 + (j >> 2) * 16 + gq * 4 + (j & 3);
+                    if (key < qlo || key > qa) e = 0.f;
+                }
+                const u32 x = __builtin_bit_cast(unsigned short, (_Float16)e);
+                pw[j][i >> 1] |= i & 1 ? x << 16 : x;
+            }
         }
-        lds_barrier();
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+            *(uint2*)(pb[now] + fr * QS +
+                      ((j >> 2) * 16 + gq * 4 + (j & 3)) * LDR + wv * 4) =
+                make_uint2(pw[j][0], pw[j][1]);
+        if (SAME)                             // for the next turn
+            load_v(kv0, min(max(k0 - 32, begin), tail));
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int qi = wv * 2 + (j >> 1), kb = (j & 1) * 16;
-            const f16x8 a =
-                *(const f16x8*)(pb + qi * QS + (kb + fr) * LDR + gq * 8);
+            const _Float16* ar =
+                pb[now ^ 1] + qi * QS + (kb + fr) * LDR + gq * 8;
+            const f16x8 a = __builtin_shufflevector(
+                *(const f16x4*)ar, *(const f16x4*)(ar + 4), 0, 1, 2, 3, 4, 5,
+                6, 7);
 #pragma unroll
             for (int b = 0; b < 2; ++b)
                 if (b == 0 || two) {
                     const f32x4 c = __builtin_amdgcn_mfma_f32_16x16x32_f16(
-                        a, tf[b], (f32x4){0.f, 0.f, 0.f, 0.f}, 0, 0, 0);
-                    *(uint2*)(wb + (b * 16 + fr) * HS + qi * LDR + kb +
-                              gq * 4) =
+                        a, *(const f16x8*)(tb + b * 512 + lane * 8),
+                        (f32x4){0.f, 0.f, 0.f, 0.f}, 0, 0, 0);
+                    *(uint2*)(wb[now ^ 1] + (b * 16 + fr) * HS + qi * LDR +
+                              kb + gq * 4) =
                         make_uint2(pack2(c[0], c[1]), pack2(c[2], c[3]));
                 }
         }
         lds_barrier();
-        int vh = kv0;
-#pragma unroll
-        for (int i = 0; i < NH; ++i)
-            if (i < mine) {
-                const int kv = (h0 + i) / rep;
-                if (kv != vh) load_v(vh = kv, k0);
-                const bf16x8 w = *(const bf16x8*)(
-                    wb + (wv * 4 + i) * HS + fr * LDR + gq * 8);
-#pragma unroll
-                for (int t = 0; t < NT; ++t)
-                    acc[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                        vf[t], w, acc[i][t], 0, 0, 0);
-            }
     }
     if (fr >= nq) return;
 #pragma unroll
     for (int i = 0; i < NH; ++i)
-        if (i < mine) {
+        if (h0 + i < H) {
             bf16_t* o = out + ((long)row * H + h0 + i) * P + gq * 4;
 #pragma unroll
             for (int t = 0; t < NT; ++t)
@@ -836,8 +915,8 @@ static int go_decode(hipStream_t st, bf16_t* out, const bf16_t* q,
         G, chunk, nsplit, cap);
     LAUNCH_CHECK();
     if (nsplit > 1) {
-        k_talk_combine<P><<<dim3(N, G, (H / G + 3) / 4), 256, 0, st>>>(
-            out, ws, talk, pos, per_slot, N, H, G, chunk, nsplit, cap.rho);
+        k_talk_combine<<<dim3(N, G, P / 32), 256, 0, st>>>(
+            out, ws, talk, pos, per_slot, N, H, G, P, chunk, nsplit, cap.rho);
         LAUNCH_CHECK();
     }
     return 0;
@@ -873,6 +952,7 @@ int gt_talk_decode(void* stream, void* out, const void* q, const void* vc,
                    float rho) {
     if (N < 1 || !sizes_ok(H, G, P, R, nrot, chunk) || nsplit < 1 ||
         nsplit > 64 || H > 64 || G * P > 1024 || R % 32 ||
+        nrot < per_slot * PAGE ||
         (nsplit > 1 && !ws)) return -100;
     const Rotation rot = rotation(cos_, sin_, R, nrot);
     const Cap cap{rate, top, rho};
@@ -936,11 +1016,13 @@ int gt_talk_prefill(void* stream, void* out, const void* q, const void* kx,
     const int nh = (H + 7) / 8;
     if (ntiles < 1 || !sizes_ok(H, G, P, 0, 1, chunk) || nh > 4 ||
         nh * P > 512) return -100;
-#define GO(A, B) k_talk_prefill<A, B><<<ntiles, 512, 0, \
+#define GO1(A, B, C) k_talk_prefill<A, B, C><<<ntiles, 512, 0, \
         (hipStream_t)stream>>>((bf16_t*)out, (const bf16_t*)q, \
         (const bf16_t*)kx, (const bf16_t*)vx, (const float*)lse, \
         (const _Float16*)talk, (const int*)meta, H, G, chunk, \
         Cap{rate, top, rho}, fin)
+#define GO(A, B) do { if (H / G % B == 0) GO1(A, B, true); \
+        else GO1(A, B, false); } while (0)
 #define PICK(A) do { if (nh == 1) GO(A, 1); else if (nh == 2) GO(A, 2); \
         else if (nh == 3) GO(A, 3); else GO(A, 4); } while (0)
     if (P == 64) PICK(64);
@@ -949,6 +1031,7 @@ int gt_talk_prefill(void* stream, void* out, const void* q, const void* kx,
     else GO(256, 2);
 #undef PICK
 #undef GO
+#undef GO1
     LAUNCH_CHECK();
     return 0;
 }

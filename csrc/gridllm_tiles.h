@@ -20,19 +20,23 @@ struct Rotation {
     int half, rows;
 };
 
-// Rotate the neighbouring pairs of 8 coordinates, the first of which is
-// coordinate c of the rotated part.
-DEV_INLINE void rotate8(float* f, int c, int p, const Rotation rot) {
-    const long at = (long)min(p, rot.rows - 1) * rot.half + c / 2;
+// Rotate the neighbouring pairs of 8 coordinates by 4 cosines and sines.
+DEV_INLINE void rotate_by(float* f, const float* cos_, const float* sin_) {
     float co[4], si[4];
-    ld4(rot.cos_ + at, co);
-    ld4(rot.sin_ + at, si);
+    ld4(cos_, co);
+    ld4(sin_, si);
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
         const float u = f[2 * i], v = f[2 * i + 1];
         f[2 * i] = u * co[i] - v * si[i];
         f[2 * i + 1] = v * co[i] + u * si[i];
     }
+}
+
+// The same by the tables; the first is coordinate c of the rotated part.
+DEV_INLINE void rotate8(float* f, int c, int p, const Rotation rot) {
+    const long at = (long)min(p, rot.rows - 1) * rot.half + c / 2;
+    rotate_by(f, rot.cos_ + at, rot.sin_ + at);
 }
 
 DEV_INLINE bf16x8 to_bf16x8(const float* f) {

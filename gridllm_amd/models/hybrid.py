@@ -154,8 +154,9 @@ class HybridModel:
 
     def _rotations(self) -> list[Optional[tuple]]:
         """Per latent- or talking-heads-attention layer, cos and sin of position
-        times frequency, f32 [max_seq, R / 2]; 1 and 0 for pairs that are not
-        rotated."""
+        times frequency, f32 [rows, R / 2] for the positions of whole pages; 1
+        and 0 for pairs that are not rotated."""
+        rows = pad64(self.max_seq)
         made: dict[tuple, tuple] = {}
 
         def table(mx) -> tuple:
@@ -166,9 +167,9 @@ class HybridModel:
                 half = mx.rot_dims // 2
                 f = mx.rot_base ** (-torch.arange(half, dtype=torch.float64)
                                     / max(half, 1))
-                a = torch.zeros(self.max_seq, r // 2, dtype=torch.float64)
+                a = torch.zeros(rows, r // 2, dtype=torch.float64)
                 a[:, :half] = torch.outer(
-                    torch.arange(self.max_seq, dtype=torch.float64), f)
+                    torch.arange(rows, dtype=torch.float64), f)
                 made[key] = tuple(t.float().to(self.device).contiguous()
                                   for t in (a.cos(), a.sin()))
             return made[key]
@@ -776,10 +777,12 @@ class HybridModel:
             pages += len(have)
         if not pages:
             return 0, [], [], []
-        t16, t128 = (np.concatenate(t) for t in tiles.values())
-        # the kernel's blocks start in this order: long spans of keys first
-        span = (t16[:, 3] + t16[:, 4]) % chunk
-        t16 = t16[np.argsort(-span, kind="stable")]
+
+        def ordered(t):             # blocks start in this order
+            span = (t[:, 3] + t[:, 4]) % chunk
+            return t[np.argsort(-span, kind="stable")]
+
+        t16, t128 = (ordered(np.concatenate(t)) for t in tiles.values())
         return pages, np.concatenate(items), t16, t128
 
     def _upload_ints(self, parts: list) -> list[torch.Tensor]:

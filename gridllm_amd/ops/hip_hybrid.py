@@ -518,9 +518,10 @@ def _talk_sizes(tk: Talk, g: int, p: int) -> tuple[bool, bool]:
     return one, one and nh <= 4 and nh * p <= 512
 
 
-def talk_tiled(tk: Talk, g: int, p: int) -> bool:
-    """Whether prompt portions of this mixer run the tiled kernels."""
-    return _talk_sizes(tk, g, p)[1]
+def _talk_splits(rows: int, heads: int, seen: int) -> int:
+    """Into how many parts a decode row's keys are split. (A part's sums are as
+    large as the values of 2 * heads keys.)"""
+    return max(1, min(256 // rows, -(-seen // max(128, 8 * heads)), 32))
 
 
 def talk_attn(q: torch.Tensor, vc: torch.Tensor, inv: torch.Tensor,
@@ -544,9 +545,7 @@ def talk_attn(q: torch.Tensor, vc: torch.Tensor, inv: torch.Tensor,
     portions = st.talk.get(tk.chunk) if tiled else None
     na = n if portions is None else st.absorbed
     if na:
-        # a split's sums are as large as the values of 2 H keys
-        seen = min(st.max_len, tk.chunk)
-        nsplit = max(1, min(256 // na, -(-seen // max(128, 8 * h)), 32))
+        nsplit = _talk_splits(na, h, min(st.max_len, tk.chunk))
         ws = torch.empty(na * nsplit * (g * h * p + h), dtype=torch.float32,
                          device=dev) if nsplit > 1 else None
         _call("gt_talk_decode", out, q, vc, inv, st.table, per, st.pos,

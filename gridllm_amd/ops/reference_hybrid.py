@@ -19,9 +19,8 @@ class ChunkPortions:
     chunk size. The keys that they see are laid out in `pages` pages:
     items    [*, 4] {page number, slot, page to write, rows} per page
     tiles16  [*, 8] {first token, length, first page, first row, start, page
-             number of that page} per 16 rows of a portion, longest spans
-             first, and
-    tiles128 per 128 rows
+             number of that page} per 16 rows of a portion, and
+    tiles128 per 128 rows; long spans of keys first
     """
     pages: int
     items: torch.Tensor
