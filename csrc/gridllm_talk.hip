@@ -25,6 +25,8 @@
 
 #include "gridllm_tiles.h"
 
+#include <type_traits>
+
 typedef __attribute__((ext_vector_type(8))) _Float16 f16x8;
 typedef __attribute__((ext_vector_type(4))) _Float16 f16x4;
 
@@ -106,6 +108,12 @@ k_talk_rows(const T* __restrict__ rows, T* __restrict__ q,
     if (c == 0) inv[at] = rs;
 }
 
+// the value of the lane 8 further on, in rounds of 16
+DEV_INLINE float from_8_lanes_on(float x) {
+    return __uint_as_float(__builtin_amdgcn_update_dpp(
+        0, __float_as_uint(x), 0x128 /* row_ror:8 */, 0xf, 0xf, true));
+}
+
 // keys a query at position p sees: from here on, up to p
 DEV_INLINE int first_seen(int p, int chunk) { return p / chunk * chunk; }
 
@@ -127,7 +135,7 @@ DEV_INLINE void split_tiles(int p, int chunk, int nsplit, int split, int* t0,
 //   ws (nsplit > 1): sums [N][nsplit][G][H][P], and behind them the weights'
 //   sums [N][nsplit][H]
 // ===========================================================================
-template <int P, int GP, int HB>
+template <int P, int GP, int HB, int R>
 struct DecodeShape {
     static constexpr int WAVES =
         GP > 8 ? 16 : GP * P / 16 < 8 ? GP * P / 16 : 8;
@@ -139,13 +147,13 @@ struct DecodeShape {
     // tiles and, if it fits, the rotation of one
     static constexpr int ELEMS = 2 * TILE + HB * 16 * PLD;
     static constexpr int FIXED = ELEMS * 2 + (HB * 32 + GP * 64) * 4;
-    static constexpr int TABLE = 32 * P * 4;
+    static constexpr int TABLE = 32 * R * 4;
     static constexpr bool TAB = FIXED + TABLE <= 160 * 1024;
     static constexpr int BYTES = FIXED + (TAB ? TABLE : 0);
 };
 
-template <int P, int GP, int HB>
-__global__ void __launch_bounds__((DecodeShape<P, GP, HB>::WAVES * 64))
+template <int P, int GP, int HB, int R>
+__global__ void __launch_bounds__((DecodeShape<P, GP, HB, R>::WAVES * 64))
 k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
               const bf16_t* __restrict__ vc, const float* __restrict__ inv,
               const int* __restrict__ table, int per_slot,
@@ -153,9 +161,9 @@ k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
               float* __restrict__ ws, const float* __restrict__ kw,
               const float* __restrict__ talk, const Rotation rot, int N,
               int H, int G, int chunk, int nsplit, const Cap cap) {
-    typedef DecodeShape<P, GP, HB> Sh;
-    constexpr int WAVES = Sh::WAVES, CW = Sh::CW, CH = P / 8, IT = 2;
-    constexpr int NS = P / 32, NT = CW / 16, PLD = Sh::PLD;
+    typedef DecodeShape<P, GP, HB, R> Sh;
+    constexpr int WAVES = Sh::WAVES, CW = Sh::CW, CH = P / 8;
+    constexpr int NS = P / 32, RS = R / 32, NT = CW / 16, PLD = Sh::PLD;
     constexpr int LOADS = GP * 32 * CH / (WAVES * 64);
     extern __shared__ __attribute__((aligned(16))) bf16_t smem[];
     bf16_t* const pb = smem + 2 * Sh::TILE;
@@ -166,16 +174,14 @@ k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
     const int lane = threadIdx.x & 63, wv = wave_number();
     const int fr = lane & 15, gq = lane >> 4;
     const int rep = H / G, rbn = (rep + 15) >> 4, items = 2 * G * rbn;
-    const int per = (items + WAVES - 1) / WAVES;    // 1 or 2, see IT
+    const int per = (items + WAVES - 1) / WAVES;    // 1 or 2
     const int p = min(pos[n], per_slot * PAGE - 1);
     const int lo = first_seen(p, chunk);
     int t0, t1;
     split_tiles(p, chunk, nsplit, split, &t0, &t1);
     const int* tab = table + (long)slot[n] * per_slot;
-    const int rotated = 2 * rot.half;
 
-    auto issue = [&](int t) {
-        const long page = tab[t >> 1];
+    auto issue = [&](int t, long page) {
         const bf16_t* src = vc + page * G * PAGE * P + (t & 1) * 32 * P;
         bf16_t* dst = smem + (t & 1) * Sh::TILE;
 #pragma unroll
@@ -194,46 +200,52 @@ k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                        (bf16_t*)(ivs + (t & 1) * GP * 32 + wv * 256));
     };
     // rotation of a tile's positions; 16-byte pieces swizzled by the row
-    const int pieces = rot.half / 4, twist = pieces % 8 ? 3 : 7;
+    constexpr int PIECES = R / 8, TWIST = PIECES % 8 ? 3 : 7;
     auto issue_rotation = [&](int t) {
         if (!Sh::TAB) return;
-        for (int i = wv * 64; i < 64 * pieces; i += WAVES * 64) {
-            const int pc = i + lane, row = pc / pieces, c = pc % pieces;
+#pragma unroll
+        for (int i = 0; i < (PIECES + WAVES - 1) / WAVES; ++i) {
+            const int w = i * WAVES + wv, pc = w * 64 + lane;
+            const int row = pc / PIECES, c = pc % PIECES;
             const float* src = row < 32 ? rot.cos_ : rot.sin_;
-            load_lds16((const bf16_t*)(
-                           src + (long)(t * 32 + (row & 31)) * rot.half +
-                           (c ^ (row & twist)) * 4),
-                       (bf16_t*)(tabs + i * 4));
+            if (w < PIECES)
+                load_lds16((const bf16_t*)(
+                               src + (long)(t * 32 + (row & 31)) * (R / 2) +
+                               (c ^ (row & TWIST)) * 4),
+                           (bf16_t*)(tabs + w * 256));
         }
     };
+    int page = tab[min(t0, t1 - 1) >> 1];
     if (t0 < t1) {
-        issue(t0);
+        issue(t0, page);
         issue_rotation(t0);
+        page = tab[min(t0 + 1, t1 - 1) >> 1];
     }
     // this wave's scores: up to 16 heads of one value head, 16 or 32 keys.
-    // Where keys are not rotated, their weights go into the queries.
+    // Behind the rotated part the keys' weights go into the queries.
     const int sg = min(wv * per >> 1, G * rbn - 1), kv = sg / rbn;
     const int hr = sg % rbn * 16 + fr, h = kv * rep + min(hr, rep - 1);
     const int mine = min(per, items - wv * per);
     bf16x8 qf[NS];
-    float kwf[NS][8];
+    float kwf[RS][8];
 #pragma unroll
     for (int s = 0; s < NS; ++s) {
         const int c = s * 32 + gq * 8;
-        float f[8];
+        float f[8], g[8];
         ld8(q + ((long)n * H + h) * P + c, f);
-        ld8(kw + c, kwf[s]);
-        if (s * 32 >= rotated)
+        ld8(kw + c, g);
 #pragma unroll
-            for (int i = 0; i < 8; ++i) f[i] *= kwf[s][i];
+        for (int i = 0; i < 8; ++i)
+            if (s < RS) kwf[s][i] = g[i]; else f[i] *= g[i];
         qf[s] = to_bf16x8(f);
     }
+    const bool few = rep <= 8;
     for (int i = threadIdx.x; i < HB * 16 * PLD / 2; i += WAVES * 64)
         ((u32*)pb)[i] = 0;
     if (threadIdx.x < HB * 32) ls[threadIdx.x] = 0.f;
 
     const int vh = wv * CW / P, part = wv * CW % P;   // value head, column
-    float l[IT] = {};
+    float l[2] = {0.f, 0.f};
     f32x4 acc[HB][NT];
 #pragma unroll
     for (int b = 0; b < HB; ++b)
@@ -244,47 +256,71 @@ k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
         const bf16_t* tile = smem + (t & 1) * Sh::TILE;
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         lds_barrier();              // tile is there, the other one is free
-        if (t + 1 < t1) issue(t + 1);
-#pragma unroll
-        for (int it = 0; it < IT; ++it) {
-            if (it >= mine) continue;
-            const int kb = (wv * per + it) & 1, row = kb * 16 + fr;
+        if (t + 1 < t1) issue(t + 1, page);
+        page = tab[min(t + 2, t1 - 1) >> 1];
+        // raw scores of 16 keys
+        auto score = [&](int kb) {
+            const int row = kb * 16 + fr;
             f32x4 sc = {0.f, 0.f, 0.f, 0.f};
+            bf16x8 kf[NS];
 #pragma unroll
-            for (int s = 0; s < NS; ++s) {
+            for (int s = 0; s < NS; ++s)
+                kf[s] = *(const bf16x8*)(tile + (kv * 32 + row) * P +
+                                         ((s * 4 + gq) ^ (row & 7)) * 8);
+#pragma unroll
+            for (int s = 0; s < RS; ++s) {
                 const int c = s * 32 + gq * 8;
-                const bf16_t* src = tile + (kv * 32 + row) * P +
-                                    ((c >> 3) ^ (row & 7)) * 8;
-                bf16x8 kf = *(const bf16x8*)src;
-                if (s * 32 < rotated) {
-                    float f[8];
+                float f[8];
 #pragma unroll
-                    for (int i = 0; i < 8; ++i)
-                        f[i] = (float)kf[i] * kwf[s][i];
-                    if (Sh::TAB) {
-                        const int at = (row * pieces + ((c >> 3) ^
-                                                        (row & twist))) * 4;
-                        rotate_by(f, tabs + at, tabs + 128 * pieces + at);
-                    } else {
-                        rotate8(f, c, t * 32 + row, rot);
-                    }
-                    kf = to_bf16x8(f);
+                for (int i = 0; i < 8; ++i)
+                    f[i] = (float)kf[s][i] * kwf[s][i];
+                if (Sh::TAB) {
+                    const int at = (row * PIECES + ((s * 4 + gq) ^
+                                                    (row & TWIST))) * 4;
+                    rotate_by(f, tabs + at, tabs + 128 * PIECES + at);
+                } else {
+                    rotate8(f, c, t * 32 + row, rot);
                 }
-                sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                    kf, qf[s], sc, 0, 0, 0);
+                kf[s] = to_bf16x8(f);
             }
+#pragma unroll
+            for (int s = 0; s < NS; ++s)
+                sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[s], qf[s], sc,
+                                                             0, 0, 0);
+            return sc;
+        };
+        // weights of head hk from its scores against 16 keys
+        auto weigh = [&](f32x4 sc, int kb, int hk, float* sum) {
             float e[4], iv[4];
-            ld4(ivs + (t & 1) * GP * 32 + kv * 32 + kb * 16 + gq * 4, iv);
             const int key = t * 32 + kb * 16 + gq * 4;
+            ld4(ivs + (t & 1) * GP * 32 + kv * 32 + kb * 16 + gq * 4, iv);
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-                e[r] = fast_exp2(capped(sc[r] * iv[r], cap, cap.top - cap.rho));
-                if (key + r < lo || key + r > p) e[r] = 0.f;
-                l[it] += e[r];
+                e[r] = fast_exp2(capped(sc[r] * iv[r], cap,
+                                        cap.top - cap.rho));
+                e[r] = (u32)(key + r - lo) <= (u32)(p - lo) ? e[r] : 0.f;
+                *sum += e[r];
             }
-            if (hr < rep)
-                *(uint2*)(pb + h * PLD + kb * 16 + gq * 4) =
+            if (hk < rep)
+                *(uint2*)(pb + (kv * rep + hk) * PLD + kb * 16 + gq * 4) =
                     make_uint2(pack2(e[0], e[1]), pack2(e[2], e[3]));
+        };
+        if (mine == 2) {
+            f32x4 a = score(0);
+            const f32x4 b = score(1);
+            if (few) {            // the second 16 keys into idle lanes
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const float x = from_8_lanes_on(b[r]);
+                    a[r] = fr < 8 ? a[r] : x;
+                }
+                weigh(a, fr >> 3, fr & 7, l);
+            } else {
+                weigh(a, 0, hr, l);
+                weigh(b, 1, hr, l + 1);
+            }
+        } else if (mine == 1) {
+            weigh(score(wv & 1), wv & 1, hr, l);
         }
         lds_barrier();              // weights are there
         if (t + 1 < t1) issue_rotation(t + 1);
@@ -313,13 +349,18 @@ k_talk_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
         }
     }
     lds_barrier();                  // ls is cleared, also without a tile
+    if (mine > 0) {
+        float s[2] = {l[0], l[1]};
 #pragma unroll
-    for (int it = 0; it < IT; ++it) {
-        if (it >= mine) continue;
-        float s = l[it];
-        s += __shfl_xor(s, 16, WAVE);
-        s += __shfl_xor(s, 32, WAVE);
-        if (gq == 0 && hr < rep) ls[(((wv * per + it) & 1)) * HB * 16 + h] = s;
+        for (int i = 0; i < 2; ++i) {
+            s[i] += __shfl_xor(s[i], 16, WAVE);
+            s[i] += __shfl_xor(s[i], 32, WAVE);
+        }
+        if (few && mine == 2) s[1] = from_8_lanes_on(s[0]);
+        if (gq == 0 && hr < rep) {
+            ls[(mine == 1 ? wv & 1 : 0) * HB * 16 + h] = s[0];
+            if (mine == 2) ls[HB * 16 + h] = s[1];
+        }
     }
     __syncthreads();
     if (nsplit > 1) {
@@ -700,37 +741,41 @@ k_talk_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                         vf[t], w[i], acc[i][t], 0, 0, 0);
             }
         }
-        const bool whole = k0 >= all_lo && k0 + 31 <= first;
-        u32 pw[8][2];                         // heads 0 | 1 and 2 | 3
+        u32 pw[8][2] = {};                    // heads 0 | 1 and 2 | 3
+        const int base = k0 + gq * 4 - qlo;   // from the first key seen
+        auto weights = [&](auto whole) {
 #pragma unroll
-        for (int j = 0; j < 8; ++j) pw[j][0] = pw[j][1] = 0;
-#pragma unroll
-        for (int i = 0; i < NH; ++i) {
-            if (other(i)) {
-                load_k(value_head(i), kt, 0);
-                load_k(value_head(i), kt, 1);
-            }
-            f32x4 sc[2];
-#pragma unroll
-            for (int b = 0; b < 2; ++b) {
-                sc[b] = (f32x4){0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-                for (int s = 0; s < NS; ++s)
-                    sc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                        kf[b][s], qf[i][s], sc[b], 0, 0, 0);
-            }
-#pragma unroll
-            for (int j = 0; j < 8; ++j) {
-                float e =
-                    fast_exp2(capped(sc[j >> 2][j & 3], cap, ls[i]));
-                if (!whole) {
-                    const int key = k0 + (j >> 2) * 16 + gq * 4 + (j & 3);
-                    if (key < qlo || key > qa) e = 0.f;
+            for (int i = 0; i < NH; ++i) {
+                if (other(i)) {
+                    load_k(value_head(i), kt, 0);
+                    load_k(value_head(i), kt, 1);
                 }
-                const u32 x = __builtin_bit_cast(unsigned short, (_Float16)e);
-                pw[j][i >> 1] |= i & 1 ? x << 16 : x;
+                f32x4 sc[2];
+#pragma unroll
+                for (int b = 0; b < 2; ++b) {
+                    sc[b] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                    for (int s = 0; s < NS; ++s)
+                        sc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                            kf[b][s], qf[i][s], sc[b], 0, 0, 0);
+                }
+#pragma unroll
+                for (int j = 0; j < 8; ++j) {
+                    float e =
+                        fast_exp2(capped(sc[j >> 2][j & 3], cap, ls[i]));
+                    if (!decltype(whole)::value)
+                        e = (u32)(base + (j >> 2) * 16 + (j & 3)) <=
+                                    (u32)(qa - qlo) ? e : 0.f;
+                    const u32 x = __builtin_bit_cast(unsigned short,
+                                                     (_Float16)e);
+                    pw[j][i >> 1] |= i & 1 ? x << 16 : x;
+                }
             }
-        }
+        };
+        if (k0 >= all_lo && k0 + 31 <= first)
+            weights(std::true_type{});
+        else
+            weights(std::false_type{});
 #pragma unroll
         for (int j = 0; j < 8; ++j)
             *(uint2*)(pb[now] + fr * QS +
@@ -899,18 +944,18 @@ static int allow_lds(int bytes) {
     return (int)e;
 }
 
-template <int P, int GP, int HB>
+template <int P, int GP, int HB, int R>
 static int go_decode(hipStream_t st, bf16_t* out, const bf16_t* q,
                      const bf16_t* vc, const float* inv, const int* table,
                      int per_slot, const int* pos, const int* slot, float* ws,
                      const float* kw, const float* talk, const Rotation rot,
                      int N, int H, int G, int chunk, int nsplit,
                      const Cap cap) {
-    typedef DecodeShape<P, GP, HB> Sh;
+    typedef DecodeShape<P, GP, HB, R> Sh;
     if (Sh::BYTES > 160 * 1024) return -102;
-    const int e = allow_lds<k_talk_decode<P, GP, HB>>(Sh::BYTES);
+    const int e = allow_lds<k_talk_decode<P, GP, HB, R>>(Sh::BYTES);
     if (e) return e;
-    k_talk_decode<P, GP, HB><<<N * nsplit, Sh::WAVES * 64, Sh::BYTES, st>>>(
+    k_talk_decode<P, GP, HB, R><<<N * nsplit, Sh::WAVES * 64, Sh::BYTES, st>>>(
         out, q, vc, inv, table, per_slot, pos, slot, ws, kw, talk, rot, N, H,
         G, chunk, nsplit, cap);
     LAUNCH_CHECK();
@@ -951,30 +996,30 @@ int gt_talk_decode(void* stream, void* out, const void* q, const void* vc,
                    int R, int chunk, int nsplit, float rate, float top,
                    float rho) {
     if (N < 1 || !sizes_ok(H, G, P, R, nrot, chunk) || nsplit < 1 ||
-        nsplit > 64 || H > 64 || G * P > 1024 || R % 32 ||
+        nsplit > 64 || H > 64 || G * P > 1024 ||
         nrot < per_slot * PAGE ||
         (nsplit > 1 && !ws)) return -100;
     const Rotation rot = rotation(cos_, sin_, R, nrot);
     const Cap cap{rate, top, rho};
-#define GO(A, B, C) return go_decode<A, B, C>((hipStream_t)stream, \
+#define GO(A, B, C, D) return go_decode<A, B, C, D>((hipStream_t)stream, \
         (bf16_t*)out, (const bf16_t*)q, (const bf16_t*)vc, \
         (const float*)inv, (const int*)table, per_slot, (const int*)pos, \
         (const int*)slot, (float*)ws, (const float*)kw, (const float*)talk, \
         rot, N, H, G, chunk, nsplit, cap)
-#define HEADS(A, B) do { if (H <= 16) GO(A, B, 1); \
-        else if (H <= 32) GO(A, B, 2); else GO(A, B, 4); } while (0)
-#define VALUES(A) do { if (G == 1) HEADS(A, 1); else if (G == 2) HEADS(A, 2); \
-        else if (G <= 4) HEADS(A, 4); } while (0)
-    if (P == 64) {
-        VALUES(64);
-        if (G <= 8) HEADS(64, 8);
-        HEADS(64, 16);
-    }
-    if (P == 128) {
-        VALUES(128);
-        HEADS(128, 8);
-    }
-    VALUES(256);
+#define HEADS(A, B, D) do { if (H <= 16) GO(A, B, 1, D); \
+        else if (H <= 32) GO(A, B, 2, D); else GO(A, B, 4, D); } while (0)
+#define VALUES(A, D) do { if (G == 1) HEADS(A, 1, D); \
+        else if (G == 2) HEADS(A, 2, D); \
+        else if (G <= 4) HEADS(A, 4, D); \
+        else if (G <= 8 && A <= 128) HEADS(A, A <= 128 ? 8 : 4, D); \
+        else if (A == 64) HEADS(A, A == 64 ? 16 : 4, D); } while (0)
+    if (P == 64 && R == 32) VALUES(64, 32);
+    if (P == 64 && R == 64) VALUES(64, 64);
+    if (P == 128 && R == 32) VALUES(128, 32);
+    if (P == 128 && R == 64) VALUES(128, 64);
+    if (P == 128 && R == 128) VALUES(128, 128);
+    if (P == 256 && R == 64) VALUES(256, 64);
+    if (P == 256 && R == 256) VALUES(256, 256);
 #undef VALUES
 #undef HEADS
 #undef GO

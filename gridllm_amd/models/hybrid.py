@@ -28,7 +28,7 @@ import numpy as np
 import torch
 
 from gridllm_amd.models.paged import (PAGE, PagedCache, head_pad, latent_pad,
-                                      pad64)
+                                      pad64, rotated_pad)
 from gridllm_amd.models.registry import (AttentionMixer, DenseFF, GlaMixer,
                                          HybridSpec, LatentMixer, PolyFF,
                                          RoutedFF, TalkingMixer)
@@ -161,7 +161,7 @@ class HybridModel:
 
         def table(mx) -> tuple:
             r = latent_pad(mx)[1] if isinstance(mx, LatentMixer) else \
-                -(-mx.rot_dims // 32) * 32
+                rotated_pad(mx)
             key = (mx.rot_base, mx.rot_dims, r)
             if key not in made:
                 half = mx.rot_dims // 2

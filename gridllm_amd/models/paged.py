@@ -58,6 +58,14 @@ def latent_pad(mixer: LatentMixer) -> tuple[int, int]:
             _next_of((64, 128), mixer.rot_dim, "rotated key parts"))
 
 
+def rotated_pad(mixer: TalkingMixer) -> int:
+    """Leading coordinates of a head that the talking-heads kernels treat as
+    rotated."""
+    p = head_pad(mixer)
+    return next(r for r in ((64, 256) if p == 256 else (32, 64, p))
+                if mixer.rot_dims <= r)
+
+
 class PagedCache:
     def __init__(self, spec: HybridSpec, slots: int, max_seq: int,
                  device: torch.device, dtype: torch.dtype,
