@@ -632,7 +632,9 @@ k_talk_lse(float* __restrict__ lse, const bf16_t* __restrict__ q,
 // (f16, times 2^14) and leaves them in LDS; one MFMA mixes 16 keys of a row for
 // 16 output heads; each wave applies its heads' mixed weights. The three steps
 // work on three successive tiles between two barriers.
+// Weights are normalised, so parts of a row's keys (grid y) just add up.
 //   talk: f16 [32][32] in that numbering; fin: factor of the result
+//   ws: null, or f32 [parts][rows][H][P] from token `row0` on
 //   SAME: the heads of a wave share a value head
 // ===========================================================================
 #define LIFT 14.f
@@ -643,7 +645,8 @@ k_talk_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                const bf16_t* __restrict__ kx, const bf16_t* __restrict__ vx,
                const float* __restrict__ lse, const _Float16* __restrict__ talk,
                const int* __restrict__ meta, int H, int G, int chunk,
-               const Cap cap, float fin) {
+               const Cap cap, float fin, float* __restrict__ ws, int row0,
+               int rows) {
     constexpr int NS = P / 32, NT = P / 16;
     // a row of 32, and 32 or 16 such rows, padded against bank conflicts
     constexpr int LDR = 36, QS = 32 * LDR + 4, HS = 16 * LDR + 4;
@@ -693,7 +696,11 @@ k_talk_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
         for (int t = 0; t < NT; ++t)
             vf[t] = *(const bf16x8*)(vr + t * 16 * PAGE);
     };
-    const int begin = first_seen(first, chunk) & ~31;
+    const int start = first_seen(first, chunk) & ~31;
+    const int tiles = (last - start) / 32 + 1;
+    const int per = (tiles + gridDim.y - 1) / gridDim.y * 32;
+    const int begin = start + blockIdx.y * per;
+    const int tail = min(last & ~31, begin + per - 32);
     // value head of a wave's head (the last head stands in for missing ones:
     // their column of talk is zero, and nobody stores their result)
     auto value_head = [&](int i) { return min(h0 + i, H - 1) / rep; };
@@ -703,13 +710,12 @@ k_talk_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
     const int kv0 = value_head(0), now0 = (begin >> 5) & 1;
     for (int i = threadIdx.x; i < 8 * QS; i += 512) ((u32*)pb[now0 ^ 1])[i] = 0;
     for (int i = threadIdx.x; i < 16 * HS; i += 512) ((u32*)wb[now0])[i] = 0;
-    if (SAME) load_v(kv0, begin);
+    if (SAME && begin <= tail) load_v(kv0, begin);
     lds_barrier();
     // Tile k0: weights; tile k0 - 32: mixing; tile k0 - 64: values. Where there
     // is no such tile the weights are zero. Keys take over the registers of
     // the values.
-    const int tail = last & ~31;
-    for (int k0 = begin; k0 <= tail + 64; k0 += 32) {
+    for (int k0 = begin; k0 <= tail + 64 && begin <= tail; k0 += 32) {
         const int now = (k0 >> 5) & 1, kt = min(k0, tail);
         bf16x8 w[NH];
 #pragma unroll
@@ -743,6 +749,7 @@ k_talk_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
         }
         u32 pw[8][2] = {};                    // heads 0 | 1 and 2 | 3
         const int base = k0 + gq * 4 - qlo;   // from the first key seen
+        const u32 until = k0 <= tail ? qa - qlo + 1 : 0;
         auto weights = [&](auto whole) {
 #pragma unroll
             for (int i = 0; i < NH; ++i) {
@@ -764,15 +771,15 @@ k_talk_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                     float e =
                         fast_exp2(capped(sc[j >> 2][j & 3], cap, ls[i]));
                     if (!decltype(whole)::value)
-                        e = (u32)(base + (j >> 2) * 16 + (j & 3)) <=
-                                    (u32)(qa - qlo) ? e : 0.f;
+                        e = (u32)(base + (j >> 2) * 16 + (j & 3)) < until
+                                ? e : 0.f;
                     const u32 x = __builtin_bit_cast(unsigned short,
                                                      (_Float16)e);
                     pw[j][i >> 1] |= i & 1 ? x << 16 : x;
                 }
             }
         };
-        if (k0 >= all_lo && k0 + 31 <= first)
+        if (k0 >= all_lo && k0 + 31 <= first && k0 <= tail)
             weights(std::true_type{});
         else
             weights(std::false_type{});
@@ -807,7 +814,13 @@ k_talk_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
     if (fr >= nq) return;
 #pragma unroll
     for (int i = 0; i < NH; ++i)
-        if (h0 + i < H) {
+        if (h0 + i < H && ws) {
+            float* o = ws + (((long)blockIdx.y * rows + row - row0) * H + h0 +
+                             i) * P + gq * 4;
+#pragma unroll
+            for (int t = 0; t < NT; ++t)
+                *(f32x4*)(o + t * 16) = acc[i][t] * fin;
+        } else if (h0 + i < H) {
             bf16_t* o = out + ((long)row * H + h0 + i) * P + gq * 4;
 #pragma unroll
             for (int t = 0; t < NT; ++t)
@@ -815,6 +828,23 @@ k_talk_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                     pack2(acc[i][t][0] * fin, acc[i][t][1] * fin),
                     pack2(acc[i][t][2] * fin, acc[i][t][3] * fin));
         }
+}
+
+// out = the sum of `parts` f32 rows [parts][n], 4 elements a thread
+__global__ void __launch_bounds__(256)
+k_talk_add(bf16_t* __restrict__ out, const float* __restrict__ ws, long n,
+           int parts) {
+    const long i = (blockIdx.x * 256L + threadIdx.x) * 4;
+    if (i >= n) return;
+    float a[4];
+    ld4(ws + i, a);
+    for (int s = 1; s < parts; ++s) {
+        float b[4];
+        ld4(ws + s * n + i, b);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) a[j] += b[j];
+    }
+    st4(out + i, a);
 }
 
 // ===========================================================================
@@ -1057,15 +1087,17 @@ int gt_talk_lse(void* stream, void* lse, const void* q, const void* kx,
 int gt_talk_prefill(void* stream, void* out, const void* q, const void* kx,
                     const void* vx, const void* lse, const void* talk,
                     const void* meta, int ntiles, int H, int G, int P,
-                    int chunk, float rate, float top, float rho, float fin) {
+                    int chunk, float rate, float top, float rho, float fin,
+                    void* ws, int parts, int row0, int rows) {
     const int nh = (H + 7) / 8;
     if (ntiles < 1 || !sizes_ok(H, G, P, 0, 1, chunk) || nh > 4 ||
-        nh * P > 512) return -100;
-#define GO1(A, B, C) k_talk_prefill<A, B, C><<<ntiles, 512, 0, \
+        nh * P > 512 || parts < 1 || (parts > 1) != !!ws || row0 < 0 ||
+        rows < 1) return -100;
+#define GO1(A, B, C) k_talk_prefill<A, B, C><<<dim3(ntiles, parts), 512, 0, \
         (hipStream_t)stream>>>((bf16_t*)out, (const bf16_t*)q, \
         (const bf16_t*)kx, (const bf16_t*)vx, (const float*)lse, \
         (const _Float16*)talk, (const int*)meta, H, G, chunk, \
-        Cap{rate, top, rho}, fin)
+        Cap{rate, top, rho}, fin, (float*)ws, row0, rows)
 #define GO(A, B) do { if (H / G % B == 0) GO1(A, B, true); \
         else GO1(A, B, false); } while (0)
 #define PICK(A) do { if (nh == 1) GO(A, 1); else if (nh == 2) GO(A, 2); \
@@ -1078,6 +1110,13 @@ int gt_talk_prefill(void* stream, void* out, const void* q, const void* kx,
 #undef GO
 #undef GO1
     LAUNCH_CHECK();
+    if (parts > 1) {
+        const long n = (long)rows * H * P;
+        k_talk_add<<<(unsigned)((n / 4 + 255) / 256), 256, 0,
+                     (hipStream_t)stream>>>(
+            (bf16_t*)out + (long)row0 * H * P, (const float*)ws, n, parts);
+        LAUNCH_CHECK();
+    }
     return 0;
 }
 

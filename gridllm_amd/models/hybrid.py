@@ -722,7 +722,7 @@ class HybridModel:
                  np.asarray(segs), np.asarray(tiles), np.asarray(chunks),
                  np.asarray(csegs), np.asarray(litems), np.asarray(ltiles)]
         for t in talks:
-            parts += t[1:]
+            parts += t[2:]
         dev = self._upload_ints(parts)
         mixed = bool(tiles)
         st = StepMeta(nd=nd, pos=dev[0], slot=dev[1], table=self.cache.table,
@@ -737,7 +737,7 @@ class HybridModel:
         for k, (c, t) in enumerate(zip(self.chunks, talks)):
             if t[0]:
                 items, t16, t128 = dev[9 + 3 * k:12 + 3 * k]
-                st.talk[c] = ChunkPortions(t[0], items.view(-1, 4),
+                st.talk[c] = ChunkPortions(*t[:2], items.view(-1, 4),
                                            t16.view(-1, 8), t128.view(-1, 8))
         x = self._run(tokens, st, trail)
         ends = np.asarray([[e[0] for e in entries],
@@ -757,8 +757,8 @@ class HybridModel:
 
     @staticmethod
     def _chunk_portions(segs: list, chunk: int) -> tuple:
-        """Pages, items, 16-row and 128-row tiles of the longer portions (see
-        ChunkPortions)."""
+        """The fields of ChunkPortions for the portions among segs, on the
+        host."""
         pages, items, tiles = 0, [], {16: [], 128: []}
         for off, ln, sl, p0 in segs:
             if ln <= _ABSORB:
@@ -776,14 +776,15 @@ class HybridModel:
                 out.append(t)
             pages += len(have)
         if not pages:
-            return 0, [], [], []
+            return 0, 0, [], [], []
 
         def ordered(t):             # blocks start in this order
             span = (t[:, 3] + t[:, 4]) % chunk
             return t[np.argsort(-span, kind="stable")]
 
         t16, t128 = (ordered(np.concatenate(t)) for t in tiles.values())
-        return pages, np.concatenate(items), t16, t128
+        span = int(((t16[:, 3] + t16[:, 4]) % chunk).max()) + 16
+        return pages, span, np.concatenate(items), t16, t128
 
     def _upload_ints(self, parts: list) -> list[torch.Tensor]:
         """int32 arrays to the device in one copy; each starts at a multiple

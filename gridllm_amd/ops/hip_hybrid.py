@@ -59,7 +59,7 @@ _SIGS = {
     "gt_talk_decode": "pppppippppppp" + "iiiiiiiifff",
     "gt_talk_gather": "pppppipppipiiii",
     "gt_talk_lse": "ppppiiiiifff",
-    "gt_talk_prefill": "pppppppiiiiiffff",
+    "gt_talk_prefill": "pppppppiiiiiffffpiii",
     "gt_talk_plain": "ipppppipppppp" + "iiiiiiiff",
 }
 _LIB_OF = {"gh": "hybrid", "gn": "latent", "gt": "talk"}
@@ -559,7 +559,12 @@ def talk_attn(q: torch.Tensor, vc: torch.Tensor, inv: torch.Tensor,
         lse = torch.empty(n, h, dtype=torch.float32, device=dev)
         _call("gt_talk_lse", lse, q, kx[0], portions.tiles128,
               portions.tiles128.shape[0], h, g, p, tk.chunk, *cap)
+        nt = portions.tiles16.shape[0]
+        # few tiles: their keys in parts, of 128 or more
+        parts = max(1, min(256 // nt, portions.span // 128, 8))
+        ws = torch.empty(parts, n - na, h, p, dtype=torch.float32,
+                         device=dev) if parts > 1 else None
         _call("gt_talk_prefill", out, q, kx[0], kx[1], lse, tk.talk16,
-              portions.tiles16, portions.tiles16.shape[0], h, g, p, tk.chunk,
-              *cap, tk.talk16_scale)
+              portions.tiles16, nt, h, g, p, tk.chunk, *cap, tk.talk16_scale,
+              ws, parts, na, n - na)
     return out

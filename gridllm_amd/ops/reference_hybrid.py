@@ -21,8 +21,10 @@ class ChunkPortions:
     tiles16  [*, 8] {first token, length, first page, first row, start, page
              number of that page} per 16 rows of a portion, and
     tiles128 per 128 rows; long spans of keys first
+    span     keys that the longest of these sees, about
     """
     pages: int
+    span: int
     items: torch.Tensor
     tiles16: torch.Tensor
     tiles128: torch.Tensor

@@ -91,8 +91,9 @@ def meta_for(cache, slot, start, ln, dev, absorb=16, chunk=0):
             p0 = start // chunk * chunk // 64          # first page seen
             n = -(-total // 64) - p0
             st.talk[chunk] = ChunkPortions(
-                n, t([[p0 + i, slot, i, min(64, total - 64 * (p0 + i))]
-                      for i in range(n)], 4),
+                n, min(total, chunk),
+                t([[p0 + i, slot, i, min(64, total - 64 * (p0 + i))]
+                   for i in range(n)], 4),
                 *(t([[0, ln, 0, q, start, p0, 0, 0]
                      for q in range(0, ln, k)], 8) for k in (16, 128)))
     return st
