@@ -1,8 +1,8 @@
 // gfx950 kernels of the layer-list models: a decoder whose layers each name a
-// mixer (grouped softmax attention over a paged cache, latent attention, mLSTM
-// or gated linear attention with a matrix memory per sequence) and a
-// feed-forward (dense gated, or routed experts). Latent attention is in
-// gridllm_latent.hip.
+// mixer (grouped softmax attention over a paged cache, latent or talking-heads
+// attention, mLSTM or gated linear attention with a matrix memory per sequence)
+// and a feed-forward (dense gated, dense with PolyNorm, or routed experts).
+// Latent attention is in gridllm_latent.hip, talking heads in gridllm_talk.hip.
 //
 // Conventions
 //  * T is the element type of activations, weights and the KV cache: bf16, or

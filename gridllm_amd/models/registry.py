@@ -88,13 +88,14 @@ class AttentionMixer:
 
 @dataclass(frozen=True)
 class TalkingMixer:
-    """Grouped softmax attention whose values are the keys as projected (with a
-    bias, ahead of norm and rotation), so that values alone are cached. RMS norms
-    of q and k with a weight over the head; pairs (i, i + rot_dims / 2) of the
-    first rot_dims coordinates turn by p rot_base^(-2 i / rot_dims); scores are
-    soft-capped at `cap`; a query sees the keys of its own chunk of `chunk`
-    positions; 1 is added to the denominator; the heads' weights are mixed by a
-    matrix."""
+    """Grouped softmax attention with one projection (and bias) for keys and
+    values: a value is the raw projection, a key is made from it by an RMS norm
+    with a weight over the head and the rotation, so that values alone are
+    cached. Queries are normed and rotated alike: pairs (i, i + rot_dims / 2) of
+    the first rot_dims coordinates turn by p rot_base^(-2 i / rot_dims). Scores
+    are soft-capped at `cap`; a query sees the keys of its own chunk of `chunk`
+    positions; the softmax's denominator holds an extra 1; a matrix mixes the
+    heads' weights."""
     heads: int
     kv_heads: int
     dim: int
@@ -186,8 +187,8 @@ class DenseFF:
 
 @dataclass(frozen=True)
 class PolyFF:
-    """Ungated feed-forward with PolyNorm between its matrices: a N(z) + b N(z^2)
-    + c N(z^3) + e, N dividing by the root mean square."""
+    """Ungated feed-forward with PolyNorm between its matrices: a polynomial of
+    third degree, each power of a row divided by its own root mean square."""
     ff: int
 
     def params(self, width: int) -> int:

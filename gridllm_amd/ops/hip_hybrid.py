@@ -1,8 +1,8 @@
 """ctypes binding to libgridllm_hybrid.so, libgridllm_latent.so and
 libgridllm_talk.so: the gfx950 kernels of the layer-list models
-(csrc/gridllm_hybrid.hip, _latent.hip and _talk.hip). Same contract as hip_ops: launches go onto torch's
-current stream, a missing library raises, shapes are checked on the host before
-a launch.
+(csrc/gridllm_hybrid.hip, _latent.hip and _talk.hip). Same contract as hip_ops:
+launches go onto torch's current stream, a missing library raises, shapes are
+checked on the host before a launch.
 
 Every function here has a CPU counterpart of the same signature in
 reference_hybrid; ops.hybrid picks one by device.

@@ -187,9 +187,9 @@ def test_poly_norm(ff, run):
     z = torch.nn.functional.pad(torch.randn(7, ff, generator=g) *
                                 torch.logspace(-3, 1, 7).view(7, 1),
                                 (0, fp - ff)).to(element(run))
-    abce = torch.tensor([0.7, -0.4, 0.3, 0.2])
-    want = oracle.poly_norm(z[:, :ff].double(), abce.double(), 1e-3)
-    got = hops.poly_norm(z.to(run[0]), abce.to(run[0]), ff, 1e-3)[:, :ff]
+    coef = torch.tensor([0.7, -0.4, 0.3, 0.2])
+    want = oracle.poly_norm(z[:, :ff].double(), coef.double(), 1e-3)
+    got = hops.poly_norm(z.to(run[0]), coef.to(run[0]), ff, 1e-3)[:, :ff]
     assert got.dtype == z.dtype
     assert float(errors(got, want).max()) < \
         (1e-5 if run[1] == "fp32" else 0.005)
@@ -413,7 +413,7 @@ def test_prompts_of_several_chunks_and_splits(heads, kv, dim, chunk, run):
     W = weights_of(cfg)
     m = build(cfg, run, W=W, max_seq=2200)
     ids = tokens(2100 if run[0] != "cpu" else 720, cfg, seed=7)
-    cuts = [n for n in (699, 1, 1, 1299, 1, 1, 17, 2, 1)]
+    cuts = [699, 1, 1, 1299, 1, 1, 17, 2, 1]
     slot, at, got, places = m.cache.alloc(0), 0, [], []
     for n in cuts:
         part = ids[at:at + n]

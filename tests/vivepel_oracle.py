@@ -85,9 +85,9 @@ def attention(h, w, c, eps):
     return out.reshape(t, H * d) @ w["o"].T
 
 
-def poly_norm(z, abce, eps):
-    a, b, c, e = abce
-    return a * rms(z, eps) + b * rms(z ** 2, eps) + c * rms(z ** 3, eps) + e
+def poly_norm(z, coef, eps):
+    """Three normed powers and a constant."""
+    return coef[3] + sum(coef[k] * rms(z ** (k + 1), eps) for k in range(3))
 
 
 def dense_ff(h, w, eps):
