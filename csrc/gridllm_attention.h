@@ -33,14 +33,59 @@ struct PagedKV {
     }
 };
 
+// Which keys up to its own a query sees. Kernels walk blocks of keys by number
+// (decode) or by first key (prefill) and leave out what no row sees.
+struct AllKeys {
+    DEV_INLINE int blocks(int seq) const { return (seq + 63) >> 6; }
+    DEV_INLINE int start(int b, int seq) const { return b << 6; }
+    DEV_INLINE int skip(int k0, int q0) const { return k0; }
+    DEV_INLINE bool sees(int q, int key) const { return true; }
+};
+
+// The last `size` keys, its own included, and the first `keep`.
+struct WindowKeys {
+    int size, keep;
+    // blocks of 64 that hold kept keys, and the first one of the window behind
+    // them, for the last of seq positions
+    DEV_INLINE int kept(int seq) const { return (min(keep, seq) + 63) >> 6; }
+    DEV_INLINE int window(int seq) const {
+        return max(kept(seq), max(0, seq - size) >> 6);
+    }
+    DEV_INLINE int blocks(int seq) const {
+        return kept(seq) + ((seq + 63) >> 6) - window(seq);
+    }
+    DEV_INLINE int start(int b, int seq) const {
+        const int k = kept(seq);
+        return (b < k ? b : window(seq) + b - k) << 6;
+    }
+    // first key, from k0 on, of a tile of 32 that rows from q0 on may see
+    DEV_INLINE int skip(int k0, int q0) const {
+        return k0 < keep ? k0 : max(k0, max(0, q0 - size + 1) & ~31);
+    }
+    DEV_INLINE bool sees(int q, int key) const {
+        return q - key < size || key < keep;
+    }
+};
+
 // What happens to a head's sums before they are stored. `sink` (nullable, one
 // per query head) adds exp(sink) to the softmax denominator; `gate` (nullable,
-// one per row and query head, row stride gate_ld) multiplies the output by
-// its sigmoid.
+// row stride gate_ld) multiplies the output by its sigmoid: one per query
+// head, or (gate_el) one per element; so does `scale`. out_ld: row stride of
+// the output, 0 if the heads fill a row.
 struct HeadEpilogue {
     const float* sink;
     const bf16_t* gate;
     int gate_ld;
+    int gate_el = 0;
+    float scale = 1.f;
+    int out_ld = 0;
+    DEV_INLINE long at(long row, int head, int Hq, int D) const {
+        return row * (out_ld ? out_ld : Hq * D) + head * D;
+    }
+    DEV_INLINE float element(int row, int col) const {
+        if (!gate_el) return 1.f;
+        return 1.f / (1.f + __expf(-bf2f(gate[(long)row * gate_ld + col])));
+    }
     // M, L: running maximum and sum of the log2-domain softmax. Returns the
     // factor for the accumulated values.
     DEV_INLINE float factor(int row, int head, float M, float L) const {
@@ -51,8 +96,8 @@ struct HeadEpilogue {
             f = (M == -INFINITY) ? 0.f : exp2f(M - m2);
             L = L * f + exp2f(s2 - m2);
         }
-        f = L > 0.f ? f / L : 0.f;
-        if (gate)
+        f = L > 0.f ? f / L * scale : 0.f;
+        if (gate && !gate_el)
             f /= 1.f + __expf(-bf2f(gate[(long)row * gate_ld + head]));
         return f;
     }
@@ -77,14 +122,15 @@ struct HeadEpilogue {
 
 // A kv head with more than MAXG query heads is served by `ngrp` blocks of G
 // query heads each. Sequence lengths are given as seqlen + seq_add.
-template <int D, int G, class KV>
+template <int D, int G, class KV, class Keys>
 __global__ void __launch_bounds__(256, 3)
 k_attn_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
               const KV kv,
               const int* __restrict__ seqlen, int seq_add,
               const int* __restrict__ slot_map,
               float* __restrict__ ws,
-              int ngrp, int nsplit, float scale, const HeadEpilogue epi) {
+              int ngrp, int nsplit, float scale, const HeadEpilogue epi,
+              const Keys keys) {
     const int Hg = kv.Hk * ngrp;
     const int split = blockIdx.x % nsplit;
     const int hg = (blockIdx.x / nsplit) % Hg;
@@ -100,12 +146,10 @@ k_attn_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
 
     const int seq = seqlen[b] + seq_add;
     // split range, 64-aligned chunks
-    const int chunks = (seq + 63) >> 6;
+    const int chunks = keys.blocks(seq);
     const int per = (chunks + nsplit - 1) / nsplit;
     const int c0 = split * per;
     const int c1 = min(chunks, c0 + per);
-    const int s0 = c0 << 6;
-    const int s1 = min(seq, c1 << 6);
 
     // stage q (scaled) into LDS as f32
     const int Hq = Hg * G;
@@ -140,14 +184,15 @@ k_attn_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
     const int rg = lane / DV;
     const int d8 = (lane % DV) * 8;
 
-    int kb = s0 + wid * 64;
-    long next = kb < s1 ? kv.off(bc, hk, kb) : 0;
-    for (; kb < s1; kb += 256) {
+    int cb = c0 + wid;
+    long next = cb < c1 ? kv.off(bc, hk, keys.start(cb, seq)) : 0;
+    for (; cb < c1; cb += 4) {
+        const int kb = keys.start(cb, seq);
         const bf16_t* kblk = kv.k + next;
         const bf16_t* vblk = kv.v + next;
-        if (kb + 256 < s1) next = kv.off(bc, hk, kb + 256);
+        if (cb + 4 < c1) next = kv.off(bc, hk, keys.start(cb + 4, seq));
         const int j = kb + lane;
-        const bool valid = j < s1;
+        const bool valid = j < seq && keys.sees(seq - 1, j);
         float s[G];
 #pragma unroll
         for (int g = 0; g < G; ++g) s[g] = 0.f;
@@ -187,7 +232,7 @@ k_attn_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
         // wave-local LDS visibility (no cross-wave traffic here)
         asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
         // accumulate P·V: RPI rows per iteration, one b128 load per lane
-        const int jmax = min(64, s1 - kb);
+        const int jmax = min(64, seq - kb);
         for (int jb = 0; jb < jmax; jb += RPI) {
             const int j2 = jb + rg;
             const uint4 vv = *(const uint4*)(
@@ -243,8 +288,9 @@ k_attn_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
         float M = fmaxf(fmaxf(wml[0][g][0], wml[1][g][0]),
                         fmaxf(wml[2][g][0], wml[3][g][0]));
         if (nsplit == 1) {
-            out[((long)b * Hq + hg * (long)G + g) * D + d] =
-                f2bf(a * epi.factor(b, hg * G + g, M, L));
+            out[epi.at(b, hg * G + g, Hq, D) + d] =
+                f2bf(a * epi.factor(b, hg * G + g, M, L) *
+                     epi.element(b, (hg * G + g) * D + d));
         } else {
             float* wsp = ws + (((long)b * Hq + hg * G + g) * nsplit + split) * (D + 2);
             wsp[d] = a;
@@ -265,14 +311,15 @@ k_attn_decode(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
 // RPI rows per b128 iteration with an end shfl ladder.
 // ===========================================================================
 
-template <int D, int G, class KV>
+template <int D, int G, class KV, class Keys>
 __global__ void __launch_bounds__(64, 3)
 k_attn_decode1(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                const KV kv,
                const int* __restrict__ seqlen, int seq_add,
                const int* __restrict__ slot_map,
                float* __restrict__ ws,
-               int ngrp, int nsplit, float scale, const HeadEpilogue epi) {
+               int ngrp, int nsplit, float scale, const HeadEpilogue epi,
+               const Keys keys) {
     const int Hg = kv.Hk * ngrp;
     const int split = blockIdx.x % nsplit;
     const int hg = (blockIdx.x / nsplit) % Hg;
@@ -285,10 +332,10 @@ k_attn_decode1(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
     __shared__ float p_lds[G * 64];
 
     const int seq = seqlen[b] + seq_add;
-    const int chunks = (seq + 63) >> 6;
+    const int chunks = keys.blocks(seq);
     const int per = (chunks + nsplit - 1) / nsplit;
-    const int s0 = (split * per) << 6;
-    const int s1 = min(seq, (split * per + per) << 6);
+    const int c0 = split * per;
+    const int c1 = min(chunks, c0 + per);
 
     const int Hq = Hg * G;
     for (int i = lane; i < G * D; i += 64)
@@ -310,13 +357,14 @@ k_attn_decode1(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
     const int rg = lane / DV;
     const int d8 = (lane % DV) * 8;
 
-    long next = s0 < s1 ? kv.off(bc, hk, s0) : 0;
-    for (int kb = s0; kb < s1; kb += 64) {
+    long next = c0 < c1 ? kv.off(bc, hk, keys.start(c0, seq)) : 0;
+    for (int cb = c0; cb < c1; ++cb) {
+        const int kb = keys.start(cb, seq);
         const bf16_t* kblk = kv.k + next;
         const bf16_t* vblk = kv.v + next;
-        if (kb + 64 < s1) next = kv.off(bc, hk, kb + 64);
+        if (cb + 1 < c1) next = kv.off(bc, hk, keys.start(cb + 1, seq));
         const int j = kb + lane;
-        const bool valid = j < s1;
+        const bool valid = j < seq && keys.sees(seq - 1, j);
         float s[G];
 #pragma unroll
         for (int g = 0; g < G; ++g) s[g] = 0.f;
@@ -356,7 +404,7 @@ k_attn_decode1(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
         // P.V: RPI rows per b128 iteration; p read from same-wave LDS
         // (an LDS hop, not shfl: it bounds how far the scheduler can
         // interleave the K and V phases — shfl spilled 1.5 KB here)
-        const int jmax = min(64, s1 - kb);
+        const int jmax = min(64, seq - kb);
         for (int jb = 0; jb < jmax; jb += RPI) {
             const int j2 = jb + rg;
             const uint4 vv = *(const uint4*)(
@@ -388,8 +436,9 @@ k_attn_decode1(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                 const float f = epi.factor(b, hg * G + g, m[g], l[g]);
 #pragma unroll
                 for (int i = 0; i < 8; ++i)
-                    out[((long)b * Hq + hg * (long)G + g) * D + d8 + i] =
-                        f2bf(facc[g][i] * f);
+                    out[epi.at(b, hg * G + g, Hq, D) + d8 + i] =
+                        f2bf(facc[g][i] * f *
+                             epi.element(b, (hg * G + g) * D + d8 + i));
             } else {
                 float* wsp = ws + (((long)b * Hq + hg * G + g) * nsplit
                                    + split) * (D + 2);
@@ -421,8 +470,9 @@ k_attn_combine(bf16_t* __restrict__ out, const float* __restrict__ ws,
         num += f * p[d];
         den += f * p[D + 1];
     }
-    out[bh * D + d] = f2bf(num * epi.factor((int)(bh / Hq), (int)(bh % Hq),
-                                            M, den));
+    const int b = (int)(bh / Hq), h = (int)(bh % Hq);
+    out[epi.at(b, h, Hq, D) + d] =
+        f2bf(num * epi.factor(b, h, M, den) * epi.element(b, h * D + d));
 }
 // ===========================================================================
 // GQA prefill attention — flash-style on MFMA (bf16), reads K/V straight
@@ -450,14 +500,14 @@ k_attn_combine(bf16_t* __restrict__ out, const float* __restrict__ ws,
 // Shared body: one 128-q-row tile of one q-head for one sequence.
 // q0 = first q row of this tile; vt/plds = caller's LDS buffers.
 // row0 = row of q[0] in the epilogue's gate.
-template <int D, class KV>
+template <int D, class KV, class Keys = AllKeys>
 __device__ __forceinline__ void
 attn_prefill_tile(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                   const KV& kv,
                   int T, int Hq, int G, int slot,
                   int s_total, int causal_off, float scale, int q0,
                   bf16_t* vt, bf16_t* plds_all, const HeadEpilogue& epi,
-                  int row0) {
+                  int row0, const Keys keys = Keys()) {
     constexpr int NS = D / 16;     // 16-wide d slices (QK^T fragments)
     constexpr int NT = D / 32;     // 32-wide d tiles (output / V^T)
     constexpr int VST = 40;        // padded k-stride of V^T tile (16B-mult)
@@ -490,7 +540,9 @@ attn_prefill_tile(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
     // causal upper bound for the workgroup's LAST q-row
     const int kmax = min(s_total, causal_off + q0 + 128);
 
-    for (int k0 = 0; k0 < kmax; k0 += 32) {
+    const int qfirst = causal_off + q0;
+    for (int k0 = keys.skip(0, qfirst); k0 < kmax;
+         k0 = keys.skip(k0 + 32, qfirst)) {
         const long blk = kv.off(slot, hk, k0);   // 32 keys lie together
         const int klast = s_total - 1 - k0;
         // ---- stage V^T tile (cooperative transpose) --------------------
@@ -530,7 +582,8 @@ attn_prefill_tile(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
             const int kg = k0 + (r & 3) + 8 * (r >> 2) + 4 * hi;
-            const bool ok = (kg < s_total) && (kg <= q_abs);
+            const bool ok = (kg < s_total) && (kg <= q_abs) &&
+                            keys.sees(q_abs, kg);
             sv[r] = ok ? s_acc[r] * scl2 : -INFINITY;
             tmax = fmaxf(tmax, sv[r]);
         }
@@ -587,17 +640,23 @@ attn_prefill_tile(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
     // ---- normalize + store: lane holds O^T[*][q=ln] — one q-row --------
     if (qw + ln < T) {
         const float inv = epi.factor(row0 + qw + ln, hq, m, l);
-        bf16_t* orow = out + ((long)(qw + ln) * Hq + hq) * D;
+        bf16_t* orow = out + epi.at(qw + ln, hq, Hq, D);
 #pragma unroll
         for (int t = 0; t < NT; ++t) {
 #pragma unroll
             for (int g = 0; g < 4; ++g) {
                 const int d = t * 32 + 8 * g + 4 * hi;
-                u32 lo = (u32)f2bf(acc[t][4 * g] * inv) |
-                         ((u32)f2bf(acc[t][4 * g + 1] * inv) << 16);
-                u32 h2 = (u32)f2bf(acc[t][4 * g + 2] * inv) |
-                         ((u32)f2bf(acc[t][4 * g + 3] * inv) << 16);
-                *(uint2*)(orow + d) = make_uint2(lo, h2);
+                float f[4];
+#pragma unroll
+                for (int i = 0; i < 4; ++i) f[i] = acc[t][4 * g + i] * inv;
+                if (epi.gate_el) {
+                    float z[4];
+                    ld4(epi.gate + (long)(row0 + qw + ln) * epi.gate_ld +
+                        hq * D + d, z);
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) f[i] /= 1.f + __expf(-z[i]);
+                }
+                st4(orow + d, f);
             }
         }
     }

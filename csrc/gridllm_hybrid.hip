@@ -1,7 +1,8 @@
 // gfx950 kernels of the layer-list models: a decoder whose layers each name a
 // mixer (grouped softmax attention over a paged cache, latent or talking-heads
-// attention, mLSTM or gated linear attention with a matrix memory per sequence)
-// and a feed-forward (dense gated, dense with PolyNorm, or routed experts).
+// attention, mLSTM, gated linear or lightning attention with a matrix memory
+// per sequence, or two of these side by side) and a feed-forward (dense gated,
+// dense with PolyNorm, or routed experts, with a shared one beside them).
 // Latent attention is in gridllm_latent.hip, talking heads in gridllm_talk.hip.
 //
 // Conventions
@@ -17,6 +18,7 @@
 // Exported extern "C" with an explicit stream; nothing here allocates.
 
 #include "gridllm_attention.h"
+#include "gridllm_tiles.h"
 
 // ===========================================================================
 // x = embed[token], f32, plus pos_table[position] if there is one, then its
@@ -333,6 +335,173 @@ k_group_norm(T* __restrict__ out, float* __restrict__ x,
 }
 
 // ===========================================================================
+// Hyper-connections: ns residual streams x_s, f32 [N][ns][W].
+//   start: x_s = embed[token] * scale for all s
+//   join:  x_t = sum_s mix[s][t] x_s + put[t] y, all from the old ones
+// and what the next sublayer reads, if there is one:
+//   h = T(norm(sum_s in[s] x_s) * w)
+// hc holds mix [from][to], then put. y is a sublayer's output; with experts
+// (top > 0) the sum of a token's pairs, and `extra` adds a row times the
+// sigmoid of a number per token. S: ns rounded up to a power of two. W <= 2048
+// NV; the mean is over Wtrue elements.
+// ===========================================================================
+template <class T, int NV>
+DEV_INLINE void store_normed(T* h, const float u[NV][8], const float* w,
+                             long n, int W, int Wtrue, float eps, float* red) {
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < NV; ++j)
+        if ((j * 256 + threadIdx.x) * 8 < W)
+#pragma unroll
+            for (int i = 0; i < 8; ++i) ss += u[j][i] * u[j][i];
+    const float rs = 1.f / sqrtf(block_sum(ss, red) / (float)Wtrue + eps);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+        const int c = (j * 256 + threadIdx.x) * 8;
+        if (c < W) {
+            float g[8];
+            ld8(w + c, g);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) g[i] *= u[j][i] * rs;
+            st8(h + n * W + c, g);
+        }
+    }
+}
+
+template <class T>
+__global__ void __launch_bounds__(256)
+k_streams_start(float* __restrict__ x, T* __restrict__ h,
+                const T* __restrict__ emb, const long long* __restrict__ tok,
+                float scale, const float* __restrict__ in,
+                const float* __restrict__ w, int ns, int W, int Wtrue,
+                float eps, int vocab) {
+    __shared__ float red[4];
+    const long n = blockIdx.x;
+    const long t = min(max(tok[n], 0ll), (long long)vocab - 1);
+    float total = 0.f, u[4][8];
+    for (int s = 0; s < ns; ++s) total += in[s];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int c = (j * 256 + threadIdx.x) * 8;
+        if (c < W) {
+            float a[8];
+            ld8(emb + t * W + c, a);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) {
+                a[i] *= scale;
+                u[j][i] = total * a[i];
+            }
+            for (int s = 0; s < ns; ++s) st8(x + (n * ns + s) * W + c, a);
+        }
+    }
+    store_normed<T, 4>(h, u, w, n, W, Wtrue, eps, red);
+}
+
+template <class T, int S, int NV, bool MOE>
+__global__ void __launch_bounds__(256)
+k_streams_join(float* __restrict__ x, T* __restrict__ h,
+               const T* __restrict__ y, int top, const T* __restrict__ extra,
+               const float* __restrict__ extra_z, int extra_ld,
+               const float* __restrict__ hc, const float* __restrict__ in,
+               const float* __restrict__ w, int ns, int W, int Wtrue,
+               float eps) {
+    constexpr bool AHEAD = S * NV <= 8;     // all loads ahead of the stores
+    constexpr int NX = AHEAD ? NV : 1;
+    __shared__ float red[4];
+    const long n = blockIdx.x;
+    float* xr = x + n * ns * W;
+    const float ge = MOE && extra ? sigmoidf_(extra_z[n * extra_ld]) : 0.f;
+    float a[NX][S][8], v[NX][8], u[NV][8];
+    auto load = [&](int j, int c) {
+#pragma unroll
+        for (int s = 0; s < S; ++s)
+            if (s < ns) ld8(xr + (long)s * W + c, a[j][s]);
+        if (!MOE) {
+            ld8(y + n * W + c, v[j]);
+            return;
+        }
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[j][i] = 0.f;
+        for (int k0 = 0; k0 < top; k0 += 4) {       // 4 rows in flight
+            float f[4][8];
+#pragma unroll
+            for (int k = 0; k < 4; ++k)
+                ld8(y + (n * top + min(k0 + k, top - 1)) * W + c, f[k]);
+#pragma unroll
+            for (int k = 0; k < 4; ++k)
+#pragma unroll
+                for (int i = 0; i < 8; ++i)
+                    v[j][i] += k0 + k < top ? f[k][i] : 0.f;
+        }
+        if (extra) {
+            float f[8];
+            ld8(extra + n * W + c, f);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) v[j][i] += ge * f[i];
+        }
+    };
+    if (AHEAD)
+#pragma unroll
+        for (int j = 0; j < NV; ++j) {
+            const int c = (j * 256 + threadIdx.x) * 8;
+            if (c < W) load(j % NX, c);
+        }
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+        const int c = (j * 256 + threadIdx.x) * 8, jx = j % NX;
+        if (c < W) {
+            if (!AHEAD) load(jx, c);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) u[j][i] = 0.f;
+#pragma unroll
+            for (int t = 0; t < S; ++t) {
+                if (t >= ns) continue;
+                const float put = hc[ns * ns + t], read = h ? in[t] : 0.f;
+                float r[8];
+#pragma unroll
+                for (int i = 0; i < 8; ++i) r[i] = put * v[jx][i];
+#pragma unroll
+                for (int s = 0; s < S; ++s) {
+                    if (s >= ns) continue;
+                    const float m = hc[s * ns + t];
+#pragma unroll
+                    for (int i = 0; i < 8; ++i) r[i] += m * a[jx][s][i];
+                }
+#pragma unroll
+                for (int i = 0; i < 8; ++i) u[j][i] += read * r[i];
+                st8(xr + (long)t * W + c, r);
+            }
+        }
+    }
+    if (h) store_normed<T, NV>(h, u, w, n, W, Wtrue, eps, red);
+}
+
+// out[r] = norm(sum_s x_s[rows[r]]) * w; rows null = identity
+template <class T>
+__global__ void __launch_bounds__(256)
+k_streams_norm(T* __restrict__ out, const float* __restrict__ x,
+               const int* __restrict__ rows, const float* __restrict__ w,
+               int ns, int W, int Wtrue, float eps) {
+    __shared__ float red[4];
+    const long n = rows ? rows[blockIdx.x] : blockIdx.x;
+    float u[4][8];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int c = (j * 256 + threadIdx.x) * 8;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) u[j][i] = 0.f;
+        if (c < W)
+            for (int s = 0; s < ns; ++s) {
+                float a[8];
+                ld8(x + (n * ns + s) * W + c, a);
+#pragma unroll
+                for (int i = 0; i < 8; ++i) u[j][i] += a[i];
+            }
+    }
+    store_normed<T, 4>(out, u, w, blockIdx.x, W, Wtrue, eps, red);
+}
+
+// ===========================================================================
 // PolyNorm: out = c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3, powers by element, N
 // dividing a row by its root mean square over Ftrue elements (columns behind
 // them are zero). NV > 0: a row of up to NV * 2048 columns stays in registers.
@@ -476,31 +645,44 @@ k_proj_f32(float* __restrict__ out, const bf16_t* __restrict__ x,
 }
 
 // ===========================================================================
-// Attention prologue: unit-RMS q and k (no weight), query temperature, and
-// the write of k and v into the paged cache, from one projection row
+// Attention prologue: rotated (if there are tables) unit-RMS q and k (no
+// weight), query temperature, and the write of k and v into the paged cache,
+// from one projection row
 //   [H*P q | G*P k | G*P v | ...], row stride ld.
 // temperature(p) = 1 + coef * ln(floor((p + 1) / every) + 1).
-// One wave per (token, head).
+// P / 8 lanes per head. Further waves put SiLU on act_n columns from act_0 on,
+// in place (q, k and v of a recurrence in the same row).
 // ===========================================================================
 template <class T, int P>
 __global__ void __launch_bounds__(256)
-k_qknorm_kv(const T* __restrict__ qkv, T* __restrict__ q_out,
+k_qknorm_kv(T* __restrict__ qkv, T* __restrict__ q_out,
             T* __restrict__ kc, T* __restrict__ vc,
             const int* __restrict__ table, int per_slot,
             const int* __restrict__ pos, const int* __restrict__ slot,
             int N, int H, int G, int ld_, int dim, float eps, float coef,
-            int every) {
-    constexpr int V = P / 64;
+            int every, const Rotation rot, int act_0, int act_n) {
+    constexpr int LPH = P / 8, HW = 64 / LPH;
     const int nh = H + 2 * G;
+    const int groups = (nh + HW - 1) / HW, per = groups + (act_n + 511) / 512;
     const long item = blockIdx.x * 4L + (threadIdx.x >> 6);
-    if (item >= (long)N * nh) return;
-    const int n = (int)(item / nh), h = (int)(item % nh);
+    if (item >= (long)N * per) return;
+    const int n = (int)(item / per), it = (int)(item % per);
     const int lane = threadIdx.x & 63;
-    const T* src = qkv + (long)n * ld_ + (long)h * P + lane * V;
-    const int p = pos[n];
-    float f[V];
+    float f[8];
+    if (it >= groups) {
+        const int c = (it - groups) * 512 + lane * 8;
+        if (c >= act_n) return;
+        T* z = qkv + (long)n * ld_ + act_0 + c;
+        ld8(z, f);
 #pragma unroll
-    for (int i = 0; i < V; ++i) f[i] = ld(src + i);
+        for (int i = 0; i < 8; ++i) f[i] *= sigmoidf_(f[i]);
+        st8(z, f);
+        return;
+    }
+    const int h = it * HW + lane / LPH, c = (lane % LPH) * 8;
+    if (h >= nh) return;
+    ld8(qkv + (long)n * ld_ + (long)h * P + c, f);
+    const int p = pos[n];
     T* dst;
     if (h < H) {
         dst = q_out + ((long)n * H + h) * P;
@@ -513,34 +695,37 @@ k_qknorm_kv(const T* __restrict__ qkv, T* __restrict__ q_out,
               ((page * G + hk) * KV_PAGE + p % KV_PAGE) * P;
     }
     if (h < H + G) {
+        if (c < 2 * rot.half) rotate8(f, c, p, rot);
         float ss = 0.f;
 #pragma unroll
-        for (int i = 0; i < V; ++i) ss += f[i] * f[i];
-        float s = 1.f / sqrtf(wave_reduce_sum(ss) / (float)dim + eps);
+        for (int i = 0; i < 8; ++i) ss += f[i] * f[i];
+#pragma unroll
+        for (int off = LPH / 2; off > 0; off >>= 1)
+            ss += __shfl_xor(ss, off, WAVE);
+        float s = 1.f / sqrtf(ss / (float)dim + eps);
         if (h < H) s *= 1.f + coef * logf((float)((p + 1) / every) + 1.f);
 #pragma unroll
-        for (int i = 0; i < V; ++i) f[i] *= s;
+        for (int i = 0; i < 8; ++i) f[i] *= s;
     }
-#pragma unroll
-    for (int i = 0; i < V; ++i) st(dst + lane * V + i, f[i]);
+    st8(dst + c, f);
 }
 
 // Varlen prefill over the paged cache. meta row (8 ints): {q_off, len, slot,
 // q0, start}: rows [q0, q0 + 128) of the portion packed at q_off, whose first
 // token stands at position `start`.
-template <int D>
+template <int D, class Keys>
 __global__ void __launch_bounds__(256, D > 128 ? 1 : 2)
 k_paged_prefill(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                 const PagedKV<D> kv, const int* __restrict__ meta, int Hq,
-                int G, float scale, const HeadEpilogue epi) {
+                int G, float scale, const HeadEpilogue epi, const Keys keys) {
     __shared__ __attribute__((aligned(16))) bf16_t vt[D * 40];
     __shared__ __attribute__((aligned(16))) bf16_t plds[4][2 * 64 * 8];
     const int* m = meta + blockIdx.x * 8;
     const int q_off = m[0], len = m[1], start = m[4];
-    attn_prefill_tile<D>(out + (long)q_off * Hq * D,
+    attn_prefill_tile<D>(out + epi.at(q_off, 0, Hq, D),
                          q + (long)q_off * Hq * D, kv, len, Hq, G, m[2],
                          start + len, start, scale, m[3], vt, &plds[0][0],
-                         epi, q_off);
+                         epi, q_off, keys);
 }
 
 // Exact mode: one block per (row, query head), f32 cache, any position.
@@ -551,7 +736,8 @@ k_attn_rows_f32(float* __restrict__ out, const float* __restrict__ q,
                 const int* __restrict__ table, int per_slot,
                 const int* __restrict__ pos, const int* __restrict__ slot,
                 int H, int G, float scale, const float* __restrict__ sink,
-                const float* __restrict__ gate, int gate_ld) {
+                const float* __restrict__ gate, int gate_ld, int gate_el,
+                float oscale, int out_ld, const WindowKeys keys) {
     const int n = blockIdx.x / H, h = blockIdx.x % H;
     const int hk = h / (H / G);
     const int* tab = table + (long)slot[n] * per_slot;
@@ -564,10 +750,12 @@ k_attn_rows_f32(float* __restrict__ out, const float* __restrict__ q,
     const int c = threadIdx.x % P, grp = threadIdx.x / P;
     const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
     float m = sink ? sink[h] : -INFINITY, l = sink ? 1.f : 0.f, acc = 0.f;
-    for (int k0 = 0; k0 < seq; k0 += 256) {
+    for (int k0 = keys.skip(0, seq - 1); k0 < seq;
+         k0 = keys.skip(k0 + 256, seq - 1)) {
         const int j = k0 + threadIdx.x;
+        const bool seen = j < seq && keys.sees(seq - 1, j);
         float s = -INFINITY;
-        if (j < seq) {
+        if (seen) {
             const float* kr = kc + (((long)tab[j / KV_PAGE] * G + hk) * KV_PAGE
                                     + j % KV_PAGE) * P;
             s = 0.f;
@@ -584,7 +772,7 @@ k_attn_rows_f32(float* __restrict__ out, const float* __restrict__ q,
         mx = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
         const float mn = fmaxf(m, mx);
         const float alpha = (m == -INFINITY) ? 0.f : expf(m - mn);
-        const float p = (j < seq) ? expf(s - mn) : 0.f;
+        const float p = seen ? expf(s - mn) : 0.f;
         sc[threadIdx.x] = p;
         m = mn;
         __syncthreads();                       // red read, sc written
@@ -606,9 +794,11 @@ k_attn_rows_f32(float* __restrict__ out, const float* __restrict__ q,
     if (threadIdx.x < P) {
         float a = 0.f;
         for (int g = 0; g < NG; ++g) a += acc_s[g * P + threadIdx.x];
-        float f = l > 0.f ? 1.f / l : 0.f;
-        if (gate) f *= sigmoidf_(gate[(long)n * gate_ld + h]);
-        out[((long)n * H + h) * P + threadIdx.x] = a * f;
+        float f = l > 0.f ? oscale / l : 0.f;
+        if (gate)
+            f *= sigmoidf_(gate[(long)n * gate_ld +
+                                (gate_el ? h * P + threadIdx.x : h)]);
+        out[(long)n * out_ld + h * P + threadIdx.x] = a * f;
     }
 }
 
@@ -642,10 +832,13 @@ DEV_INLINE int4 segment(const int4* seg, const int* pos, const int* slot,
 
 // Token by token. Block = (segment, head, `rpb` state rows); LPR lanes hold
 // one row of DK as NJ float4 each, and a wave works on 64 / LPR rows at once,
-// U of them in flight. With CH the memory decays per key channel instead: gr
-// is the logarithm of the decay, f32 [n][H*DK], and there is neither an input
-// gate nor a normaliser row (gated linear attention; S is [H][DV][DK]).
-template <class T, int LPR, int NJ, bool CH>
+// U of them in flight. The other kinds have neither an input gate nor a
+// normaliser row (S is [H][DV][DK]): their memory decays per key channel, gr
+// being the logarithm of the decay, f32 [n][H*DK] (gated linear attention), or
+// by a constant per head, gr f32 [H] (lightning attention).
+enum Rec { MLSTM = 0, CHANNELS = 1, CONSTANT = 2 };
+
+template <class T, int LPR, int NJ, int KIND>
 __global__ void __launch_bounds__(256)
 k_rec_step(float* __restrict__ o, float* __restrict__ S,
            const float* __restrict__ mst, const T* __restrict__ qkv,
@@ -655,19 +848,20 @@ k_rec_step(float* __restrict__ o, float* __restrict__ S,
            int rpb) {
     constexpr int RW = 64 / LPR;
     constexpr int U = NJ == 1 ? 4 : 2;
-    const int R = CH ? DV : DV + 1;
+    constexpr bool CH = KIND == CHANNELS, GATED = KIND == MLSTM;
+    const int R = GATED ? DV + 1 : DV;
     const int4 sg = segment(segs, pos, slot, blockIdx.x);
     const int h = blockIdx.y;
     const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
     const int c0 = (lane % LPR) * 4, rl = lane / LPR;
     const int rbeg = blockIdx.z * rpb, rend = min(R, rbeg + rpb);
     float* Sb = S + ((long)sg.z * H + h) * R * DK;
-    float m = CH || sg.w == 0 ? 0.f : mst[(long)sg.z * H + h];
+    float m = !GATED || sg.w == 0 ? 0.f : mst[(long)sg.z * H + h];
     for (int t = 0; t < sg.y; ++t) {
         const long n = sg.x + t;
         const bool fresh = sg.w + t == 0;
-        float keep1 = 0.f, put = 1.f;
-        if (!CH) {
+        float keep1 = KIND == CONSTANT ? gr[h] : 0.f, put = 1.f;
+        if (GATED) {
             float gi, gf;
             mlstm_gates(gr + n * 2 * H, h, H, cap, gi, gf);
             const float mn = fmaxf(gf + m, gi);
@@ -798,6 +992,64 @@ k_rec_out(T* __restrict__ out, const float* __restrict__ o,
     if (is_seg && lane == 0) mst[(long)sg.z * H + h] = m;
 }
 
+// The same for heads that are normed together and have no denominators
+// (lightning attention): one block per token, out rows of stride out_ld. NV > 0:
+// a row of up to NV * 1024 columns stays in registers.
+template <class T, int NV>
+__global__ void __launch_bounds__(256)
+k_rec_row_out(T* __restrict__ out, const float* __restrict__ o,
+              const T* __restrict__ gate, const float* __restrict__ norm,
+              int H, int DV, int ld_, int out_ld, int true_cols, float eps) {
+    __shared__ float red[4];
+    constexpr int KEEP = NV ? NV : 1;
+    const long n = blockIdx.x;
+    const int cols = H * DV;
+    const float* ob = o + n * H * (DV + 4);
+    float v[KEEP][4], ss = 0.f;
+    auto load = [&](int c, float* f) {
+        ld4(ob + (c / DV) * (DV + 4) + c % DV, f);
+    };
+    auto add = [&](const float* f) {
+        ss += f[0] * f[0] + f[1] * f[1] + f[2] * f[2] + f[3] * f[3];
+    };
+    if (NV) {
+#pragma unroll
+        for (int j = 0; j < KEEP; ++j) {
+            const int c = (j * 256 + threadIdx.x) * 4;
+            if (c < cols) {
+                load(c, v[j]);
+                add(v[j]);
+            }
+        }
+    } else {
+        for (int c = threadIdx.x * 4; c < cols; c += 1024) {
+            load(c, v[0]);
+            add(v[0]);
+        }
+    }
+    const float rs = 1.f / sqrtf(block_sum(ss, red) / (float)true_cols + eps);
+    auto put = [&](int c, float* f) {
+        float z[4], w[4];
+        ld4(gate + n * ld_ + c, z);
+        ld4(norm + c, w);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) f[i] *= rs * w[i] * sigmoidf_(z[i]);
+        st4(out + n * out_ld + c, f);
+    };
+    if (NV) {
+#pragma unroll
+        for (int j = 0; j < KEEP; ++j) {
+            const int c = (j * 256 + threadIdx.x) * 4;
+            if (c < cols) put(c, v[j]);
+        }
+    } else {
+        for (int c = threadIdx.x * 4; c < cols; c += 1024) {
+            load(c, v[0]);
+            put(c, v[0]);
+        }
+    }
+}
+
 // ---------------------------------------------------------------------------
 // Prompt portions in chunks of 64 tokens. With F_t the running sum of f
 // inside a chunk, a_s = i_s - F_s and M_t = max(m_in, max_{s<=t} a_s):
@@ -817,12 +1069,24 @@ k_rec_out(T* __restrict__ out, const float* __restrict__ o,
 #define MCH 64
 #define MLD 72      // padded row of 64 tokens in LDS
 
+// Lightning attention (CONST) is the case i = 0, f the same for every token: m
+// then stays 0. It has no normaliser and no head norm; gr is f by head, f32
+// [H]. Score weights are (hi, lo) pairs of bf16, too.
+
 // running sum of f, a, running max of a; lane = token, wave-wide
+template <bool CONST>
 DEV_INLINE void chunk_scan(const float* gr, int tok0, int clen, int h, int H,
                            float cap, float& F, float& a, float& amax) {
     const int t = threadIdx.x & 63;
     float gi = -INFINITY, gf = 0.f;
-    if (t < clen) mlstm_gates(gr + (long)(tok0 + t) * 2 * H, h, H, cap, gi, gf);
+    if (t < clen) {
+        if (CONST) {
+            gi = 0.f;
+            gf = gr[h];
+        } else {
+            mlstm_gates(gr + (long)(tok0 + t) * 2 * H, h, H, cap, gi, gf);
+        }
+    }
     F = gf;
 #pragma unroll
     for (int off = 1; off < 64; off <<= 1) {
@@ -838,6 +1102,7 @@ DEV_INLINE void chunk_scan(const float* gr, int tok0, int clen, int h, int H,
     }
 }
 
+template <bool CONST>
 __global__ void __launch_bounds__(256)
 k_mlstm_chunk_state(float* __restrict__ dS, float* __restrict__ scal,
                     const float* __restrict__ mst,
@@ -857,7 +1122,7 @@ k_mlstm_chunk_state(float* __restrict__ dS, float* __restrict__ scal,
     const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
     if (wid == 0) {
         float F, a, amax;
-        chunk_scan(gr, ch.x, ch.y, h, H, cap, F, a, amax);
+        chunk_scan<CONST>(gr, ch.x, ch.y, h, H, cap, F, a, amax);
         const float A = __shfl(amax, 63, WAVE);
         wgt[lane] = lane < ch.y ? expf(a - A) : 0.f;
         if (blockIdx.z == 0 && lane == 63) {
@@ -865,7 +1130,7 @@ k_mlstm_chunk_state(float* __restrict__ dS, float* __restrict__ scal,
             float* sp = scal + ((long)blockIdx.x * H + h) * 4;
             sp[0] = A;
             sp[1] = F;
-            sp[2] = sg.y == 0 ? 0.f : mst[(long)sg.x * H + h];
+            sp[2] = CONST || sg.y == 0 ? 0.f : mst[(long)sg.x * H + h];
         }
     }
     __syncthreads();
@@ -887,7 +1152,8 @@ k_mlstm_chunk_state(float* __restrict__ dS, float* __restrict__ scal,
         }
     }
     __syncthreads();
-    float* Db = dS + ((long)blockIdx.x * H + h) * (DV + 1) * DK;
+    const int R = CONST ? DV : DV + 1;
+    float* Db = dS + ((long)blockIdx.x * H + h) * R * DK;
     const int fr = lane & 15, kg = (lane >> 4) * 8;
     f32x4 acc[4];
 #pragma unroll
@@ -911,7 +1177,7 @@ k_mlstm_chunk_state(float* __restrict__ dS, float* __restrict__ scal,
         for (int r = 0; r < 4; ++r)
             Db[(long)(v0 + wid * 16 + (lane >> 4) * 4 + r) * DK + d0 + c * 16 +
                fr] = acc[c][r];
-    if (v0 == 0 && threadIdx.x < 64) {
+    if (!CONST && v0 == 0 && threadIdx.x < 64) {
         float s = 0.f;
         for (int t = 0; t < MCH; ++t)
             s += bf2f(kh[lane * MLD + t]) + bf2f(kl[lane * MLD + t]);
@@ -919,13 +1185,14 @@ k_mlstm_chunk_state(float* __restrict__ dS, float* __restrict__ scal,
     }
 }
 
+template <bool CONST>
 __global__ void __launch_bounds__(256)
 k_mlstm_chunk_scan(float* __restrict__ dS, float* __restrict__ scal,
                    float* __restrict__ S, float* __restrict__ mst,
                    const int4* __restrict__ segs, int H, int DK, int DV) {
     const int4 sg = segs[blockIdx.x];
     const int h = blockIdx.y;
-    const long size = (long)(DV + 1) * DK;
+    const long size = (long)(CONST ? DV : DV + 1) * DK;
     const long e = (blockIdx.z * 256L + threadIdx.x) * 4;
     if (e >= size) return;
     float* Sb = S + ((long)sg.x * H + h) * size + e;
@@ -965,7 +1232,7 @@ k_mlstm_chunk_scan(float* __restrict__ dS, float* __restrict__ scal,
         }
     }
     *(float4*)Sb = s;
-    if (e == 0) mst[(long)sg.x * H + h] = m;
+    if (!CONST && e == 0) mst[(long)sg.x * H + h] = m;
 }
 
 // 8 (hi | lo << 16) pairs -> the two bf16 fragments
@@ -981,6 +1248,7 @@ DEV_INLINE void split8(const u32* p, bf16x8& hi, bf16x8& lo) {
 }
 
 // Block = (chunk, head, 128 value columns); a wave owns 16 tokens.
+template <bool CONST>
 __global__ void __launch_bounds__(256, 2)
 k_mlstm_chunk_out(float* __restrict__ o, const float* __restrict__ dS,
                   const float* __restrict__ scal,
@@ -990,6 +1258,7 @@ k_mlstm_chunk_out(float* __restrict__ o, const float* __restrict__ dS,
                   int ld_, float qscale, float cap) {
     __shared__ __attribute__((aligned(16))) bf16_t vt[128 * MLD];
     __shared__ __attribute__((aligned(16))) bf16_t ps[64 * MLD];
+    __shared__ __attribute__((aligned(16))) bf16_t pl[CONST ? 64 * MLD : 8];
     __shared__ float sa[MCH], sM[MCH], sm[MCH], sin_[MCH], snq[MCH];
     const int4 ch = chunks[blockIdx.x];
     const int h = blockIdx.y, v0 = blockIdx.z * 128;
@@ -997,7 +1266,7 @@ k_mlstm_chunk_out(float* __restrict__ o, const float* __restrict__ dS,
     const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
     if (wid == 0) {
         float F, a, amax;
-        chunk_scan(gr, ch.x, ch.y, h, H, cap, F, a, amax);
+        chunk_scan<CONST>(gr, ch.x, ch.y, h, H, cap, F, a, amax);
         const float m_in = scal[((long)blockIdx.x * H + h) * 4 + 3];
         const float M = fmaxf(m_in, amax);
         sa[lane] = a;
@@ -1016,7 +1285,8 @@ k_mlstm_chunk_out(float* __restrict__ o, const float* __restrict__ dS,
     }
     __syncthreads();
     const int fr = lane & 15, kg = (lane >> 4) * 8, r0 = wid * 16;
-    const u32* Sb = (const u32*)dS + ((long)blockIdx.x * H + h) * (DV + 1) * DK;
+    const u32* Sb = (const u32*)dS +
+                    ((long)blockIdx.x * H + h) * (CONST ? DV : DV + 1) * DK;
     const bf16_t* qr = qkv + (long)(ch.x + min(r0 + fr, ch.y - 1)) * ld_ +
                        h * DK + kg;
 
@@ -1032,14 +1302,16 @@ k_mlstm_chunk_out(float* __restrict__ o, const float* __restrict__ dS,
     float nq = 0.f;
     for (int k0 = 0; k0 < DK; k0 += 32) {
         const bf16x8 a = *(const bf16x8*)(qr + k0);
-        float qf[8];
-        unpack8(*(const uint4*)&a, qf);
-        const u32* np = Sb + (long)DV * DK + k0 + kg;
+        if (!CONST) {
+            float qf[8];
+            unpack8(*(const uint4*)&a, qf);
+            const u32* np = Sb + (long)DV * DK + k0 + kg;
 #pragma unroll
-        for (int i = 0; i < 8; ++i) {
-            const u32 w = np[i];
-            nq += qf[i] * (__uint_as_float(w << 16) +
-                           __uint_as_float(w & 0xffff0000u));
+            for (int i = 0; i < 8; ++i) {
+                const u32 w = np[i];
+                nq += qf[i] * (__uint_as_float(w << 16) +
+                               __uint_as_float(w & 0xffff0000u));
+            }
         }
 #pragma unroll
         for (int j = 0; j < 4; ++j)
@@ -1047,9 +1319,11 @@ k_mlstm_chunk_out(float* __restrict__ o, const float* __restrict__ dS,
                 sc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
                     a, *(const bf16x8*)(kr[j] + k0), sc[j], 0, 0, 0);
     }
-    nq += __shfl_xor(nq, 16, WAVE);
-    nq += __shfl_xor(nq, 32, WAVE);
-    if (lane < 16) snq[r0 + lane] = nq;
+    if (!CONST) {
+        nq += __shfl_xor(nq, 16, WAVE);
+        nq += __shfl_xor(nq, 32, WAVE);
+        if (lane < 16) snq[r0 + lane] = nq;
+    }
     float den[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
@@ -1063,6 +1337,8 @@ k_mlstm_chunk_out(float* __restrict__ o, const float* __restrict__ dS,
                 ? sc[j][r] * qscale * expf(ak - sM[row]) : 0.f;
             den[r] += p;
             ps[row * MLD + key] = f2bf(p);
+            if (CONST)
+                pl[row * MLD + key] = f2bf(p - bf2f(f2bf(p)));
         }
     }
 #pragma unroll
@@ -1094,19 +1370,29 @@ k_mlstm_chunk_out(float* __restrict__ o, const float* __restrict__ dS,
     for (int r = 0; r < 4; ++r) {
         const int row = r0 + (lane >> 4) * 4 + r;
         const float in = sin_[row] * qscale;
-        const float d = den[r] + in * snq[row];
-        inv[r] = 1.f / (fmaxf(fabsf(d), expf(-sm[row])) + 1e-6f);
+        inv[r] = 1.f;
+        if (!CONST) {
+            const float d = den[r] + in * snq[row];
+            inv[r] = 1.f / (fmaxf(fabsf(d), expf(-sm[row])) + 1e-6f);
+        }
 #pragma unroll
         for (int c = 0; c < 8; ++c) acc[c][r] *= in;
     }
     for (int ks = 0; ks <= (wid >> 1); ++ks) {
-        const bf16x8 a = *(const bf16x8*)(ps + (r0 + fr) * MLD + ks * 32 + kg);
+        const int at = (r0 + fr) * MLD + ks * 32 + kg;
+        const bf16x8 a = *(const bf16x8*)(ps + at);
+        bf16x8 al;
+        if (CONST) al = *(const bf16x8*)(pl + at);
 #pragma unroll
         for (int c = 0; c < 8; ++c) {
             if (c * 16 >= nv) continue;
-            acc[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                a, *(const bf16x8*)(vt + (c * 16 + fr) * MLD + ks * 32 + kg),
-                acc[c], 0, 0, 0);
+            const bf16x8 v =
+                *(const bf16x8*)(vt + (c * 16 + fr) * MLD + ks * 32 + kg);
+            acc[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, v, acc[c],
+                                                             0, 0, 0);
+            if (CONST)
+                acc[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                    al, v, acc[c], 0, 0, 0);
         }
     }
 #pragma unroll
@@ -1486,18 +1772,19 @@ k_gla_chunk_out(float* __restrict__ o, const float* __restrict__ dS,
 // ===========================================================================
 // Routed experts.
 //   route:   top experts of every token by f32 logits (ties: lower index),
-//            their weights; counts per expert and each pair's rank. The choice
-//            may add a correction per expert to the softmax scores and be
+//            their weights, by softmax or (plain) sigmoids; counts per expert
+//            and each pair's rank. The choice may add a correction per expert to the softmax scores and be
 //            confined to the best of equal groups; router outputs beyond the
 //            experts are identities, whose weights are summed up apart
 //   scatter: pairs (token * top + k) sorted by expert, and the tile list
 //            {expert, first sorted row, rows, -}; entry max_tiles holds the
 //            number of tiles
 //   gemm:    rows of one expert against its weights, once for the up
-//            projection (gathers token rows; squared ReLU or silu(gate) * up)
-//            and once for the down projection (writes each pair's row back in
+//            projection (gathers token rows, times the pairs' weights if these
+//            go with the input; squared ReLU or a gated unit) and once for the down projection (writes each pair's row back in
 //            pair order)
-// The weighted sum over a token's pairs is taken in k_post_norm / k_sum_norm.
+// The (weighted) sum over a token's pairs is taken in k_post_norm, k_sum_norm
+// or k_streams_join.
 // ===========================================================================
 //
 // A wave routes `tpw` tokens, one expert per lane and VPL experts deep. The
@@ -1508,9 +1795,10 @@ template <int VPL>
 __global__ void __launch_bounds__(256)
 k_moe_route(int* __restrict__ idx, float* __restrict__ wt,
             int* __restrict__ rank, int* __restrict__ counts,
-            const float* __restrict__ z, const float* __restrict__ corr,
-            float* __restrict__ ident, int N, int E, int experts, int top,
-            int groups, int keep, float eps, float scale, int tpw) {
+            const float* __restrict__ z, int ldz,
+            const float* __restrict__ corr, float* __restrict__ ident, int N,
+            int E, int experts, int top, int groups, int keep, float eps,
+            float scale, int sigmoid, int tpw) {
     __shared__ int cnt[VPL * 64], base[VPL * 64];
     __shared__ float cs[4][VPL * 64], gm[4][VPL * 64];
     for (int e = threadIdx.x; e < VPL * 64; e += 256) cnt[e] = 0;
@@ -1524,7 +1812,7 @@ k_moe_route(int* __restrict__ idx, float* __restrict__ wt,
 #pragma unroll
         for (int i = 0; i < VPL; ++i) {
             const int e = i * 64 + lane;
-            v[i] = e < E ? z[(long)n * E + e] : -INFINITY;
+            v[i] = e < E ? z[(long)n * ldz + e] : -INFINITY;
             if (v[i] != v[i]) v[i] = -INFINITY;   // keeps the choice in range
             place[i] = 0;
             mx = fmaxf(mx, v[i]);
@@ -1533,10 +1821,11 @@ k_moe_route(int* __restrict__ idx, float* __restrict__ wt,
         float total = 0.f;
 #pragma unroll
         for (int i = 0; i < VPL; ++i) {
-            s[i] = i * 64 + lane < E ? expf(v[i] - mx) : 0.f;
+            s[i] = i * 64 + lane >= E ? 0.f
+                   : sigmoid ? sigmoidf_(v[i]) : expf(v[i] - mx);
             total += s[i];
         }
-        total = wave_reduce_sum(total);
+        total = sigmoid ? 1.f : wave_reduce_sum(total);
 #pragma unroll
         for (int i = 0; i < VPL; ++i) {
             const int e = i * 64 + lane;
@@ -1599,7 +1888,7 @@ k_moe_route(int* __restrict__ idx, float* __restrict__ wt,
             const int e = i * 64 + lane;
             if (place[i] >= top || e >= E) continue;
             const long at = (long)n * top + place[i];
-            const float w = s[i] / (sum + eps) * scale;
+            const float w = sigmoid ? s[i] : s[i] / (sum + eps) * scale;
             idx[at] = e;
             wt[at] = e < experts ? w : 0.f;
             if (e >= experts) same += w;
@@ -1692,20 +1981,16 @@ DEV_INLINE bool moe_work(const int4* tiles, int max_tiles, int ntn, int4& tl,
 // With few rows per expert the same pipeline streams the weights.
 // ACT != 0 (up projection): row r of the tile is token sorted[row0 + r] / top,
 // output in sorted order through squared ReLU (1) or, with weight rows in turns
-// of 16 gate | 16 up, silu(gate) * up in N / 2 columns (2). ACT 0: row r is
-// sorted row row0 + r and its output goes to pair order. The MFMA computes
+// of 16 gate | 16 up, the gated unit `glu` in N / 2 columns (2); pw (nullable):
+// a weight per pair on the unit's input. ACT 0: row r is sorted row row0 + r and its output goes to pair order. The MFMA computes
 // W x^T, so a lane ends up with 4 neighbouring columns of one row.
 // K % 64 == 0, N % 64 == 0 (ACT 2: N % 128 == 0).
-DEV_INLINE float silu_mul(float g, float u) {
-    return g / (1.f + __expf(-g)) * u;
-}
-
 template <int ACT, int NB>
 __global__ void __launch_bounds__(256, 2)
 k_moe_gemm(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
            const bf16_t* __restrict__ w, const int4* __restrict__ tiles,
            const int* __restrict__ sorted, int top, int N, int K, int ntn,
-           int max_tiles) {
+           int max_tiles, const GluParams glu, const float* __restrict__ pw) {
     constexpr int BK = 64, TB = 256 * BK, GL = 8;
     constexpr bool UP = ACT != 0;
     const int NO = ACT == 2 ? N / 2 : N;
@@ -1788,6 +2073,7 @@ k_moe_gemm(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
         if (m >= tl.z) continue;
         bf16_t* orow = out + (UP ? (long)tl.y + m : sorted[tl.y + m]) *
                                  (long)NO;
+        const float wi = ACT == 2 && pw ? pw[sorted[tl.y + m]] : 1.f;
 #pragma unroll
         for (int c = 0; c < 4; c += ACT == 2 ? 2 : 1) {
             const int n = (ACT == 2 ? (n0 + wc + c * 16) / 2
@@ -1795,7 +2081,8 @@ k_moe_gemm(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
             float f[4];
 #pragma unroll
             for (int r = 0; r < 4; ++r)
-                f[r] = ACT == 2 ? silu_mul(acc[a][c][r], acc[a][(c + 1) & 3][r])
+                f[r] = ACT == 2 ? glu_act(wi * acc[a][c][r],
+                                          wi * acc[a][(c + 1) & 3][r], glu)
                      : ACT == 1 ? sq_relu(acc[a][c][r]) : acc[a][c][r];
             if (n < NO) st4(orow + n, f);
         }
@@ -1810,7 +2097,8 @@ __global__ void __launch_bounds__(256)
 k_moe_gemm_few(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
                const bf16_t* __restrict__ w, const int4* __restrict__ tiles,
                const int* __restrict__ sorted, int top, int N, int K,
-               int ntn, int max_tiles) {
+               int ntn, int max_tiles, const GluParams glu,
+               const float* __restrict__ pw) {
     constexpr int U = 8, NW = ACT == 2 ? 2 : 1;
     constexpr bool UP = ACT != 0;
     __shared__ __attribute__((aligned(16))) float red[NW][4][16][20];
@@ -1857,8 +2145,9 @@ k_moe_gemm_few(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
     for (int t = 0; t < NW; ++t)
         v[t] = red[t][0][m][c] + red[t][1][m][c] + red[t][2][m][c] +
                red[t][3][m][c];
+    const float wi = ACT == 2 && pw ? pw[sorted[tl.y + m]] : 1.f;
     out[(UP ? (long)tl.y + m : sorted[tl.y + m]) * (long)(N / NW) + nti * 16 +
-        c] = f2bf(ACT == 2 ? silu_mul(v[0], v[NW - 1])
+        c] = f2bf(ACT == 2 ? glu_act(wi * v[0], wi * v[NW - 1], glu)
                            : ACT == 1 ? sq_relu(v[0]) : v[0]);
 }
 
@@ -1868,7 +2157,8 @@ __global__ void __launch_bounds__(256)
 k_moe_gemm_f32(float* __restrict__ out, const float* __restrict__ x,
                const float* __restrict__ w, const int4* __restrict__ tiles,
                const int* __restrict__ sorted, int top, int N, int K,
-               int ntn, int max_tiles) {
+               int ntn, int max_tiles, const GluParams glu,
+               const float* __restrict__ pw) {
     constexpr bool UP = ACT != 0;
     __shared__ float xs[16][33], ws[64][33];
     int4 tl;
@@ -1898,7 +2188,14 @@ k_moe_gemm_f32(float* __restrict__ out, const float* __restrict__ x,
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
         float v = ACT == 1 ? sq_relu(acc[r]) : acc[r];
-        if (ACT == 2) v = v / (1.f + expf(-v)) * __shfl_down(v, 16, WAVE);
+        if (ACT == 2) {
+            if (pw) v *= pw[sorted[tl.y + min(r4 + r, tl.z - 1)]];
+            const float u = fminf(fmaxf(__shfl_down(v, 16, WAVE), -glu.limit),
+                                  glu.limit);
+            v = fminf(v, glu.limit);
+            const float z = glu.alpha * v * (1.f + glu.cubic * v * v);
+            v = v / (1.f + expf(-z)) * (u + glu.shift);
+        }
         if (r4 + r >= tl.z) continue;
         const long dst = UP ? tl.y + r4 + r : sorted[tl.y + r4 + r];
         if (ACT != 2)
@@ -1916,16 +2213,17 @@ static void launch_paged_decode(hipStream_t st, void* out, const void* q,
                                 const PagedKV<D>& kv, const int* pos,
                                 const int* slot, float* ws, int B, int ngrp,
                                 int nsplit, float scale,
-                                const HeadEpilogue& epi) {
+                                const HeadEpilogue& epi,
+                                const WindowKeys& keys) {
     const dim3 grid((unsigned)(B * kv.Hk * ngrp * nsplit));
     if (nsplit == 1 && B * kv.Hk * ngrp >= 2048)
         k_attn_decode1<D, G><<<grid, dim3(64), 0, st>>>(
             (bf16_t*)out, (const bf16_t*)q, kv, pos, 1, slot, ws, ngrp,
-            nsplit, scale, epi);
+            nsplit, scale, epi, keys);
     else
         k_attn_decode<D, G><<<grid, dim3(256), 0, st>>>(
             (bf16_t*)out, (const bf16_t*)q, kv, pos, 1, slot, ws, ngrp,
-            nsplit, scale, epi);
+            nsplit, scale, epi, keys);
 }
 
 template <int D>
@@ -1933,7 +2231,8 @@ static int paged_decode(hipStream_t st, void* out, const void* q,
                         const void* kc, const void* vc, const int* table,
                         int per_slot, const int* pos, const int* slot,
                         float* ws, int B, int Hq, int Hk, int nsplit,
-                        float scale, const HeadEpilogue& epi) {
+                        float scale, const HeadEpilogue& epi,
+                        const WindowKeys& keys) {
     const PagedKV<D> kv{(const bf16_t*)kc, (const bf16_t*)vc, table, Hk,
                         per_slot};
     const int per = Hq / Hk;
@@ -1941,7 +2240,7 @@ static int paged_decode(hipStream_t st, void* out, const void* q,
     if (g > MAXG) for (g = MAXG; per % g; --g) {}
     switch (g) {
 #define CASE_G(GG) case GG: launch_paged_decode<D, GG>(st, out, q, kv, pos, \
-        slot, ws, B, per / GG, nsplit, scale, epi); break;
+        slot, ws, B, per / GG, nsplit, scale, epi, keys); break;
         CASE_G(1) CASE_G(2) CASE_G(3) CASE_G(4)
         CASE_G(5) CASE_G(6) CASE_G(7) CASE_G(8)
 #undef CASE_G
@@ -2085,16 +2384,80 @@ int gh_proj_f32(void* stream, void* out, const void* x, const void* w,
     return 0;
 }
 
-int gh_qknorm_kv(void* stream, int f32, const void* qkv, void* q_out,
+int gh_streams_start(void* stream, int f32, void* x, void* h, const void* emb,
+                     const void* tok, float scale, const void* in,
+                     const void* w, int N, int ns, int W, int Wtrue, float eps,
+                     int vocab) {
+    if (N < 1 || ns < 1 || W % 64 || W > 8192) return -100;
+#define GO(T) k_streams_start<T><<<N, 256, 0, (hipStream_t)stream>>>( \
+        (float*)x, (T*)h, (const T*)emb, (const long long*)tok, scale, \
+        (const float*)in, (const float*)w, ns, W, Wtrue, eps, vocab)
+    if (f32) GO(float); else GO(bf16_t);
+#undef GO
+    LAUNCH_CHECK();
+    return 0;
+}
+
+// moe: y holds `top` rows per token, and extra (nullable) one more
+int gh_streams_join(void* stream, int f32, int moe, void* x, void* h,
+                    const void* y, int top, const void* extra,
+                    const void* extra_z, int extra_ld, const void* hc,
+                    const void* in, const void* w, int N, int ns, int W,
+                    int Wtrue, float eps) {
+    if (N < 1 || ns < 1 || ns > 16 || W % 64 || W > 8192 ||
+        (moe && top < 1) || (h && !(in && w)) || (extra && !extra_z))
+        return -100;
+#define GO(T, S, NV, M) k_streams_join<T, S, NV, M><<<N, 256, 0, \
+        (hipStream_t)stream>>>((float*)x, (T*)h, (const T*)y, top, \
+        (const T*)extra, (const float*)extra_z, extra_ld, (const float*)hc, \
+        (const float*)in, (const float*)w, ns, W, Wtrue, eps)
+#define PICKV(T, S, M) do { if (W <= 4096) GO(T, S, 2, M); \
+        else GO(T, S, 4, M); } while (0)
+#define PICK(T, M) do { if (ns == 1) PICKV(T, 1, M); \
+        else if (ns == 2) PICKV(T, 2, M); else if (ns <= 4) PICKV(T, 4, M); \
+        else if (ns <= 8) GO(T, 8, 4, M); else GO(T, 16, 4, M); } while (0)
+    if (f32) { if (moe) PICK(float, true); else PICK(float, false); }
+    else { if (moe) PICK(bf16_t, true); else PICK(bf16_t, false); }
+#undef PICK
+#undef PICKV
+#undef GO
+    LAUNCH_CHECK();
+    return 0;
+}
+
+int gh_streams_norm(void* stream, int f32, void* out, const void* x,
+                    const void* rows, const void* w, int M, int ns, int W,
+                    int Wtrue, float eps) {
+    if (M < 1 || ns < 1 || W % 64 || W > 8192) return -100;
+#define GO(T) k_streams_norm<T><<<M, 256, 0, (hipStream_t)stream>>>((T*)out, \
+        (const float*)x, (const int*)rows, (const float*)w, ns, W, Wtrue, eps)
+    if (f32) GO(float); else GO(bf16_t);
+#undef GO
+    LAUNCH_CHECK();
+    return 0;
+}
+
+// cos_ and sin_ (nullable): tables of rot_rows x rot_half; act_0, act_n:
+// columns that get SiLU in place (which may be all there is: H and G 0)
+int gh_qknorm_kv(void* stream, int f32, void* qkv, void* q_out,
                  void* kc, void* vc, const void* table, int per_slot,
                  const void* pos, const void* slot, int N, int H, int G,
-                 int P, int ld_, int dim, float eps, float coef, int every) {
-    if (N < 1 || H % G || every < 1) return -100;
+                 int P, int ld_, int dim, float eps, float coef, int every,
+                 const void* cos_, const void* sin_, int rot_half,
+                 int rot_rows, int act_0, int act_n) {
+    if (N < 1 || (G ? H % G : H) || every < 1 || rot_half % 4 || 2 * rot_half > P ||
+        act_0 % 8 || act_n % 8 || act_0 + act_n > ld_ || ld_ % 8)
+        return -100;
     hipStream_t st_ = (hipStream_t)stream;
-    const unsigned grid = (unsigned)(((long)N * (H + 2 * G) + 3) / 4);
-#define GO(T, PP) k_qknorm_kv<T, PP><<<grid, 256, 0, st_>>>((const T*)qkv, \
+    const Rotation rot{(const float*)cos_, (const float*)sin_,
+                       cos_ ? rot_half : 0, rot_rows};
+    const int hw = 512 / P;
+    const long per = (H + 2 * G + hw - 1) / hw + (act_n + 511) / 512;
+    const unsigned grid = (unsigned)((N * per + 3) / 4);
+#define GO(T, PP) k_qknorm_kv<T, PP><<<grid, 256, 0, st_>>>((T*)qkv, \
         (T*)q_out, (T*)kc, (T*)vc, (const int*)table, per_slot, \
-        (const int*)pos, (const int*)slot, N, H, G, ld_, dim, eps, coef, every)
+        (const int*)pos, (const int*)slot, N, H, G, ld_, dim, eps, coef, \
+        every, rot, act_0, act_n)
     if (P == 64) { if (f32) GO(float, 64); else GO(bf16_t, 64); }
     else if (P == 128) { if (f32) GO(float, 128); else GO(bf16_t, 128); }
     else if (P == 256) { if (f32) GO(float, 256); else GO(bf16_t, 256); }
@@ -2104,17 +2467,22 @@ int gh_qknorm_kv(void* stream, int f32, const void* qkv, void* q_out,
     return 0;
 }
 
+// Keys seen: the last `window` (0: all) and the first `keep`. Epilogue: see
+// HeadEpilogue
 int gh_paged_decode(void* stream, void* out, const void* q, const void* kc,
                     const void* vc, const void* table, int per_slot,
                     const void* pos, const void* slot, void* ws, int B,
                     int Hq, int Hk, int D, int nsplit, float scale,
-                    const void* sink, const void* gate, int gate_ld) {
-    if (B < 1 || Hq % Hk || nsplit < 1) return -100;
-    const HeadEpilogue epi{(const float*)sink, (const bf16_t*)gate, gate_ld};
+                    int window, int keep, const void* sink, const void* gate,
+                    int gate_ld, int gate_el, float oscale, int out_ld) {
+    if (B < 1 || Hq % Hk || nsplit < 1 || window < 0 || keep < 0) return -100;
+    const HeadEpilogue epi{(const float*)sink, (const bf16_t*)gate, gate_ld,
+                           gate && gate_el, oscale, out_ld};
+    const WindowKeys keys{window ? window : 1 << 30, keep};
     hipStream_t st_ = (hipStream_t)stream;
 #define GO(DD) return paged_decode<DD>(st_, out, q, kc, vc, \
         (const int*)table, per_slot, (const int*)pos, (const int*)slot, \
-        (float*)ws, B, Hq, Hk, nsplit, scale, epi)
+        (float*)ws, B, Hq, Hk, nsplit, scale, epi, keys)
     if (D == 64) GO(64);
     if (D == 128) GO(128);
     if (D == 256) GO(256);
@@ -2125,19 +2493,27 @@ int gh_paged_decode(void* stream, void* out, const void* q, const void* kc,
 int gh_paged_prefill(void* stream, void* out, const void* q, const void* kc,
                      const void* vc, const void* table, int per_slot,
                      const void* meta, int ntiles, int Hq, int Hk, int D,
-                     float scale, const void* sink, const void* gate,
-                     int gate_ld) {
-    if (ntiles < 1 || Hq % Hk) return -100;
-    const HeadEpilogue epi{(const float*)sink, (const bf16_t*)gate, gate_ld};
+                     float scale, int window, int keep, const void* sink,
+                     const void* gate, int gate_ld, int gate_el, float oscale,
+                     int out_ld) {
+    if (ntiles < 1 || Hq % Hk || window < 0 || keep < 0 ||
+        (gate && gate_el && gate_ld % 4) || out_ld % 4)
+        return -100;
+    const HeadEpilogue epi{(const float*)sink, (const bf16_t*)gate, gate_ld,
+                           gate && gate_el, oscale, out_ld};
     hipStream_t st_ = (hipStream_t)stream;
-#define GO(DD) k_paged_prefill<DD><<<dim3(ntiles, Hq), 256, 0, st_>>>( \
-        (bf16_t*)out, (const bf16_t*)q, \
+#define GO(DD, K, ...) k_paged_prefill<DD, K><<<dim3(ntiles, Hq), 256, 0, \
+        st_>>>((bf16_t*)out, (const bf16_t*)q, \
         PagedKV<DD>{(const bf16_t*)kc, (const bf16_t*)vc, (const int*)table, \
-                    Hk, per_slot}, (const int*)meta, Hq, Hq / Hk, scale, epi)
-    if (D == 64) GO(64);
-    else if (D == 128) GO(128);
-    else if (D == 256) GO(256);
+                    Hk, per_slot}, (const int*)meta, Hq, Hq / Hk, scale, epi, \
+        K{__VA_ARGS__})
+#define PICK(DD) do { if (window) GO(DD, WindowKeys, window, keep); \
+        else GO(DD, AllKeys); } while (0)
+    if (D == 64) PICK(64);
+    else if (D == 128) PICK(128);
+    else if (D == 256) PICK(256);
     else return -101;
+#undef PICK
 #undef GO
     LAUNCH_CHECK();
     return 0;
@@ -2146,14 +2522,17 @@ int gh_paged_prefill(void* stream, void* out, const void* q, const void* kc,
 int gh_attn_rows_f32(void* stream, void* out, const void* q, const void* kc,
                      const void* vc, const void* table, int per_slot,
                      const void* pos, const void* slot, int N, int H, int G,
-                     int P, float scale, const void* sink, const void* gate,
-                     int gate_ld) {
-    if (N < 1 || H % G) return -100;
+                     int P, float scale, int window, int keep,
+                     const void* sink, const void* gate, int gate_ld,
+                     int gate_el, float oscale, int out_ld) {
+    if (N < 1 || H % G || window < 0 || keep < 0) return -100;
     hipStream_t st_ = (hipStream_t)stream;
+    const WindowKeys keys{window ? window : 1 << 30, keep};
 #define GO(PP) k_attn_rows_f32<PP><<<(unsigned)((long)N * H), 256, 0, st_>>>( \
         (float*)out, (const float*)q, (const float*)kc, (const float*)vc, \
         (const int*)table, per_slot, (const int*)pos, (const int*)slot, H, G, \
-        scale, (const float*)sink, (const float*)gate, gate_ld)
+        scale, (const float*)sink, (const float*)gate, gate_ld, gate_el, \
+        oscale, out_ld ? out_ld : H * P, keys)
     if (P == 64) GO(64);
     else if (P == 128) GO(128);
     else if (P == 256) GO(256);
@@ -2163,15 +2542,17 @@ int gh_attn_rows_f32(void* stream, void* out, const void* q, const void* kc,
     return 0;
 }
 
-// mst null: decay per key channel (gated linear attention)
-int gh_rec_step(void* stream, int f32, void* o, void* S, const void* mst,
+// kind: Rec
+int gh_rec_step(void* stream, int f32, int kind, void* o, void* S, const void* mst,
                 const void* qkv, const void* gr, const void* segs,
                 const void* pos, const void* slot, int nseg, int H, int DK,
                 int DV, int ld_, float qscale, float cap, int rpb) {
-    if (nseg < 1 || DK % 64 || DV % 64 || DK > 1024 || rpb < 1) return -100;
+    if (nseg < 1 || DK % 64 || DV % 64 || DK > 1024 || rpb < 1 || kind < 0 ||
+        kind > CONSTANT || (kind == MLSTM && !mst))
+        return -100;
     hipStream_t st_ = (hipStream_t)stream;
     const dim3 grid((unsigned)nseg, (unsigned)H,
-                    (unsigned)((DV + (mst ? 1 : 0) + rpb - 1) / rpb));
+                    (unsigned)((DV + (kind == MLSTM) + rpb - 1) / rpb));
 #define GO(T, L, J, C) k_rec_step<T, L, J, C><<<grid, 256, 0, st_>>>( \
         (float*)o, (float*)S, (const float*)mst, (const T*)qkv, \
         (const float*)gr, (const int4*)segs, (const int*)pos, \
@@ -2180,8 +2561,13 @@ int gh_rec_step(void* stream, int f32, void* o, void* S, const void* mst,
         else if (DK <= 128) GO(T, 32, 1, C); \
         else if (DK <= 256) GO(T, 64, 1, C); \
         else if (DK <= 512) GO(T, 64, 2, C); else GO(T, 64, 4, C); } while (0)
-    if (mst) { if (f32) PICK(float, false); else PICK(bf16_t, false); }
-    else { if (f32) PICK(float, true); else PICK(bf16_t, true); }
+    if (kind == MLSTM) {
+        if (f32) PICK(float, MLSTM); else PICK(bf16_t, MLSTM);
+    } else if (kind == CHANNELS) {
+        if (f32) PICK(float, CHANNELS); else PICK(bf16_t, CHANNELS);
+    } else {
+        if (f32) PICK(float, CONSTANT); else PICK(bf16_t, CONSTANT);
+    }
 #undef PICK
 #undef GO
     LAUNCH_CHECK();
@@ -2208,27 +2594,50 @@ int gh_rec_out(void* stream, int f32, int silu, void* out, const void* o,
     return 0;
 }
 
-int gh_mlstm_chunks(void* stream, void* o, void* S, void* mst, void* dS,
-                    void* scal, const void* qkv, const void* gr,
+int gh_rec_row_out(void* stream, int f32, void* out, const void* o,
+                   const void* gate, const void* norm, int N, int H, int DV,
+                   int ld_, int out_ld, int true_cols, float eps) {
+    if (N < 1 || H < 1 || DV % 64 || ld_ % 4 || out_ld % 4 || true_cols < 1)
+        return -100;
+#define GO(T, NV) k_rec_row_out<T, NV><<<N, 256, 0, (hipStream_t)stream>>>( \
+        (T*)out, (const float*)o, (const T*)gate, (const float*)norm, H, DV, \
+        ld_, out_ld, true_cols, eps)
+#define PICK(T) do { if (H * DV <= 4096) GO(T, 4); \
+        else if (H * DV <= 8192) GO(T, 8); else GO(T, 0); } while (0)
+    if (f32) PICK(float); else PICK(bf16_t);
+#undef PICK
+#undef GO
+    LAUNCH_CHECK();
+    return 0;
+}
+
+// constant: lightning attention (gr: log decay by head; mst unused)
+int gh_mlstm_chunks(void* stream, int constant, void* o, void* S, void* mst,
+                    void* dS, void* scal, const void* qkv, const void* gr,
                     const void* chunks, const void* segs, int nchunks,
                     int nseg, int H, int DK, int DV, int ld_, float qscale,
                     float cap) {
-    if (nchunks < 1 || nseg < 1 || DK % 64 || DV % 64) return -100;
+    if (nchunks < 1 || nseg < 1 || DK % 64 || DV % 64 || (!constant && !mst))
+        return -100;
     hipStream_t st_ = (hipStream_t)stream;
-    k_mlstm_chunk_state<<<dim3(nchunks, H, (DK / 64) * (DV / 64)), 256, 0,
-                          st_>>>((float*)dS, (float*)scal, (const float*)mst,
-        (const bf16_t*)qkv, (const float*)gr, (const int4*)chunks,
-        (const int4*)segs, H, DK, DV, ld_, cap);
-    LAUNCH_CHECK();
-    const long quads = (long)(DV + 1) * DK / 4;
-    k_mlstm_chunk_scan<<<dim3(nseg, H, (unsigned)((quads + 255) / 256)), 256,
-                         0, st_>>>((float*)dS, (float*)scal, (float*)S,
-        (float*)mst, (const int4*)segs, H, DK, DV);
-    LAUNCH_CHECK();
-    k_mlstm_chunk_out<<<dim3(nchunks, H, (DV + 127) / 128), 256, 0, st_>>>(
-        (float*)o, (const float*)dS, (const float*)scal, (const bf16_t*)qkv,
-        (const float*)gr, (const int4*)chunks, H, DK, DV, ld_, qscale, cap);
-    LAUNCH_CHECK();
+    const long quads = (long)(DV + !constant) * DK / 4;
+#define GO(C) do { \
+    k_mlstm_chunk_state<C><<<dim3(nchunks, H, (DK / 64) * (DV / 64)), 256, 0, \
+        st_>>>((float*)dS, (float*)scal, (const float*)mst, \
+        (const bf16_t*)qkv, (const float*)gr, (const int4*)chunks, \
+        (const int4*)segs, H, DK, DV, ld_, cap); \
+    LAUNCH_CHECK(); \
+    k_mlstm_chunk_scan<C><<<dim3(nseg, H, (unsigned)((quads + 255) / 256)), \
+        256, 0, st_>>>((float*)dS, (float*)scal, (float*)S, (float*)mst, \
+        (const int4*)segs, H, DK, DV); \
+    LAUNCH_CHECK(); \
+    k_mlstm_chunk_out<C><<<dim3(nchunks, H, (DV + 127) / 128), 256, 0, \
+        st_>>>((float*)o, (const float*)dS, (const float*)scal, \
+        (const bf16_t*)qkv, (const float*)gr, (const int4*)chunks, H, DK, DV, \
+        ld_, qscale, cap); \
+    LAUNCH_CHECK(); } while (0)
+    if (constant) GO(true); else GO(false);
+#undef GO
     return 0;
 }
 
@@ -2272,13 +2681,15 @@ int gh_gla_chunks(void* stream, void* o, void* S, void* dS, const void* qkv,
     return 0;
 }
 
-// E router outputs, of which the first `experts` have weights. corr (nullable):
-// correction of the choice; ident (nullable): sum of a token's weights beyond
+// E router outputs (rows of stride ldz), of which the first `experts` have
+// weights. corr (nullable): correction of the choice; ident (nullable): sum of a token's weights beyond
 // the experts
 int gh_moe_route(void* stream, void* idx, void* wt, void* rank, void* counts,
-                 void* sorted, void* tiles, const void* z, const void* corr,
-                 void* ident, int N, int E, int experts, int top, int groups,
-                 int keep, float eps, float scale, int bm, int max_tiles) {
+                 void* sorted, void* tiles, const void* z, int ldz,
+                 const void* corr, void* ident, int N, int E, int experts, int top, int groups,
+                 int keep, float eps, float scale, int sigmoid, int bm,
+                 int max_tiles) {
+    if (ldz < E || (sigmoid && (corr || ident))) return -100;
     if (N < 1 || E < 1 || E > 1024 || top < 1 || experts < 1 || experts > E ||
         groups < 1 || E % groups || keep < 1 || keep > groups ||
         top > E / groups * keep)
@@ -2286,8 +2697,8 @@ int gh_moe_route(void* stream, void* idx, void* wt, void* rank, void* counts,
     hipStream_t st_ = (hipStream_t)stream;
 #define GO(V) k_moe_route<V><<<(N + 4 * tpw - 1) / (4 * tpw), 256, 0, st_>>>((int*)idx, \
         (float*)wt, (int*)rank, (int*)counts, (const float*)z, \
-        (const float*)corr, (float*)ident, N, E, experts, top, groups, keep, \
-        eps, scale, tpw)
+        ldz, (const float*)corr, (float*)ident, N, E, experts, top, groups, \
+        keep, eps, scale, sigmoid, tpw)
     const int tpw = min(max(N / 2048, 1), 16);
     if (E <= 64) GO(1);
     else if (E <= 128) GO(2);
@@ -2304,14 +2715,17 @@ int gh_moe_route(void* stream, void* idx, void* wt, void* rank, void* counts,
 }
 
 // act: 0 down, 1 up with squared ReLU, 2 gate and up (N weight rows, in turns
-// of 16 | 16). bm: rows per tile of the list: 16 (few pairs; the exact mode) or
+// of 16 | 16) with the gated unit's constants; pw (nullable): weights of the
+// pairs on its input. bm: rows per tile of the list: 16 (few pairs; the exact mode) or
 // 128
 int gh_moe_gemm(void* stream, int f32, int act, void* out, const void* x,
                 const void* w, const void* tiles, const void* sorted,
-                int top, int N, int K, int bm, int max_tiles) {
+                int top, int N, int K, int bm, int max_tiles, float alpha,
+                float limit, float shift, float cubic, const void* pw) {
     if (N % (act == 2 ? 128 : 64) || K % 64 || max_tiles < 1 || act < 0 ||
         act > 2)
         return -100;
+    const GluParams glu{alpha, limit, shift, cubic};
     hipStream_t st_ = (hipStream_t)stream;
     if (f32) {
         if (bm != 16) return -103;
@@ -2319,14 +2733,15 @@ int gh_moe_gemm(void* stream, int f32, int act, void* out, const void* x,
         const unsigned grid = (unsigned)((max_tiles * ntn + 7) / 8 * 8);
 #define GO(U) k_moe_gemm_f32<U><<<grid, 256, 0, st_>>>((float*)out, \
         (const float*)x, (const float*)w, (const int4*)tiles, \
-        (const int*)sorted, top, N, K, ntn, max_tiles)
+        (const int*)sorted, top, N, K, ntn, max_tiles, glu, (const float*)pw)
         if (act == 2) GO(2); else if (act) GO(1); else GO(0);
 #undef GO
         LAUNCH_CHECK();
         return 0;
     }
 #define ARGS (bf16_t*)out, (const bf16_t*)x, (const bf16_t*)w, \
-        (const int4*)tiles, (const int*)sorted, top, N, K, ntn, max_tiles
+        (const int4*)tiles, (const int*)sorted, top, N, K, ntn, max_tiles, \
+        glu, (const float*)pw
     if (bm == 128) {
         const int ntn = (N + 127) / 128;
         const unsigned grid = (unsigned)((max_tiles * ntn + 7) / 8 * 8);

@@ -748,9 +748,11 @@ static int launch_attn_decode(hipStream_t st, bf16_t* out, const bf16_t* q,
     switch (G) {   // compile-time G keeps softmax state in registers
 #define CASE_G(GG) \
         case GG: if (onewave) k_attn_decode1<D, GG><<<grid, dim3(64), 0, st>>>( \
-                out, q, kv, seqlen, 0, slot_map, ws, 1, nsplit, scale, epi); \
+                out, q, kv, seqlen, 0, slot_map, ws, 1, nsplit, scale, epi, \
+                AllKeys()); \
             else k_attn_decode<D, GG><<<grid, dim3(256), 0, st>>>( \
-                out, q, kv, seqlen, 0, slot_map, ws, 1, nsplit, scale, epi); \
+                out, q, kv, seqlen, 0, slot_map, ws, 1, nsplit, scale, epi, \
+                AllKeys()); \
             break;
         CASE_G(1) CASE_G(2) CASE_G(3) CASE_G(4)
         CASE_G(5) CASE_G(6) CASE_G(7) CASE_G(8)

@@ -1,7 +1,8 @@
 """Layer-list models: a decoder in which every layer names its mixer (softmax,
-latent or talking-heads attention over a paged cache, mLSTM or gated linear
-attention with a state per sequence) and its feed-forward (dense gated, dense
-with PolyNorm, or routed experts).
+latent or talking-heads attention over a paged cache, mLSTM, gated linear or
+lightning attention with a state per sequence, or attention and a recurrence
+side by side) and its feed-forward (dense gated, dense with PolyNorm, or routed
+experts, with or without a shared one).
 
 One step function serves prompts, portions of prompts and decoding, also mixed
 in one batch: `forward_step`. Its tokens are ordered decode rows first, so each
@@ -30,14 +31,15 @@ import torch
 from gridllm_amd.models.paged import (PAGE, PagedCache, head_pad, latent_pad,
                                       pad64, rotated_pad)
 from gridllm_amd.models.registry import (AttentionMixer, DenseFF, GlaMixer,
-                                         HybridSpec, LatentMixer, PolyFF,
-                                         RoutedFF, TalkingMixer)
+                                         HybridSpec, LatentMixer,
+                                         LightningMixer, ParallelMixer, PolyFF,
+                                         Rotary, RoutedFF, TalkingMixer)
 from gridllm_amd.ops import hybrid as hops
 from gridllm_amd.ops.autotune import linear as _linear
 from gridllm_amd.ops.autotune import linear_gateup as _linear_gateup
-from gridllm_amd.ops.hybrid import (ChunkPortions, Choice, DepthAverage,
+from gridllm_amd.ops.hybrid import (ChunkPortions, Choice, DepthAverage, Keys,
                                     StepMeta, Talk)
-from gridllm_amd.ops.reference import Glu
+from gridllm_amd.ops.reference import SWIGLU, Glu
 from gridllm_amd.parallel.tp import TPContext
 
 _DTYPES = {"bf16": torch.bfloat16, "fp32": torch.float32}
@@ -51,7 +53,8 @@ _ABSORB = 16
 class BlockWeights:
     """One layer's tensors, fused and padded. Dense: gateup and down are 2-D;
     routed: up [E, F, W] (gated: [E, 2 F, W], rows in turns of 16 gate | 16
-    up), down [E, W, F]."""
+    up), down [E, W, F]; gateup and sdown are the shared expert's, and the last
+    row of router is its gate's."""
     wmix: torch.Tensor                    # q, k, v, output gate; or the
                                           # projections to latents, gate
     wo: torch.Tensor
@@ -73,11 +76,17 @@ class BlockWeights:
     act: Optional[torch.Tensor] = None        # PolyNorm's numbers
     pre1: Optional[torch.Tensor] = None       # norms ahead of the sublayers
     pre2: Optional[torch.Tensor] = None
+    decay: Optional[torch.Tensor] = None      # by head: decays, logarithms
+    hc1: Optional[torch.Tensor] = None        # streams: mix, then put
+    hc2: Optional[torch.Tensor] = None
+    read1: Optional[torch.Tensor] = None      # weights of what is read
+    read2: Optional[torch.Tensor] = None
     corr: Optional[torch.Tensor] = None
     avg: Optional[torch.Tensor] = None        # depth average
     wgateup: Optional[torch.Tensor] = None
     up: Optional[torch.Tensor] = None
     down: Optional[torch.Tensor] = None
+    sdown: Optional[torch.Tensor] = None
     router: Optional[torch.Tensor] = None
 
 
@@ -103,6 +112,11 @@ def _pair_order(dim: int, rot_dims: int) -> torch.Tensor:
     i = torch.arange(rot_dims // 2)
     pairs = torch.stack([i, i + rot_dims // 2], dim=1).flatten()
     return torch.cat([pairs, torch.arange(rot_dims, dim)])
+
+
+def _glu(ff: Optional[DenseFF]) -> Glu:
+    return SWIGLU if ff is None else Glu(ff.alpha, ff.limit, ff.shift,
+                                         ff.cubic)
 
 
 class HybridModel:
@@ -153,30 +167,35 @@ class HybridModel:
             self._init_weights(seed)
 
     def _rotations(self) -> list[Optional[tuple]]:
-        """Per latent- or talking-heads-attention layer, cos and sin of position
+        """Per layer with rotated queries and keys, cos and sin of position
         times frequency, f32 [rows, R / 2] for the positions of whole pages; 1
         and 0 for pairs that are not rotated."""
         rows = pad64(self.max_seq)
         made: dict[tuple, tuple] = {}
 
-        def table(mx) -> tuple:
-            r = latent_pad(mx)[1] if isinstance(mx, LatentMixer) else \
-                rotated_pad(mx)
-            key = (mx.rot_base, mx.rot_dims, r)
-            if key not in made:
-                half = mx.rot_dims // 2
-                f = mx.rot_base ** (-torch.arange(half, dtype=torch.float64)
-                                    / max(half, 1))
-                a = torch.zeros(rows, r // 2, dtype=torch.float64)
-                a[:, :half] = torch.outer(
-                    torch.arange(rows, dtype=torch.float64), f)
-                made[key] = tuple(t.float().to(self.device).contiguous()
-                                  for t in (a.cos(), a.sin()))
-            return made[key]
+        def table(mx) -> Optional[tuple]:
+            if isinstance(mx, AttentionMixer):
+                rot = mx.rot
+                r = -(-rot.dims // 8) * 8 if rot else 0
+            elif mx is not None:
+                rot = Rotary(mx.rot_base, mx.rot_dims)
+                r = latent_pad(mx)[1] if isinstance(mx, LatentMixer) else \
+                    rotated_pad(mx)
+            if mx is None or rot is None:
+                return None
+            if (rot, r) not in made:
+                f, grow = rot.frequencies()
+                half = len(f)
+                a = torch.outer(torch.arange(rows, dtype=torch.float64),
+                                torch.tensor(f, dtype=torch.float64))
+                cos = torch.ones(rows, r // 2, dtype=torch.float64)
+                sin = torch.zeros_like(cos)
+                cos[:, :half], sin[:, :half] = a.cos() * grow, a.sin() * grow
+                made[rot, r] = tuple(t.float().to(self.device).contiguous()
+                                     for t in (cos, sin))
+            return made[rot, r]
 
-        return [table(ly.mixer)
-                if isinstance(ly.mixer, (LatentMixer, TalkingMixer)) else None
-                for ly in self.spec.layers]
+        return [table(ly.attention()) for ly in self.spec.layers]
 
     # -- weights -----------------------------------------------------------
 
@@ -197,10 +216,14 @@ class HybridModel:
                 out[f"l{i}.dwa"] = (i + 2,)
             if ly.weights_of is not None:
                 continue
-            p, mx, ff = f"l{i}.", ly.mixer, ly.ff
+            p, mx, ff = f"l{s.number(i)}.", ly.mixer, ly.ff
             out |= self._mixer_shapes(p + "mix.", mx)
             for k in (1, 2) if ff is not None else (1,):
                 out[f"{p}norm{k}"] = norm
+                if s.streams:
+                    out |= {f"{p}hc{k}.in": (s.streams,),
+                            f"{p}hc{k}.out": (s.streams,),
+                            f"{p}hc{k}.mix": (s.streams, s.streams)}
                 if s.pre_norms:
                     out[f"{p}norm{k}b"] = norm
                 if s.layer_scale:
@@ -223,9 +246,17 @@ class HybridModel:
                         f"{p}mlp.e{e}.down": (w, ff.ff)}
                 if ff.gated:
                     out[f"{p}mlp.e{e}.gate"] = (ff.ff, w)
+            if ff.shared is not None:
+                out |= {p + "mlp.shared.gate": (ff.shared.ff, w),
+                        p + "mlp.shared.up": (ff.shared.ff, w),
+                        p + "mlp.shared.down": (w, ff.shared.ff),
+                        p + "mlp.shared.sg": (1, w)}
         return out
 
     def _mixer_shapes(self, p: str, mx) -> dict[str, tuple]:
+        if isinstance(mx, ParallelMixer):
+            return self._mixer_shapes(p + "left.", mx.left) | \
+                self._mixer_shapes(p + "right.", mx.right)
         w, h = self.spec.hidden, mx.heads
         if isinstance(mx, LatentMixer):
             qr, k = mx.q_rank, mx.kv_rank
@@ -245,8 +276,13 @@ class HybridModel:
         out = {p + "q": (h * mx.dim, w), p + "k": (kv * mx.dim, w),
                p + "v": (kv * mx.vdim, w), p + "o": (w, h * mx.vdim)}
         if attn:
-            return out | {p + "sink": (h,), p + "g": (h, w)}
+            if mx.sink:
+                out[p + "sink"] = (h,)
+            gates = h * mx.vdim if mx.gate == "element" else h
+            return out | {p + "g": (gates, w)}
         out[p + "g"] = (h * mx.vdim, w)
+        if isinstance(mx, LightningMixer):
+            return out | {p + "norm": (h * mx.vdim,)}
         if isinstance(mx, GlaMixer):
             return out | {p + "norm": (mx.vdim,), p + "a1": (mx.rank, w),
                           p + "a2": (h * mx.dim, mx.rank),
@@ -272,6 +308,12 @@ class HybridModel:
                 return torch.ones(sh, device=self.device)
             if last in ("ls1", "ls2"):
                 return torch.ones(sh, device=self.device)
+            if last == "in":               # streams: read their mean, add the
+                return torch.full(sh, 1.0 / sh[0], device=self.device)
+            if last == "out":              # result to all, keep them apart
+                return torch.ones(sh, device=self.device)
+            if last == "mix":
+                return torch.eye(sh[0], device=self.device)
             if last == "act":              # odd powers, as an activation's
                 return torch.tensor([0.5, 0.0, 0.5, 0.0], device=self.device)
             if last == "talk":             # mostly each head's own weights
@@ -363,6 +405,7 @@ class HybridModel:
         return dict(
             wmix=wmix, wuq=uq.reshape(h * (pd + r), qr).contiguous(),
             wuk=uk.transpose(1, 2).contiguous(), wuv=uv.contiguous(),
+            wo=_pad_heads(get(p + "o").to(self.dtype).T, h, pd).T,
             wukv=torch.cat([uk, uv], dim=1).contiguous()
             if self.dtype == torch.bfloat16 else None,
             qnorm=_pad(get(p + "dq.norm").float(), qr),
@@ -402,22 +445,26 @@ class HybridModel:
                       *((talk16, 2.0 ** (lift - 14)) if nh <= 4 else ())))
 
     def _assemble_layer(self, i: int, ly, get, mat, norm) -> BlockWeights:
-        s, mx, ff, wp, p = self.spec, ly.mixer, ly.ff, self.width, f"l{i}."
-        h = mx.heads
+        s, mx, ff, wp = self.spec, ly.mixer, ly.ff, self.width
+        p = f"l{s.number(i)}."
         if isinstance(mx, TalkingMixer):
             parts = self._assemble_talk(i, mx, get, mat)
-            dv = head_pad(mx)
         elif isinstance(mx, LatentMixer):
             parts = self._assemble_latent(p + "mix.", mx, get, mat)
-            dv = head_pad(mx)
+        elif isinstance(mx, ParallelMixer):
+            # one row of projections, and one output projection: the parts'
+            # scales go into the kernels behind which their outputs are rounded
+            parts = self._assemble_rows(p + "mix.left.", mx.left, get, mat)
+            right = self._assemble_rows(p + "mix.right.", mx.right, get, mat)
+            for name, dim in (("wmix", 0), ("wo", 1)):
+                right[name] = torch.cat([parts[name], right[name]], dim=dim)
+            right["mnorm"] = right["mnorm"] * mx.right_scale
+            parts |= right
         else:
-            parts, dv = self._assemble_rows(p + "mix.", mx, get, mat)
+            parts = self._assemble_rows(p + "mix.", mx, get, mat)
         wmix = parts.pop("wmix")
         wmix = _pad(wmix, -(-wmix.shape[0] // 128) * 128, wp).contiguous()
-        # columns of the output projection follow the padded heads
-        wo = parts.pop("wo", None)
-        if wo is None:
-            wo = _pad_heads(get(p + "mix.o").to(self.dtype).T, h, dv).T
+        wo = parts.pop("wo")
 
         def norms(k):               # behind a sublayer (scaled), ahead of it
             t = norm(get(f"{p}norm{k}b" if s.pre_norms else f"{p}norm{k}"))
@@ -425,25 +472,42 @@ class HybridModel:
                 t *= _pad(get(f"{p}ls{k}").float(), wp)
             return t, norm(get(f"{p}norm{k}")) if s.pre_norms else None
 
+        def streams(k):             # how a sublayer mixes them, and reads
+            if not s.streams:
+                return None, None
+            t = f"{p}hc{k}."
+            return torch.cat([get(t + "mix").float().flatten(),
+                              get(t + "out").float()]), \
+                get(t + "in").float().contiguous()
+
         norm1, pre1 = norms(1)
         w = BlockWeights(
-            wmix=wmix, wo=_pad(wo, wp, h * dv).contiguous(),
+            wmix=wmix, wo=_pad(wo, wp, wo.shape[1]).contiguous(),
             norm1=norm1, pre1=pre1, **parts)
+        w.hc1, w.read1 = streams(1)
         if ff is None:
             return w
         w.norm2, w.pre2 = norms(2)
+        w.hc2, w.read2 = streams(2)
         fp = pad64(ff.ff)
         if isinstance(ff, PolyFF):
             w.up = mat(get(p + "mlp.up"), fp).contiguous()
             w.down = mat(get(p + "mlp.down"), wp)
             w.act = get(p + "mlp.act").float().contiguous()
             return w
+        def gated(t, n):
+            return torch.cat([mat(get(t + "gate"), n), mat(get(t + "up"), n)])
+
         if isinstance(ff, DenseFF):
-            w.wgateup = torch.cat([mat(get(p + "mlp.gate"), fp),
-                                   mat(get(p + "mlp.up"), fp)])
+            w.wgateup = gated(p + "mlp.", fp)
             w.down = mat(get(p + "mlp.down"), wp)
             return w
         w.router = mat(get(p + "mlp.router"))
+        if ff.shared is not None:
+            t = p + "mlp.shared."
+            w.wgateup = gated(t, pad64(ff.shared.ff))
+            w.sdown = mat(get(t + "down"), wp)
+            w.router = torch.cat([w.router, mat(get(t + "sg"))])
         if ff.corrected:
             w.corr = get(p + "mlp.correction").float().contiguous()
         w.up = torch.empty(ff.experts, fp * (2 if ff.gated else 1), wp,
@@ -460,21 +524,29 @@ class HybridModel:
             w.down[e] = mat(get(f"{p}mlp.e{e}.down"), wp)
         return w
 
-    def _assemble_rows(self, p: str, mx, get, mat) -> tuple[dict, int]:
-        """Tensors of a mixer with one row [q | k | v | output gate], and its
-        padded value size."""
+    def _assemble_rows(self, p: str, mx, get, mat) -> dict:
+        """Tensors of a mixer with one row [q | k | v | output gate]."""
         h = mx.heads
         attn = isinstance(mx, AttentionMixer)
         kv = mx.kv_heads if attn else h
         dk = head_pad(mx) if attn else pad64(mx.dim)
         dv = dk if attn else pad64(mx.vdim)
         g = mat(get(p + "g"))
+        by_head = attn and mx.gate == "head"
         out = {"wmix": torch.cat([_pad_heads(mat(get(p + "q")), h, dk),
                                   _pad_heads(mat(get(p + "k")), kv, dk),
                                   _pad_heads(mat(get(p + "v")), kv, dv),
-                                  g if attn else _pad_heads(g, h, dv)])}
+                                  g if by_head else _pad_heads(g, h, dv)]),
+               # columns follow the padded heads
+               "wo": _pad_heads(get(p + "o").to(self.dtype).T, h, dv).T}
         if attn:
-            out["sink"] = get(p + "sink").float()
+            if mx.sink:
+                out["sink"] = get(p + "sink").float()
+        elif isinstance(mx, LightningMixer):
+            d = torch.tensor(mx.decay, dtype=torch.float64)
+            out["decay"] = torch.stack([d, d.clamp(min=1e-30).log()]).float() \
+                .to(self.device).contiguous()
+            out["mnorm"] = _pad_heads(get(p + "norm").float(), h, dv)
         elif isinstance(mx, GlaMixer):
             out["wgates"] = mat(get(p + "a1")).contiguous()
             wa2 = _pad_heads(get(p + "a2").float(), h, dk)
@@ -487,7 +559,7 @@ class HybridModel:
             out["bgates"] = torch.cat([get(p + "i.b"),
                                        get(p + "f.b")]).float()
             out["mnorm"] = _pad_heads(get(p + "norm").float(), h, dv)
-        return out, dv
+        return out
 
     def unique_layers(self) -> list[BlockWeights]:
         return list({id(w): w for w in self.layers}.values())
@@ -502,7 +574,8 @@ class HybridModel:
                 plain.add(tuple(w.wuq.shape))
             if w.wgateup is not None:
                 gu.add(tuple(w.wgateup.shape))
-                plain.add(tuple(w.down.shape))
+                plain.add(tuple((w.down if w.sdown is None
+                                 else w.sdown).shape))
             if w.act is not None:
                 plain |= {tuple(w.up.shape), tuple(w.down.shape)}
         return sorted(plain), sorted(gu)
@@ -537,13 +610,23 @@ class HybridModel:
              st: StepMeta) -> torch.Tensor:
         c, eps = self.cache, self.spec.norm_eps
         rows = _linear(xb, w.wmix)
-        if isinstance(mx, AttentionMixer):
-            h, g, p = mx.heads, mx.kv_heads, c.k[i].shape[3]
-            q = hops.qknorm_kv(rows, c.k[i], c.v[i], st, h, g, mx.dim, eps,
-                               mx.q_coef, mx.q_every)
-            gate = rows[:, (h + 2 * g) * p:(h + 2 * g) * p + h]
-            o = hops.paged_attn(q, c.k[i], c.v[i], st, mx.scale, w.sink,
-                                gate).view(xb.shape[0], -1)
+        if isinstance(mx, ParallelMixer):
+            o = torch.empty(xb.shape[0], w.wo.shape[1], dtype=xb.dtype,
+                            device=xb.device)
+            at = self._attend(i, w, mx.left, rows, st, o, mx.left_scale,
+                              mx.right)
+            hops.lightning(rows[:, at:], c.S[i], w.decay, w.mnorm, st,
+                           mx.right.vdim, eps,
+                           o[:, mx.left.heads * c.k[i].shape[3]:])
+        elif isinstance(mx, LightningMixer):
+            dv, dk = c.S[i].shape[2:]
+            hops.silu_cols(rows, 0, mx.heads * (2 * dk + dv))
+            o = hops.lightning(rows, c.S[i], w.decay, w.mnorm, st, mx.vdim,
+                               eps)
+        elif isinstance(mx, AttentionMixer):
+            o = torch.empty(xb.shape[0], w.wo.shape[1], dtype=xb.dtype,
+                            device=xb.device)
+            self._attend(i, w, mx, rows, st, o)
         elif isinstance(mx, LatentMixer):
             cq = hops.latent_rows(rows, c.lat[i], st, self.rot[i], w.qnorm,
                                   w.kvnorm, mx.q_rank, mx.kv_rank, eps)
@@ -565,30 +648,65 @@ class HybridModel:
                            mx.vdim, mx.gate_cap, eps)
         return _linear(o, w.wo)
 
+    def _attend(self, i: int, w: BlockWeights, mx: AttentionMixer,
+                rows: torch.Tensor, st: StepMeta, out: torch.Tensor,
+                scale: float = 1.0,
+                right: Optional[LightningMixer] = None) -> int:
+        """Attention of projection rows [q | k | v | gate | ...] into the first
+        columns of out, times scale; returns where its part of the rows ends.
+        `right` is a recurrence whose part follows: its q, k and v get SiLU."""
+        c, h, g = self.cache, mx.heads, mx.kv_heads
+        p = c.k[i].shape[3]
+        at = (h + 2 * g) * p
+        end = at + (h * p if mx.gate == "element" else h)
+        silu = (0, 0)
+        if right is not None:
+            dv, dk = c.S[i].shape[2:]
+            silu = (end, right.heads * (2 * dk + dv))
+        q = hops.qknorm_kv(rows, c.k[i], c.v[i], st, h, g, mx.dim,
+                           self.spec.norm_eps, mx.q_coef, mx.q_every,
+                           self.rot[i], silu)
+        hops.paged_attn(q, c.k[i], c.v[i], st, mx.scale, w.sink,
+                        rows[:, at:end], Keys(mx.window, mx.keep_first),
+                        out[:, :h * p], scale)
+        return end
+
+    def _gated(self, w: BlockWeights, ff: DenseFF,
+               xb: torch.Tensor) -> torch.Tensor:
+        if self.gateup_il:
+            return _linear_gateup(xb, w.wgateup, _glu(ff))
+        return hops.glu(_linear(xb, w.wgateup), _glu(ff))
+
     def _feed(self, w: BlockWeights, ff, xb: torch.Tensor):
         """Feed-forward output, and, if it is still a row per (token, chosen
-        expert), the pairs' weights and those of identity experts."""
+        expert), the pairs' weights and those of identity experts; with weighted
+        inputs the rows just add up."""
         if isinstance(ff, DenseFF):
-            glu = Glu(ff.alpha, ff.limit, ff.shift, ff.cubic)
-            act = _linear_gateup(xb, w.wgateup, glu) if self.gateup_il else \
-                hops.glu(_linear(xb, w.wgateup), glu)
-            return _linear(act, w.down), None, None
+            return _linear(self._gated(w, ff, xb), w.down), None, None
         if isinstance(ff, PolyFF):
             z = hops.poly_norm(_linear(xb, w.up), w.act, ff.ff,
                                self.spec.norm_eps)
             return _linear(z, w.down), None, None
         assert isinstance(ff, RoutedFF)
-        how = Choice(ff.top, w.corr, ff.groups, ff.keep,
-                     1e-20 if ff.corrected else 0.0, ff.scale)
-        return hops.moe(xb, hops.proj_f32(xb, w.router), w.up, w.down, how)
+        return hops.moe(xb, hops.proj_f32(xb, w.router), w.up, w.down,
+                        self._choice(w, ff))
+
+    @staticmethod
+    def _choice(w: BlockWeights, ff: RoutedFF) -> Choice:
+        return Choice(ff.top, w.corr, ff.groups, ff.keep,
+                      1e-20 if ff.corrected else 0.0, ff.scale, ff.sigmoid,
+                      ff.weigh_input, _glu(ff.unit))
 
     def _run(self, tokens: torch.Tensor, st: StepMeta,
              trail: Optional[list] = None) -> torch.Tensor:
-        """The residual stream behind the last layer, f32 [n, W]; trail
-        collects it behind every layer."""
+        """The residual stream behind the last layer, f32 [n, W] (or all of
+        them, [n, streams, W]); trail collects it (or their sum) behind every
+        layer."""
         s = self.spec
         if s.pre_norms:
             return self._run_between_norms(tokens, st, trail)
+        if s.streams:
+            return self._run_streams(tokens, st, trail)
         n, size, norm = tokens.shape[0], (s.hidden, s.norm_eps), self.norm_off
         hist = None
         if s.depth_average:
@@ -644,9 +762,49 @@ class HybridModel:
                 trail.append(x[:, :s.hidden].clone())
         return x
 
+    def _run_streams(self, tokens: torch.Tensor, st: StepMeta,
+                     trail: Optional[list]) -> torch.Tensor:
+        """_run for several residual streams: taking a sublayer's output in and
+        reading the next one's input are one kernel."""
+        s, run = self.spec, self.layers
+        size = (s.hidden, s.norm_eps)
+        x, h = hops.streams_start(tokens, self.embed, s.embed_scale,
+                                  run[0].read1, run[0].norm1, *size)
+        for i, (ly, w) in enumerate(zip(s.layers, run)):
+            ahead = (run[i + 1].read1, run[i + 1].norm1) \
+                if i + 1 < len(run) else (None, None)
+            y = self._mix(i, w, ly.mixer, h, st)
+            h = hops.streams_join(x, y, w.hc1, *(
+                ahead if ly.ff is None else (w.read2, w.norm2)), *size)
+            if isinstance(ly.ff, RoutedFF):
+                y, extra = self._feed_pairs(w, ly.ff, h)
+                h = hops.streams_join(x, y, w.hc2, *ahead, *size, ly.ff.top,
+                                      extra)
+            elif ly.ff is not None:
+                h = hops.streams_join(x, self._feed(w, ly.ff, h)[0], w.hc2,
+                                      *ahead, *size)
+            if trail is not None:
+                trail.append(x[..., :s.hidden].sum(1))
+        return x
+
+    def _feed_pairs(self, w: BlockWeights, ff: RoutedFF, h: torch.Tensor
+                    ) -> tuple[torch.Tensor, Optional[tuple]]:
+        """Experts' outputs by (token, chosen expert), which just add up; and
+        the shared expert's with the logits of its gate."""
+        z = hops.proj_f32(h, w.router)
+        y, _, _ = hops.moe(h, z[:, :ff.outputs], w.up, w.down,
+                           self._choice(w, ff))
+        if ff.shared is None:
+            return y, None
+        return y, (_linear(self._gated(w, ff.shared, h), w.sdown),
+                   z[:, ff.outputs:])
+
     def _normed(self, x: torch.Tensor, rows: Optional[torch.Tensor],
                 w: torch.Tensor) -> torch.Tensor:
         s = self.spec
+        if s.streams:
+            return hops.streams_norm(x, rows, w, s.hidden, s.norm_eps,
+                                     self.dtype)
         if s.norm_groups > 1:
             return hops.group_norm(x, rows, w, s.norm_groups, s.hidden,
                                    s.norm_eps, self.dtype)

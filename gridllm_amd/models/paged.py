@@ -27,7 +27,8 @@ import torch
 
 from gridllm_amd.models.registry import (AttentionMixer, GlaMixer,
                                          HybridSpec, LatentMixer,
-                                         TalkingMixer)
+                                         LightningMixer, MlstmMixer,
+                                         ParallelMixer, TalkingMixer)
 
 PAGE = 64
 
@@ -87,7 +88,9 @@ class PagedCache:
         self.S: list[Optional[torch.Tensor]] = []
         self.m: list[Optional[torch.Tensor]] = []
         for ly in spec.layers:
-            mx = ly.mixer
+            mx = rec = ly.mixer
+            if isinstance(mx, ParallelMixer):     # pages and a state
+                mx, rec = mx.left, mx.right
             k = v = lat = inv = s = m = None
             if isinstance(mx, AttentionMixer):
                 shape = (pages + 1, mx.kv_heads, PAGE, head_pad(mx))
@@ -101,13 +104,13 @@ class PagedCache:
                 v = torch.zeros(*shape, head_pad(mx), dtype=dtype,
                                 device=device)
                 inv = torch.zeros(shape, device=device)
-            elif isinstance(mx, GlaMixer):
-                s = torch.zeros(slots, mx.heads, pad64(mx.vdim),
-                                pad64(mx.dim), device=device)
-            else:
-                s = torch.zeros(slots, mx.heads, pad64(mx.vdim) + 1,
-                                pad64(mx.dim), device=device)
-                m = torch.zeros(slots, mx.heads, device=device)
+            if isinstance(rec, (GlaMixer, LightningMixer)):
+                s = torch.zeros(slots, rec.heads, pad64(rec.vdim),
+                                pad64(rec.dim), device=device)
+            elif isinstance(rec, MlstmMixer):
+                s = torch.zeros(slots, rec.heads, pad64(rec.vdim) + 1,
+                                pad64(rec.dim), device=device)
+                m = torch.zeros(slots, rec.heads, device=device)
             self.k.append(k)
             self.v.append(v)
             self.lat.append(lat)

@@ -68,10 +68,51 @@ class ModelSpec:
 
 
 @dataclass(frozen=True)
+class Yarn:
+    """YaRN: pairs that turn fewer than `slow` times within the `original`
+    length turn `factor` times slower, those that turn more than `fast` times
+    keep their speed, those between are interpolated; cosines and sines grow by
+    0.1 ln(factor) + 1."""
+    factor: float
+    original: int
+    fast: float
+    slow: float
+
+
+@dataclass(frozen=True)
+class Rotary:
+    """Neighbouring pairs of a head's first `dims` coordinates turn by
+    p base^(-2 i / dims)."""
+    base: float
+    dims: int
+    scaling: Optional[Yarn] = None
+
+    def frequencies(self) -> tuple[list[float], float]:
+        """Angle of each pair per position, and the factor on cosines and
+        sines."""
+        d, y = self.dims, self.scaling
+        f = [self.base ** (-2 * i / d) for i in range(d // 2)]
+        if y is None:
+            return f, 1.0
+
+        def pair(turns: float) -> float:
+            return d * math.log(y.original / (2 * math.pi * turns)) \
+                / (2 * math.log(self.base))
+
+        lo = max(math.floor(pair(y.fast)), 0)
+        hi = min(math.ceil(pair(y.slow)), d - 1)
+        slower = [min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+                  for i in range(d // 2)]
+        return [a / y.factor * r + a * (1 - r) for a, r in zip(f, slower)], \
+            0.1 * math.log(y.factor) + 1
+
+
+@dataclass(frozen=True)
 class AttentionMixer:
-    """Grouped softmax attention: unit-RMS q and k, a query temperature
-    1 + q_coef ln(floor((p + 1) / q_every) + 1), a sink term and an output
-    gate per head; no rotation."""
+    """Grouped softmax attention: rotated (if `rot`) unit-RMS q and k, a query
+    temperature 1 + q_coef ln(floor((p + 1) / q_every) + 1), a sink term, an
+    output gate per head or per element. With a window a query sees the last
+    `window` positions, its own included, and the first keep_first."""
     heads: int
     kv_heads: int
     dim: int
@@ -79,11 +120,17 @@ class AttentionMixer:
     scale: float
     q_coef: float = 0.0
     q_every: int = 1
+    rot: Optional[Rotary] = None
+    window: int = 0                # 0: all
+    keep_first: int = 0
+    sink: bool = True
+    gate: str = "head"             # or "element"
 
     def params(self, width: int) -> int:
         h, g = self.heads, self.kv_heads
-        return width * (h * self.dim + g * (self.dim + self.vdim) + h
-                        + h * self.vdim) + h
+        gates = h * self.vdim if self.gate == "element" else h
+        return width * (h * self.dim + g * (self.dim + self.vdim) + gates
+                        + h * self.vdim) + h * self.sink
 
 
 @dataclass(frozen=True)
@@ -166,6 +213,34 @@ class GlaMixer:
 
 
 @dataclass(frozen=True)
+class LightningMixer:
+    """Linear attention with SiLU on q, k and v: a matrix memory per head that
+    decays by a constant per token. The heads' outputs are normed together and
+    gated by element."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: tuple[float, ...]
+
+    def params(self, width: int) -> int:
+        return width * self.heads * (2 * self.dim + 3 * self.vdim) \
+            + self.heads * self.vdim
+
+
+@dataclass(frozen=True)
+class ParallelMixer:
+    """Attention and a recurrence on the same input; a weighted sum of their
+    outputs."""
+    left: AttentionMixer
+    right: LightningMixer
+    left_scale: float = 1.0
+    right_scale: float = 1.0
+
+    def params(self, width: int) -> int:
+        return self.left.params(width) + self.right.params(width)
+
+
+@dataclass(frozen=True)
 class DenseFF:
     """Gated feed-forward, act(g, u) = g sigmoid(alpha g (1 + cubic g^2))
     (u + shift) with g capped at limit and u clamped to +-limit."""
@@ -197,12 +272,16 @@ class PolyFF:
 
 @dataclass(frozen=True)
 class RoutedFF:
-    """Routed experts: squared ReLU, or (gated) silu(gate) * up.
+    """Routed experts: squared ReLU, or (gated) silu(gate) * up, or another
+    unit of DenseFF's form by `unit`.
 
-    Weights are the softmax scores of the chosen, made to sum to `scale`. The
-    choice is by score, plus a correction per expert if `corrected`, among the
-    `keep` of `groups` equal groups that hold the largest ones. The last
-    `identity` router outputs stand for experts that return their input."""
+    Weights are the softmax scores of the chosen, made to sum to `scale`; with
+    `sigmoid` the scores are sigmoids, and stay as they are. They multiply the
+    experts' outputs, or (weigh_input) inputs. The choice is by score, plus a
+    correction per expert if `corrected`, among the `keep` of `groups` equal
+    groups that hold the largest ones. The last `identity` router outputs stand
+    for experts that return their input. A `shared` expert takes every token,
+    its output times a sigmoid gate per token."""
     experts: int
     top: int
     ff: int
@@ -212,6 +291,10 @@ class RoutedFF:
     keep: int = 1
     identity: int = 0
     scale: float = 1.0
+    sigmoid: bool = False
+    weigh_input: bool = False
+    unit: Optional[DenseFF] = None
+    shared: Optional[DenseFF] = None
 
     @property
     def outputs(self) -> int:
@@ -220,15 +303,37 @@ class RoutedFF:
 
     def params(self, width: int) -> int:
         return self.experts * width * (3 if self.gated else 2) * self.ff \
-            + self.outputs * (width + self.corrected)
+            + self.outputs * (width + self.corrected) \
+            + (self.shared.params(width) + width if self.shared else 0)
 
 
 @dataclass(frozen=True)
 class LayerSpec:
     mixer: Union[AttentionMixer, LatentMixer, TalkingMixer, MlstmMixer,
-                 GlaMixer]
+                 GlaMixer, LightningMixer, ParallelMixer]
     ff: Union[DenseFF, PolyFF, RoutedFF, None] = None
     weights_of: Optional[int] = None
+    number: Optional[int] = None   # in tensor names; None: the layer's place
+
+    def attention(self):
+        """The mixer's attention part, if any."""
+        mx = self.mixer.left if isinstance(self.mixer, ParallelMixer) \
+            else self.mixer
+        return mx if isinstance(mx, (AttentionMixer, LatentMixer,
+                                     TalkingMixer)) else None
+
+
+def looped(layers: list[LayerSpec], start: int, stop: int,
+           times: int) -> tuple[LayerSpec, ...]:
+    """Layers in the order they run in if start .. stop - 1 run `times` times
+    in a row with the same weights."""
+    if not 0 <= start < stop <= len(layers) or times < 1:
+        raise ValueError(f"{times} loops over layers {start} .. {stop - 1} of "
+                         f"{len(layers)}")
+    again = [replace(layers[i], weights_of=i) for i in range(start, stop)]
+    return (*layers[:stop], *again * (times - 1),
+            *(replace(ly, number=i) for i, ly in enumerate(layers)
+              if i >= stop))
 
 
 @dataclass(frozen=True)
@@ -256,6 +361,11 @@ class HybridSpec:
     depth_average: bool = False
     tied: bool = True              # the head is the embedding
     logit_scale: float = 1.0
+    embed_scale: float = 1.0
+    # hyper-connections: this many residual streams x_s; a sublayer reads the
+    # norm of sum_s in[s] x_s, then x_t <- sum_s mix[s, t] x_s + out[t] y. The
+    # norm is ahead of the sublayer alone
+    streams: int = 0
 
     def __post_init__(self) -> None:
         bound = self.positions or self.max_seq_len or 8192
@@ -274,6 +384,21 @@ class HybridSpec:
             raise ValueError(f"{self.name}: norms on both sides exclude norms "
                              "behind the sum, of the embedding, and depth "
                              "averages")
+        if self.streams and (
+                self.pre_norms or self.post_alpha is not None or
+                self.depth_average or self.embed_norm or self.positions or
+                self.scalar_norms or not self.plain_norms):
+            raise ValueError(f"{self.name}: residual streams go with plain "
+                             "norms ahead of the sublayers alone")
+        if not 0 <= self.streams <= 16:
+            raise ValueError(f"{self.name}: {self.streams} residual streams")
+        if self.embed_scale != 1.0 and not self.streams:
+            raise ValueError(f"{self.name}: a scaled embedding goes with "
+                             "residual streams")
+        numbers = [self.number(i) for i, ly in enumerate(self.layers)
+                   if ly.weights_of is None]
+        if len(set(numbers)) != len(numbers):
+            raise ValueError(f"{self.name}: two layers of one number")
         for i, ly in enumerate(self.layers):
             j = self.owner(i)
             own = self.layers[j]
@@ -281,6 +406,23 @@ class HybridSpec:
                 raise ValueError(f"layer {i} uses layer {j}'s weights but "
                                  "differs from it")
             mx, ff = ly.mixer, ly.ff
+            if isinstance(mx, ParallelMixer):
+                _check_lightning(i, mx.right)
+                mx = mx.left
+            elif isinstance(mx, LightningMixer):
+                _check_lightning(i, mx)
+            if isinstance(mx, AttentionMixer):
+                if mx.rot and (mx.rot.dims % 2 or
+                               not 0 < mx.rot.dims <= mx.dim):
+                    raise ValueError(f"layer {i}: rotates {mx.rot.dims} of "
+                                     f"{mx.dim} dimensions")
+                if mx.window < 0 or mx.keep_first < 0 or \
+                        mx.gate not in ("head", "element") or \
+                        mx.sink and (mx.window or mx.gate == "element"):
+                    raise ValueError(
+                        f"layer {i}: a window of {mx.window}, the first "
+                        f"{mx.keep_first} kept, sink {mx.sink}, a gate per "
+                        f"{mx.gate}")
             if isinstance(mx, (AttentionMixer, TalkingMixer)) and \
                     mx.heads % mx.kv_heads:
                 raise ValueError(f"layer {i}: {mx.heads} heads over "
@@ -299,12 +441,28 @@ class HybridSpec:
             if self.pre_norms and isinstance(ff, RoutedFF):
                 raise ValueError(f"layer {i}: routed experts between norms")
             if isinstance(ff, RoutedFF):
+                if (ff.weigh_input or ff.unit) and not ff.gated or \
+                        ff.sigmoid and (ff.corrected or ff.groups > 1 or
+                                        ff.identity or ff.scale != 1.0):
+                    raise ValueError(f"layer {i}: weighted inputs and units "
+                                     "go with gated experts, sigmoid scores "
+                                     "with a plain choice")
+                if (ff.sigmoid or ff.weigh_input or ff.shared) and \
+                        not self.streams:
+                    raise ValueError(f"layer {i}: sigmoid scores, weighted "
+                                     "inputs and shared experts go with "
+                                     "residual streams")
                 if ff.outputs % ff.groups or not 0 < ff.keep <= ff.groups:
                     raise ValueError(f"layer {i}: {ff.keep} of {ff.groups} "
                                      f"groups of {ff.outputs} experts")
                 choice = ff.outputs // ff.groups * ff.keep
                 if not 0 < ff.top <= choice:
                     raise ValueError(f"layer {i}: top {ff.top} of {choice}")
+
+    def number(self, i: int) -> int:
+        """Layer i's number in tensor names."""
+        n = self.layers[i].number
+        return i if n is None else n
 
     def owner(self, i: int) -> int:
         """The layer whose tensors layer i uses (itself, usually)."""
@@ -318,9 +476,7 @@ class HybridSpec:
 
     def model_info(self) -> dict:
         """Ollama-style model_info of /api/show."""
-        attn = [ly.mixer for ly in self.layers
-                if isinstance(ly.mixer, (AttentionMixer, LatentMixer,
-                                         TalkingMixer))]
+        attn = [mx for ly in self.layers if (mx := ly.attention())]
         routed = [ly.ff for ly in self.layers if isinstance(ly.ff, RoutedFF)]
         f = self.family
         info = {
@@ -346,6 +502,12 @@ class HybridSpec:
                          f"{f}.attention.logit_softcapping": attn[0].cap,
                          f"{f}.rope.dimension_count": attn[0].rot_dims,
                          f"{f}.rope.freq_base": attn[0].rot_base}
+            else:
+                if attn[0].window:
+                    info[f"{f}.attention.sliding_window"] = attn[0].window
+                if attn[0].rot:
+                    info |= {f"{f}.rope.dimension_count": attn[0].rot.dims,
+                             f"{f}.rope.freq_base": attn[0].rot.base}
         if routed:
             info |= {f"{f}.expert_count": routed[0].experts,
                      f"{f}.expert_used_count": routed[0].top}
@@ -365,7 +527,14 @@ class HybridSpec:
                 total += ly.mixer.params(w) + sub
                 if ly.ff is not None:
                     total += ly.ff.params(w) + sub
+                total += (2 + self.streams) * self.streams * (
+                    1 if ly.ff is None else 2)
         return total
+
+
+def _check_lightning(i: int, mx: LightningMixer) -> None:
+    if len(mx.decay) != mx.heads or not all(0 <= d <= 1 for d in mx.decay):
+        raise ValueError(f"layer {i}: decays {mx.decay} of {mx.heads} heads")
 
 
 Spec = Union[ModelSpec, HybridSpec]
@@ -522,11 +691,84 @@ def read_vivepel(cfg: dict, name: str = "vivepel", shape=None) -> HybridSpec:
 _VIVEPEL = dict(family="vivepel", plain_norms=True, pre_norms=True,
                 layer_scale=True, tied=False)
 
+
+def _read_rotary(d: dict) -> Rotary:
+    _take(d, "rot", ("base", "dims"), ("scaling",))
+    y = d.get("scaling")
+    if y is not None:
+        _take(y, "rot scaling", ("factor", "original", "fast", "slow"))
+        y = Yarn(float(y["factor"]), y["original"], float(y["fast"]),
+                 float(y["slow"]))
+    return Rotary(float(d["base"]), d["dims"], y)
+
+
+def _read_zinavik_layer(i: int, ly: dict) -> LayerSpec:
+    _take(ly, f"layer {i}", ("type", "mixer"), ("mlp",))
+    kind, d, ff = ly["type"], ly["mixer"], ly.get("mlp")
+    if kind != "parallel":
+        raise ValueError(f"config: unknown mixer {kind!r}")
+    _take(d, kind, ("left", "right", "left_scale", "right_scale"))
+    a = _take(d["left"], "left", ("heads", "kv_heads", "dim", "vdim", "scale",
+                                  "rot", "mask"))
+    b = _take(d["right"], "right", ("heads", "dim", "vdim", "decay"))
+    mask = _take(a["mask"], "mask", ("size", "keep_first"))
+    if mask["size"] < 1:
+        raise ValueError(f"config: a window of {mask['size']}")
+    mixer = ParallelMixer(
+        AttentionMixer(heads=a["heads"], kv_heads=a["kv_heads"], dim=a["dim"],
+                       vdim=a["vdim"], scale=float(a["scale"]),
+                       rot=_read_rotary(a["rot"]), window=mask["size"],
+                       keep_first=mask["keep_first"], sink=False,
+                       gate="element"),
+        LightningMixer(b["heads"], b["dim"], b["vdim"],
+                       tuple(float(x) for x in b["decay"])),
+        float(d["left_scale"]), float(d["right_scale"]))
+    if ff is None:
+        return LayerSpec(mixer)
+    if ff.get("kind") != "moe":
+        raise ValueError(f"config: unknown mlp kind {ff.get('kind')!r}")
+    _take(ff, "moe mlp", ("kind", "expert", "router"), ("shared",))
+    e = _take(ff["expert"], "expert", ("ff", "limit"))
+    r = _take(ff["router"], "router", ("experts", "top"))
+    sh = ff.get("shared")
+    if sh is not None:
+        _take(sh, "shared expert", ("ff", "limit"))
+        sh = DenseFF(sh["ff"], float(sh["limit"]))
+    return LayerSpec(mixer, RoutedFF(
+        experts=r["experts"], top=r["top"], ff=e["ff"],
+        unit=DenseFF(e["ff"], float(e["limit"])), shared=sh, **_ZINAVIK_MOE))
+
+
+_ZINAVIK = dict(family="zinavik", plain_norms=True)
+_ZINAVIK_MOE = dict(gated=True, sigmoid=True, weigh_input=True)
+
+
+def read_zinavik(cfg: dict, name: str = "zinavik", shape=None) -> HybridSpec:
+    """Zinavik's config.json -> spec."""
+    _take(cfg, "model", ("layers", "vocab", "width", "norm", "streams",
+                         "embedding"), ("architecture", "loop"))
+    layers = [_read_zinavik_layer(i, ly) for i, ly in enumerate(cfg["layers"])]
+    loop = cfg.get("loop")
+    if loop is not None:
+        layers = looped(layers, **_take(loop, "loop", ("start", "stop",
+                                                       "times")))
+    if cfg["streams"] < 1:
+        raise ValueError(f"config: {cfg['streams']} streams")
+    return HybridSpec(
+        name=name, vocab=cfg["vocab"], hidden=cfg["width"],
+        layers=tuple(layers),
+        norm_eps=float(_take(cfg["norm"], "norm", ("eps",))["eps"]),
+        embed_scale=float(_take(cfg["embedding"], "embedding",
+                                ("scale",))["scale"]),
+        streams=cfg["streams"], **_ZINAVIK)
+
+
 # "architecture" in config.json -> reader. Checkpoints without that key (HF
 # layout) are loaded into the architecture that the model name gives.
 _READERS: dict[str, Callable[..., Spec]] = {"Birepel": read_birepel,
                                             "Maferax": read_maferax,
-                                            "Vivepel": read_vivepel}
+                                            "Vivepel": read_vivepel,
+                                            "Zinavik": read_zinavik}
 
 
 def _shape_reader(path: str) -> Callable[[str], Optional[tuple]]:
@@ -718,6 +960,45 @@ _reg(vivepel_stack("vivepel:2b", vocab=128256, hidden=3072, ff=12288,
                    attn=TalkingMixer(24, 8, 128, 128 ** -0.5, 30.0, 4096, 5e5,
                                      64)),
      "vivepel-2b")
+
+
+# Zinavik: window attention and lightning attention side by side, sigmoid-routed
+# experts beside a shared one, hyper-connections, layers that run more than once
+def zinavik_stack(name: str, *, vocab: int, hidden: int, mixer: ParallelMixer,
+                  experts: int, top: int, ff: int, shared: int, limit: float,
+                  layers: int, loop: tuple[int, int, int], streams: int,
+                  max_seq_len: int) -> HybridSpec:
+    routed = RoutedFF(experts, top, ff, unit=DenseFF(ff, limit),
+                      shared=DenseFF(shared, limit), **_ZINAVIK_MOE)
+    return HybridSpec(name, vocab=vocab, hidden=hidden,
+                      layers=looped([LayerSpec(mixer, routed)] * layers, *loop),
+                      norm_eps=1e-5, embed_scale=hidden ** 0.5,
+                      streams=streams, max_seq_len=max_seq_len, **_ZINAVIK)
+
+
+_reg(zinavik_stack("tiny-zinavik", vocab=512, hidden=128, experts=8, top=2,
+                   ff=64, shared=64, limit=7.0, layers=3, loop=(1, 2, 2),
+                   streams=2, max_seq_len=256,
+                   mixer=ParallelMixer(
+                       AttentionMixer(4, 2, 32, 32, 32 ** -0.5, window=48,
+                                      keep_first=4, sink=False, gate="element",
+                                      rot=Rotary(1e4, 16, Yarn(2.0, 128, 32.0,
+                                                               1.0))),
+                       LightningMixer(2, 32, 48, (0.9, 0.99)))),
+     "tiny-zinavik:latest")
+_reg(zinavik_stack("zinavik:4b", vocab=128256, hidden=3072, experts=64, top=7,
+                   ff=1024, shared=1024, limit=7.0, layers=6, loop=(2, 4, 2),
+                   streams=4, max_seq_len=16384,
+                   mixer=ParallelMixer(
+                       AttentionMixer(24, 8, 128, 128, 128 ** -0.5,
+                                      window=2048, keep_first=64, sink=False,
+                                      gate="element",
+                                      rot=Rotary(5e5, 128, Yarn(4.0, 4096,
+                                                                32.0, 1.0))),
+                       LightningMixer(12, 128, 256, tuple(
+                           1 - 2.0 ** (-5 - 7 * h / 11) for h in range(12))),
+                       0.5, 0.5)),
+     "zinavik-4b")
 
 
 def get_spec(name: str, max_seq_len: int = 0) -> Spec:

@@ -21,10 +21,12 @@ from gridllm_amd.ops.build import lib_path
 from gridllm_amd.ops.hip_ops import (HipExtensionMissing, _check,
                                      _check_range)
 from gridllm_amd.ops.reference import Glu
-from gridllm_amd.ops.reference_hybrid import Choice, StepMeta, Talk
+from gridllm_amd.ops.reference_hybrid import (ALL_KEYS, Choice, Keys, StepMeta,
+                                              Talk)
 
 _libs: dict[str, ctypes.CDLL] = {}
 PAGE = 64
+_MLSTM, _CHANNELS, _CONSTANT = 0, 1, 2      # kinds of recurrence
 LOG2E = 1.4426950408889634
 
 # argument kinds of each entry point after the stream: p pointer, i int,
@@ -38,17 +40,21 @@ _SIGS = {
     "gh_poly_norm": "ipppiiif",
     "gh_glu_f32": "ppliffff",
     "gh_proj_f32": "ppppiii",
-    "gh_qknorm_kv": "ipppppippiiiiiiffi",
-    "gh_paged_decode": "pppppipppiiiiifppi",
-    "gh_paged_prefill": "pppppipiiiifppi",
-    "gh_attn_rows_f32": "pppppippiiiifppi",
-    "gh_rec_step": "ippppppppiiiiiffi",
+    "gh_streams_start": "ippppfppiiiifi",
+    "gh_streams_join": "iipppippipppiiiif",
+    "gh_streams_norm": "ippppiiiif",
+    "gh_qknorm_kv": "ipppppippiiiiiiffippiiii",
+    "gh_paged_decode": "pppppipppiiiiifiippiifi",
+    "gh_paged_prefill": "pppppipiiiifiippiifi",
+    "gh_attn_rows_f32": "pppppippiiiifiippiifi",
+    "gh_rec_step": "iippppppppiiiiiffi",
+    "gh_rec_row_out": "ippppiiiiiif",
     "gh_rec_out": "iipppppppppiiiiiiiiff",
-    "gh_mlstm_chunks": "pppppppppiiiiiiff",
+    "gh_mlstm_chunks": "ipppppppppiiiiiiff",
     "gh_gla_decay": "pppppiiiif",
     "gh_gla_chunks": "pppppppiiiiiif",
-    "gh_moe_route": "pppppppppiiiiiiffii",
-    "gh_moe_gemm": "iipppppiiiii",
+    "gh_moe_route": "pppppppippiiiiiiffiii",
+    "gh_moe_gemm": "iipppppiiiiiffffp",
     "gn_latent_rows": "ippppippppppiiiiiiiif",
     "gn_head_gemm": "ippppiiiiili",
     "gn_latent_decode": "pppppipppppiiiiiiif",
@@ -251,52 +257,136 @@ def proj_f32(x: torch.Tensor, w: torch.Tensor,
     return out
 
 
+def streams_start(tok: torch.Tensor, emb: torch.Tensor, scale: float,
+                  read: torch.Tensor, w: torch.Tensor, width: int,
+                  eps: float) -> tuple[torch.Tensor, torch.Tensor]:
+    """Residual streams f32 [n, streams, W], all embed[tok] * scale, and
+    norm(sum_s read[s] x_s) * w in the weights' type. read: f32 [streams]."""
+    n, (vocab, wp), ns = tok.shape[0], emb.shape, read.shape[0]
+    _dense(tok, emb, read, w)
+    assert w.shape == (wp,) and tok.dtype == torch.int64
+    x = torch.empty(n, ns, wp, dtype=torch.float32, device=tok.device)
+    h = torch.empty(n, wp, dtype=emb.dtype, device=tok.device)
+    _call("gh_streams_start", _f32(emb), x, h, emb, tok, scale, read, w, n, ns,
+          wp, width, eps, vocab)
+    return x, h
+
+
+def streams_join(x: torch.Tensor, y: torch.Tensor, hc: torch.Tensor,
+                 read: Optional[torch.Tensor], w: Optional[torch.Tensor],
+                 width: int, eps: float, top: int = 0,
+                 extra: Optional[tuple] = None) -> Optional[torch.Tensor]:
+    """x_t <- sum_s mix[s, t] x_s + put[t] y, in place; then norm(sum_s read[s]
+    x_s) * w in y's type, if there is a w. hc f32: mix, then put. With top, y
+    [n * top, W] is first summed over a token's pairs; extra (rows [n, W], z f32
+    [n, 1], a column view is fine) adds rows times sigmoid(z)."""
+    n, ns, wp = x.shape
+    _dense(x, y, hc, read, w)
+    assert y.shape == (n * max(1, top), wp) and hc.shape == (ns * ns + ns,)
+    assert w is None or w.shape == (wp,) and read.shape == (ns,)
+    rows = z = None
+    if extra is not None:
+        rows, z = extra
+        _dense(rows)
+        assert top and rows.shape == (n, wp) and rows.dtype == y.dtype
+        assert z.shape == (n, 1) and z.dtype == torch.float32
+    h = None if w is None else torch.empty(n, wp, dtype=y.dtype,
+                                           device=y.device)
+    _call("gh_streams_join", _f32(y), int(top > 0), x, h, y, top, rows, z,
+          0 if z is None else z.stride(0), hc, read, w, n, ns, wp, width, eps)
+    return h
+
+
+def streams_norm(x: torch.Tensor, rows: Optional[torch.Tensor],
+                 w: torch.Tensor, width: int, eps: float,
+                 dtype: torch.dtype) -> torch.Tensor:
+    """norm of the streams' sum at x[rows], times w, in dtype; rows int32, None
+    for all."""
+    n, ns, wp = x.shape
+    m = n if rows is None else rows.shape[0]
+    _dense(x, rows, w)
+    assert w.shape == (wp,)
+    if rows is not None:
+        _check_range("streams_norm.rows", rows, n)
+    out = torch.empty(m, wp, dtype=dtype, device=x.device)
+    _call("gh_streams_norm", _f32(out), out, x, rows, w, m, ns, wp, width, eps)
+    return out
+
+
 def qknorm_kv(qkv: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor,
               st: StepMeta, heads: int, kv_heads: int, dim: int, eps: float,
-              coef: float, every: int) -> torch.Tensor:
+              coef: float, every: int, rot: Optional[tuple] = None,
+              silu: tuple[int, int] = (0, 0)) -> torch.Tensor:
     """Unit-RMS q (with temperature) -> [n, heads, P]; unit-RMS k and v go to
-    the pages of kc / vc [pages, kv_heads, 64, P]."""
+    the pages of kc / vc [pages, kv_heads, 64, P]. rot: cos and sin tables
+    [positions, R / 2] by which the first R coordinates of q and k turn first.
+    silu: first column and number of columns of qkv that get SiLU in place."""
     n, p = qkv.shape[0], kc.shape[3]
-    _dense(qkv, kc, vc, st.table)
+    _dense(qkv, kc, vc, st.table, *(rot or ()))
     assert qkv.shape[1] >= (heads + 2 * kv_heads) * p
+    assert sum(silu) <= qkv.shape[1]
+    assert rot is None or rot[0].shape == rot[1].shape
     _check_range("qknorm_kv.slot", st.slot, st.table.shape[0])
     q = torch.empty(n, heads, p, dtype=qkv.dtype, device=qkv.device)
+    tables = (None, None, 0, 0) if rot is None else \
+        (*rot, rot[0].shape[1], rot[0].shape[0])
     _call("gh_qknorm_kv", _f32(qkv), qkv, q, kc, vc, st.table,
           st.table.shape[1], st.pos, st.slot, n, heads, kv_heads, p,
-          qkv.shape[1], dim, eps, coef, every)
+          qkv.shape[1], dim, eps, coef, every, *tables, *silu)
     return q
+
+
+def silu_cols(rows: torch.Tensor, at: int, count: int) -> None:
+    """SiLU on `count` columns of rows from `at` on, in place."""
+    n, ld = rows.shape
+    _dense(rows)
+    assert 0 <= at and 0 < count <= ld - at
+    _call("gh_qknorm_kv", _f32(rows), rows, None, None, None, None, 0, None,
+          None, n, 0, 0, 64, ld, 1, 0.0, 0.0, 1, None, None, 0, 0, at, count)
 
 
 def paged_attn(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor,
                st: StepMeta, scale: float, sink: Optional[torch.Tensor],
-               gate: Optional[torch.Tensor]) -> torch.Tensor:
+               gate: Optional[torch.Tensor], keys: Keys = ALL_KEYS,
+               out: Optional[torch.Tensor] = None,
+               oscale: float = 1.0) -> torch.Tensor:
     """Causal attention of a step's tokens over their sequences' pages.
-    q/out [n, heads, P]; sink [heads] f32; gate [n, >= heads] (a column view
-    of the projection rows is fine)."""
+    q [n, heads, P]; sink [heads] f32; gate [n, heads], or [n, heads * P] for a
+    gate per element (a column view of the projection rows is fine). `out`
+    takes the result [n, heads * P], a column view too; oscale multiplies it.
+    Without it the result is [n, heads, P]."""
     n, h, p = q.shape
+    if out is None:
+        out = torch.empty_like(q)
+        paged_attn(q, kc, vc, st, scale, sink, gate, keys,
+                   out.view(n, h * p), oscale)
+        return out
     g = kc.shape[1]
     _dense(q, kc, vc, st.table, sink)
-    out = torch.empty_like(q)
-    ld = 0
+    assert out.shape == (n, h * p) and out.stride(1) == 1
+    ld = el = 0
     if gate is not None:
         assert gate.stride(1) == 1 and gate.dtype == q.dtype
-        ld = gate.stride(0)
+        assert gate.shape in ((n, h), (n, h * p))
+        ld, el = gate.stride(0), int(gate.shape[1] != h)
+    how = (scale, keys.window, keys.keep, sink, gate, ld, el, oscale,
+           out.stride(0))
     per = st.table.shape[1]
     if _f32(q):
         _call("gh_attn_rows_f32", out, q, kc, vc, st.table, per, st.pos,
-              st.slot, n, h, g, p, scale, sink, gate, ld)
+              st.slot, n, h, g, p, *how)
         return out
     if st.nd:
         groups = h // max(d for d in range(1, 9) if (h // g) % d == 0)
         nsplit = max(1, min(512 // max(1, st.nd * groups),
-                            (st.max_len + 255) // 256, 32))
+                            (keys.most(st.max_len) + 255) // 256, 32))
         ws = torch.empty(st.nd * h * nsplit * (p + 2), dtype=torch.float32,
                          device=q.device) if nsplit > 1 else None
         _call("gh_paged_decode", out, q, kc, vc, st.table, per, st.pos,
-              st.slot, ws, st.nd, h, g, p, nsplit, scale, sink, gate, ld)
+              st.slot, ws, st.nd, h, g, p, nsplit, *how)
     if st.tiles is not None:
         _call("gh_paged_prefill", out, q, kc, vc, st.table, per, st.tiles,
-              st.tiles.shape[0], h, g, p, scale, sink, gate, ld)
+              st.tiles.shape[0], h, g, p, *how)
     return out
 
 
@@ -319,7 +409,7 @@ def mlstm(qkv: torch.Tensor, gates: torch.Tensor, S: torch.Tensor,
         # rows of the state per block: more for large batches, where the grid
         # is full anyway and a block amortises its loads of q and k
         rpb = 128 if nseg * h * (dv + 1) >= 128 * 2048 else 32
-        _call("gh_rec_step", f, o, S, m, qkv, gates, segs, st.pos, st.slot,
+        _call("gh_rec_step", f, _MLSTM, o, S, m, qkv, gates, segs, st.pos, st.slot,
               nseg, h, dk, dv, ld, qscale, cap, rpb)
     nplain = 0
     if not f and st.chunks is not None:
@@ -328,12 +418,49 @@ def mlstm(qkv: torch.Tensor, gates: torch.Tensor, S: torch.Tensor,
         ds = torch.empty(nch, h, dv + 1, dk, dtype=torch.float32,
                          device=qkv.device)
         scal = torch.empty(nch, h, 4, dtype=torch.float32, device=qkv.device)
-        _call("gh_mlstm_chunks", o, S, m, ds, scal, qkv, gates, st.chunks,
+        _call("gh_mlstm_chunks", 0, o, S, m, ds, scal, qkv, gates, st.chunks,
               st.chunk_segs, nch, st.chunk_segs.shape[0], h, dk, dv, ld,
               qscale, cap)
     out = torch.empty(n, h * dv, dtype=qkv.dtype, device=qkv.device)
     _call("gh_rec_out", f, 0, out, o, m, qkv, gates, segs, st.pos, st.slot,
           norm, nseg, st.nd, nplain, h, dk, dv, ld, vdim, cap, eps)
+    return out
+
+
+def lightning(rows: torch.Tensor, S: torch.Tensor, decay: torch.Tensor,
+              norm: torch.Tensor, st: StepMeta, vdim: int, eps: float,
+              out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Lightning attention over a step's tokens. rows [H*DK q | H*DK k | H*DV v
+    | H*DV gate | ...] with SiLU on q, k and v already (a column view is fine);
+    decay f32 [2, H]: the decays and their logarithms; S f32 [slots, H, DV, DK]
+    is advanced in place. -> [n, H * DV], in `out` if given."""
+    n, ld = rows.shape[0], rows.stride(0)
+    h, dv, dk = S.shape[1:]
+    _dense(S, decay, norm)
+    assert rows.stride(1) == 1 and rows.shape[1] >= h * (2 * dk + 2 * dv)
+    assert decay.shape == (2, h) and norm.shape == (h * dv,)
+    f, dev = _f32(rows), rows.device
+    if out is None:
+        out = torch.empty(n, h * dv, dtype=rows.dtype, device=dev)
+    assert out.shape == (n, h * dv) and out.stride(1) == 1
+    o = torch.empty(n, h, dv + 4, dtype=torch.float32, device=dev)
+    # the exact mode walks every portion token by token
+    segs, nseg = (st.segs, st.segs.shape[0]) if f and st.segs is not None \
+        else (None, st.nd)
+    if nseg:
+        rpb = 128 if nseg * h * dv >= 128 * 2048 else 32
+        _call("gh_rec_step", f, _CONSTANT, o, S, None, rows, decay[0], segs,
+              st.pos, st.slot, nseg, h, dk, dv, ld, 1.0, 0.0, rpb)
+    if not f and st.chunks is not None:
+        nch = st.chunks.shape[0]
+        ds = torch.empty(nch, h, dv, dk, dtype=torch.float32, device=dev)
+        scal = torch.empty(nch, h, 4, dtype=torch.float32, device=dev)
+        _call("gh_mlstm_chunks", 1, o, S, None, ds, scal, rows, decay[1],
+              st.chunks, st.chunk_segs, nch, st.chunk_segs.shape[0], h, dk, dv,
+              ld, 1.0, 0.0)
+    at = h * (2 * dk + dv)
+    _call("gh_rec_row_out", f, out, o, rows[:, at:], norm, n, h, dv, ld,
+          out.stride(0), h * vdim, eps)
     return out
 
 
@@ -345,9 +472,9 @@ _FEW_PAIRS = 64
 def moe(x: torch.Tensor, logits: torch.Tensor, up: torch.Tensor,
         down: torch.Tensor, how: Union[int, Choice]
         ) -> tuple[torch.Tensor, torch.Tensor, Optional[torch.Tensor]]:
-    """Routed experts. x [n, W]; logits f32 [n, E + identities]; down
-    [E, W, F]; up [E, F, W] with squared ReLU, or [E, 2 F, W] in turns of 16
-    gate | 16 up rows for silu(gate) * up. Returns the chosen experts' outputs
+    """Routed experts. x [n, W]; logits f32 [n, E + identities] (a column view
+    is fine); down [E, W, F]; up [E, F, W] with squared ReLU, or [E, 2 F, W] in
+    turns of 16 gate | 16 up rows for the gated unit how.glu. Returns the chosen experts' outputs
     [n * top, W] in pair order, their weights f32 [n, top] (zero, and the row
     undefined, where the choice is an identity) and the identities' summed
     weights [n]."""
@@ -356,7 +483,9 @@ def moe(x: torch.Tensor, logits: torch.Tensor, up: torch.Tensor,
     n, w = x.shape
     e, rows, ff = up.shape[0], up.shape[1], down.shape[2]
     outs, top = logits.shape[1], how.top
-    _dense(x, logits, up, down, how.corr)
+    _dense(x, up, down, how.corr)
+    assert logits.stride(1) == 1 and logits.dtype == torch.float32
+    assert not (how.sigmoid and (how.corr is not None or outs > e))
     assert rows in (ff, 2 * ff) and up.shape[2] == w == down.shape[1]
     assert outs >= e and (how.corr is None or how.corr.shape == (outs,))
     dev, f = x.device, _f32(x)
@@ -371,14 +500,14 @@ def moe(x: torch.Tensor, logits: torch.Tensor, up: torch.Tensor,
     ident = torch.empty(n, dtype=torch.float32, device=dev) \
         if outs > e else None
     _call("gh_moe_route", idx, wt, rank, counts, order, tiles, logits,
-          how.corr, ident, n, outs, e, top, how.groups, how.keep, how.eps,
-          how.scale, bm, max_tiles)
+          logits.stride(0), how.corr, ident, n, outs, e, top, how.groups,
+          how.keep, how.eps, how.scale, int(how.sigmoid), bm, max_tiles)
     act = torch.empty(pairs, ff, dtype=x.dtype, device=dev)
     _call("gh_moe_gemm", f, rows // ff, act, x, up, tiles, order, top, rows, w,
-          bm, max_tiles)
+          bm, max_tiles, *how.glu, wt if how.weigh_input else None)
     ye = torch.empty(pairs, w, dtype=x.dtype, device=dev)
     _call("gh_moe_gemm", f, 0, ye, act, down, tiles, order, top, w, ff, bm,
-          max_tiles)
+          max_tiles, *how.glu, None)
     return ye, wt, ident
 
 
@@ -479,7 +608,7 @@ def gla(rows: torch.Tensor, u: torch.Tensor, wa2: torch.Tensor,
         else (None, st.nd)
     if nseg:
         rpb = 128 if nseg * h * dv >= 128 * 2048 else 32
-        _call("gh_rec_step", f, o, S, None, rows, b, segs, st.pos, st.slot,
+        _call("gh_rec_step", f, _CHANNELS, o, S, None, rows, b, segs, st.pos, st.slot,
               nseg, h, dk, dv, ld, qscale, 0.0, rpb)
     if nch:
         ds = torch.empty(nch, h, dv, dk, dtype=torch.float32, device=dev)

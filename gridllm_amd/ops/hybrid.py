@@ -8,7 +8,7 @@ import torch
 from gridllm_amd.ops import hip_hybrid, reference_hybrid
 from gridllm_amd.ops import reference
 from gridllm_amd.ops.reference_hybrid import (  # noqa: F401
-    ChunkPortions, Choice, DepthAverage, StepMeta, Talk)
+    ALL_KEYS, ChunkPortions, Choice, DepthAverage, Keys, StepMeta, Talk)
 
 
 def _dispatch(name: str):
@@ -28,8 +28,12 @@ norm_rows = _dispatch("norm_rows")
 group_norm = _dispatch("group_norm")
 join_norm = _dispatch("join_norm")
 poly_norm = _dispatch("poly_norm")
+streams_start = _dispatch("streams_start")
+streams_join = _dispatch("streams_join")
+streams_norm = _dispatch("streams_norm")
 proj_f32 = _dispatch("proj_f32")
 qknorm_kv = _dispatch("qknorm_kv")
+silu_cols = _dispatch("silu_cols")
 paged_attn = _dispatch("paged_attn")
 latent_rows = _dispatch("latent_rows")
 latent_attn = _dispatch("latent_attn")
@@ -37,6 +41,7 @@ talk_rows = _dispatch("talk_rows")
 talk_attn = _dispatch("talk_attn")
 mlstm = _dispatch("mlstm")
 gla = _dispatch("gla")
+lightning = _dispatch("lightning")
 moe = _dispatch("moe")
 
 

@@ -10,6 +10,8 @@ from typing import Optional
 import torch
 import torch.nn.functional as F
 
+from gridllm_amd.ops.reference import SWIGLU, Glu, swiglu
+
 PAGE = 64
 
 
@@ -76,18 +78,40 @@ class StepMeta:
             zip(self.slot.tolist(), self.pos.tolist()))]
 
 
+@dataclass(frozen=True)
+class Keys:
+    """Which keys up to its own a query sees: the last `window` (0: all), its
+    own included, and the first `keep`."""
+    window: int = 0
+    keep: int = 0
+
+    def most(self, length: int) -> int:
+        """Bound of the keys that lie in pages with a seen one."""
+        if not self.window:
+            return length
+        return min(length, self.window + self.keep + 2 * PAGE)
+
+
+ALL_KEYS = Keys()
+
+
 @dataclass
 class Choice:
     """How experts are chosen: `top` of them, by softmax score plus `corr` (f32,
     one per router output), among the `keep` best of `groups` equal groups.
-    Weights are the scores over (their sum + eps), times scale. Router outputs
-    behind the experts are identities."""
+    Weights are the scores over (their sum + eps), times scale; or (sigmoid) the
+    sigmoids of the logits as they are. They go with the experts' outputs, or
+    (weigh_input) are put on their inputs. Router outputs behind the experts are
+    identities. glu: the unit of gated experts."""
     top: int
     corr: Optional[torch.Tensor] = None
     groups: int = 1
     keep: int = 1
     eps: float = 0.0
     scale: float = 1.0
+    sigmoid: bool = False
+    weigh_input: bool = False
+    glu: Glu = SWIGLU
 
 
 @dataclass
@@ -195,6 +219,32 @@ def poly_norm(z, coef, ff, eps):
     return out
 
 
+def streams_start(tok, emb, scale, read, w, width, eps):
+    x = (emb[tok].float() * scale).unsqueeze(1).repeat(1, read.shape[0], 1)
+    return x, _read_streams(x, read, w, width, eps).to(emb.dtype)
+
+
+def _read_streams(x, read, w, width, eps):
+    return _norm(torch.einsum("s,nsw->nw", read, x), w, 0.0, width, eps)
+
+
+def streams_join(x, y, hc, read, w, width, eps, top=0, extra=None):
+    n, ns, _ = x.shape
+    out = y.float().view(n, max(1, top), -1).sum(1)
+    if extra is not None:
+        out = out + extra[0].float() * torch.sigmoid(extra[1])
+    mix, put = hc[:ns * ns].view(ns, ns), hc[ns * ns:]
+    x.copy_(torch.einsum("st,nsw->ntw", mix, x) +
+            put.view(1, ns, 1) * out.unsqueeze(1))
+    return None if w is None else _read_streams(x, read, w, width,
+                                                eps).to(y.dtype)
+
+
+def streams_norm(x, rows, w, width, eps, dtype):
+    z = x if rows is None else x[rows.long()]
+    return _norm(z.sum(1), w, 0.0, width, eps).to(dtype)
+
+
 def proj_f32(x, w, bias=None):
     return F.linear(x.float(), w.float(), bias)
 
@@ -205,7 +255,13 @@ def _rows_of(cache, table, slot, lo, hi):
     return table[slot, p // PAGE].long(), p % PAGE
 
 
-def qknorm_kv(qkv, kc, vc, st, heads, kv_heads, dim, eps, coef, every):
+def silu_cols(rows, at, count):
+    cols = rows[:, at:at + count]
+    cols.copy_(F.silu(cols.float()))
+
+
+def qknorm_kv(qkv, kc, vc, st, heads, kv_heads, dim, eps, coef, every,
+              rot=None, silu=(0, 0)):
     n, p = qkv.shape[0], kc.shape[3]
     cols = qkv[:, :(heads + 2 * kv_heads) * p].float().view(n, -1, p)
     q, k, v = cols.split([heads, kv_heads, kv_heads], dim=1)
@@ -213,6 +269,10 @@ def qknorm_kv(qkv, kc, vc, st, heads, kv_heads, dim, eps, coef, every):
     def unit(z):
         return z * torch.rsqrt(z.pow(2).sum(-1, keepdim=True) / dim + eps)
 
+    if silu[1]:
+        silu_cols(qkv, *silu)
+    if rot is not None:
+        q, k = (_rotate_first(z, st.pos, rot) for z in (q, k))
     steps = torch.div(st.pos + 1, every, rounding_mode="floor").float()
     q = unit(q) * (1 + coef * torch.log(steps + 1)).view(n, 1, 1)
     k = unit(k)
@@ -223,26 +283,31 @@ def qknorm_kv(qkv, kc, vc, st, heads, kv_heads, dim, eps, coef, every):
     return q.to(qkv.dtype)
 
 
-def paged_attn(q, kc, vc, st, scale, sink, gate):
+def paged_attn(q, kc, vc, st, scale, sink, gate, keys=ALL_KEYS, out=None,
+               oscale=1.0):
     n, h, p = q.shape
     g = kc.shape[1]
-    out = torch.empty_like(q)
+    o = torch.empty(n, h, p)
     for off, ln, slot, start in st.entries():
         total = start + ln
         page, row = _rows_of(kc, st.table, slot, 0, total)
         k = kc[page, :, row].float().repeat_interleave(h // g, dim=1)
         v = vc[page, :, row].float().repeat_interleave(h // g, dim=1)
         s = torch.einsum("thd,shd->hts", q[off:off + ln].float(), k) * scale
-        ahead = torch.arange(total).view(1, 1, -1) > \
-            torch.arange(start, total).view(1, -1, 1)
-        s = s.masked_fill(ahead, float("-inf"))
+        j = torch.arange(total).view(1, 1, -1)
+        i = torch.arange(start, total).view(1, -1, 1)
+        hidden = j > i
+        if keys.window:
+            hidden |= (i - j >= keys.window) & (j >= keys.keep)
+        s = s.masked_fill(hidden, float("-inf"))
         if sink is not None:
             s = torch.cat([s, sink.view(h, 1, 1).expand(h, ln, 1)], dim=-1)
         w = torch.softmax(s, dim=-1)[..., :total]
-        out[off:off + ln] = torch.einsum("hts,shd->thd", w, v).to(q.dtype)
+        o[off:off + ln] = torch.einsum("hts,shd->thd", w, v)
     if gate is not None:
-        out *= torch.sigmoid(gate[:, :h].float()).unsqueeze(-1).to(q.dtype)
-    return out
+        o *= torch.sigmoid(gate.float()).view(n, h, -1)
+    o = (o * oscale).to(q.dtype)
+    return o if out is None else out.copy_(o.view(n, h * p))
 
 
 def _rotate(x, pos, rot):
@@ -335,11 +400,30 @@ def mlstm(qkv, gates, S, m, norm, st, dim, vdim, cap, eps):
     return (o.reshape(n, -1) * norm * torch.sigmoid(g)).to(qkv.dtype)
 
 
+def lightning(rows, S, decay, norm, st, vdim, eps, out=None):
+    n = rows.shape[0]
+    h, dv, dk = S.shape[1:]
+    q, k, v, g = rows[:, :h * 2 * (dk + dv)].float().split(
+        [h * dk, h * dk, h * dv, h * dv], dim=1)
+    q, k, v = (t.view(n, h, -1) for t in (q, k, v))
+    keep = decay[0].view(h, 1, 1)
+    o = torch.empty(n, h, dv)
+    for off, ln, slot, start in st.entries():
+        s = torch.zeros_like(S[slot]) if start == 0 else S[slot]
+        for t in range(off, off + ln):
+            s = keep * s + v[t].unsqueeze(2) * k[t].unsqueeze(1)
+            o[t] = torch.matmul(s, q[t].unsqueeze(2)).squeeze(2)
+        S[slot] = s
+    o = (_norm(o.view(n, -1), norm, 0.0, h * vdim, eps) *
+         torch.sigmoid(g)).to(rows.dtype)
+    return o if out is None else out.copy_(o)
+
+
 def moe(x, logits, up, down, how):
     if isinstance(how, int):
         how = Choice(how)
     n, experts = x.shape[0], up.shape[0]
-    s = torch.softmax(logits, dim=-1)
+    s = torch.sigmoid(logits) if how.sigmoid else torch.softmax(logits, dim=-1)
     choice = logits if how.corr is None else s + how.corr
     if how.groups > 1:
         by = choice.view(n, how.groups, -1)
@@ -349,7 +433,8 @@ def moe(x, logits, up, down, how):
         choice = by.masked_fill(out.unsqueeze(-1), float("-inf")).view(n, -1)
     idx = torch.topk(choice, how.top, dim=-1).indices
     wt = s.gather(1, idx)
-    wt = wt / (wt.sum(-1, keepdim=True) + how.eps) * how.scale
+    if not how.sigmoid:
+        wt = wt / (wt.sum(-1, keepdim=True) + how.eps) * how.scale
     ident = None
     if logits.shape[1] > experts:
         same = idx >= experts
@@ -364,9 +449,12 @@ def moe(x, logits, up, down, how):
             continue
         r = (flat == e).nonzero().squeeze(1)
         a = xs[r] @ up[e].float().T
+        if how.weigh_input:
+            a = a * wt.reshape(-1)[r].unsqueeze(1)
         if gated:                          # rows in turns of 16 gate | 16 up
             g, u = a.view(len(r), -1, 2, 16).unbind(2)
-            a = (F.silu(g) * u).reshape(len(r), -1)
+            a = swiglu(torch.cat([g.reshape(len(r), -1),
+                                  u.reshape(len(r), -1)], dim=1), how.glu)
         else:
             a = torch.relu(a) ** 2
         ye[r] = (a @ down[e].float().T).to(x.dtype)
