@@ -502,9 +502,11 @@ def engine_mode(args, rank, world, local_rank, dist, device, on_gpu):
 
 def layers_twin(spec):
     """The closest model of another design at the size of a layer-list model,
-    and its key in the results: Birepel beside Maferax, layer by layer, a Llama
-    of equal active feed-forward size beside Birepel, and of as many
-    feed-forward weights beside Vivepel."""
+    and its key in the results: Birepel beside Maferax, layer by layer, and
+    beside Zinavik, two layers for one (attention, then a recurrence with gated
+    experts, as many as chosen and shared ones); a Llama of equal active
+    feed-forward size beside Birepel, and of as many feed-forward weights beside
+    Vivepel."""
     from gridllm_amd.models.registry import (AttentionMixer, DenseFF,
                                              HybridSpec, LatentMixer,
                                              LayerSpec, MlstmMixer, ModelSpec,
@@ -524,6 +526,21 @@ def layers_twin(spec):
             elif isinstance(ff, RoutedFF):
                 ff = RoutedFF(ff.experts, ff.top, ff.ff)
             layers.append(LayerSpec(mx, ff))
+        return "birepel_twin", HybridSpec(
+            f"{spec.name}-birepel-twin", vocab=spec.vocab, hidden=spec.hidden,
+            layers=tuple(layers), norm_eps=spec.norm_eps,
+            positions=spec.max_seq_len)
+    if spec.family == "zinavik":
+        layers = []
+        for ly in spec.layers:
+            at = None if ly.weights_of is None else 2 * ly.weights_of
+            a, r, ff = ly.mixer.left, ly.mixer.right, ly.ff
+            layers += [
+                LayerSpec(AttentionMixer(a.heads, a.kv_heads, a.dim, a.vdim,
+                                         a.scale), None, at),
+                LayerSpec(MlstmMixer(r.heads, r.dim, r.vdim, 15.0),
+                          RoutedFF(ff.experts, ff.top + 1, ff.ff, gated=True),
+                          None if at is None else at + 1)]
         return "birepel_twin", HybridSpec(
             f"{spec.name}-birepel-twin", vocab=spec.vocab, hidden=spec.hidden,
             layers=tuple(layers), norm_eps=spec.norm_eps,
@@ -648,7 +665,8 @@ def main() -> None:
     ap.add_argument("--model", default="llama3.2:3b")
     ap.add_argument("--layers-model", default="",
                     help="layers: layer-list model to time beside its twin "
-                         "(default birepel:3b; others: maferax:5b, vivepel:2b)")
+                         "(default birepel:3b; others: maferax:5b, vivepel:2b, "
+                         "zinavik:4b)")
     ap.add_argument("--concurrency", type=int, default=1024,
                     help="serving: concurrent streams per GPU")
     ap.add_argument("--num-predict", type=int, default=128,

@@ -2378,6 +2378,7 @@ int gh_proj_f32(void* stream, void* out, const void* x, const void* w,
     // few rows: narrow blocks, so that more of them stream the weights
     if (M <= 512 || N <= 16) GO(1);
     else if (N <= 32) GO(2);
+    else if ((N + 79) / 80 < (N + 63) / 64) GO(5);
     else GO(4);
 #undef GO
     LAUNCH_CHECK();

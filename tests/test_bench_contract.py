@@ -46,7 +46,8 @@ def test_bench_engine_mode_contract():
 @pytest.mark.parametrize("argv,twin", [
     ([], "llama_twin"),
     (["--layers-model", "tiny-maferax"], "birepel_twin"),
-    (["--layers-model", "tiny-vivepel"], "llama_twin")])
+    (["--layers-model", "tiny-vivepel"], "llama_twin"),
+    (["--layers-model", "tiny-zinavik"], "birepel_twin")])
 def test_bench_layers_mode_contract(argv, twin):
     res = _run(["--mode", "layers", "--steps", "1", "--warmup", "1"] + argv)
     assert REQUIRED <= set(res)

@@ -186,7 +186,7 @@ def random_weights(cfg, seed=0, dtype=torch.bfloat16):
 
     def glu(p, ff):
         return {p + "gate": r(ff, wd), p + "up": r(ff, wd),
-                p + "down": r(wd, ff)}
+                p + "down": r(wd, ff, std=0.4 * ff ** -0.5)}
 
     W = {"embed": r(cfg["vocab"], wd, std=1 / cfg["embedding"]["scale"]),
          "final.norm": one()}
@@ -204,9 +204,9 @@ def random_weights(cfg, seed=0, dtype=torch.bfloat16):
               right + "g": r(vr, wd), right + "o": r(wd, vr),
               right + "norm": one(vr)}
         for k in (1, 2) if ml is not None else (1,):
-            W |= {f"{p}norm{k}": one(), f"{p}hc{k}.in": r(s, mean=0.6, std=0.3),
-                  f"{p}hc{k}.out": r(s, mean=0.8, std=0.3),
-                  f"{p}hc{k}.mix": (torch.eye(s) * 0.8 + r(s, s, std=0.25)
+            W |= {f"{p}norm{k}": one(), f"{p}hc{k}.in": r(s, mean=0.6, std=0.2),
+                  f"{p}hc{k}.out": r(s, mean=0.5, std=0.2),
+                  f"{p}hc{k}.mix": (torch.eye(s) * 0.9 + r(s, s, std=0.15)
                                     ).to(dtype)}
         if ml is None:
             continue
