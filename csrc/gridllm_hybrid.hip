@@ -1773,16 +1773,17 @@ k_gla_chunk_out(float* __restrict__ o, const float* __restrict__ dS,
 // Routed experts.
 //   route:   top experts of every token by f32 logits (ties: lower index),
 //            their weights, by softmax or (plain) sigmoids; counts per expert
-//            and each pair's rank. The choice may add a correction per expert to the softmax scores and be
-//            confined to the best of equal groups; router outputs beyond the
-//            experts are identities, whose weights are summed up apart
+//            and each pair's rank. The choice may add a correction per expert
+//            to the softmax scores and be confined to the best of equal groups;
+//            router outputs beyond the experts are identities, whose weights
+//            are summed up apart
 //   scatter: pairs (token * top + k) sorted by expert, and the tile list
 //            {expert, first sorted row, rows, -}; entry max_tiles holds the
 //            number of tiles
 //   gemm:    rows of one expert against its weights, once for the up
 //            projection (gathers token rows, times the pairs' weights if these
-//            go with the input; squared ReLU or a gated unit) and once for the down projection (writes each pair's row back in
-//            pair order)
+//            go with the input; squared ReLU or a gated unit) and once for the
+//            down projection (writes each pair's row back in pair order)
 // The (weighted) sum over a token's pairs is taken in k_post_norm, k_sum_norm
 // or k_streams_join.
 // ===========================================================================
@@ -1982,8 +1983,9 @@ DEV_INLINE bool moe_work(const int4* tiles, int max_tiles, int ntn, int4& tl,
 // ACT != 0 (up projection): row r of the tile is token sorted[row0 + r] / top,
 // output in sorted order through squared ReLU (1) or, with weight rows in turns
 // of 16 gate | 16 up, the gated unit `glu` in N / 2 columns (2); pw (nullable):
-// a weight per pair on the unit's input. ACT 0: row r is sorted row row0 + r and its output goes to pair order. The MFMA computes
-// W x^T, so a lane ends up with 4 neighbouring columns of one row.
+// a weight per pair on the unit's input. ACT 0: row r is sorted row row0 + r and
+// its output goes to pair order. The MFMA computes W x^T, so a lane ends up with
+// 4 neighbouring columns of one row.
 // K % 64 == 0, N % 64 == 0 (ACT 2: N % 128 == 0).
 template <int ACT, int NB>
 __global__ void __launch_bounds__(256, 2)
@@ -2683,12 +2685,12 @@ int gh_gla_chunks(void* stream, void* o, void* S, void* dS, const void* qkv,
 }
 
 // E router outputs (rows of stride ldz), of which the first `experts` have
-// weights. corr (nullable): correction of the choice; ident (nullable): sum of a token's weights beyond
-// the experts
+// weights. corr (nullable): correction of the choice; ident (nullable): sum of
+// a token's weights beyond the experts
 int gh_moe_route(void* stream, void* idx, void* wt, void* rank, void* counts,
                  void* sorted, void* tiles, const void* z, int ldz,
-                 const void* corr, void* ident, int N, int E, int experts, int top, int groups,
-                 int keep, float eps, float scale, int sigmoid, int bm,
+                 const void* corr, void* ident, int N, int E, int experts,
+                 int top, int groups, int keep, float eps, float scale, int sigmoid, int bm,
                  int max_tiles) {
     if (ldz < E || (sigmoid && (corr || ident))) return -100;
     if (N < 1 || E < 1 || E > 1024 || top < 1 || experts < 1 || experts > E ||

@@ -711,14 +711,14 @@ def _read_zinavik_layer(i: int, ly: dict) -> LayerSpec:
     a = _take(d["left"], "left", ("heads", "kv_heads", "dim", "vdim", "scale",
                                   "rot", "mask"))
     b = _take(d["right"], "right", ("heads", "dim", "vdim", "decay"))
-    mask = _take(a["mask"], "mask", ("size", "keep_first"))
+    mask = _take(a["mask"], "mask", ("size",), ("keep_first",))
     if mask["size"] < 1:
         raise ValueError(f"config: a window of {mask['size']}")
     mixer = ParallelMixer(
         AttentionMixer(heads=a["heads"], kv_heads=a["kv_heads"], dim=a["dim"],
                        vdim=a["vdim"], scale=float(a["scale"]),
                        rot=_read_rotary(a["rot"]), window=mask["size"],
-                       keep_first=mask["keep_first"], sink=False,
+                       keep_first=mask.get("keep_first") or 0, sink=False,
                        gate="element"),
         LightningMixer(b["heads"], b["dim"], b["vdim"],
                        tuple(float(x) for x in b["decay"])),

@@ -24,7 +24,8 @@ ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950")
 
 # library name -> source. "hip": what every model shares and the Llama
 # family's attention; "hybrid": layer-list models (paged attention, mLSTM,
-# gated linear attention, routed experts); "latent": their latent attention;
+# gated linear and lightning attention, routed experts, residual streams);
+# "latent": their latent attention;
 # "talk": their talking-heads attention
 LIBS = {"hip": "gridllm_kernels.hip", "hybrid": "gridllm_hybrid.hip",
         "latent": "gridllm_latent.hip", "talk": "gridllm_talk.hip"}

@@ -409,8 +409,8 @@ def mlstm(qkv: torch.Tensor, gates: torch.Tensor, S: torch.Tensor,
         # rows of the state per block: more for large batches, where the grid
         # is full anyway and a block amortises its loads of q and k
         rpb = 128 if nseg * h * (dv + 1) >= 128 * 2048 else 32
-        _call("gh_rec_step", f, _MLSTM, o, S, m, qkv, gates, segs, st.pos, st.slot,
-              nseg, h, dk, dv, ld, qscale, cap, rpb)
+        _call("gh_rec_step", f, _MLSTM, o, S, m, qkv, gates, segs, st.pos,
+              st.slot, nseg, h, dk, dv, ld, qscale, cap, rpb)
     nplain = 0
     if not f and st.chunks is not None:
         nplain = n - st.nd
@@ -474,10 +474,10 @@ def moe(x: torch.Tensor, logits: torch.Tensor, up: torch.Tensor,
         ) -> tuple[torch.Tensor, torch.Tensor, Optional[torch.Tensor]]:
     """Routed experts. x [n, W]; logits f32 [n, E + identities] (a column view
     is fine); down [E, W, F]; up [E, F, W] with squared ReLU, or [E, 2 F, W] in
-    turns of 16 gate | 16 up rows for the gated unit how.glu. Returns the chosen experts' outputs
-    [n * top, W] in pair order, their weights f32 [n, top] (zero, and the row
-    undefined, where the choice is an identity) and the identities' summed
-    weights [n]."""
+    turns of 16 gate | 16 up rows for the gated unit how.glu. Returns the chosen
+    experts' outputs [n * top, W] in pair order, their weights f32 [n, top]
+    (zero, and the row undefined, where the choice is an identity) and the
+    identities' summed weights [n]."""
     if isinstance(how, int):
         how = Choice(how)
     n, w = x.shape
@@ -608,8 +608,8 @@ def gla(rows: torch.Tensor, u: torch.Tensor, wa2: torch.Tensor,
         else (None, st.nd)
     if nseg:
         rpb = 128 if nseg * h * dv >= 128 * 2048 else 32
-        _call("gh_rec_step", f, _CHANNELS, o, S, None, rows, b, segs, st.pos, st.slot,
-              nseg, h, dk, dv, ld, qscale, 0.0, rpb)
+        _call("gh_rec_step", f, _CHANNELS, o, S, None, rows, b, segs, st.pos,
+              st.slot, nseg, h, dk, dv, ld, qscale, 0.0, rpb)
     if nch:
         ds = torch.empty(nch, h, dv, dk, dtype=torch.float32, device=dev)
         _call("gh_gla_chunks", o, S, ds, rows, b, st.chunks, st.chunk_segs,
