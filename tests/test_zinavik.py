@@ -139,7 +139,7 @@ ALONE = {
     "wide-state": config((mixer(b=right(2, 300, 200, (0.8, 0.99))), None)),
     "experts": config((mixer(), moe(shared=0))),
     "shared": config((mixer(), moe())),
-    "top-one": config((mixer(), moe(16, 1))),
+    "top-one": config((mixer(), moe(19, 1))),
     "all-experts": config((mixer(), moe(5, 5))),
     "loose-limits": config((mixer(), moe(limit=50.0, shared_limit=50.0))),
     "tight-limits": config((mixer(), moe(limit=0.1, shared_limit=0.05))),
@@ -303,7 +303,7 @@ def test_streams(width, ns, run):
 
 @pytest.mark.parametrize("run", RUNS)
 @pytest.mark.parametrize("n", [1, 7, 90])
-@pytest.mark.parametrize("experts,top", [(6, 2), (16, 1), (70, 5)])
+@pytest.mark.parametrize("experts,top", [(6, 2), (19, 1), (70, 5)])
 def test_weights_on_the_experts_inputs(experts, top, n, run):
     """Small and large weights against tight limits: weighting the output
     instead, or summing the weights to one, would show."""
@@ -343,7 +343,7 @@ CUTS = {"whole": [330], "decode-tail": [185, 1], "pairs": [250, 2],
 @pytest.mark.parametrize("run", RUNS)
 @pytest.mark.parametrize("how", sorted(CUTS))
 @pytest.mark.parametrize("sizes", [
-    (4, 2, 64, 40, 100, 7, 64), (24, 8, 128, 128, 64, 64, 32),
+    (6, 2, 64, 40, 100, 7, 64), (24, 8, 128, 128, 64, 64, 32),
     (11, 1, 48, 64, 33, 0, 16), (2, 1, 160, 200, 1, 90, 96),
     (3, 3, 20, 20, 500, 2, 20)], ids=str)
 def test_one_key_stands_out(sizes, how, run):
